@@ -1,0 +1,365 @@
+// Kernels of the gated delta rule with a decay per key channel (gfx950).
+//
+// The mixer's products leave, per token, [q | k | v | b] (proj) and [z | gate] (up).
+//
+// delta_inputs: q, k and v pass a short causal convolution per channel and SiLU (the last tap meets the token
+//   itself; the inputs before a step's first token come from the request's state, zeros at a sequence's start); q
+//   and k become unit vectors per head, x / sqrt(sum(x^2) + 1e-6), q times q_scale; the decay of a key channel is
+//   exp(-exp(A_log) softplus(z + dt_bias)); beta = sigmoid(b).  All of it lands in one float32 row per token,
+//   [q: kv dim | k: kv dim | v: heads vdim | decay: heads dim | beta: heads], rounded up to a multiple of four.
+// delta_scan: per (request, head), over the step's tokens in order, with the state S [dim, vdim] in float32
+//   registers (q and k of kv head head / (heads / kv)):
+//     S <- diag(decay) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
+//
+// Convolution, norms, decays with their exponentials, beta, the recurrence and its state are float32 whatever
+// the storage type.
+#include "common.h"
+#include "short_conv.h"
+#include "slots.h"
+
+using namespace tk;
+
+namespace {
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));   // (arrays of HIP's float4 struct may end up in scratch)
+
+constexpr int kSegment = 16;      // tokens of a request that a wave of delta_inputs walks
+constexpr float kUnitEps = 1e-6f;
+
+struct DeltaShape {
+  int heads, kv, dim, vdim, taps;
+  __host__ __device__ int conv_channels() const { return 2 * kv * dim + heads * vdim; }
+  __host__ __device__ int row() const { return (2 * kv * dim + heads * vdim + heads * dim + heads + 3) / 4 * 4; }   // (whole 16-byte pieces)
+};
+
+// A wave a unit (a q or k head, or a run of 64 * CPL channels of v or of the decays) and a segment of a request's
+// tokens: a lane walks CPL channels with the taps' inputs in registers.  grid (units / 4, requests, segments).
+// update: a request's tokens are this one segment, whose wave also writes the convolution's new state.
+template <typename T, int CPL>
+__global__ __launch_bounds__(256) void delta_inputs_kernel(
+    RowsIn proj, long ld, RowsIn up, long uld, const float* __restrict__ conv, float* __restrict__ state,
+    const float* __restrict__ a_log, const float* __restrict__ dt_bias, const int* __restrict__ q_start,
+    const int* __restrict__ state_slots, float* __restrict__ out, DeltaShape sh, float q_scale, int update) {
+  const int lane = threadIdx.x & (kWave - 1);
+  int unit = blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
+  const int req = blockIdx.y;
+  const int first = q_start[req], end = q_start[req + 1];
+  const int t_lo = first + blockIdx.z * kSegment, t_hi = min(end, t_lo + kSegment);
+  if (t_lo >= end) return;                 // (nothing below synchronises across waves)
+  constexpr int RUN = kWave * CPL;
+  const int kdim = sh.kv * sh.dim, vall = sh.heads * sh.vdim, gall = sh.heads * sh.dim;
+  const int vunits = (vall + RUN - 1) / RUN, gunits = (gall + RUN - 1) / RUN;
+  const int C = sh.conv_channels(), row = sh.row(), taps = sh.taps;
+  if (unit >= 2 * sh.kv + vunits) {
+    unit -= 2 * sh.kv + vunits;
+    if (unit >= gunits) return;
+    // decays, and (its first unit) the heads' step sizes
+    float* dst = out + C;
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) {
+      const int c = unit * RUN + i * kWave + lane;
+      if (c < gall) {
+        const float rate = expf(a_log[c / sh.dim]), bias = dt_bias[c];
+        for (int t = t_lo; t < t_hi; ++t)
+          dst[(size_t)t * row + c] = expf(-rate * softplus(load_in<T>(up, (size_t)t * uld + c) + bias));
+      }
+    }
+    if (unit == 0) {
+      for (int i = lane; i < (t_hi - t_lo) * sh.heads; i += kWave) {
+        const int t = t_lo + i / sh.heads, head = i % sh.heads;
+        out[(size_t)t * row + C + gall + head] = sigmoid(load_in<T>(proj, (size_t)t * ld + C + head));
+      }
+    }
+    return;
+  }
+  const bool qk = unit < 2 * sh.kv;
+  const int col0 = qk ? unit * sh.dim : 2 * kdim + (unit - 2 * sh.kv) * RUN;     // (q's heads, then k's)
+  const int count = qk ? sh.dim : min(RUN, vall - (unit - 2 * sh.kv) * RUN);
+  const float scale = unit < sh.kv ? q_scale : 1.f;
+  float* st = taps > 1 ? state + (size_t)state_slots[req] * (taps - 1) * C + col0 : nullptr;
+  // taps and window sit at the END of arrays of kMaxTaps: index kMaxTaps - 1 is the token itself
+  float wv[CPL][kMaxTaps], win[CPL][kMaxTaps];
+#pragma unroll
+  for (int i = 0; i < CPL; ++i) {
+    const int c = i * kWave + lane;
+#pragma unroll
+    for (int k = 0; k < kMaxTaps; ++k) {
+      const int j = k - (kMaxTaps - taps);
+      wv[i][k] = (j >= 0 && c < count) ? conv[(size_t)(col0 + c) * taps + j] : 0.f;
+      win[i][k] = 0.f;
+    }
+#pragma unroll
+    for (int d = 1; d < kMaxTaps; ++d) {
+      if (d < taps && c < count) {
+        const int local = t_lo - first - d;     // the input d positions before the segment's first token
+        win[i][kMaxTaps - d] = local >= 0 ? load_in<T>(proj, (size_t)(t_lo - d) * ld + col0 + c)
+                                          : st[(size_t)(taps - 1 + local) * C + c];
+      }
+    }
+  }
+  for (int t = t_lo; t < t_hi; ++t) {
+    float y[CPL];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) {
+      const int c = i * kWave + lane;
+#pragma unroll
+      for (int k = 0; k < kMaxTaps - 1; ++k) win[i][k] = win[i][k + 1];
+      win[i][kMaxTaps - 1] = c < count ? load_in<T>(proj, (size_t)t * ld + col0 + c) : 0.f;
+      float acc = 0.f;
+#pragma unroll
+      for (int k = 0; k < kMaxTaps; ++k) acc = fmaf(wv[i][k], win[i][k], acc);
+      y[i] = silu(acc);        // (channels behind the unit's: zero)
+      ss = fmaf(y[i], y[i], ss);
+    }
+    float r = 1.f;
+    if (qk) r = scale / sqrtf(wave_sum(ss) + kUnitEps);
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) {
+      const int c = i * kWave + lane;
+      if (c < count) out[(size_t)t * row + col0 + c] = y[i] * r;
+    }
+  }
+  if (update) {      // (the window now ends at the request's last token)
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) {
+      const int c = i * kWave + lane;
+#pragma unroll
+      for (int k = 1; k < kMaxTaps; ++k) {
+        const int j = k - (kMaxTaps - (taps - 1));
+        if (j >= 0 && c < count) st[(size_t)j * C + c] = win[i][k];
+      }
+    }
+  }
+}
+
+// Sum over each run of 16 neighbouring lanes, in every lane of the run: quads by permutation, then the mirrored
+// half of eight and of sixteen (after each step all lanes of the mirrored group hold the same number).
+template <int CTRL>
+__device__ __forceinline__ float lane_move(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float sum16(float v) {
+  v += lane_move<0xB1>(v);       // quad_perm [1, 0, 3, 2]
+  v += lane_move<0x4E>(v);       // quad_perm [2, 3, 0, 1]
+  v += lane_move<0x141>(v);      // row_half_mirror
+  v += lane_move<0x140>(v);      // row_mirror
+  return v;
+}
+
+constexpr int kLanes = 16;        // lanes that share a value column
+constexpr int kColumns = 16;      // value columns of a block of four waves
+constexpr int kScanThreads = 256;
+
+// One round's operands, tokens t0 .. t0 + tb, on their way from memory: piece e of the round is
+// [k | q | decay] as [TB][DP / 4] each, then v as [TB][4].  *_at: where they lie in a token's row; columns: the value
+// columns that exist from the block's first one on.
+template <int PER, int TB, int DP, bool WIDE>
+__device__ __forceinline__ void fetch_round(const float* __restrict__ in, int row, int k_at, int q_at, int g_at,
+                                            int v_at, int b_at, int dim, int columns, int t0, int tb,
+                                            f32x4 (&held)[PER], float& beta) {
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = i * kScanThreads + threadIdx.x;
+    int t, c, most, from;
+    if (e < 3 * TB * DP / 4) {
+      const int set = e / (TB * DP / 4), in_set = e - set * (TB * DP / 4);
+      t = in_set / (DP / 4);
+      c = (in_set - t * (DP / 4)) * 4;
+      most = dim;
+      from = set == 0 ? k_at : set == 1 ? q_at : g_at;
+    } else {
+      t = (e - 3 * TB * DP / 4) / (kColumns / 4);
+      c = ((e - 3 * TB * DP / 4) - t * (kColumns / 4)) * 4;
+      most = columns;
+      from = v_at;
+    }
+    if (t >= tb) most = 0;
+    const float* p = in + (size_t)(t0 + t) * row + from + c;
+    held[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (WIDE) {
+      if (c < most) held[i] = *reinterpret_cast<const f32x4*>(p);
+    } else {
+      if (c < most) held[i].x = p[0];
+      if (c + 1 < most) held[i].y = p[1];
+      if (c + 2 < most) held[i].z = p[2];
+      if (c + 3 < most) held[i].w = p[3];
+    }
+  }
+  beta = (int)threadIdx.x < tb ? in[(size_t)(t0 + threadIdx.x) * row + b_at] : 0.f;
+}
+
+// A block a (request, head, 16 value columns).  The 16 neighbouring lanes that share a column hold its rows of the
+// state in registers, PIECES pieces of four rows a lane (lane l: rows 64 i + 4 l .. + 4), so that both dot
+// products of a token are sums of 4 PIECES multiply-adds and four lane moves, with no LDS and no barrier in
+// between.  The tokens' k, q and decays are staged in LDS, TB at a time, the next round's on their way
+// to registers meanwhile; the columns of a head never meet, so a head's blocks run side by side.
+// The state lies as [head][column][dim rounded up to 4].
+// WIDE: dim and vdim are multiples of four, so that rows are read in 16-byte pieces.
+template <int PIECES, int TB, bool WIDE>
+__global__ __launch_bounds__(kScanThreads) void delta_scan_kernel(
+    const float* __restrict__ in, float* __restrict__ state, const int* __restrict__ q_start,
+    const int* __restrict__ state_slots, float* __restrict__ y, DeltaShape sh) {
+  constexpr int DP = kLanes * 4 * PIECES;      // rows with the padding (zeros behind dim)
+  constexpr int SET = TB * DP;
+  constexpr int ALL = (3 * SET + TB * kColumns) / 4;      // pieces of four numbers that a round stages
+  constexpr int PER = (ALL + kScanThreads - 1) / kScanThreads;
+  __shared__ __attribute__((aligned(16))) float lds[3 * SET + TB * kColumns + TB];
+  float* vv = lds + 3 * SET;
+  float* bb = vv + TB * kColumns;
+  const int req = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
+  const int first = q_start[req], end = q_start[req + 1];
+  const int ks = tid & (kLanes - 1), jl = tid / kLanes;
+  const int col0 = blockIdx.z * kColumns, j = col0 + jl;
+  const int dim = sh.dim, vdim = sh.vdim, row = sh.row();
+  const int rows4 = (dim + 3) & ~3;
+  const bool owns = j < vdim;
+  const int kvh = head / (sh.heads / sh.kv);
+  const int kdim = sh.kv * dim, gall = sh.heads * dim;
+  const int behind = 2 * kdim + sh.heads * vdim;      // of q, k and v
+  const int q_at = kvh * dim, k_at = kdim + q_at, v_at = 2 * kdim + head * vdim + col0, g_at = behind + head * dim;
+  const int b_at = behind + gall + head;
+  float* S = state + (((size_t)state_slots[req] * sh.heads + head) * vdim + (owns ? j : 0)) * rows4;
+  f32x4 s[PIECES];
+#pragma unroll
+  for (int i = 0; i < PIECES; ++i) {
+    const int r = i * (kLanes * 4) + ks * 4;
+    s[i] = owns && r < rows4 ? *reinterpret_cast<const f32x4*>(S + r) : f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  f32x4 held[PER];
+  float held_beta = 0.f;
+  fetch_round<PER, TB, DP, WIDE>(in, row, k_at, q_at, g_at, v_at, b_at, dim, vdim - col0, first, min(TB, end - first), held, held_beta);
+  for (int t0 = first; t0 < end; t0 += TB) {
+    const int tb = min(TB, end - t0);
+    __syncthreads();     // (the round before has been read)
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int e = i * kScanThreads + tid;
+      if (e < ALL) *reinterpret_cast<f32x4*>(lds + 4 * e) = held[i];
+    }
+    if (tid < TB) bb[tid] = held_beta;
+    __syncthreads();
+    if (t0 + TB < end) fetch_round<PER, TB, DP, WIDE>(in, row, k_at, q_at, g_at, v_at, b_at, dim, vdim - col0, t0 + TB,
+                                                      min(TB, end - t0 - TB), held, held_beta);
+    float kept = 0.f;
+    for (int t = 0; t < tb; ++t) {
+      f32x4 k[PIECES], g[PIECES], q[PIECES];
+#pragma unroll
+      for (int i = 0; i < PIECES; ++i) {
+        const int piece = t * DP + i * (kLanes * 4) + ks * 4;
+        k[i] = *reinterpret_cast<const f32x4*>(lds + piece);
+        g[i] = *reinterpret_cast<const f32x4*>(lds + 2 * SET + piece);
+        q[i] = *reinterpret_cast<const f32x4*>(lds + SET + piece);
+      }
+      const float beta = bb[t], v = vv[t * kColumns + jl];
+      float d0 = 0.f, d1 = 0.f;
+#pragma unroll
+      for (int i = 0; i < PIECES; ++i) {
+        s[i] *= g[i];
+        d0 = fmaf(s[i].x, k[i].x, d0);
+        d1 = fmaf(s[i].y, k[i].y, d1);
+        d0 = fmaf(s[i].z, k[i].z, d0);
+        d1 = fmaf(s[i].w, k[i].w, d1);
+      }
+      const float u = beta * (v - sum16(d0 + d1));
+      float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+      for (int i = 0; i < PIECES; ++i) {
+        s[i] = f32x4{fmaf(k[i].x, u, s[i].x), fmaf(k[i].y, u, s[i].y), fmaf(k[i].z, u, s[i].z), fmaf(k[i].w, u, s[i].w)};
+        o0 = fmaf(s[i].x, q[i].x, o0);
+        o1 = fmaf(s[i].y, q[i].y, o1);
+        o0 = fmaf(s[i].z, q[i].z, o0);
+        o1 = fmaf(s[i].w, q[i].w, o1);
+      }
+      const float o = sum16(o0 + o1);
+      if (ks == t) kept = o;      // (lane t of a column keeps token t's output: one store a round)
+    }
+    static_assert(TB <= kLanes, "a lane of a column keeps one token's output");
+    if (owns && ks < tb) y[(size_t)(t0 + ks) * sh.heads * vdim + (size_t)head * vdim + j] = kept;
+  }
+  if (owns) {
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i) {
+      const int r = i * (kLanes * 4) + ks * 4;
+      if (r < rows4) *reinterpret_cast<f32x4*>(S + r) = s[i];
+    }
+  }
+}
+
+template <typename T>
+int launch_inputs(RowsIn proj, long ld, RowsIn up, long uld, const float* conv, float* state, const float* a_log,
+                  const float* dt_bias, const int* q_start, const int* slots, float* out, int R, DeltaShape sh,
+                  float q_scale, int max_tokens, hipStream_t stream) {
+  const int segments = (max_tokens + kSegment - 1) / kSegment;
+  const int update = segments == 1 && sh.taps > 1;
+  const int cpl = sh.dim <= 64 ? 1 : sh.dim <= 128 ? 2 : sh.dim <= 256 ? 4 : 8;
+  const int run = kWave * cpl;
+  const long units = 2L * sh.kv + ((long)sh.heads * sh.vdim + run - 1) / run + ((long)sh.heads * sh.dim + run - 1) / run;
+  const dim3 grid((unsigned)((units + 3) / 4), R, segments);
+  if (grid.y > 65535 || grid.z > 65535) return -1;
+#define TK_DI(CPL)                                                                                              \
+  delta_inputs_kernel<T, CPL><<<grid, 256, 0, stream>>>(proj, ld, up, uld, conv, state, a_log, dt_bias, q_start, \
+                                                        slots, out, sh, q_scale, update)
+  if (cpl == 1) TK_DI(1);
+  else if (cpl == 2) TK_DI(2);
+  else if (cpl == 4) TK_DI(4);
+  else TK_DI(8);
+#undef TK_DI
+  if (!update && sh.taps > 1) {
+    const int C = sh.conv_channels();
+    conv_carry_kernel<T><<<dim3((C + 255) / 256, R), 256, 0, stream>>>(proj, ld, 0, state, q_start, slots, C, sh.taps);
+  }
+  return launch_status();
+}
+
+}  // namespace
+
+// proj: [N, ld] in dtype, float32 (in_f32) or float32 partial sums, its columns [q: kv dim | k: kv dim | v: heads vdim |
+// b: heads | ...]; up: [N, uld] likewise, its first heads * dim columns the decays' pre-activations.  conv float32
+// [2 kv dim + heads vdim, taps]; state float32 [slots, taps - 1, 2 kv dim + heads vdim]; a_log float32 [heads], dt_bias
+// float32 [heads * dim]; out float32 [N, 2 kv dim + heads vdim + heads dim + heads rounded up to four].
+// max_tokens: the most tokens a request brings to the step.
+TK_API int tk_delta_inputs(int dtype, const void* proj, int in_f32, int parts, long part_stride, long ld, const void* up,
+                           int up_f32, int up_parts, long up_stride, long uld, const float* conv, float* state,
+                           const float* a_log, const float* dt_bias, const int* q_start, const int* state_slots,
+                           float* out, int R, int heads, int kv, int dim, int vdim, int taps, float q_scale,
+                           int max_tokens, hipStream_t stream) {
+  if (R <= 0 || max_tokens <= 0) return 0;
+  const DeltaShape sh{heads, kv, dim, vdim, taps};
+  if (heads < 1 || kv < 1 || heads % kv != 0 || dim < 1 || dim > 512 || vdim < 1 || taps < 1 || taps > kMaxTaps ||
+      (taps > 1 && state == nullptr) || parts < 1 || (parts > 1 && !in_f32) || up_parts < 1 || (up_parts > 1 && !up_f32) ||
+      ld < (long)sh.conv_channels() + heads || uld < (long)heads * dim)
+    return -1;
+  const RowsIn p{proj, in_f32 || dtype == 0, parts, part_stride}, u{up, up_f32 || dtype == 0, up_parts, up_stride};
+  if (dtype == 0)
+    return launch_inputs<float>(p, ld, u, uld, conv, state, a_log, dt_bias, q_start, state_slots, out, R, sh, q_scale,
+                                max_tokens, stream);
+  return launch_inputs<bf16_t>(p, ld, u, uld, conv, state, a_log, dt_bias, q_start, state_slots, out, R, sh, q_scale,
+                               max_tokens, stream);
+}
+
+// in: what tk_delta_inputs left; state float32 [slots, heads, vdim, dim rounded up to 4]; y float32 [N, heads * vdim].
+TK_API int tk_delta_scan(const float* in, float* state, const int* q_start, const int* state_slots, float* y, int R,
+                         int heads, int kv, int dim, int vdim, hipStream_t stream) {
+  if (R <= 0) return 0;
+  if (heads < 1 || heads > 65535 || kv < 1 || heads % kv != 0 || dim < 1 || dim > 512 || vdim < 1) return -1;
+  const DeltaShape sh{heads, kv, dim, vdim, 1};
+  const dim3 grid(R, heads, (vdim + kColumns - 1) / kColumns);
+  if (grid.z > 65535) return -1;
+  const bool wide = dim % 4 == 0 && vdim % 4 == 0 && (uintptr_t)in % 16 == 0;
+#define TK_DS(PIECES, TB)                                                                                              \
+  {                                                                                                                    \
+    if (wide) delta_scan_kernel<PIECES, TB, true><<<grid, kScanThreads, 0, stream>>>(in, state, q_start, state_slots, y, sh); \
+    else delta_scan_kernel<PIECES, TB, false><<<grid, kScanThreads, 0, stream>>>(in, state, q_start, state_slots, y, sh);     \
+  }
+  if (dim <= 64) TK_DS(1, 16)
+  else if (dim <= 128) TK_DS(2, 16)
+  else if (dim <= 192) TK_DS(3, 8)
+  else if (dim <= 256) TK_DS(4, 8)
+  else TK_DS(8, 4)
+#undef TK_DS
+  return launch_status();
+}
+
+TK_SLOTS(tk_delta_inputs)
+TK_SLOTS(tk_delta_scan)

@@ -40,6 +40,44 @@ TK_API int tk_embed_gather(int dtype, const void* table, const int* ids, float* 
   return launch_status();
 }
 
+// resid[n, :] (+)= r / sqrt(mean(r^2) + eps) * weight with r = float(table[ids[n], :]) * scale: an embedding with a
+// norm of its own.  A block a token; the row is read twice (the second time from the cache).
+template <typename T>
+__global__ __launch_bounds__(256) void embed_norm_kernel(const T* __restrict__ table, const int* __restrict__ ids,
+                                                         const float* __restrict__ weight, float* __restrict__ resid,
+                                                         int H, int V, float scale, float eps, int accumulate) {
+  __shared__ float scratch[16];
+  const int n = blockIdx.x;
+  const int id = ids[n];
+  float* out = resid + (size_t)n * H;
+  if (id < 0 || id >= V) {      // (the whole block, before any barrier)
+    for (int d = threadIdx.x; d < H; d += blockDim.x) out[d] = __uint_as_float(0x7fc00000u);
+    return;
+  }
+  const T* row = table + (size_t)id * H;
+  float ss = 0.f;
+  for (int d = threadIdx.x; d < H; d += blockDim.x) {
+    const float v = Elem<T>::load(row + d) * scale;
+    ss = fmaf(v, v, ss);
+  }
+  ss = block_sum(ss, scratch);
+  const float rstd = 1.f / sqrtf(ss / (float)H + eps);
+  for (int d = threadIdx.x; d < H; d += blockDim.x) {
+    const float v = Elem<T>::load(row + d) * scale * rstd * weight[d];
+    out[d] = accumulate ? out[d] + v : v;
+  }
+}
+
+TK_API int tk_embed_norm(int dtype, const void* table, const int* ids, const float* weight, float* resid, int N, int H,
+                         int V, float scale, float eps, int accumulate, hipStream_t stream) {
+  if (N <= 0) return 0;
+  if (dtype == 0)
+    embed_norm_kernel<float><<<N, 256, 0, stream>>>((const float*)table, ids, weight, resid, H, V, scale, eps, accumulate);
+  else
+    embed_norm_kernel<bf16_t><<<N, 256, 0, stream>>>((const bf16_t*)table, ids, weight, resid, H, V, scale, eps, accumulate);
+  return launch_status();
+}
+
 // ---------------------------------------------------------------------------
 // Token ids that are still on the GPU: ids[slots[i]] = sampled[rows[i]].  A step may be
 // launched before the host has read the tokens that the step before it sampled; its
@@ -537,16 +575,19 @@ TK_API int tk_qknorm_rope_store(int dtype, const void* qkv, int in_f32, int part
 
 // ---------------------------------------------------------------------------
 // out[n, i] = act(gu[n, i]) * gu[n, I + i]; act 0: silu(z) = z / (1 + exp(-z)), act 1: the tanh
-// form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
+// form of gelu, 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))).  act 2, a gate with clamped halves:
+// with g = min(gu[n, i], limit) and u = clamp(gu[n, I + i], -limit, limit), out = g sigmoid(1.702 g) (u + 1)
 // ---------------------------------------------------------------------------
-__device__ __forceinline__ float gate_act(float z, int act) {
-  if (act == 0) return z / (1.f + expf(-z));
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+__device__ __forceinline__ float gated_value(float z, float u, int act, float limit) {
+  if (act == 0) return z / (1.f + expf(-z)) * u;
+  if (act == 1) return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) * u;
+  const float g = fminf(z, limit);
+  return g / (1.f + expf(-1.702f * g)) * (fminf(fmaxf(u, -limit), limit) + 1.f);
 }
 
 template <typename T>
 __global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total, int act,
-                                const float* __restrict__ bias) {
+                                float limit, const float* __restrict__ bias) {
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const size_t n = idx / I;
@@ -557,7 +598,7 @@ __global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, i
     g += bias[i];
     u += bias[I + i];
   }
-  Elem<T>::store(out + idx, gate_act(g, act) * u);
+  Elem<T>::store(out + idx, gated_value(g, u, act, limit));
 }
 
 // x[n, c] += bias[c] in place (float32 bias, the sum formed in float32)
@@ -570,7 +611,7 @@ __global__ void add_bias_kernel(T* __restrict__ x, const float* __restrict__ bia
 
 // 8 elements a thread (16-byte loads): I a multiple of 8, pointers 16-byte aligned
 __global__ void silu_mul_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __restrict__ out,
-                                       int I, size_t total8, int act) {
+                                       int I, size_t total8, int act, float limit) {
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total8) return;
   const int per_row = I / 8;
@@ -584,7 +625,7 @@ __global__ void silu_mul_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __
   for (int k = 0; k < 4; ++k) {
     const float g0 = __uint_as_float(gw[k] << 16), g1 = __uint_as_float(gw[k] & 0xffff0000u);
     const float u0 = __uint_as_float(uw[k] << 16), u1 = __uint_as_float(uw[k] & 0xffff0000u);
-    ow[k] = pack_bf16x2(gate_act(g0, act) * u0, gate_act(g1, act) * u1);
+    ow[k] = pack_bf16x2(gated_value(g0, u0, act, limit), gated_value(g1, u1, act, limit));
   }
   *reinterpret_cast<uint4*>(out + n * I + i) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
 }
@@ -599,22 +640,22 @@ TK_API int tk_add_bias(int dtype, void* x, const float* bias, int N, int H, hipS
 }
 
 // bias: null, or float32 [2 I] added to the gate's and the up projection's halves before the activation
-TK_API int tk_silu_mul(int dtype, const void* gu, void* out, int N, int I, int act, const float* bias,
+TK_API int tk_silu_mul(int dtype, const void* gu, void* out, int N, int I, int act, float limit, const float* bias,
                        hipStream_t stream) {
   if (N <= 0 || I <= 0) return 0;
-  if (act != 0 && act != 1) return -1;
+  if (act < 0 || act > 2) return -1;
   const size_t total = (size_t)N * I;
   if (bias == nullptr && dtype == 1 && I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0) {
     const size_t total8 = total / 8;
     silu_mul_bf16x8_kernel<<<(unsigned)((total8 + 255) / 256), 256, 0, stream>>>(
-        (const bf16_t*)gu, (bf16_t*)out, I, total8, act);
+        (const bf16_t*)gu, (bf16_t*)out, I, total8, act, limit);
     return launch_status();
   }
   const unsigned blocks = (unsigned)((total + 255) / 256);
   if (dtype == 0)
-    silu_mul_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total, act, bias);
+    silu_mul_kernel<float><<<blocks, 256, 0, stream>>>((const float*)gu, (float*)out, I, total, act, limit, bias);
   else
-    silu_mul_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total, act, bias);
+    silu_mul_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, I, total, act, limit, bias);
   return launch_status();
 }
 
@@ -900,6 +941,233 @@ TK_API int tk_add_norm2(int dtype, float* resid, const void* a, int a_f32, int a
 }
 
 // ---------------------------------------------------------------------------
+// Residual add of a sub-layer's NORMED output (a layer whose norm stands behind its sub-layers).
+//   A = a[row] + bias, B = b[row];  with a gain of its own each is divided by its root mean square first: A <- A / rms(A) gain_a
+//   m = wa A + wb B;  with `gain`: m <- m / rms(m) gain
+//   x = resid[row] + m;  if write_resid: resid[row] = x
+//   out[m] = weight ? x * rsqrt(mean(x^2) + eps_out) * weight : x
+// All of it in float32, one rounding into out (which may be absent: the stream itself is read).  A branch is T,
+// float32, or float32 partial sums (added in order); b, the bias, every gain and the weight may be absent, and so
+// may both branches (m = 0).  A block a row.
+// ---------------------------------------------------------------------------
+struct NormedAdds {
+  NormBranch a, b;
+  const float *bias, *gain_a, *gain_b, *gain;
+  float wa, wb, eps;
+};
+
+// sums of two values over a block (scratch: 32 floats)
+__device__ __forceinline__ void block_sum2(float& u, float& v, float* scratch) {
+  u = wave_sum(u);
+  v = wave_sum(v);
+  const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave, nwaves = (blockDim.x + kWave - 1) / kWave;
+  __syncthreads();
+  if (lane == 0) {
+    scratch[wave] = u;
+    scratch[16 + wave] = v;
+  }
+  __syncthreads();
+  u = v = 0.f;
+  for (int i = 0; i < nwaves; ++i) {
+    u += scratch[i];
+    v += scratch[16 + i];
+  }
+}
+
+__device__ __forceinline__ float square_sum(const float4& v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; }
+__device__ __forceinline__ void scale_by(float4& v, float s, const float* w) {
+  const float4 g = *reinterpret_cast<const float4*>(w);
+  v = make_float4(v.x * s * g.x, v.y * s * g.y, v.z * s * g.z, v.w * s * g.w);
+}
+
+// Vector form: a thread keeps up to GROUPS pieces of four elements of the row in registers.
+template <typename T, int GROUPS>
+__global__ __launch_bounds__(1024) void add_normed_vec_kernel(
+    float* __restrict__ resid, NormedAdds n, const int* __restrict__ rows, const float* __restrict__ weight,
+    T* __restrict__ out, int H, float eps_out, int write_resid) {
+  __shared__ float scratch[32];
+  const int m = blockIdx.x;
+  const size_t row = rows ? (size_t)rows[m] : (size_t)m;
+  float* x = resid + row * H;
+  float4 av[GROUPS], bv[GROUPS], xv[GROUPS];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    av[g] = bv[g] = xv[g] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (d < H) {
+      xv[g] = *reinterpret_cast<const float4*>(x + d);
+      if (n.a.p) av[g] = branch_four<T>(n.a, row * H + d);
+      if (n.b.p) bv[g] = branch_four<T>(n.b, row * H + d);
+      if (n.bias) {
+        const float4 t = *reinterpret_cast<const float4*>(n.bias + d);
+        av[g].x += t.x; av[g].y += t.y; av[g].z += t.z; av[g].w += t.w;
+      }
+      sa += square_sum(av[g]);
+      sb += square_sum(bv[g]);
+    }
+  }
+  if (n.gain_a || n.gain_b) {      // (every thread of the block alike)
+    block_sum2(sa, sb, scratch);
+    const float ra = 1.f / sqrtf(sa / (float)H + n.eps), rb = 1.f / sqrtf(sb / (float)H + n.eps);
+#pragma unroll
+    for (int g = 0; g < GROUPS; ++g) {
+      const int d = (g * blockDim.x + threadIdx.x) * 4;
+      if (d < H) {
+        if (n.gain_a) scale_by(av[g], ra, n.gain_a + d);
+        if (n.gain_b) scale_by(bv[g], rb, n.gain_b + d);
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    av[g] = make_float4(n.wa * av[g].x + n.wb * bv[g].x, n.wa * av[g].y + n.wb * bv[g].y,
+                        n.wa * av[g].z + n.wb * bv[g].z, n.wa * av[g].w + n.wb * bv[g].w);
+    ss += square_sum(av[g]);
+  }
+  float rstd = 1.f;
+  if (n.gain) rstd = 1.f / sqrtf(block_sum(ss, scratch) / (float)H + n.eps);
+  ss = 0.f;
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    if (d < H) {
+      if (n.gain) scale_by(av[g], rstd, n.gain + d);
+      xv[g].x += av[g].x; xv[g].y += av[g].y; xv[g].z += av[g].z; xv[g].w += av[g].w;
+      if (write_resid) *reinterpret_cast<float4*>(x + d) = xv[g];
+      ss += square_sum(xv[g]);
+    }
+  }
+  if (!out) return;
+  if (weight) rstd = 1.f / sqrtf(block_sum(ss, scratch) / (float)H + eps_out);
+  T* o = out + (size_t)m * H;
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    if (d < H) {
+      if (weight) scale_by(xv[g], rstd, weight + d);
+      Store4<T>::at(o + d, xv[g]);
+    }
+  }
+}
+
+// Any width and alignment: the row's m and x wait in LDS (H floats) between the passes.
+template <typename T>
+__global__ __launch_bounds__(256) void add_normed_kernel(
+    float* __restrict__ resid, NormedAdds n, const int* __restrict__ rows, const float* __restrict__ weight,
+    T* __restrict__ out, int H, float eps_out, int write_resid) {
+  __shared__ float scratch[32];
+  extern __shared__ float held[];
+  const int m = blockIdx.x;
+  const size_t row = rows ? (size_t)rows[m] : (size_t)m;
+  float* x = resid + row * H;
+  auto first = [&](int d) {
+    return (n.a.p ? branch_value<T>(n.a.p, n.a.f32, n.a.parts, n.a.stride, row * H + d) : 0.f) + (n.bias ? n.bias[d] : 0.f);
+  };
+  auto second = [&](int d) { return n.b.p ? branch_value<T>(n.b.p, n.b.f32, n.b.parts, n.b.stride, row * H + d) : 0.f; };
+  float ra = 1.f, rb = 1.f;
+  if (n.gain_a || n.gain_b) {
+    float sa = 0.f, sb = 0.f;
+    for (int d = threadIdx.x; d < H; d += blockDim.x) {
+      const float a = first(d), b = second(d);
+      sa = fmaf(a, a, sa);
+      sb = fmaf(b, b, sb);
+    }
+    block_sum2(sa, sb, scratch);
+    ra = 1.f / sqrtf(sa / (float)H + n.eps);
+    rb = 1.f / sqrtf(sb / (float)H + n.eps);
+  }
+  float ss = 0.f;
+  for (int d = threadIdx.x; d < H; d += blockDim.x) {      // (a thread reads back only what it wrote itself)
+    const float a = n.gain_a ? first(d) * ra * n.gain_a[d] : first(d), b = n.gain_b ? second(d) * rb * n.gain_b[d] : second(d);
+    const float v = n.wa * a + n.wb * b;
+    held[d] = v;
+    ss = fmaf(v, v, ss);
+  }
+  float rstd = 1.f;
+  if (n.gain) rstd = 1.f / sqrtf(block_sum(ss, scratch) / (float)H + n.eps);
+  ss = 0.f;
+  for (int d = threadIdx.x; d < H; d += blockDim.x) {
+    const float v = x[d] + (n.gain ? held[d] * rstd * n.gain[d] : held[d]);
+    if (write_resid) x[d] = v;
+    held[d] = v;
+    ss = fmaf(v, v, ss);
+  }
+  if (!out) return;
+  if (weight) rstd = 1.f / sqrtf(block_sum(ss, scratch) / (float)H + eps_out);
+  for (int d = threadIdx.x; d < H; d += blockDim.x)
+    Elem<T>::store(out + (size_t)m * H + d, weight ? held[d] * rstd * weight[d] : held[d]);
+}
+
+TK_API int tk_add_normed(int dtype, float* resid, const void* a, int a_f32, int a_parts, long a_stride, const float* bias,
+                         const float* gain_a, float wa, const void* b, int b_f32, int b_parts, long b_stride,
+                         const float* gain_b, float wb, const float* gain, float eps, const int* rows,
+                         const float* weight, float eps_out, void* out, int M, int H, int write_resid, hipStream_t stream) {
+  if (M <= 0) return 0;
+  if (rows && write_resid) return -1;
+  if (a_parts < 1 || b_parts < 1 || (a_parts > 1 && !a_f32) || (b_parts > 1 && !b_f32) || (weight && !out)) return -1;
+  const NormedAdds adds{{a, a_f32 || dtype == 0, a_parts, a_stride}, {b, b_f32 || dtype == 0, b_parts, b_stride},
+                        bias, gain_a, gain_b, gain, wa, wb, eps};
+  int threads = 64;
+  while (threads < 1024 && threads * 4 * (M >= 512 ? kNormGroups : 1) < H) threads *= 2;
+  const bool vec = H % 4 == 0 && H <= threads * 4 * kNormGroups && a_stride % 4 == 0 && b_stride % 4 == 0 &&
+                   (uintptr_t)resid % 16 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)b % 16 == 0 && (uintptr_t)bias % 16 == 0 &&
+                   (uintptr_t)gain_a % 16 == 0 && (uintptr_t)gain_b % 16 == 0 && (uintptr_t)gain % 16 == 0 &&
+                   (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0;
+#define TK_AN(KERNEL, T_, THREADS_, LDS_) \
+  KERNEL<<<M, THREADS_, LDS_, stream>>>(resid, adds, rows, weight, (T_*)out, H, eps_out, write_resid)
+  if (vec) {
+    const bool one = threads * 4 >= H;
+    if (dtype == 0) {
+      if (one) TK_AN((add_normed_vec_kernel<float, 1>), float, threads, 0);
+      else TK_AN((add_normed_vec_kernel<float, kNormGroups>), float, threads, 0);
+    } else {
+      if (one) TK_AN((add_normed_vec_kernel<bf16_t, 1>), bf16_t, threads, 0);
+      else TK_AN((add_normed_vec_kernel<bf16_t, kNormGroups>), bf16_t, threads, 0);
+    }
+    return launch_status();
+  }
+  const size_t lds = (size_t)H * 4;
+  if (lds > 60 * 1024) return -1;
+  if (dtype == 0) TK_AN((add_normed_kernel<float>), float, 256, lds);
+  else TK_AN((add_normed_kernel<bf16_t>), bf16_t, 256, lds);
+#undef TK_AN
+  return launch_status();
+}
+
+// ---------------------------------------------------------------------------
+// x[n, head, d] *= sigmoid(gate[n, head * vd + d]) in place: the gate behind attention.  x rows hold `heads`
+// heads of vdp >= vd columns (those behind vd stay as they are); gate rows are ld long and start at column col0,
+// in T, float32, or float32 partial sums.
+// ---------------------------------------------------------------------------
+template <typename T>
+__global__ void sigmoid_gate_kernel(T* __restrict__ x, const void* __restrict__ gate, int f32, int parts, long part_stride,
+                                    long ld, int col0, int width, int vd, int vdp, size_t total) {
+  const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const size_t n = idx / width;
+  const int c = (int)(idx - n * width);
+  const int head = c / vd, d = c - head * vd;
+  const float g = branch_value<T>(gate, f32, parts, part_stride, n * ld + col0 + c);
+  T* at = x + n * ((size_t)(width / vd) * vdp) + (size_t)head * vdp + d;
+  Elem<T>::store(at, Elem<T>::load(at) / (1.f + expf(-g)));
+}
+
+TK_API int tk_sigmoid_gate(int dtype, void* x, const void* gate, int f32, int parts, long part_stride, long ld, int col0,
+                           int N, int heads, int vd, int vdp, hipStream_t stream) {
+  if (N <= 0) return 0;
+  if (heads < 1 || vd < 1 || vdp < vd || parts < 1 || (parts > 1 && !f32 && dtype != 0) || col0 < 0 || ld < (long)col0 + (long)heads * vd)
+    return -1;
+  const size_t total = (size_t)N * heads * vd;
+  const unsigned blocks = (unsigned)((total + 255) / 256);
+  if (dtype == 0)
+    sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, gate, 1, parts, part_stride, ld, col0, heads * vd, vd, vdp, total);
+  else
+    sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)x, gate, f32, parts, part_stride, ld, col0, heads * vd, vd, vdp, total);
+  return launch_status();
+}
+
 // ---------------------------------------------------------------------------
 // Rotation of the first `rot` dims of q and k (half-split pairs, dim j with j + rot/2, or
 // `interleaved` pairs, dim 2j with 2j + 1), THEN (unit) each head of q and k divided by
@@ -911,6 +1179,8 @@ TK_API int tk_add_norm2(int dtype, float* resid, const void* a, int a_f32, int a
 // hdp >= hd and vdp >= vd are the sizes the pages and q_out are laid out for (hd rounded up to 8,
 // vd to 16): the channels behind hd are written as zeros into q_out and never written in the
 // pages (which start as zeros), so they add nothing to a score or an output.
+// norm_first: the norm comes before the rotation instead.  bias (float32, one for every q, k and v column that
+// the input holds) is added before anything else.  Input rows are in_ld long (columns behind the heads are not read).
 // Values may be mixed with those another layer made for the same tokens (v_keep, float32
 // [N, nkv * vd]): v_mode 1 leaves this layer's values there as they are projected; v_mode 2
 // caches (1 - lambda) v + lambda v_keep with lambda = *v_lambda.
@@ -924,7 +1194,7 @@ __global__ void rope_norm_store_kernel(
     const int* __restrict__ block_tables, T* __restrict__ q_out, T* __restrict__ k_cache,
     T* __restrict__ v_cache, int nh, int nkv_in, int nkv, int hd, int vd, int hdp, int vdp, int rot, int ps,
     int max_pages, int unit, float eps, int num_pairs, int interleaved, float* __restrict__ v_keep, int v_mode,
-    const float* __restrict__ v_lambda) {
+    const float* __restrict__ v_lambda, long in_ld, const float* __restrict__ bias, int norm_first) {
   __shared__ float vecs[kPairsPerBlock][kMaxHeadDim];
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
   const int heads = nh + 2 * nkv_in;
@@ -932,19 +1202,28 @@ __global__ void rope_norm_store_kernel(
   if (pair >= num_pairs) return;  // nothing below synchronises across waves
   const int n = pair / heads, head = pair - n * heads;
   float* vec = vecs[wave];
-  const size_t row_width = (size_t)(nh + nkv_in) * hd + (size_t)nkv_in * vd;
   const bool is_q = head < nh;
   const bool is_k = !is_q && head < nh + nkv_in;
   const int width = (is_q || is_k) ? hd : vd;
   const size_t head_at = (is_q || is_k) ? (size_t)head * hd : (size_t)(nh + nkv_in) * hd + (size_t)(head - nh - nkv_in) * vd;
-  const TIN* src = qkv + (size_t)n * row_width + head_at;
+  const TIN* src = qkv + (size_t)n * in_ld + head_at;
   for (int d = lane; d < width; d += kWave) {
-    float v = 0.f;
+    float v = bias ? bias[head_at + d] : 0.f;
     for (int p = 0; p < parts; ++p) v += Elem<TIN>::load(src + (size_t)p * part_stride + d);
     vec[d] = v;
   }
   wave_lds_sync();
+  auto norm_head = [&]() {
+    float ss = 0.f;
+    for (int d = lane; d < hd; d += kWave) ss += vec[d] * vec[d];
+    ss = wave_sum(ss);
+    const float rstd = 1.f / sqrtf(ss / (float)hd + eps);
+    const float* w = is_q ? q_weight : k_weight;
+    for (int d = lane; d < hd; d += kWave) vec[d] = vec[d] * rstd * (w ? w[d] : 1.f);   // (a lane rewrites what it read)
+    wave_lds_sync();
+  };
   if (is_q || is_k) {
+    if (unit && norm_first) norm_head();
     const int half = rot / 2;
     float lo[kMaxHeadDim / 2 / kWave], hi[kMaxHeadDim / 2 / kWave];
     int cnt = 0;
@@ -961,15 +1240,7 @@ __global__ void rope_norm_store_kernel(
       vec[interleaved ? 2 * j + 1 : j + half] = hi[cnt];
     }
     wave_lds_sync();
-    if (unit) {
-      float ss = 0.f;
-      for (int d = lane; d < hd; d += kWave) ss += vec[d] * vec[d];
-      ss = wave_sum(ss);
-      const float rstd = 1.f / sqrtf(ss / (float)hd + eps);
-      const float* w = is_q ? q_weight : k_weight;
-      for (int d = lane; d < hd; d += kWave) vec[d] = vec[d] * rstd * (w ? w[d] : 1.f);   // (a lane rewrites what it read)
-      wave_lds_sync();
-    }
+    if (unit && !norm_first) norm_head();
   }
   if (is_q) {
     T* dst = q_out + ((size_t)n * nh + head) * hdp;
@@ -1005,7 +1276,8 @@ TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts,
                               const int* block_tables, void* q_out, void* k_cache, void* v_cache,
                               int N, int nh, int nkv_in, int nkv, int hd, int vd, int hdp, int vdp, int rot,
                               int ps, int max_pages, int unit, float eps, int interleaved, float* v_keep,
-                              int v_mode, const float* v_lambda, hipStream_t stream) {
+                              int v_mode, const float* v_lambda, long in_ld, const float* bias, int norm_first,
+                              hipStream_t stream) {
   if (N <= 0) return 0;
   if (hdp > kMaxHeadDim || vdp > kMaxHeadDim || hd < 1 || vd < 1 || hdp < hd || vdp < vd || hdp % 8 != 0 ||
       vdp % 16 != 0 || ps % 4 != 0 || rot > hd || rot % 2 != 0)
@@ -1013,6 +1285,7 @@ TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts,
   if (v_mode < 0 || v_mode > 2 || (v_mode != 0 && v_keep == nullptr) || (v_mode == 2 && v_lambda == nullptr)) return -1;
   if (nkv_in != 0 && nkv_in != nkv) return -1;
   if (parts < 1 || (parts > 1 && !in_f32 && dtype != 0)) return -1;
+  if (in_ld < (long)(nh + nkv_in) * hd + (long)nkv_in * vd) return -1;
   const long pairs = (long)N * (nh + 2 * nkv_in);
   if (pairs > 0x7fffffffL) return -1;
   const unsigned grid = (unsigned)((pairs + kPairsPerBlock - 1) / kPairsPerBlock);
@@ -1020,7 +1293,7 @@ TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts,
   rope_norm_store_kernel<T_, TIN_><<<grid, kWave * kPairsPerBlock, 0, stream>>>(                 \
       (const TIN_*)qkv, parts, part_stride, q_weight, k_weight, cos_t, sin_t, positions,         \
       req_of_token, block_tables, (T_*)q_out, (T_*)k_cache, (T_*)v_cache, nh, nkv_in, nkv, hd,   \
-      vd, hdp, vdp, rot, ps, max_pages, unit, eps, (int)pairs, interleaved, v_keep, v_mode, v_lambda)
+      vd, hdp, vdp, rot, ps, max_pages, unit, eps, (int)pairs, interleaved, v_keep, v_mode, v_lambda, in_ld, bias, norm_first)
   if (dtype == 0) TK_RN(float, float);
   else if (in_f32) TK_RN(bf16_t, float);
   else TK_RN(bf16_t, bf16_t);
@@ -1048,6 +1321,8 @@ TK_API int tk_scale_softcap(float* x, long total, float scale, float cap, hipStr
 // the same entry points in slot form (slots.h), for launch lists
 TK_SLOTS(tk_add_rmsnorm)
 TK_SLOTS(tk_add_norm2)
+TK_SLOTS(tk_add_normed)
+TK_SLOTS(tk_sigmoid_gate)
 TK_SLOTS(tk_rope_tables)
 TK_SLOTS(tk_qknorm_rope_store)
 TK_SLOTS(tk_silu_mul)

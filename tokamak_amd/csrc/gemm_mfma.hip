@@ -246,12 +246,16 @@ struct RowScale {
   const float* sumsq;  // [slabs][M]: sums of squares of the rows over slabs of columns; nullptr: no scaling
   int slabs;
   float eps;
-  int act;             // the gated form's activation: 0 silu, 1 the tanh form of gelu
+  int act;             // the gated form's activation: 0 silu, 1 the tanh form of gelu, 2 the clamped gate
+  float limit;         // of the clamped gate
 };
 
-__device__ __forceinline__ float gate_act(float z, int act) {
-  if (act == 0) return z / (1.f + __expf(-z));
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+// act(z) * u; 2: with g = min(z, limit), g sigmoid(1.702 g) (clamp(u, -limit, limit) + 1)
+__device__ __forceinline__ float gated_value(float z, float u, const RowScale& s) {
+  if (s.act == 0) return z / (1.f + __expf(-z)) * u;
+  if (s.act == 1) return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) * u;
+  const float g = fminf(z, s.limit);
+  return g / (1.f + __expf(-1.702f * g)) * (fminf(fmaxf(u, -s.limit), s.limit) + 1.f);
 }
 
 template <int MT, typename TO, bool GATED, int WAVES>
@@ -440,10 +444,10 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_kernel(
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
       const float4 u = *reinterpret_cast<const float4*>(up + ((size_t)(wave * MT + j) * 64 + lane) * 4);
-      acc[j][0] = gate_act(acc[j][0], scale.act) * u.x;
-      acc[j][1] = gate_act(acc[j][1], scale.act) * u.y;
-      acc[j][2] = gate_act(acc[j][2], scale.act) * u.z;
-      acc[j][3] = gate_act(acc[j][3], scale.act) * u.w;
+      acc[j][0] = gated_value(acc[j][0], u.x, scale);
+      acc[j][1] = gated_value(acc[j][1], u.y, scale);
+      acc[j][2] = gated_value(acc[j][2], u.z, scale);
+      acc[j][3] = gated_value(acc[j][3], u.w, scale);
     }
   }
 
@@ -525,17 +529,17 @@ TK_API int tk_gemm_stream(int out_dtype, const void* A, const void* W, void* C, 
 }
 
 // C[M, N] = act(A W_gate^T) * (A W_up^T) with W = [W_gate; W_up] of 2N rows; bfloat16 out.  act: 0 silu, 1 the
-// tanh form of gelu.
+// tanh form of gelu, 2 the gate whose halves are clamped at `limit`.
 TK_API int tk_gemm_stream_swiglu(const void* A, const void* W, void* C, int M, int N, int K, long lda,
                                  long ldw, long ldc, int waves, const float* sumsq, int slabs, float eps,
-                                 int act, hipStream_t stream) {
+                                 int act, float limit, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
-  if (act != 0 && act != 1) return -1;
+  if (act < 0 || act > 2) return -1;
   if (M > 64 || K < 8 || K % 8 != 0 || lda % 8 != 0 || ldw % 8 != 0) return -1;
   if (sumsq != nullptr && (M > 16 || slabs < 1 || slabs > kRowScaleSlabs || waves >= 6)) return -1;
   const int total_chunks = (K + SBK - 1) / SBK;
   return launch_stream<bf16_t, true>(waves, A, W, C, M, N, K, lda, ldw, ldc, total_chunks, 1, 0,
-                                     RowScale{sumsq, slabs, eps, act}, stream);
+                                     RowScale{sumsq, slabs, eps, act, limit}, stream);
 }
 
 // the same entry points in slot form (slots.h), for launch lists

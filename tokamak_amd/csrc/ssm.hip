@@ -11,47 +11,26 @@
 //     dt = softplus(dt_in + dt_bias),  S <- exp(-exp(A_log) dt) S + dt B_t x_t^T,  y_t = S^T C_t + D x_t
 //   with the state S [state, vdim] in float32 registers (a thread owns a few state rows of one value
 //   column); head h reads the B and C of group h / (heads / groups).
+// fixed_decay_scan: linear attention with one constant decay a head,
+//     S <- a S + k_t v_t^T,  o_t = S^T q_t,  q, k, v = silu(.) of the projection's columns [v | k | q | ...],
+//   in the same kernels (SILU: the operands are the projection itself, and every head has a B and a C of its own).
 // gated_group_norm: y * silu(z), divided by its root mean square over each of `norm_groups` equal parts
-//   of the row, times a weight.
+//   of the row, times a weight; or (`after`) y divided by its root mean square first, times the weight, times sigmoid(z).
 //
 // Step sizes, decays with their exponentials, the recurrence, its state, the gate's product and the
 // norm are float32 whatever the storage type; x, B and C enter as the convolution stored them.
 #include "common.h"
+#include "short_conv.h"
 #include "slots.h"
 
 using namespace tk;
 
 namespace {
 
-constexpr int kMaxTaps = 8;
 constexpr int kConvSegment = 64;   // tokens of a request that one thread of the convolution walks
 constexpr int kScanTokens = 8;     // tokens staged in LDS at a time by the scan
 
-// an input of [rows, ld] elements: T, or float32, or `parts` float32 partial sums `stride` elements apart
-struct SsmIn {
-  const void* p;
-  int f32;
-  int parts;
-  long stride;
-};
-
-template <typename T>
-__device__ __forceinline__ float load_in(const SsmIn& in, size_t idx) {
-  if (!in.f32) return Elem<T>::load(reinterpret_cast<const T*>(in.p) + idx);
-  const float* f = reinterpret_cast<const float*>(in.p) + idx;
-  float s = f[0];
-  int i = 1;
-  for (; i + 3 < in.parts; i += 4) {      // four loads in flight; the sums in the order of the parts
-    const float a = f[(size_t)i * in.stride], b = f[(size_t)(i + 1) * in.stride];
-    const float c = f[(size_t)(i + 2) * in.stride], d = f[(size_t)(i + 3) * in.stride];
-    s = (((s + a) + b) + c) + d;
-  }
-  for (; i < in.parts; ++i) s += f[(size_t)i * in.stride];
-  return s;
-}
-
-__device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
-__device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+using SsmIn = RowsIn;
 
 // grid (channel blocks, requests, segments of kConvSegment tokens).  proj rows are ld long, the
 // convolution's channels start at column col0.  state: float32 [slots][taps - 1][C], oldest first.
@@ -99,31 +78,6 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(
       if (j >= 0) st[(size_t)j * C] = win[k];
     }
   }
-}
-
-// The state after a step: the last taps - 1 inputs of every request, from the step's rows or, where the
-// step brought fewer, from the state before it.  A thread a (request, channel): it reads what it needs, then writes.
-template <typename T>
-__global__ __launch_bounds__(256) void conv_carry_kernel(
-    SsmIn proj, long ld, int col0, float* __restrict__ state, const int* __restrict__ q_start,
-    const int* __restrict__ state_slots, int C, int taps) {
-  const int c = blockIdx.x * blockDim.x + threadIdx.x;
-  const int req = blockIdx.y;
-  if (c >= C) return;
-  const int first = q_start[req], count = q_start[req + 1] - first;
-  float* st = state + (size_t)state_slots[req] * (taps - 1) * C + c;
-  float keep[kMaxTaps - 1];
-#pragma unroll
-  for (int j = 0; j < kMaxTaps - 1; ++j) {
-    keep[j] = 0.f;
-    if (j < taps - 1) {
-      const int local = count - (taps - 1) + j;
-      keep[j] = local >= 0 ? load_in<T>(proj, (size_t)(first + local) * ld + col0 + c) : st[(size_t)(taps - 1 + local) * C];
-    }
-  }
-#pragma unroll
-  for (int j = 0; j < kMaxTaps - 1; ++j)
-    if (j < taps - 1) st[(size_t)j * C] = keep[j];
 }
 
 // Sums over the KS neighbouring lanes that share a column group, for the COUNT values v[0 .. COUNT) that
@@ -177,7 +131,9 @@ struct ScanShape {
 //   MODE 2: the same blocks again, each from its S_start, with the outputs.
 // MODE 0 walks a request's tokens in one block from the request's state.  A chunk's place in the scratch
 // arrays is its number among all chunks of the step (requests in order).
-template <typename T, int RS, int KS, int MODE>
+// SILU: u is not read; dt_in is the projection [x | B | C | ...], whose columns pass silu as they are loaded, the
+// step size is 1, the decay of a head is a_log[head] itself and there is no skip term.
+template <typename T, int RS, int KS, int MODE, bool SILU>
 __global__ __launch_bounds__(1024) void ssd_scan_kernel(
     const T* __restrict__ u, int C, SsmIn dt_in, long ld, int dt_col, const float* __restrict__ dt_bias,
     const float* __restrict__ a_log, const float* __restrict__ skip, float* __restrict__ state,
@@ -223,7 +179,8 @@ __global__ __launch_bounds__(1024) void ssd_scan_kernel(
     if (MODE != 1 && owns && k0 + r < ns) row = *reinterpret_cast<const float4*>(S + r * 4);
     s[r][0] = row.x; s[r][1] = row.y; s[r][2] = row.z; s[r][3] = row.w;
   }
-  const float rate = expf(a_log[head]), bias = dt_bias[head], d_skip = skip[head];
+  const float rate = SILU ? a_log[head] : expf(a_log[head]);
+  const float bias = SILU ? 0.f : dt_bias[head], d_skip = SILU ? 0.f : skip[head];
   float decayed = 1.f;      // the product of the chunk's decays (MODE 1)
 
   for (int t0 = first; t0 < end; t0 += TB) {
@@ -232,17 +189,27 @@ __global__ __launch_bounds__(1024) void ssd_scan_kernel(
       const int t = i / nsp, n = i - t * nsp;
       const size_t row = (size_t)(t0 + t) * C;
       // (every element forms its token's step size itself: the same float32 operations, no barrier for it)
-      const float dt = softplus(load_in<T>(dt_in, (size_t)(t0 + t) * ld + dt_col + head) + bias);
-      bb[i] = n < ns ? dt * Elem<T>::load(u + row + b_col + n) : 0.f;
-      cc[i] = n < ns ? Elem<T>::load(u + row + c_col + n) : 0.f;
-      if (n == 0) aa[t] = expf(-rate * dt);
+      if constexpr (SILU) {
+        const size_t at = (size_t)(t0 + t) * ld;
+        bb[i] = n < ns ? silu(load_in<T>(dt_in, at + b_col + n)) : 0.f;
+        cc[i] = n < ns ? silu(load_in<T>(dt_in, at + c_col + n)) : 0.f;
+        if (n == 0) aa[t] = rate;
+      } else {
+        const float dt = softplus(load_in<T>(dt_in, (size_t)(t0 + t) * ld + dt_col + head) + bias);
+        bb[i] = n < ns ? dt * Elem<T>::load(u + row + b_col + n) : 0.f;
+        cc[i] = n < ns ? Elem<T>::load(u + row + c_col + n) : 0.f;
+        if (n == 0) aa[t] = expf(-rate * dt);
+      }
     }
     float xloc[TB][CS];
 #pragma unroll
     for (int t = 0; t < TB; ++t) {
 #pragma unroll
-      for (int c = 0; c < CS; ++c)
-        xloc[t][c] = (t < tb && owns && j0 + c < vdim) ? Elem<T>::load(u + (size_t)(t0 + t) * C + head * vdim + j0 + c) : 0.f;
+      for (int c = 0; c < CS; ++c) {
+        const bool there = t < tb && owns && j0 + c < vdim;
+        if constexpr (SILU) xloc[t][c] = there ? silu(load_in<T>(dt_in, (size_t)(t0 + t) * ld + head * vdim + j0 + c)) : 0.f;
+        else xloc[t][c] = there ? Elem<T>::load(u + (size_t)(t0 + t) * C + head * vdim + j0 + c) : 0.f;
+      }
     }
     __syncthreads();
     float outs[TB * CS];      // this thread's share of the round's outputs: [token][column]
@@ -324,10 +291,14 @@ __global__ __launch_bounds__(256) void ssd_chunk_starts_kernel(
 }
 
 // A wave a (token, part of the row): out = g / rms(g) * weight with g = y * silu(z).
+// `after`: out = y / rms(y) * weight * sigmoid(z).  `shared`: one weight for all parts.
+__device__ __forceinline__ float before_norm(float y, float z, int after) { return after ? y : y * silu(z); }
+__device__ __forceinline__ float behind_norm(float v, float z, int after) { return after ? v * sigmoid(z) : v; }
+
 template <typename T>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(
     const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
-    T* __restrict__ out, long pairs, int inner, int groups, float eps) {
+    T* __restrict__ out, long pairs, int inner, int groups, float eps, int shared, int after) {
   const int lane = threadIdx.x & (kWave - 1);
   const long pair = (long)blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
   if (pair >= pairs) return;
@@ -337,14 +308,15 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
   const size_t zat = (size_t)n * ld + z_col + (size_t)g * size;
   float ss = 0.f;
   for (int x = lane; x < size; x += kWave) {
-    const float v = y[at + x] * silu(load_in<T>(z_in, zat + x));
+    const float v = before_norm(y[at + x], after ? 0.f : load_in<T>(z_in, zat + x), after);
     ss = fmaf(v, v, ss);
   }
   ss = wave_sum(ss);
   const float rstd = 1.f / sqrtf(ss / (float)size + eps);
   for (int x = lane; x < size; x += kWave) {
-    const float v = y[at + x] * silu(load_in<T>(z_in, zat + x));
-    Elem<T>::store(out + at + x, v * rstd * weight[(size_t)g * size + x]);
+    const float z = load_in<T>(z_in, zat + x);
+    const float v = before_norm(y[at + x], z, after);
+    Elem<T>::store(out + at + x, behind_norm(v * rstd * weight[shared ? x : g * size + x], z, after));
   }
 }
 
@@ -354,23 +326,24 @@ constexpr int kHold = 8;
 template <typename T>
 __global__ __launch_bounds__(1024) void gated_group_norm_block_kernel(
     const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
-    T* __restrict__ out, int inner, int groups, float eps) {
+    T* __restrict__ out, int inner, int groups, float eps, int shared, int after) {
   __shared__ float scratch[16];
   const long pair = blockIdx.x;
   const long n = pair / groups;
   const int g = (int)(pair - n * groups), size = inner / groups;
   const size_t at = (size_t)n * inner + (size_t)g * size;
   const size_t zat = (size_t)n * ld + z_col + (size_t)g * size;
-  float held[kHold];
+  float held[kHold], gate[kHold];
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < kHold; ++i) {
     const int x = threadIdx.x + i * blockDim.x;
-    held[i] = x < size ? y[at + x] * silu(load_in<T>(z_in, zat + x)) : 0.f;
+    gate[i] = x < size ? load_in<T>(z_in, zat + x) : 0.f;
+    held[i] = x < size ? before_norm(y[at + x], gate[i], after) : 0.f;
     ss = fmaf(held[i], held[i], ss);
   }
   for (int x = threadIdx.x + kHold * blockDim.x; x < size; x += blockDim.x) {
-    const float v = y[at + x] * silu(load_in<T>(z_in, zat + x));
+    const float v = before_norm(y[at + x], load_in<T>(z_in, zat + x), after);
     ss = fmaf(v, v, ss);
   }
   ss = block_sum(ss, scratch);
@@ -378,15 +351,16 @@ __global__ __launch_bounds__(1024) void gated_group_norm_block_kernel(
 #pragma unroll
   for (int i = 0; i < kHold; ++i) {
     const int x = threadIdx.x + i * blockDim.x;
-    if (x < size) Elem<T>::store(out + at + x, held[i] * rstd * weight[(size_t)g * size + x]);
+    if (x < size) Elem<T>::store(out + at + x, behind_norm(held[i] * rstd * weight[shared ? x : g * size + x], gate[i], after));
   }
   for (int x = threadIdx.x + kHold * blockDim.x; x < size; x += blockDim.x) {
-    const float v = y[at + x] * silu(load_in<T>(z_in, zat + x));
-    Elem<T>::store(out + at + x, v * rstd * weight[(size_t)g * size + x]);
+    const float z = load_in<T>(z_in, zat + x);
+    const float v = before_norm(y[at + x], z, after);
+    Elem<T>::store(out + at + x, behind_norm(v * rstd * weight[shared ? x : g * size + x], z, after));
   }
 }
 
-template <typename T>
+template <typename T, bool SILU = false>
 int launch_scan(const void* u, int C, SsmIn dt, long ld, int dt_col, const float* dt_bias, const float* a_log,
                 const float* skip, float* state, const int* q_start, const int* state_slots, float* y, int R,
                 int heads, int groups, int ns, int vdim, int splits, int chunk, int max_chunks, float* chunk_state,
@@ -412,13 +386,13 @@ int launch_scan(const void* u, int C, SsmIn dt, long ld, int dt_col, const float
     if (lds > 48 * 1024) {                                                                                    \
       static bool raised = false;                                                                             \
       if (!raised) {                                                                                          \
-        if (hipFuncSetAttribute(reinterpret_cast<const void*>(&ssd_scan_kernel<T, RS, KS, MODE>),             \
+        if (hipFuncSetAttribute(reinterpret_cast<const void*>(&ssd_scan_kernel<T, RS, KS, MODE, SILU>),             \
                                 hipFuncAttributeMaxDynamicSharedMemorySize, 72 * 1024) != hipSuccess)         \
           return -1;                                                                                          \
         raised = true;                                                                                        \
       }                                                                                                       \
     }                                                                                                         \
-    ssd_scan_kernel<T, RS, KS, MODE><<<grid, threads, lds, stream>>>((const T*)u, C, dt, ld, dt_col, dt_bias, \
+    ssd_scan_kernel<T, RS, KS, MODE, SILU><<<grid, threads, lds, stream>>>((const T*)u, C, dt, ld, dt_col, dt_bias, \
                                                                     a_log, skip, state, q_start, state_slots, \
                                                                     y, sh, chunk, max_chunks, chunk_state,    \
                                                                     chunk_decay);                             \
@@ -500,10 +474,32 @@ TK_API int tk_ssd_scan(int dtype, const void* u, const void* dt, int dt_f32, int
                              groups, ns, vdim, splits, chunk, max_chunks, chunk_state, chunk_decay, stream);
 }
 
-// y float32 [N, inner]; z: column z_col .. + inner of rows ld long; weight float32 [inner]; out [N, inner] in dtype.
+// proj: [N, ld] (dtype, float32 or partial sums), its columns [v: heads * vdim | k: heads * dim | q: heads * dim | ...]
+// before silu; decay float32 [heads].  State, y, splits and chunks as in tk_ssd_scan (dim is the state's size).
+TK_API int tk_fixed_decay_scan(int dtype, const void* proj, int in_f32, int parts, long part_stride, long ld,
+                               const float* decay, float* state, const int* q_start, const int* state_slots, float* y,
+                               int R, int heads, int dim, int vdim, int splits, int chunk, int max_chunks,
+                               float* chunk_state, float* chunk_decay, hipStream_t stream) {
+  if (R <= 0) return 0;
+  if (chunk < 0 || (chunk > 0 && (max_chunks < 1 || chunk_state == nullptr || chunk_decay == nullptr ||
+                                  (long)R * max_chunks > 0x7fffffffL)))
+    return -1;
+  if (heads < 1 || dim < 1 || dim > 1024 || vdim < 1 || vdim > 1024 || splits < 1 || R > 65535 || heads > 65535 ||
+      parts < 1 || (parts > 1 && !in_f32) || ld < (long)heads * (vdim + 2 * dim))
+    return -1;
+  const SsmIn in{proj, in_f32 || dtype == 0, parts, part_stride};
+  if (dtype == 0)
+    return launch_scan<float, true>(nullptr, 0, in, ld, 0, nullptr, decay, nullptr, state, q_start, state_slots, y, R, heads,
+                                    heads, dim, vdim, splits, chunk, max_chunks, chunk_state, chunk_decay, stream);
+  return launch_scan<bf16_t, true>(nullptr, 0, in, ld, 0, nullptr, decay, nullptr, state, q_start, state_slots, y, R, heads,
+                                   heads, dim, vdim, splits, chunk, max_chunks, chunk_state, chunk_decay, stream);
+}
+
+// y float32 [N, inner]; z: column z_col .. + inner of rows ld long; weight float32 [inner], or
+// (shared) [inner / groups], the same for every part; out [N, inner] in dtype.  after: norm first, then sigmoid(z).
 TK_API int tk_gated_group_norm(int dtype, const float* y, const void* z, int z_f32, int z_parts, long z_stride, long ld,
                                int z_col, const float* weight, void* out, int N, int inner, int groups, float eps,
-                               hipStream_t stream) {
+                               int shared, int after, hipStream_t stream) {
   if (N <= 0) return 0;
   if (inner < 1 || groups < 1 || inner % groups != 0 || z_parts < 1 || (z_parts > 1 && !z_f32)) return -1;
   const SsmIn in{z, z_f32 || dtype == 0, z_parts, z_stride};
@@ -514,16 +510,17 @@ TK_API int tk_gated_group_norm(int dtype, const float* y, const void* z, int z_f
     int threads = 64;
     while (threads < 1024 && threads * 4 < size) threads *= 2;
     if (pairs > 0x7fffffffL) return -1;
-    if (dtype == 0) gated_group_norm_block_kernel<float><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, inner, groups, eps);
-    else gated_group_norm_block_kernel<bf16_t><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, inner, groups, eps);
+    if (dtype == 0) gated_group_norm_block_kernel<float><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, inner, groups, eps, shared, after);
+    else gated_group_norm_block_kernel<bf16_t><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, inner, groups, eps, shared, after);
     return launch_status();
   }
   const unsigned blocks = (unsigned)((pairs + 3) / 4);
-  if (dtype == 0) gated_group_norm_kernel<float><<<blocks, 256, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, pairs, inner, groups, eps);
-  else gated_group_norm_kernel<bf16_t><<<blocks, 256, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, pairs, inner, groups, eps);
+  if (dtype == 0) gated_group_norm_kernel<float><<<blocks, 256, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, pairs, inner, groups, eps, shared, after);
+  else gated_group_norm_kernel<bf16_t><<<blocks, 256, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, pairs, inner, groups, eps, shared, after);
   return launch_status();
 }
 
 TK_SLOTS(tk_conv_silu)
 TK_SLOTS(tk_ssd_scan)
+TK_SLOTS(tk_fixed_decay_scan)
 TK_SLOTS(tk_gated_group_norm)

@@ -50,7 +50,10 @@ def pending_tensors(pending) -> list[tuple[str, torch.Tensor]]:
 
 def pending_kind(pending) -> tuple:
     """What must agree between the recorded layer's incoming sub-layer output and another's."""
-    return (type(pending).__name__, tuple((name, tuple(t.shape), t.dtype, t.stride()) for name, t in pending_tensors(pending)))
+    plain = () if pending is None or isinstance(pending, torch.Tensor) else tuple(
+        (name, value) for name, value in sorted(vars(pending).items()) if isinstance(value, (int, float, bool)))
+    return (type(pending).__name__, plain,
+            tuple((name, tuple(t.shape), t.dtype, t.stride()) for name, t in pending_tensors(pending)))
 
 
 def _stores(store) -> list[tuple[str, object]]:

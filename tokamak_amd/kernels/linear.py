@@ -132,12 +132,13 @@ def _sink_fits(sink: StreamSink, m: int, n: int) -> bool:
             and (g is None or (g.dtype == torch.float32 and g.numel() == n and g.is_contiguous() and g.data_ptr() % 16 == 0)))
 
 
-def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activation: str = "silu") -> torch.Tensor:
+def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activation: str = "silu",
+                 limit: float | None = None) -> torch.Tensor:
     """act(x @ gate^T) * (x @ up^T) for ``gate_up`` = [gate; up] ([2I, K]) -> [M, I].
 
     bfloat16 with up to 64 rows: one fused weight-streaming kernel (the whole-K form for very small
     matrices has the SiLU gate only).  Otherwise the product, then the gate kernel (``activation``:
-    "silu" or "gelu_tanh").
+    "silu", "gelu_tanh", or "clamped" with its ``limit``: both halves clamped, see ``ops.silu_mul``).
     """
     m = x.shape[0]
     if activation != "silu":
@@ -149,9 +150,9 @@ def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activati
         from tokamak_amd.kernels import gemm_bf16
 
         if x.dtype == torch.bfloat16 and m <= 64 and gemm_bf16.skinny_fits(x, gate_up):
-            ops.gemm_stream_swiglu(x, gate_up, out, activation=activation)
+            ops.gemm_stream_swiglu(x, gate_up, out, activation=activation, limit=limit)
         else:
-            ops.silu_mul(linear(x, gate_up), out, activation)
+            ops.silu_mul(linear(x, gate_up), out, activation, limit=limit)
         return out
     inter = gate_up.shape[0] // 2
     # A very small pair of matrices (0.6B-shaped: 13 MB) goes to the whole-K form, whose blocks of 16

@@ -167,12 +167,17 @@ def _check(status: int, name: str) -> None:
 _SIGS = {
     "elementwise": {
         "tk_embed_gather": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_int, c_void_p],
+        "tk_embed_norm": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float, c_int, c_void_p],
         "tk_feed_tokens": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
         "tk_add_rmsnorm": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p,
                            c_void_p, c_int, c_int, c_float, c_int, c_void_p],
         "tk_add_norm2": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_int, c_int, c_long,
                          c_void_p, c_int, c_int, c_long, c_void_p, c_float, c_void_p,
                          c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_int, c_void_p],
+        "tk_add_normed": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float,
+                          c_void_p, c_int, c_int, c_long, c_void_p, c_float, c_void_p, c_float, c_void_p,
+                          c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+        "tk_sigmoid_gate": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p],
         "tk_rope_tables": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p],
         "tk_qknorm_rope_store": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                  c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
@@ -180,9 +185,9 @@ _SIGS = {
         "tk_rope_norm_store": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                               c_int, c_void_p, c_int, c_void_p, c_void_p],
+                               c_int, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_void_p],
         "tk_scale_softcap": [c_void_p, c_long, c_float, c_float, c_void_p],
-        "tk_silu_mul": [c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
+        "tk_silu_mul": [c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p],
         "tk_add_bias": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
         "tk_scaled_sum": [c_int, c_void_p, c_int, c_int, c_long, c_float, c_void_p, c_int, c_int, c_long, c_float,
                           c_void_p, c_void_p, c_int, c_int, c_void_p],
@@ -237,7 +242,7 @@ _SIGS = {
         "tk_gemm_stream": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long,
                            c_long, c_int, c_long, c_int, c_void_p, c_int, c_float, c_void_p],
         "tk_gemm_stream_swiglu": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long, c_long,
-                                  c_int, c_void_p, c_int, c_float, c_int, c_void_p],
+                                  c_int, c_void_p, c_int, c_float, c_int, c_float, c_void_p],
         "tk_gemm_skinny": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long,
                            c_long, c_int, c_int, c_void_p],
     },
@@ -283,8 +288,16 @@ _SIGS = {
         "tk_ssd_scan": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_void_p, c_void_p, c_void_p,
                         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                         c_void_p, c_void_p, c_void_p],
+        "tk_fixed_decay_scan": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
+                                c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p],
         "tk_gated_group_norm": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_void_p, c_void_p,
-                                c_int, c_int, c_int, c_float, c_void_p],
+                                c_int, c_int, c_int, c_float, c_int, c_int, c_void_p],
+    },
+    "delta": {
+        "tk_delta_inputs": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_void_p, c_int, c_int, c_long, c_long,
+                            c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                            c_int, c_int, c_int, c_float, c_int, c_void_p],
+        "tk_delta_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     },
     "attention_fused": {
         "tk_attention_decode_fused": [c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
@@ -400,6 +413,22 @@ def embed_gather(table: torch.Tensor, ids: torch.Tensor, resid: torch.Tensor, sc
            "embed_gather")
 
 
+def embed_norm(table: torch.Tensor, ids: torch.Tensor, weight: torch.Tensor, resid: torch.Tensor, eps: float,
+               scale: float = 1.0, accumulate: bool = False) -> None:
+    """resid[n] = r / sqrt(mean(r^2) + eps) * weight with r = float(table[ids[n]]) * scale (``accumulate``: added to
+    what resid[n] holds); resid is float32 [N, H]."""
+    _gpu(table, ids, weight, resid)
+    n = ids.numel()
+    v, h = table.shape
+    _need(ids.dtype == torch.int32, "token ids must be int32")
+    _need(weight.dtype == torch.float32 and weight.numel() == h, "the norm's weight is float32 [H]")
+    _need(resid.dtype == torch.float32 and resid.shape[-1] == h and resid.numel() >= n * h,
+          "residual buffer must be float32 [>=N, H]")
+    _note(f"{n}x{h}", n * h * (table.element_size() + 4))
+    _check(_fn("elementwise", "tk_embed_norm")(_code(table.dtype), _p(table), _p(ids), _p(weight), _p(resid), n, h, v,
+                                               float(scale), float(eps), int(bool(accumulate)), _stream()), "embed_norm")
+
+
 def feed_tokens(ids: torch.Tensor, sampled: torch.Tensor, slots: torch.Tensor, rows: torch.Tensor, count: int,
                 num_sampled: int) -> None:
     """ids[slots[i]] = sampled[rows[i]] for i < count: token ids of a step that the sampler
@@ -487,6 +516,49 @@ def add_norm2(resid: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | Non
            "add_norm2")
 
 
+def add_normed(resid: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | None, out: torch.Tensor | None, *,
+               dtype: torch.dtype, eps: float = 0.0, bias: torch.Tensor | None = None, gain_a: torch.Tensor | None = None,
+               gain_b: torch.Tensor | None = None, gain: torch.Tensor | None = None, weight_a: float = 1.0,
+               weight_b: float = 1.0, out_weight: torch.Tensor | None = None, out_eps: float = 0.0,
+               rows: torch.Tensor | None = None, write_resid: bool = True) -> None:
+    """A = a[row] + bias and B = b[row], each divided by its root mean square and multiplied by its gain if it has one;
+    m = weight_a A + weight_b B, normed likewise if ``gain`` is given; x = resid[row] + m, optionally stored back; out
+    = rms norm of x times ``out_weight``, or (None) x itself.  ``a`` and ``b`` are each None, [M, H] in ``dtype`` (the
+    compute dtype, which out has) or float32, or float32 partial sums [P, M, H]; bias, gains and the weight are
+    float32 [H] or None.  ``out`` None: only the stream is written."""
+    _gpu(resid, a, b, out, bias, gain_a, gain_b, gain, out_weight, rows)
+    h = resid.shape[-1]
+    m = resid.shape[0] if rows is None else rows.numel()
+    _need(resid.dtype == torch.float32, "the residual stream is float32")
+    for t in (bias, gain_a, gain_b, gain, out_weight):
+        _need(t is None or (t.dtype == torch.float32 and t.numel() == h), "bias, gains and weight are float32 [H]")
+    _need(out is None or (out.dtype == dtype and out.shape[-1] == h and out.shape[0] >= m), "add_normed shapes disagree")
+    _need(out_weight is None or out is not None, "an output weight goes with an output")
+    if rows is not None:
+        _need(rows.dtype == torch.int32 and not write_resid and out is not None, "a row-indexed norm cannot write the residual")
+    pa, fa, na, sa = _branch(a, resid.shape[0], h, dtype, "a")
+    pb, fb, nb, sb = _branch(b, resid.shape[0], h, dtype, "b")
+    _note(f"{m}x{h}", m * h * (4 + (4 if write_resid else 0) + (out.element_size() if out is not None else 0))
+          + sum(t.element_size() * parts * m * h for t, parts in ((a, na), (b, nb)) if t is not None))
+    _check(_fn("elementwise", "tk_add_normed")(
+        _code(dtype), _p(resid), pa, fa, na, sa, _p(bias), _p(gain_a), float(weight_a), pb, fb, nb, sb, _p(gain_b),
+        float(weight_b), _p(gain), float(eps), _p(rows), _p(out_weight), float(out_eps), _p(out), m, h,
+        int(bool(write_resid)), _stream()), "add_normed")
+
+
+def sigmoid_gate(x: torch.Tensor, gate: torch.Tensor, col0: int, *, heads: int, vdim: int, vdim_padded: int) -> None:
+    """x[n, head, d] *= sigmoid(gate[n, col0 + head * vdim + d]) in place.  x [N, heads * vdim_padded]; ``gate`` [N, ld]
+    in x's dtype or float32, or float32 partial sums [P, N, ld]."""
+    _gpu(x, gate)
+    n = x.shape[0]
+    _need(x.shape == (n, heads * vdim_padded) and 1 <= vdim <= vdim_padded, "the gated heads' shape disagrees")
+    pointer, is_f32, parts, stride, ld = _ssm_in(gate, n, x.dtype, "gate")
+    _need(0 <= col0 and col0 + heads * vdim <= ld, "the gate lies outside the projections")
+    _note(f"{n}x{heads * vdim}", n * heads * vdim * (2 * x.element_size() + gate.element_size() * parts))
+    _check(_fn("elementwise", "tk_sigmoid_gate")(_code(x.dtype), _p(x), pointer, is_f32, parts, stride, ld, int(col0), n,
+                                                 heads, vdim, vdim_padded, _stream()), "sigmoid_gate")
+
+
 def rope_tables(positions: torch.Tensor, inv_freq: torch.Tensor, cos: torch.Tensor,
                 sin: torch.Tensor, amplitude: float = 1.0) -> None:
     """cos and sin of float(position) * inv_freq[j], float32 [N, half], both times ``amplitude``."""
@@ -544,7 +616,8 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
                     k_cache: torch.Tensor | None, v_cache: torch.Tensor | None, *, num_heads: int, num_kv_heads: int,
                     head_dim: int, value_dim: int, rotary_dim: int, page_size: int, unit_norm: bool, eps: float,
                     store: bool = True, interleaved: bool = False, value_keep: torch.Tensor | None = None,
-                    value_mode: int = 0, value_lambda: torch.Tensor | None = None) -> None:
+                    value_mode: int = 0, value_lambda: torch.Tensor | None = None, bias: torch.Tensor | None = None,
+                    norm_first: bool = False) -> None:
     """Rotation of the first ``rotary_dim`` dims of every q and k head, then (``unit_norm``) each
     head divided by its root mean square over ``head_dim`` (times a weight, if given); q written to
     q_out, k and v into pages.  Values are ``value_dim`` wide.  ``rotary_dim`` 0: no rotation.
@@ -552,9 +625,11 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
     the true sizes hold zeros.  ``interleaved``: the rotation pairs dim 2j with 2j + 1 instead of j with
     j + rotary_dim / 2.  ``value_mode`` 1: the values, as projected, are also left in ``value_keep`` (float32
     [N, kv heads * value_dim]); 2: what is cached is (1 - lambda) v + lambda value_keep with lambda =
-    ``value_lambda`` (one float32 number on the device)."""
+    ``value_lambda`` (one float32 number on the device).  ``norm_first``: the norm comes before the rotation.
+    ``bias``: float32, one number per q, k and v column, added first.  Rows of ``qkv`` may be longer than
+    q, k and v together (what lies behind them is not read)."""
     _gpu(qkv, q_weight, k_weight, cos, sin, positions, req_of_token, block_tables, q_out, k_cache, v_cache,
-         value_keep, value_lambda)
+         value_keep, value_lambda, bias)
     n = positions.numel()
     nkv_in = num_kv_heads if store else 0
     if not store:
@@ -567,7 +642,10 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
         _need(value_lambda is not None and value_lambda.dtype == torch.float32 and value_lambda.numel() == 1,
               "the mixing weight is one float32 number")
     width = (num_heads + nkv_in) * head_dim + nkv_in * value_dim
-    in_f32, parts, stride = _partials(qkv, n, width, q_out.dtype, "qkv")
+    ld = qkv.shape[-1]
+    _need(ld >= width, f"qkv rows hold {ld} columns, q, k and v are {width}")
+    in_f32, parts, stride = _partials(qkv, n, ld, q_out.dtype, "qkv")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() >= width), "the bias is float32, one number a column")
     hdp, vdp = padded_sizes(head_dim, value_dim)
     _need(q_out.numel() >= n * num_heads * hdp, "q_out too small")
     _need(min(head_dim, value_dim) >= 1 and max(hdp, vdp) <= 512 and page_size % 8 == 0,
@@ -593,7 +671,7 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
         _p(req_of_token), _p(block_tables), _p(q_out), _p(k_cache), _p(v_cache), n, num_heads,
         nkv_in, num_kv_heads, head_dim, value_dim, hdp, vdp, rotary_dim, page_size, block_tables.shape[1],
         int(bool(unit_norm)), float(eps), int(bool(interleaved)), _p(value_keep if value_mode else None), int(value_mode),
-        _p(value_lambda if value_mode == 2 else None), _stream()), "rope_norm_store")
+        _p(value_lambda if value_mode == 2 else None), ld, _p(bias), int(bool(norm_first)), _stream()), "rope_norm_store")
 
 
 def padded_sizes(head_dim: int, value_dim: int) -> tuple[int, int]:
@@ -610,12 +688,15 @@ def scale_softcap(logits: torch.Tensor, scale: float, cap: float | None) -> None
            "scale_softcap")
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
 
 
-def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu", bias: torch.Tensor | None = None) -> None:
+def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu", bias: torch.Tensor | None = None,
+             limit: float | None = None) -> None:
     """out[n, i] = act(gate_up[n, i]) * gate_up[n, I + i]; act is silu, or the tanh form of gelu.  ``bias``:
-    float32 [2 I], added to both halves before the activation."""
+    float32 [2 I], added to both halves before the activation.  "clamped": with g = min(gate_up[n, i], limit) and
+    u = clamp(gate_up[n, I + i], -limit, limit), out = g sigmoid(1.702 g) (u + 1)."""
+    _need((activation == "clamped") == (limit is not None), "a limit goes with the clamped gate")
     _gpu(gate_up, out, bias)
     _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == gate_up.shape[1]), "the bias is float32 [2 I]")
     n, two_i = gate_up.shape
@@ -623,7 +704,7 @@ def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu",
     _note(f"{n}x{two_i // 2}", n * two_i * out.element_size() * 1.5)
     _need(activation in GATE_ACTIVATIONS, f"the gate's activation is one of {sorted(GATE_ACTIVATIONS)}")
     _check(_fn("elementwise", "tk_silu_mul")(_code(out.dtype), _p(gate_up), _p(out), n, two_i // 2,
-                                             GATE_ACTIVATIONS[activation], _p(bias), _stream()), "silu_mul")
+                                             GATE_ACTIVATIONS[activation], float(limit or 0.0), _p(bias), _stream()), "silu_mul")
 
 
 def add_bias(x: torch.Tensor, bias: torch.Tensor) -> None:
@@ -1003,9 +1084,43 @@ def ssd_scan(u: torch.Tensor, proj: torch.Tensor, dt_col: int, dt_bias: torch.Te
     _need(1 <= vdim <= 1024 and 1 <= state_size <= 1024 and batch.num_tokens == n, "the scan takes sizes up to 1,024")
     pointer, is_f32, parts, stride, ld = _ssm_in(proj, n, u.dtype, "projections")
     _need(0 <= dt_col and dt_col + heads <= ld, "the step sizes lie outside the projections")
-    # Long portions: chunks of SSM_CHUNK_TOKENS tokens side by side (a chunk acts on the state as S -> P S + L, with P
-    # and L found from zeros; the chunks' start states follow from those in order; then every chunk runs again
-    # from its own start and writes its outputs): twice the arithmetic of one walk, a thirtieth of its length.
+    plan = _scan_chunks(batch, n, heads, state_size, vdim, y.device)
+    _note(f"{n}x{heads}x{state_size}x{vdim}", n * (c * u.element_size() + heads * vdim * 4), 6.0 * n * heads * state_size * vdim)
+    _check(_fn("ssm", "tk_ssd_scan")(_code(u.dtype), _p(u), pointer, is_f32, parts, stride, ld, int(dt_col), _p(dt_bias),
+                                     _p(a_log), _p(skip), _p(state), _p(batch.q_start), _p(batch.state_slots), _p(y),
+                                     batch.num_requests, heads, groups, state_size, vdim, *plan, _stream()), "ssd_scan")
+
+
+def fixed_decay_scan(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, y: torch.Tensor, batch, *, heads: int,
+                     dim: int, vdim: int) -> None:
+    """Linear attention with one constant decay a head: per request and head over the step's tokens in order
+    S <- decay S + k_t v_t^T, y_t = S^T q_t, with v, k and q the silu of ``proj``'s columns [v: heads * vdim |
+    k: heads * dim | q: heads * dim | ...] ([N, ld] in the compute dtype or float32, or float32 partial sums
+    [P, N, ld]); decay float32 [heads]; y float32 [N, heads * vdim]; S float32 [slots, heads, ceil(vdim / 4), dim, 4]."""
+    _gpu(proj, decay, state, y)
+    n = y.shape[0]
+    _need(y.dtype == torch.float32 and y.shape == (n, heads * vdim) and batch.num_tokens == n, "the scan's operands do not match its sizes")
+    _need(decay.dtype == torch.float32 and decay.numel() == heads, "the decays are float32 [heads]")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, -(-vdim // 4), dim, 4),
+          "the state is float32 [slots, heads, ceil(vdim / 4), dim, 4]")
+    _need(1 <= vdim <= 1024 and 1 <= dim <= 1024, "the scan takes sizes up to 1,024")
+    dtype = torch.bfloat16 if proj.dtype == torch.bfloat16 else torch.float32
+    pointer, is_f32, parts, stride, ld = _ssm_in(proj, n, dtype, "projections")
+    _need(ld >= heads * (vdim + 2 * dim), "the projections hold v, k and q of every head")
+    plan = _scan_chunks(batch, n, heads, dim, vdim, y.device)
+    _note(f"{n}x{heads}x{dim}x{vdim}", n * heads * ((2 * dim + vdim) * proj.element_size() * parts + vdim * 4),
+          4.0 * n * heads * dim * vdim)
+    _check(_fn("ssm", "tk_fixed_decay_scan")(_code(dtype), pointer, is_f32, parts, stride, ld, _p(decay), _p(state),
+                                             _p(batch.q_start), _p(batch.state_slots), _p(y), batch.num_requests, heads,
+                                             dim, vdim, *plan, _stream()), "fixed_decay_scan")
+
+
+def _scan_chunks(batch, n: int, heads: int, state_size: int, vdim: int, device):
+    """(blocks that share a head's value columns, tokens a chunk, most chunks a request, scratch of the chunks' states,
+    of their decays) of a scan with a scalar decay a head.  Long portions: chunks of SSM_CHUNK_TOKENS tokens side by
+    side (a chunk acts on the state as S -> P S + L, with P and L found from zeros; the chunks' start states follow from
+    those in order; then every chunk runs again from its own start and writes its outputs): twice the arithmetic of
+    one walk, a thirtieth of its length."""
     chunk = max_chunks = 0
     chunk_state = chunk_decay = None
     blocks = batch.num_requests
@@ -1013,29 +1128,88 @@ def ssd_scan(u: torch.Tensor, proj: torch.Tensor, dt_col: int, dt_bias: torch.Te
         chunk = SSM_CHUNK_TOKENS
         max_chunks = -(-batch.max_q_len // chunk)
         blocks = n // chunk + batch.num_requests        # (no step has more chunks than this)
-        chunk_state = torch.empty((blocks, heads, -(-vdim // 4), state_size, 4), dtype=torch.float32, device=y.device)
-        chunk_decay = torch.empty((blocks, heads), dtype=torch.float32, device=y.device)
+        chunk_state = torch.empty((blocks, heads, -(-vdim // 4), state_size, 4), dtype=torch.float32, device=device)
+        chunk_decay = torch.empty((blocks, heads), dtype=torch.float32, device=device)
     splits = ssd_column_splits(blocks, heads, vdim, batch.max_q_len)
-    _note(f"{n}x{heads}x{state_size}x{vdim}", n * (c * u.element_size() + heads * vdim * 4), 6.0 * n * heads * state_size * vdim)
-    _check(_fn("ssm", "tk_ssd_scan")(_code(u.dtype), _p(u), pointer, is_f32, parts, stride, ld, int(dt_col), _p(dt_bias),
-                                     _p(a_log), _p(skip), _p(state), _p(batch.q_start), _p(batch.state_slots), _p(y),
-                                     batch.num_requests, heads, groups, state_size, vdim, splits, chunk, max_chunks,
-                                     _p(chunk_state), _p(chunk_decay), _stream()), "ssd_scan")
+    return splits, chunk, max_chunks, _p(chunk_state), _p(chunk_decay)
+
+
+DELTA_MAX_DIM = 512          # key channels of a head of the delta-rule scan (csrc/delta.hip)
+
+
+def delta_row(heads: int, kv_heads: int, dim: int, vdim: int) -> int:
+    """Numbers a token has in the row that ``delta_inputs`` leaves for ``delta_scan``."""
+    return -(-(2 * kv_heads * dim + heads * (vdim + dim + 1)) // 4) * 4
+
+
+def delta_inputs(proj: torch.Tensor, up: torch.Tensor, conv: torch.Tensor, conv_state: torch.Tensor | None, a_log: torch.Tensor,
+                 dt_bias: torch.Tensor, out: torch.Tensor, batch, *, heads: int, kv_heads: int, dim: int, vdim: int,
+                 q_scale: float) -> None:
+    """The operands of the delta-rule scan, float32 [N, delta_row]: [q | k | v | decay | beta].  q, k, v: the columns
+    [q: kv dim | k: kv dim | v: heads vdim] of ``proj`` through a causal convolution per channel (``conv`` float32
+    [channels, taps], the last tap on the token itself) and silu; q and k per head divided by sqrt(sum(x^2) + 1e-6), q times
+    ``q_scale``; decay = exp(-exp(a_log) softplus(up + dt_bias)) over the first heads * dim columns of ``up``; beta = sigmoid
+    of proj's next ``heads`` columns.  ``conv_state`` float32 [slots, taps - 1, channels] (None with one tap) is carried.
+    proj and up: [N, ld] in one compute dtype or float32, or float32 partial sums [P, N, ld]."""
+    _gpu(proj, up, conv, conv_state, a_log, dt_bias, out)
+    n = out.shape[0]
+    c, taps = conv.shape
+    _need(kv_heads >= 1 and heads % kv_heads == 0 and 1 <= dim <= DELTA_MAX_DIM and vdim >= 1, "the delta rule's sizes do not fit its kernels")
+    _need(conv.dtype == torch.float32 and c == 2 * kv_heads * dim + heads * vdim and 1 <= taps <= SSM_MAX_TAPS,
+          f"the convolution is float32 [channels, taps] with 1 to {SSM_MAX_TAPS} taps")
+    _need(taps == 1 or (conv_state is not None and conv_state.dtype == torch.float32 and tuple(conv_state.shape[1:]) == (taps - 1, c)),
+          "the convolution's state is float32 [slots, taps - 1, channels]")
+    _need(a_log.dtype == torch.float32 and a_log.numel() == heads and dt_bias.dtype == torch.float32
+          and dt_bias.numel() == heads * dim, "a_log is float32 [heads], dt_bias float32 [heads * dim]")
+    _need(out.dtype == torch.float32 and out.shape == (n, delta_row(heads, kv_heads, dim, vdim)) and batch.num_tokens == n,
+          "the operands' rows are float32 [N, delta_row]")
+    dtype = torch.bfloat16 if torch.bfloat16 in (proj.dtype, up.dtype) else torch.float32
+    pp, pf, pn, ps, ld = _ssm_in(proj, n, dtype, "projections")
+    up_, uf, un, us, uld = _ssm_in(up, n, dtype, "decay projection")
+    _need(ld >= c + heads and uld >= heads * dim, "the projections are too narrow")
+    _note(f"{n}x{out.shape[1]}", n * ((c + heads) * proj.element_size() * pn + heads * dim * up.element_size() * un + out.shape[1] * 4))
+    _check(_fn("delta", "tk_delta_inputs")(
+        _code(dtype), pp, pf, pn, ps, ld, up_, uf, un, us, uld, _p(conv), _p(conv_state), _p(a_log), _p(dt_bias),
+        _p(batch.q_start), _p(batch.state_slots), _p(out), batch.num_requests, heads, kv_heads, dim, vdim, taps,
+        float(q_scale), batch.max_q_len, _stream()), "delta_inputs")
+
+
+def delta_scan(operands: torch.Tensor, state: torch.Tensor, y: torch.Tensor, batch, *, heads: int, kv_heads: int, dim: int,
+               vdim: int) -> None:
+    """Per request and head over the step's tokens in order: S <- diag(decay) S, u = beta (v - S^T k), S <- S + k u^T,
+    y = S^T q, from the rows that ``delta_inputs`` leaves.  S float32 [slots, heads, vdim, dim rounded up to 4] (kept;
+    a value column's rows next to each other), y float32 [N, heads * vdim]."""
+    _gpu(operands, state, y)
+    n = y.shape[0]
+    _need(kv_heads >= 1 and heads % kv_heads == 0 and 1 <= dim <= DELTA_MAX_DIM and vdim >= 1, "the delta rule's sizes do not fit its kernels")
+    _need(operands.dtype == torch.float32 and operands.shape == (n, delta_row(heads, kv_heads, dim, vdim))
+          and y.dtype == torch.float32 and y.shape == (n, heads * vdim) and batch.num_tokens == n,
+          "the scan's operands do not match its sizes")
+    _need(state.dtype == torch.float32 and tuple(state.shape[1:]) == (heads, vdim, -(-dim // 4) * 4),
+          "the state is float32 [slots, heads, vdim, dim rounded up to 4]")
+    # (what a call has to move: the rows, the outputs, and every request's state in and out)
+    _note(f"{n}x{heads}x{dim}x{vdim}", (operands.numel() + y.numel() + 2 * batch.num_requests * heads * dim * vdim) * 4,
+          7.0 * n * heads * dim * vdim)
+    _check(_fn("delta", "tk_delta_scan")(_p(operands), _p(state), _p(batch.q_start), _p(batch.state_slots), _p(y),
+                                         batch.num_requests, heads, kv_heads, dim, vdim, _stream()), "delta_scan")
 
 
 def gated_group_norm(y: torch.Tensor, proj: torch.Tensor, z_col: int, weight: torch.Tensor, out: torch.Tensor, *,
-                     groups: int, eps: float) -> None:
+                     groups: int, eps: float, gate_after: bool = False) -> None:
     """g = y * silu(z) with z the columns z_col .. z_col + inner of ``proj``; out = g / rms(g) * weight, the root
-    mean square taken over each of ``groups`` equal parts of the row.  y float32 [N, inner], weight float32 [inner]."""
+    mean square taken over each of ``groups`` equal parts of the row.  y float32 [N, inner], weight float32 [inner], or
+    [inner / groups]: the same for every part.  ``gate_after``: out = y / rms(y) * weight * sigmoid(z)."""
     _gpu(y, proj, weight, out)
     n, inner = out.shape
-    _need(y.dtype == torch.float32 and y.shape == (n, inner) and weight.dtype == torch.float32 and weight.numel() == inner
-          and groups >= 1 and inner % groups == 0, "the gated norm's operands do not match")
+    _need(y.dtype == torch.float32 and y.shape == (n, inner) and groups >= 1 and inner % groups == 0
+          and weight.dtype == torch.float32 and weight.numel() in (inner, inner // groups), "the gated norm's operands do not match")
+    shared = groups > 1 and weight.numel() == inner // groups
     pointer, is_f32, parts, stride, ld = _ssm_in(proj, n, out.dtype, "projections")
     _need(0 <= z_col and z_col + inner <= ld, "the gate lies outside the projections")
     _note(f"{n}x{inner}/{groups}", n * inner * (4 + proj.element_size() * parts + out.element_size()))
     _check(_fn("ssm", "tk_gated_group_norm")(_code(out.dtype), _p(y), pointer, is_f32, parts, stride, ld, int(z_col),
-                                             _p(weight), _p(out), n, inner, groups, float(eps), _stream()), "gated_group_norm")
+                                             _p(weight), _p(out), n, inner, groups, float(eps), int(shared),
+                                             int(bool(gate_after)), _stream()), "gated_group_norm")
 
 
 MOE_LDS_BYTES = 96 * 1024      # of a row of activations in float32 that a block of the expert kernels stages
@@ -1326,12 +1500,14 @@ def gemm_stream(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, splits: 
 
 
 def gemm_stream_swiglu(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, waves: int = 0,
-                       sumsq: torch.Tensor | None = None, eps: float = 0.0, activation: str = "silu") -> None:
+                       sumsq: torch.Tensor | None = None, eps: float = 0.0, activation: str = "silu",
+                       limit: float | None = None) -> None:
     """out[M, I] = act(a @ w[:I]^T) * (a @ w[I:]^T) for M <= 64: the gate and up
     projections and the gate product in one weight-streaming kernel (bfloat16); act is silu or the tanh
     form of gelu.  ``sumsq``, ``eps``: the rows' scale, applied to both products before the gate, as in
     ``gemm_stream``."""
     _need(activation in GATE_ACTIVATIONS, f"the gate's activation is one of {sorted(GATE_ACTIVATIONS)}")
+    _need((activation == "clamped") == (limit is not None), "a limit goes with the clamped gate")
     for t in (a, w, out):
         _need(t.is_cuda and t.dim() == 2 and t.stride(1) == 1, "gemm operands are 2-D GPU tensors with unit inner stride")
     m, k = a.shape
@@ -1345,7 +1521,7 @@ def gemm_stream_swiglu(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, w
     _check(_fn("gemm_mfma", "tk_gemm_stream_swiglu")(_p(a), _p(w), _p(out), m, w.shape[0] // 2, k, a.stride(0),
                                                      w.stride(0), out.stride(0), waves,
                                                      _p(sumsq), slabs, float(eps), GATE_ACTIVATIONS[activation],
-                                                     _stream()), "gemm_stream_swiglu")
+                                                     float(limit or 0.0), _stream()), "gemm_stream_swiglu")
 
 
 WHOLEK_MAX_ROWS = 16    # rows of activations that the whole-K product takes

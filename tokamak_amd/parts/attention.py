@@ -141,6 +141,13 @@ class RotatedUnitAttention(Mixer):
     its own tensor ``vmix`` (one number; the source has the tensor too and does not use it).  All
     layers of one model that mix have kv heads and value sizes alike.  The rotation pairs dimensions
     as the layer's position encoding says (half-split or interleaved).
+
+    ``norm_first``: the norm of q and k comes before the rotation.  ``norm_names``: it has a weight per dim, one
+    for q and one for k (tensors of these names, [head_dim], shared by the heads).  ``bias_suffix``: q, k, v and o have biases (the
+    projection's tensor name plus this suffix), float32; the last one may be left to whoever adds the output to
+    the residual stream (``output_bias``, ``forward(defer_bias=True)``).  ``gate_name``: the concatenated heads are
+    multiplied by sigmoid(W_g h) ahead of the o projection (W_g: the tensor of this name, [heads * value_dim, H]; one
+    product with q, k and v).
     """
 
     capturable = True
@@ -150,7 +157,9 @@ class RotatedUnitAttention(Mixer):
                  softmax_scale: float, norm_eps: float | None, chunk: int | None, dtype, device,
                  names: tuple[str, str, str, str] = ("q", "k", "v", "o"), window: int | None = None,
                  sink: bool = False, value_mix: str | None = None,
-                 extra_names: tuple[str, str] = ("sink", "vmix"), keep_first: int = 0) -> None:
+                 extra_names: tuple[str, str] = ("sink", "vmix"), keep_first: int = 0, norm_first: bool = False,
+                 norm_names: tuple[str, str] | None = None, bias_suffix: str | None = None,
+                 gate_name: str | None = None) -> None:
         super().__init__(dtype=dtype, device=device)
         if num_heads < 1 or num_kv_heads < 1 or num_heads % num_kv_heads:
             raise ValueError(f"num_heads ({num_heads}) must be a multiple of num_kv_heads ({num_kv_heads})")
@@ -179,8 +188,17 @@ class RotatedUnitAttention(Mixer):
         self.sink: torch.Tensor | None = None
         self.vmix: torch.Tensor | None = None
         self.names = tuple(names)
-        self.qkv: torch.Tensor | None = None
+        if (norm_first or norm_names is not None) and norm_eps is None:
+            raise ValueError("norm_first and norm_names go with norm_eps")
+        self.norm_first, self.gate_name = bool(norm_first), gate_name
+        self.norm_names = None if norm_names is None else tuple(norm_names)
+        self.bias_suffix = None if bias_suffix is None else str(bias_suffix)
+        self.qkv: torch.Tensor | None = None        # with a gate: [q; k; v; gate]
         self.o: torch.Tensor | None = None
+        self.qkv_bias: torch.Tensor | None = None
+        self.output_bias: torch.Tensor | None = None
+        self.q_norm: torch.Tensor | None = None
+        self.k_norm: torch.Tensor | None = None
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
         h, nh, nkv, hd, vd = self.hidden_size, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
@@ -191,12 +209,26 @@ class RotatedUnitAttention(Mixer):
             out[prefix + self.extra_names[0]] = TensorSpec((nh,), role="vector")
         if self.value_mix is not None:
             out[prefix + self.extra_names[1]] = TensorSpec((), role="vector")
+        if self.bias_suffix is not None:
+            for name, width in ((q, nh * hd), (k, nkv * hd), (v, nkv * vd), (o, h)):
+                out[prefix + name + self.bias_suffix] = TensorSpec((width,), held="float32")
+        if self.norm_names is not None:
+            for name in self.norm_names:
+                out[prefix + name] = TensorSpec((hd,), role="vector")
+        if self.gate_name is not None:
+            out[prefix + self.gate_name] = TensorSpec((nh * vd, h))
         return out
 
     def bind(self, prefix: str, fetch: Fetch) -> None:
         q, k, v, o = self.names
-        self.qkv = torch.cat([fetch(prefix + n) for n in (q, k, v)], dim=0).contiguous()
+        gate = () if self.gate_name is None else (self.gate_name,)
+        self.qkv = torch.cat([fetch(prefix + n) for n in (q, k, v, *gate)], dim=0).contiguous()
         self.o = fetch(prefix + o)
+        if self.bias_suffix is not None:
+            self.qkv_bias = torch.cat([fetch(prefix + n + self.bias_suffix) for n in (q, k, v)]).contiguous()
+            self.output_bias = fetch(prefix + o + self.bias_suffix)
+        if self.norm_names is not None:
+            self.q_norm, self.k_norm = (fetch(prefix + n) for n in self.norm_names)
         if self.has_sink:
             self.sink = fetch(prefix + self.extra_names[0])
         if self.value_mix is not None:
@@ -241,11 +273,16 @@ class RotatedUnitAttention(Mixer):
                                   "is their source (or its kv heads and value size differ)")
         return kept, 2
 
-    def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None):
+    def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None,
+                defer_bias: bool = False):
         nh, nkv, hd, vd = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         n = h.shape[0]
+        behind = (nh + nkv) * hd + nkv * vd     # rows of the matrix ahead of the gate's
         weight = self.qkv if writes_cache else self.qkv[: nh * hd]
         qkv = linear(h, weight, allow_partials=True)
+        gate, gate_at = qkv, behind
+        if self.gate_name is not None and not writes_cache:
+            gate, gate_at = linear(h, self.qkv[behind:], allow_partials=True), 0
         cos = sin = None
         rotary_dim, interleaved = 0, False
         if position is not None:
@@ -256,16 +293,24 @@ class RotatedUnitAttention(Mixer):
         q = torch.empty((n, nh * self.key_size), dtype=h.dtype, device=h.device)
         kept, value_mode = self._shared_values(batch, n, h.device) if writes_cache else (None, 0)
         ops.rope_norm_store(
-            qkv, None, None, cos, sin, batch.positions, batch.req_of_token, tables, q, store.arrays["k"],
+            qkv, self.q_norm, self.k_norm, cos, sin, batch.positions, batch.req_of_token, tables, q, store.arrays["k"],
             store.arrays["v"], num_heads=nh, num_kv_heads=nkv, head_dim=hd, value_dim=vd, rotary_dim=rotary_dim,
             page_size=store.page_size, unit_norm=self.norm_eps is not None, eps=self.norm_eps or 0.0, store=writes_cache,
-            interleaved=interleaved, value_keep=kept, value_mode=value_mode, value_lambda=self.vmix)
+            interleaved=interleaved, value_keep=kept, value_mode=value_mode, value_lambda=self.vmix, bias=self.qkv_bias,
+            norm_first=self.norm_first)
         attended = torch.empty((n, nh * self.value_size), dtype=h.dtype, device=h.device)
         paged_attention(q, store.arrays["k"], store.arrays["v"], tables, batch, attended, num_heads=nh,
                         num_kv_heads=nkv, head_dim=self.key_size, value_dim=self.value_size, page_size=store.page_size,
                         scale=self.softmax_scale, chunk=self.chunk, window=self.window, sinks=self.sink,
                         keep_first=self.keep_first)
-        return linear(attended, self.o, allow_partials=True)
+        if self.gate_name is not None:
+            ops.sigmoid_gate(attended, gate, gate_at, heads=nh, vdim=vd, vdim_padded=self.value_size)
+        if self.output_bias is None or defer_bias:
+            # (a deferred bias: the caller adds ``output_bias`` where it adds the output to the stream)
+            return linear(attended, self.o, allow_partials=True)
+        out = linear(attended, self.o)
+        ops.add_bias(out, self.output_bias)
+        return out
 
 
 register_part("mixer", "gqa_attention", GQAAttention)

@@ -168,6 +168,25 @@ class BranchPair:
     scale: float = 1.0
 
 
+@dataclass
+class NormedSum:
+    """A sub-layer's output that is normed BEFORE it joins the stream (a norm behind the sub-layer), not yet
+    added: with A = ``first`` + ``bias`` and B = ``second``, each divided by its root mean square and multiplied by its
+    gain where it has one (``first_gain``, ``second_gain``), m = first_weight A + second_weight B, normed likewise if
+    there is a ``gain``; whoever reads the stream next adds m to it.  The branches are [N, H] in the compute dtype or
+    float32, or float32 partial sums [P, N, H]; bias and gains are float32 [H]."""
+
+    first: torch.Tensor
+    second: torch.Tensor | None = None
+    bias: torch.Tensor | None = None
+    first_gain: torch.Tensor | None = None
+    second_gain: torch.Tensor | None = None
+    gain: torch.Tensor | None = None
+    first_weight: float = 1.0
+    second_weight: float = 1.0
+    eps: float = 0.0
+
+
 class Embedding(Part):
     def forward(self, batch) -> torch.Tensor:
         raise NotImplementedError

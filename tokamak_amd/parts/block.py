@@ -4,7 +4,8 @@ from __future__ import annotations
 
 from tokamak_amd.config.registry import register_part
 from tokamak_amd.kernels.linear import Added, StreamSink
-from tokamak_amd.parts.base import Block, BranchPair
+from tokamak_amd.parts.base import Block, BranchPair, NormedSum
+from tokamak_amd.parts.norm import read_stream
 from tokamak_amd.parts.scale import scaled_sum
 
 
@@ -169,6 +170,70 @@ class ParallelSublayersBlock(Block):
         return BranchPair(mixed, *terms, bias=bias, scale=self.branch_scale)
 
 
+class PostNormBlock(Block):
+    """x = x + mixer_norm(mixer(x)); x = x + feed_forward_norm(feed_forward(x)).
+
+    The norms stand behind the sub-layers, which read the stream itself (rounded to the compute dtype).  A sub-layer's
+    output is left pending as a ``NormedSum``: one kernel norms it, adds it to the float32 stream and writes what
+    the next sub-layer reads (or, behind the last layer, norms the sum for the head).
+
+    Instead of one ``mixer`` there may be two side by side, ``left`` and ``right``, each with a cache slot of its
+    own; then mixer(x) = ``left_weight`` left_norm(left(x)) + ``right_weight`` right_norm(right(x)), the two norms and
+    the norm of their sum in the same kernel (both norms or neither; they and the layer's own share one eps).  A left
+    or single mixer, or a feed-forward, that leaves a bias of its last product to the add says so (``output_bias``,
+    ``forward(defer_bias=True)``).  The feed-forward and its norm may be absent together.  An optional ``position``
+    part prepares the step's position data for the mixers.
+    """
+
+    roles = ("mixer_norm",)
+    optional = ("mixer", "left", "right", "left_norm", "right_norm", "position", "feed_forward_norm", "feed_forward")
+    replays_parts = True
+
+    def __init__(self, parts, *, left_weight: float = 0.5, right_weight: float = 0.5) -> None:
+        super().__init__(parts)
+        self.left_weight, self.right_weight = float(left_weight), float(right_weight)
+        self.mixer_norm, self.position = parts["mixer_norm"], parts.get("position")
+        self.left, self.right = parts.get("mixer", parts.get("left")), parts.get("right")
+        self.left_norm, self.right_norm = parts.get("left_norm"), parts.get("right_norm")
+        self.feed_forward, self.feed_forward_norm = parts.get("feed_forward"), parts.get("feed_forward_norm")
+        if ("mixer" in parts) == ("left" in parts) or ("left" in parts) != ("right" in parts):
+            raise ValueError("a layer has one mixer, or a left and a right one")
+        if (self.left_norm is None) != (self.right_norm is None) or (self.left_norm is not None and self.right is None):
+            raise ValueError("the norms of two mixers' outputs come together")
+        if (self.feed_forward is None) != (self.feed_forward_norm is None):
+            raise ValueError("a feed-forward and its norm come together")
+        norms = [n for n in (self.mixer_norm, self.left_norm, self.right_norm, self.feed_forward_norm) if n is not None]
+        if any(getattr(n, "weight_only", False) is not True or n.eps != self.mixer_norm.eps for n in norms):
+            raise ValueError("the norms behind the sub-layers are RMS norms with one eps")
+
+    def forward(self, resid, pending, batch, store, writes_cache):
+        position = None if self.position is None else self.position.prepare(batch)
+        h = read_stream(resid, pending, self.mixer_norm.dtype)
+        if self.right is None:
+            mixed, bias = _biasless(self.left, h, batch, store, writes_cache, position)
+            pending = NormedSum(mixed, bias=bias, gain=self.mixer_norm.weight, eps=self.mixer_norm.eps)
+        else:
+            left, bias = _biasless(self.left, h, batch, store["left"], writes_cache, position)
+            right = self.right.forward(h, batch, store["right"], writes_cache, position)
+            pending = NormedSum(left, right, bias=bias, gain=self.mixer_norm.weight, eps=self.mixer_norm.eps,
+                                first_gain=None if self.left_norm is None else self.left_norm.weight,
+                                second_gain=None if self.right_norm is None else self.right_norm.weight,
+                                first_weight=self.left_weight, second_weight=self.right_weight)
+        if self.feed_forward is None:
+            return pending
+        h = read_stream(resid, pending, self.feed_forward_norm.dtype)
+        out, bias = _biasless(self.feed_forward, h, batch)
+        first, second = out if isinstance(out, tuple) else (out, None)
+        return NormedSum(first, second, bias=bias, gain=self.feed_forward_norm.weight, eps=self.feed_forward_norm.eps)
+
+
+def _biasless(part, *args):
+    """(the part's output, the bias of its last product if it leaves that to the add)."""
+    bias = getattr(part, "output_bias", None)
+    return (part.forward(*args), None) if bias is None else (part.forward(*args, defer_bias=True), bias)
+
+
 register_part("block", "pre_norm", PreNormBlock)
+register_part("block", "post_norm", PostNormBlock)
 register_part("block", "parallel_sublayers", ParallelSublayersBlock)
 register_part("block", "parallel_mixers", ParallelMixersBlock)

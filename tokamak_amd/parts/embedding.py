@@ -14,33 +14,49 @@ from tokamak_amd.weights.spec import TensorSpec
 class TokenEmbedding(Embedding):
     """Row gather into the float32 residual stream (reference: src/tokamak/model/transformer.py:140),
     times ``scale`` if the design has one.  ``add_to`` adds the same rows into a stream once more,
-    for a model that feeds its input in again further up (``LayerCall.adds_embedding``)."""
+    for a model that feeds its input in again further up (``LayerCall.adds_embedding``).  With ``norm_eps``
+    the rows pass an RMS norm with the weight ``norm_tensor``: the normed rows are the stream."""
 
     capturable = True
 
-    def __init__(self, *, vocab_size: int, dim: int, dtype, device, tensor: str = "weight", scale: float = 1.0) -> None:
+    def __init__(self, *, vocab_size: int, dim: int, dtype, device, tensor: str = "weight", scale: float = 1.0,
+                 norm_eps: float | None = None, norm_tensor: str = "norm.weight") -> None:
         super().__init__(dtype=dtype, device=device)
         self.vocab_size, self.dim = int(vocab_size), int(dim)
         self.scale = float(scale)
+        self.norm_eps = None if norm_eps is None else float(norm_eps)
+        self.norm_tensor = str(norm_tensor)
+        self.norm_weight: torch.Tensor | None = None
         self.tensor = str(tensor)       # the matrix's name behind the part's prefix
         self.weight: torch.Tensor | None = None
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
-        return {prefix + self.tensor: TensorSpec((self.vocab_size, self.dim))}
+        out = {prefix + self.tensor: TensorSpec((self.vocab_size, self.dim))}
+        if self.norm_eps is not None:
+            out[prefix + self.norm_tensor] = TensorSpec((self.dim,), role="vector")
+        return out
 
     def bind(self, prefix: str, fetch: Fetch) -> None:
         self.weight = fetch(prefix + self.tensor)
+        if self.norm_eps is not None:
+            self.norm_weight = fetch(prefix + self.norm_tensor)
 
     def tied_matrix(self) -> torch.Tensor:
         return self.weight
 
     def forward(self, batch) -> torch.Tensor:
         resid = torch.empty((batch.num_tokens, self.dim), dtype=torch.float32, device=self.device)
-        ops.embed_gather(self.weight, batch.token_ids, resid, self.scale)
+        self._gather(batch, resid, False)
         return resid
 
     def add_to(self, batch, resid: torch.Tensor) -> None:
-        ops.embed_gather(self.weight, batch.token_ids, resid, self.scale, accumulate=True)
+        self._gather(batch, resid, True)
+
+    def _gather(self, batch, resid: torch.Tensor, accumulate: bool) -> None:
+        if self.norm_eps is None:
+            ops.embed_gather(self.weight, batch.token_ids, resid, self.scale, accumulate=accumulate)
+        else:
+            ops.embed_norm(self.weight, batch.token_ids, self.norm_weight, resid, self.norm_eps, self.scale, accumulate)
 
 
 class LinearHead(Head):

@@ -18,7 +18,8 @@ class SwiGLU(FeedForward):
 
     ``gate_proj`` and ``up_proj`` are held as one [2I, H] matrix so one product
     yields both halves.  ``activation``: what the gate passes through, ``"silu"`` or
-    ``"gelu_tanh"`` (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))).
+    ``"gelu_tanh"`` (0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))); or ``"clamped"`` with a ``limit``: with
+    g = min(gate(x), limit) and u = clamp(up(x), -limit, limit), down(g sigmoid(1.702 g) (u + 1)).
     ``bias_suffix``: every projection has a bias, whose tensor is the projection's name plus this
     suffix: down(act(gate(x) + b_g) * (up(x) + b_u)) + b_d.  The biases are float32 and are added to
     the products' results in float32; the last one may be left to whoever adds the output to the
@@ -30,11 +31,14 @@ class SwiGLU(FeedForward):
 
     def __init__(self, *, hidden_size: int, intermediate_size: int, dtype, device,
                  names: tuple[str, str, str] = ("gate_proj.weight", "up_proj.weight", "down_proj.weight"),
-                 activation: str = "silu", bias_suffix: str | None = None) -> None:
+                 activation: str = "silu", bias_suffix: str | None = None, limit: float | None = None) -> None:
         super().__init__(dtype=dtype, device=device)
         if activation not in GATE_ACTIVATIONS:
             raise ValueError(f"activation is one of {sorted(GATE_ACTIVATIONS)}, got {activation!r}")
+        if (activation == "clamped") != (limit is not None):
+            raise ValueError("a limit goes with the clamped gate")
         self.activation = activation
+        self.limit = None if limit is None else float(limit)
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.names = tuple(names)       # gate, up, down behind the part's prefix
@@ -68,9 +72,9 @@ class SwiGLU(FeedForward):
 
     def forward(self, h, batch, add_into=None, defer_bias: bool = False):
         if self.bias_suffix is None:
-            return linear(gated_linear(h, self.gate_up, self.activation), self.down, allow_partials=True, add_into=add_into)
+            return linear(gated_linear(h, self.gate_up, self.activation, self.limit), self.down, allow_partials=True, add_into=add_into)
         act = torch.empty((h.shape[0], self.intermediate_size), dtype=h.dtype, device=h.device)
-        ops.silu_mul(linear(h, self.gate_up), act, self.activation, bias=self.gate_up_bias)
+        ops.silu_mul(linear(h, self.gate_up), act, self.activation, bias=self.gate_up_bias, limit=self.limit)
         if defer_bias:
             # (the caller adds ``output_bias`` where it adds the output to the stream)
             return linear(act, self.down, allow_partials=True)

@@ -1,4 +1,4 @@
-"""Gated linear attention: a recurrence with a decayed matrix state per head."""
+"""Linear attention: recurrences with a decayed matrix state per head."""
 
 from __future__ import annotations
 
@@ -85,4 +85,59 @@ class GatedLinearAttention(Mixer):
         return linear(out, self.o, allow_partials=True)
 
 
+class FixedDecayLinearAttention(Mixer):
+    """Linear attention whose heads each have one constant decay (the lightning-attention form).
+
+    q = silu(W_q h), k = silu(W_k h) (``num_heads`` heads of ``head_dim``), v = silu(W_v h) (heads of
+    ``value_dim``).  Per head a, with the state S [head_dim, value_dim] (zeros before a sequence's first token):
+    S <- decay_a S + k_t v_t^T, o_t = S^T q_t (no other scale).  The concatenated heads are divided by their common
+    root mean square (``norm_eps``), multiplied by ``norm`` [heads * value_dim] and by sigmoid(W_g h), and projected
+    by W_o.  S is the request's state (float32, a head's value columns in groups of four, as the scan's threads own
+    them).  v, k, q and the gate are one product.  Tensors: q, k, v, g, o, norm behind the part's prefix.
+    """
+
+    capturable = True
+    replayable = True
+
+    def __init__(self, *, hidden_size: int, num_heads: int, head_dim: int, value_dim: int, decay: tuple[float, ...],
+                 norm_eps: float, dtype, device) -> None:
+        super().__init__(dtype=dtype, device=device)
+        self.hidden_size, self.num_heads = int(hidden_size), int(num_heads)
+        self.head_dim, self.value_dim = int(head_dim), int(value_dim)
+        if min(self.hidden_size, self.num_heads, self.head_dim, self.value_dim) < 1 or max(self.head_dim, self.value_dim) > 1024:
+            raise ValueError("head_dim and value_dim are 1 to 1,024 for the scan kernel")
+        if len(decay) != self.num_heads:
+            raise ValueError(f"one decay a head: {self.num_heads} heads, {len(decay)} decays")
+        self.decay = torch.tensor([float(x) for x in decay], dtype=torch.float32, device=self.device)
+        self.norm_eps = float(norm_eps)
+        self.vkqg = self.o = self.gain = None
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        h, kw, vw = self.hidden_size, self.num_heads * self.head_dim, self.num_heads * self.value_dim
+        return {
+            prefix + "q": TensorSpec((kw, h)), prefix + "k": TensorSpec((kw, h)), prefix + "v": TensorSpec((vw, h)),
+            prefix + "g": TensorSpec((vw, h)), prefix + "o": TensorSpec((h, vw)),
+            prefix + "norm": TensorSpec((vw,), role="vector"),
+        }
+
+    def bind(self, prefix: str, fetch: Fetch) -> None:
+        self.vkqg = torch.cat([fetch(prefix + n) for n in ("v", "k", "q", "g")]).contiguous()
+        self.o, self.gain = fetch(prefix + "o"), fetch(prefix + "norm")
+
+    def state_request(self) -> dict[str, StateArray]:
+        return {"S": StateArray((self.num_heads, -(-self.value_dim // 4), self.head_dim, 4), torch.float32)}
+
+    def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None):
+        n, kw, vw = h.shape[0], self.num_heads * self.head_dim, self.num_heads * self.value_dim
+        # (split products leave float32 partial sums, which the kernels below add as they load)
+        proj = linear(h, self.vkqg, allow_partials=True)
+        y = torch.empty((n, vw), dtype=torch.float32, device=h.device)
+        ops.fixed_decay_scan(proj, self.decay, store.state["S"], y, batch, heads=self.num_heads, dim=self.head_dim,
+                             vdim=self.value_dim)
+        gated = torch.empty((n, vw), dtype=self.dtype, device=h.device)
+        ops.gated_group_norm(y, proj, vw + 2 * kw, self.gain, gated, groups=1, eps=self.norm_eps, gate_after=True)
+        return linear(gated, self.o, allow_partials=True)
+
+
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "fixed_decay_linear_attention", FixedDecayLinearAttention)

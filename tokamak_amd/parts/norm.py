@@ -7,8 +7,49 @@ import torch
 from tokamak_amd.config.registry import register_part
 from tokamak_amd.kernels import ops
 from tokamak_amd.kernels.linear import Added, DeferredNorm, StreamSink
-from tokamak_amd.parts.base import BranchPair, Fetch, Norm
+from tokamak_amd.parts.base import BranchPair, Fetch, Norm, NormedSum
 from tokamak_amd.weights.spec import TensorSpec
+
+
+def _normed_sum(pending) -> NormedSum | None:
+    """``pending`` (None, a sub-layer's output, a ``BranchPair`` of up to two terms, a ``NormedSum``) as a ``NormedSum``."""
+    if pending is None or isinstance(pending, NormedSum):
+        return pending
+    if not isinstance(pending, BranchPair):
+        return NormedSum(pending)
+    if pending.third is not None:
+        raise ops.KernelError("a sum of three terms is added by a norm, not by a bare reading of the stream")
+    return NormedSum(pending.first, pending.second, bias=pending.bias, first_weight=pending.scale, second_weight=pending.scale)
+
+
+def _add_normed(resid, p: NormedSum, out, dtype, **kw) -> None:
+    ops.add_normed(resid, p.first, p.second, out, dtype=dtype, eps=p.eps, bias=p.bias, gain_a=p.first_gain,
+                   gain_b=p.second_gain, gain=p.gain, weight_a=p.first_weight, weight_b=p.second_weight, **kw)
+
+
+def read_stream(resid: torch.Tensor, pending, dtype: torch.dtype) -> torch.Tensor:
+    """The stream itself, in ``dtype``, once ``pending`` has been added to it (a layer without a norm ahead of its
+    sub-layers).  One kernel, one rounding; in float32 the stream serves as it is: it must be read before it is
+    written again."""
+    p = _normed_sum(pending)
+    if dtype == torch.float32:
+        if p is not None:
+            _add_normed(resid, p, None, dtype)
+        return resid
+    out = torch.empty(resid.shape, dtype=dtype, device=resid.device)
+    if p is None:
+        ops.add_normed(resid, None, None, out, dtype=dtype, write_resid=False)
+    else:
+        _add_normed(resid, p, out, dtype)
+    return out
+
+
+def settle(resid: torch.Tensor, pending, dtype: torch.dtype):
+    """``pending`` as a norm takes it: a ``NormedSum`` is added to the stream now, anything else is handed back."""
+    if not isinstance(pending, NormedSum):
+        return pending
+    _add_normed(resid, pending, None, dtype)
+    return None
 
 
 class RMSNorm(Norm):
@@ -24,6 +65,7 @@ class RMSNorm(Norm):
     capturable = True
     fuses_residual = True
     replayable = True
+    weight_only = True      # x / rms(x) times ``weight`` and nothing else: other kernels may apply it
 
     def __init__(self, *, dim: int, eps: float, dtype, device, tensor: str = "weight", offset: float = 0.0) -> None:
         super().__init__(dtype=dtype, device=device)
@@ -53,6 +95,10 @@ class RMSNorm(Norm):
             delta = None
         m = resid.shape[0] if rows is None else rows.numel()
         out = torch.empty((m, self.dim), dtype=self.dtype, device=resid.device)
+        if isinstance(delta, NormedSum):
+            # a sub-layer's output with a norm of its own: both norms and the add in one kernel
+            _add_normed(resid, delta, out, self.dtype, out_weight=self.weight, out_eps=self.eps, rows=rows, write_resid=write_resid)
+            return out
         if isinstance(delta, BranchPair):
             # branches that belong to one residual add: their sum is formed first, then added
             ops.add_norm2(resid, delta.first, delta.second, self.weight, self.eps, out, center=False, rows=rows,
@@ -69,6 +115,7 @@ class RMSNorm(Norm):
             return None
         if isinstance(delta, Added):
             delta = None
+        delta = settle(resid, delta, self.dtype)
         pair = delta if isinstance(delta, BranchPair) else BranchPair(delta) if delta is not None else None
         out = torch.empty((resid.shape[0], self.dim), dtype=self.dtype, device=resid.device)
         out2 = torch.empty_like(out)
@@ -114,6 +161,7 @@ class LayerNorm(Norm):
         self.weight = fetch(prefix + self.tensor)
 
     def forward(self, resid, delta, *, rows=None, write_resid=True):
+        delta = settle(resid, delta, self.dtype)
         pair = delta if isinstance(delta, BranchPair) else BranchPair(delta)
         m = resid.shape[0] if rows is None else rows.numel()
         out = torch.empty((m, self.dim), dtype=self.dtype, device=resid.device)
