@@ -2,7 +2,9 @@
 per mechanism, whole sequences at a time, no cache, no kernels, nothing shared with the engine.
 
 ``cfg`` is the parsed ``config.json`` (a dict), ``w`` maps tensor names to torch tensors.  Everything
-is computed in the dtype of ``DTYPE`` (float64 by default).
+is computed in the dtype of ``DTYPE`` (float64 by default).  With ``ROUNDED`` set the rows that enter a
+product with a weight matrix and those that leave it are rounded to bfloat16: how far that alone moves a
+logit is what a bfloat16 engine's error at that position is measured with.
 """
 
 from __future__ import annotations
@@ -10,10 +12,18 @@ from __future__ import annotations
 import torch
 
 DTYPE = torch.float64
+ROUNDED = False
 
 
 def _f(t: torch.Tensor) -> torch.Tensor:
     return t.to(DTYPE)
+
+
+def product(x: torch.Tensor, matrix: torch.Tensor) -> torch.Tensor:
+    """x @ matrix^T for rows x [T, in] and a matrix [out, in]."""
+    if not ROUNDED:
+        return x @ _f(matrix).T
+    return (x.to(torch.bfloat16).to(DTYPE) @ _f(matrix).T).to(torch.bfloat16).to(DTYPE)
 
 
 def rms_norm(x: torch.Tensor, weight: torch.Tensor | None, eps: float) -> torch.Tensor:
@@ -49,12 +59,12 @@ def delta_operands(h: torch.Tensor, w: dict, p: str, m: dict):
     """(q, k [T, heads, dim], v [T, heads, vdim], beta [T, heads], decay [T, heads, dim])."""
     t = h.shape[0]
     heads, kv, dim, vdim = int(m["heads"]), int(m.get("kv_heads") or m["heads"]), int(m["dim"]), int(m["vdim"])
-    q, k, v = (silu(causal_conv(h @ _f(w[p + n]).T, w[p + n + ".conv"])) for n in ("q", "k", "v"))
+    q, k, v = (silu(causal_conv(product(h, w[p + n]), w[p + n + ".conv"])) for n in ("q", "k", "v"))
     q, k, v = q.view(t, kv, dim), k.view(t, kv, dim), v.view(t, heads, vdim)
     q, k = unit(q) * dim ** -0.5, unit(k)
     of_head = [a // (heads // kv) for a in range(heads)]
-    beta = torch.sigmoid(h @ _f(w[p + "b"]).T)
-    step = softplus((h @ _f(w[p + "a1"]).T) @ _f(w[p + "a2"]).T + _f(w[p + "dt_bias"])).view(t, heads, dim)
+    beta = torch.sigmoid(product(h, w[p + "b"]))
+    step = softplus(product(product(h, w[p + "a1"]), w[p + "a2"]) + _f(w[p + "dt_bias"])).view(t, heads, dim)
     decay = torch.exp(-torch.exp(_f(w[p + "A_log"]))[None, :, None] * step)
     return q[:, of_head], k[:, of_head], v, beta, decay
 
@@ -76,8 +86,8 @@ def delta_rule(q, k, v, beta, decay, state=None):
 def channel_delta(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch.Tensor:
     t = h.shape[0]
     o, _ = delta_rule(*delta_operands(h, w, p, m))
-    gate = torch.sigmoid((h @ _f(w[p + "g1"]).T) @ _f(w[p + "g2"]).T)
-    return (rms_norm(o, w[p + "norm"], eps).reshape(t, -1) * gate) @ _f(w[p + "o"]).T
+    gate = torch.sigmoid(product(product(h, w[p + "g1"]), w[p + "g2"]))
+    return product(rms_norm(o, w[p + "norm"], eps).reshape(t, -1) * gate, w[p + "o"])
 
 
 # ---------------------------------------------------------------------------------------------
@@ -117,11 +127,11 @@ def softmax_attention(q, k, v, scale: float, mask: dict | None) -> torch.Tensor:
 def chunked_attention(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch.Tensor:
     t = h.shape[0]
     heads, kv, dim, vdim = int(m["heads"]), int(m.get("kv_heads") or m["heads"]), int(m["dim"]), int(m["vdim"])
-    q, k, v = (h @ _f(w[p + n]).T + _f(w[p + n + ".b"]) for n in ("q", "k", "v"))
+    q, k, v = (product(h, w[p + n]) + _f(w[p + n + ".b"]) for n in ("q", "k", "v"))
     q = rotate(rms_norm(q.view(t, heads, dim), w[p + "q.norm"], eps), m.get("rot"))
     k = rotate(rms_norm(k.view(t, kv, dim), w[p + "k.norm"], eps), m.get("rot"))
     o = softmax_attention(q, k, v.view(t, kv, vdim), float(m["scale"]), m.get("mask")).reshape(t, heads * vdim)
-    return (o * torch.sigmoid(h @ _f(w[p + "g"]).T)) @ _f(w[p + "o"]).T + _f(w[p + "o.b"])
+    return product(o * torch.sigmoid(product(h, w[p + "g"])), w[p + "o"]) + _f(w[p + "o.b"])
 
 
 # ---------------------------------------------------------------------------------------------
@@ -140,11 +150,11 @@ def fixed_decay_scan(q, k, v, decay, state=None):
 def lightning_attention(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch.Tensor:
     t = h.shape[0]
     heads, dim, vdim = int(m["heads"]), int(m["dim"]), int(m["vdim"])
-    q, k = (silu(h @ _f(w[p + n]).T).view(t, heads, dim) for n in ("q", "k"))
-    v = silu(h @ _f(w[p + "v"]).T).view(t, heads, vdim)
+    q, k = (silu(product(h, w[p + n])).view(t, heads, dim) for n in ("q", "k"))
+    v = silu(product(h, w[p + "v"])).view(t, heads, vdim)
     o, _ = fixed_decay_scan(q, k, v, torch.tensor([float(x) for x in m["decay"]], dtype=DTYPE))
-    y = rms_norm(o.reshape(t, heads * vdim), w[p + "norm"], eps) * torch.sigmoid(h @ _f(w[p + "g"]).T)
-    return y @ _f(w[p + "o"]).T
+    y = rms_norm(o.reshape(t, heads * vdim), w[p + "norm"], eps) * torch.sigmoid(product(h, w[p + "g"]))
+    return product(y, w[p + "o"])
 
 
 def parallel(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> torch.Tensor:
@@ -160,7 +170,7 @@ def clamped_gate(g: torch.Tensor, u: torch.Tensor, limit: float) -> torch.Tensor
 
 
 def feed_forward(h: torch.Tensor, w: dict, p: str, mlp: dict) -> torch.Tensor:
-    return clamped_gate(h @ _f(w[p + "gate"]).T, h @ _f(w[p + "up"]).T, float(mlp["limit"])) @ _f(w[p + "down"]).T
+    return product(clamped_gate(product(h, w[p + "gate"]), product(h, w[p + "up"]), float(mlp["limit"])), w[p + "down"])
 
 
 def embedding(w: dict, tokens: list[int], eps: float) -> torch.Tensor:
@@ -179,5 +189,5 @@ def forward(cfg: dict, w: dict, tokens: list[int]) -> tuple[torch.Tensor, torch.
         if layer.get("mlp") is not None:
             x = x + rms_norm(feed_forward(x, w, p + "mlp.", layer["mlp"]), w[p + "norm2"], eps)
         after.append(x)
-    logits = rms_norm(x, w["final.norm"], eps) @ _f(w["head"]).T * float(cfg.get("logit_scale", 1.0))
+    logits = product(rms_norm(x, w["final.norm"], eps), w["head"]) * float(cfg.get("logit_scale", 1.0))
     return logits, torch.stack(after)

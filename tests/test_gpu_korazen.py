@@ -1,0 +1,617 @@
+"""The Korazen design in the engine against the plain implementation (plain_korazen.py): each
+mechanism alone, then whole models of several small shapes through the step function: whole
+prompts, tails one by one, portions down to two tokens, mixed batches with pages and state slots
+used again, edges of chunks with sharp attention, a far key that stands out among hundreds, the delta
+rule holding one write for hundreds of tokens, long decoding through recorded steps, greedy generation
+through ``LLM.generate``, and the trace runner."""
+
+import json
+import subprocess
+import sys
+from pathlib import Path
+
+import numpy as np
+import pytest
+import torch
+
+import plain_korazen as plain
+from kernel_util import make_batch
+from korazen_util import (Expected, delta, dense, double, left, model_json, oracle_logits, parallel, random_weights, right,
+                          tokens, write_folder)
+from replay_util import mixed, portions, tail_one_by_one, whole
+from rorosun_util import run_steps
+from test_gpu_mepupel import BOTH, DEV, close, fresh_store, row_errors, summed
+
+pytestmark = pytest.mark.gpu
+ROOT = Path(__file__).resolve().parent.parent
+LIMIT = 1e-4           # float32: every row, |difference| over the row's largest |logit|
+
+
+def check_rows(steps, got, expected, dtype, what=""):
+    """float32: every row within ``LIMIT``.  bfloat16: a row's limit is three times the error that rounding alone
+    causes there (or typically in that model, if that is more: a single row's luck is no measure); one row in fifty may
+    pass it (a norm behind a nearly cancelled sum magnifies rounding), none by more than four times."""
+    errors = row_errors(steps, got, {rid: e.logits for rid, e in expected.items()})
+    if dtype == "float32":
+        assert max(errors)[0] <= LIMIT, (what, max(errors), len(errors))
+        return len(errors)
+    usual = float(np.quantile(np.concatenate([e.noise for e in expected.values()]), 0.75))
+    over = [(err / (3.0 * max(usual, float(expected[where[1]].noise[where[2]]))), err, where) for err, where in errors]
+    bad = sorted(o for o in over if not o[0] <= 1.0)
+    assert len(bad) * 50 <= len(over) and all(o[0] <= 4.0 for o in bad), (what, usual, len(bad), len(over), bad[-3:])
+    return len(errors)
+
+
+def fetcher(tensors, dtype):
+    def fetch(name):
+        t = tensors[name]
+        held = dtype if t.dim() == 2 and not name.endswith(".conv") else torch.float32
+        return t.to(DEV, held).contiguous()
+    return fetch
+
+
+def cut_spans(part, store, hs, slots, cuts):
+    """Run a mixer over several requests' rows in the given cuts; {request: output rows}.  Requests are left out
+    of a step now and then."""
+    from tokamak_amd.engine.batch import StepSpan, build_batch
+    from tokamak_amd.kernels.attention import ATTENTION_WORK
+
+    done = {r: 0 for r in hs}
+    got = {r: [] for r in hs}
+    step = 0
+    while any(done[r] < len(hs[r]) for r in hs):
+        spans, names = [], []
+        for i, r in enumerate(hs):
+            if done[r] >= len(hs[r]) or (step % 3 == 1 and i == 1 and any(done[q] < len(hs[q]) for q in hs if q != r)):
+                continue
+            n = cuts[r][len(got[r])] if len(got[r]) < len(cuts[r]) else len(hs[r]) - done[r]
+            n = min(n, len(hs[r]) - done[r])
+            spans.append(StepSpan(request=r, tokens=[0] * n, ctx_len=done[r], state_slot=slots[r],
+                                  tables=[[0]]))
+            names.append((r, n))
+        batch = build_batch(spans, 1, DEV, [ATTENTION_WORK])
+        h = torch.cat([hs[r][done[r]:done[r] + n] for r, n in names]).to(DEV)
+        out = summed(part.forward(h, batch, store))
+        at = 0
+        for r, n in names:
+            got[r].append(out[at:at + n])
+            at += n
+            done[r] += n
+        step += 1
+    return {r: torch.cat(rows) for r, rows in got.items()}
+
+
+# -- mechanisms alone -------------------------------------------------------------
+@BOTH
+@pytest.mark.parametrize("width", [64, 50, 328, 4100])
+@pytest.mark.parametrize("rows", [3, 700])
+def test_normed_outputs_join_the_stream(dtype, width, rows):
+    """One branch with a bias and a norm behind it; two branches, each normed, half their sum normed again;
+    the stream read back as it is, or through a norm at picked rows; partial sums, both ways a norm's rows fit a block."""
+    from tokamak_amd.config import get_part
+    from tokamak_amd.parts.base import BranchPair, NormedSum
+    from tokamak_amd.parts.norm import read_stream
+
+    if rows > 100 and width > 400:
+        rows = 520
+    g = torch.Generator().manual_seed(width + rows)
+    gains = [1.0 + 0.3 * torch.randn(width, generator=g) for _ in range(4)]
+    x = 2.0 * torch.randn(rows, width, generator=g)
+    a = 3.0 * torch.randn(rows, width, generator=g).to(dtype)
+    b = 0.2 * torch.randn(3, rows, width, generator=g)
+    bias = torch.randn(width, generator=g)
+    dev = [t.to(DEV) for t in gains]
+    one = plain.rms_norm(a.double() + bias.double(), gains[0], 1e-4)
+    two = plain.rms_norm(0.5 * (plain.rms_norm(a.double() + bias.double(), gains[1], 1e-4)
+                                + plain.rms_norm(b.double().sum(0), gains[2], 1e-4)), gains[0], 1e-4)
+    bare = 0.3 * (a.double() + b.double().sum(0) + bias.double())
+    final = get_part("norm", "rmsnorm")(dim=width, eps=1e-2, tensor="", dtype=dtype, device=DEV)
+    final.bind("n", lambda name: dev[3])
+    layer_norm = get_part("norm", "layernorm")(dim=width, eps=1e-2, tensor="", dtype=dtype, device=DEV)
+    layer_norm.bind("n", lambda name: dev[3])
+    for m, pending in (
+            (one, NormedSum(a.to(DEV), bias=bias.to(DEV), gain=dev[0], eps=1e-4)),
+            (two, NormedSum(a.to(DEV), b.to(DEV), bias=bias.to(DEV), first_gain=dev[1], second_gain=dev[2], gain=dev[0],
+                            first_weight=0.5, second_weight=0.5, eps=1e-4)),
+            (bare, BranchPair(a.to(DEV), b.to(DEV), bias=bias.to(DEV), scale=0.3)),
+            (a.double(), a.to(DEV))):
+        resid = x.to(DEV)
+        got = read_stream(resid, pending, dtype)
+        assert torch.allclose(resid.cpu().double(), x.double() + m, atol=3e-5)
+        assert got.dtype == dtype and torch.equal(got, resid.to(dtype))
+        # through the norm that follows the last layer, at picked rows: the stream stays
+        picked = torch.tensor([rows - 1, 0, rows - 1], dtype=torch.int32, device=DEV)
+        resid = x.to(DEV)
+        out = final.forward(resid, pending, rows=picked, write_resid=False)
+        close(out.float().cpu(), plain.rms_norm(x.double() + m, gains[3], 1e-2).float()[picked.cpu().long()], dtype)
+        assert torch.equal(resid.cpu(), x)
+        # a layer norm, which has no form of its own for such a sum, adds it first
+        resid = x.to(DEV)
+        out = layer_norm.forward(resid, pending)
+        y = x.double() + m
+        y = y - y.mean(-1, keepdim=True)
+        close(out.float().cpu(), plain.rms_norm(y, gains[3], 1e-2).float(), dtype)
+        assert torch.allclose(resid.cpu().double(), x.double() + m, atol=3e-5)
+    # nothing pending: the stream as it is
+    resid = x.to(DEV)
+    assert torch.equal(read_stream(resid, None, dtype), resid.to(dtype)) and torch.equal(resid.cpu(), x)
+
+
+@BOTH
+@pytest.mark.parametrize("width", [64, 50, 1032])
+def test_embedding_with_a_norm(dtype, width):
+    from tokamak_amd.config import get_part
+
+    g = torch.Generator().manual_seed(width)
+    table, weight = torch.randn(31, width, generator=g).to(dtype), 1.0 + 0.3 * torch.randn(width, generator=g)
+    part = get_part("embedding", "token_embedding")(vocab_size=31, dim=width, tensor="", norm_eps=1e-3, norm_tensor=".norm",
+                                                    dtype=dtype, device=DEV)
+    assert set(part.expected_tensors("embed")) == {"embed", "embed.norm"}
+    part.bind("embed", {"embed": table.to(DEV), "embed.norm": weight.to(DEV)}.__getitem__)
+    batch = make_batch([(5, 0, [0]), (1, 3, [1])])
+    ids = torch.tensor([0, 30, 7, 7, 1, 12], dtype=torch.int32)
+    batch.token_ids.copy_(ids)
+    want = plain.rms_norm(table.double()[ids.long()], weight, 1e-3)
+    resid = part.forward(batch)
+    assert torch.allclose(resid.cpu().double(), want, atol=2e-5)
+    part.add_to(batch, resid)
+    assert torch.allclose(resid.cpu().double(), 2 * want, atol=4e-5)
+
+
+DELTAS = {
+    "base": dict(heads=4, kv_heads=2, dim=16, vdim=24, conv=4),
+    "odd": dict(heads=3, kv_heads=1, dim=21, vdim=18, conv=3),
+    "ones": dict(heads=2, kv_heads=2, dim=1, vdim=1, conv=1),
+    "wide": dict(heads=2, kv_heads=1, dim=128, vdim=64, conv=8),
+    "taps2": dict(heads=6, kv_heads=3, dim=100, vdim=40, conv=2),
+    "long-k": dict(heads=1, kv_heads=1, dim=264, vdim=20, conv=5),
+    "mid-k": dict(heads=2, kv_heads=2, dim=160, vdim=33, conv=4),
+    "quarter-k": dict(heads=5, kv_heads=5, dim=252, vdim=16, conv=4),
+}
+RANKS = {"base": (8, 8), "odd": (5, 12), "ones": (1, 1), "wide": (24, 40), "taps2": (16, 3), "long-k": (8, 16), "mid-k": (7, 9),
+         "quarter-k": (8, 8)}
+
+
+@BOTH
+@pytest.mark.parametrize("name", list(DELTAS))
+def test_delta_rule_in_portions_over_state_slots(dtype, name):
+    """Three requests in portions of unlike sizes (down to one and two tokens, shorter than the convolution;
+    one of 150 tokens, which the operands' kernel walks in several segments), state slots out of order, foreign
+    slots untouched; the final states compared."""
+    from tokamak_amd.config import get_part
+
+    m = DELTAS[name]
+    width = 64
+    cfg = model_json([delta(**m)], width=width)
+    w = random_weights(cfg, seed=m["dim"], ranks=RANKS[name])
+    part = get_part("mixer", "channel_delta_rule")(
+        hidden_size=width, num_heads=m["heads"], num_kv_heads=m["kv_heads"], head_dim=m["dim"], value_dim=m["vdim"],
+        conv_taps=m["conv"], norm_eps=1e-5, dtype=dtype, device=DEV)
+    expected = part.expected_tensors("l0.mix.")
+    assert set(expected) == {n for n in w if n.startswith("l0.mix.")} and all(expected[n].fits(w[n].shape) for n in expected)
+    part.bind("l0.mix.", fetcher(w, dtype))
+    store = fresh_store(part, 16, 1, dtype, 0.0, slots=5)
+    for array in store.state.values():
+        array[3].fill_(7.0)            # a slot that belongs to nobody here
+    g = torch.Generator().manual_seed(5)
+    hs = {r: torch.randn(n, width, generator=g).to(dtype) for r, n in {"a": 190, "b": 23, "c": 9}.items()}
+    slots = {"a": 2, "b": 0, "c": 4}
+    cuts = {"a": [150, 1, 2, 30, 1, 1, 5], "b": [2, 1, 1, 3, 16], "c": [1, 1, 1, 2, 4]}
+    got = cut_spans(part, store, hs, slots, cuts)
+    mixer = cfg["layers"][0]["mixer"]
+    for r, h in hs.items():
+        close(got[r], plain.channel_delta(h.double(), double(w), "l0.mix.", mixer, 1e-5).float(), dtype, slack=2.0)
+        _, state = plain.delta_rule(*plain.delta_operands(h.double(), double(w), "l0.mix.", mixer))
+        held = store.state["S"][slots[r]].cpu()          # [heads, vdim, dim rounded up to 4]
+        close(held[:, :, :m["dim"]].permute(0, 2, 1), state.float(), dtype, slack=2.0)
+        assert bool((held[:, :, m["dim"]:] == 0).all())
+        if m["conv"] > 1:      # the convolution's state is the last taps - 1 inputs, oldest first
+            rows = torch.cat([h.double() @ double(w)["l0.mix." + n].T for n in ("q", "k", "v")], dim=1)
+            close(store.state["conv"][slots[r]].cpu(), rows[-(m["conv"] - 1):].float(), dtype)
+    for array in store.state.values():
+        assert bool((array[3] == 7.0).all()) and bool((array[1] == 0.0).all())
+
+
+@pytest.mark.parametrize("tokens_a", [40, 700])
+def test_delta_scan_remembers_one_write_and_replaces_it(tokens_a):
+    """Decays of one: a value written under one key is read back hundreds of tokens later among writes under keys
+    orthogonal to it, and a second write under that key (beta one) replaces it instead of adding to it."""
+    from tokamak_amd.kernels import ops
+
+    heads, kv, dim, vdim = 2, 1, 24, 20
+    n = tokens_a
+    g = torch.Generator().manual_seed(n)
+    q = torch.zeros(n, kv, dim, dtype=torch.float64)
+    k = torch.zeros(n, kv, dim, dtype=torch.float64)
+    v = torch.randn(n, heads, vdim, generator=g, dtype=torch.float64)
+    for t in range(n):
+        k[t, 0, 1 + t % (dim - 1)] = 1.0           # channel 0 belongs to the marked key
+    k[3] = 0.0
+    k[3, 0, 0] = 1.0
+    k[n // 2] = 0.0
+    k[n // 2, 0, 0] = 1.0
+    q[:, :, 0] = 1.0
+    beta, decay = torch.ones(n, heads, dtype=torch.float64), torch.ones(n, heads, dim, dtype=torch.float64)
+    row = ops.delta_row(heads, kv, dim, vdim)
+    flat = torch.cat([q.reshape(n, -1), k.reshape(n, -1), v.reshape(n, -1), decay.reshape(n, -1), beta], dim=1)
+    operands = torch.zeros(n, row, dtype=torch.float32)
+    operands[:, :flat.shape[1]] = flat.float()
+    state = torch.zeros(2, heads, vdim, dim, dtype=torch.float32, device=DEV)
+    y = torch.empty(n, heads * vdim, dtype=torch.float32, device=DEV)
+    ops.delta_scan(operands.to(DEV), state, y, make_batch([(n, 0, [0])]), heads=heads, kv_heads=kv, dim=dim, vdim=vdim)
+    y = y.cpu().double().view(n, heads, vdim)
+    assert torch.equal(y[:3], torch.zeros_like(y[:3]))
+    assert torch.allclose(y[3:n // 2], v[3].expand(n // 2 - 3, -1, -1), atol=1e-5)
+    assert torch.allclose(y[n // 2:], v[n // 2].expand(n - n // 2, -1, -1), atol=1e-5)
+
+
+LIGHTNINGS = {
+    "base": dict(heads=2, dim=16, vdim=24),
+    "odd": dict(heads=3, dim=20, vdim=18, decay=(0.5, 0.9, 0.997)),
+    "ones": dict(heads=1, dim=1, vdim=1, decay=(0.75,)),
+    "wide": dict(heads=5, dim=64, vdim=64, decay=(1.0, 0.0, 0.3, 0.99, 0.9999)),
+    "long": dict(heads=4, dim=130, vdim=36, decay=(0.2, 0.6, 0.95, 0.998)),
+}
+
+
+@BOTH
+@pytest.mark.parametrize("name", list(LIGHTNINGS))
+def test_fixed_decay_attention_in_portions_over_state_slots(dtype, name):
+    """Portions below and above the length from which they run as chunks side by side, single tokens, state
+    slots out of order; decays of one and zero among them; final states compared."""
+    from tokamak_amd.config import get_part
+
+    r = right(**LIGHTNINGS[name])
+    width = 72
+    cfg = model_json([{"type": "parallel", "mixer": {"left": left(), "right": r}, "mlp": None}], width=width)
+    w = random_weights(cfg, seed=r["dim"])
+    part = get_part("mixer", "fixed_decay_linear_attention")(
+        hidden_size=width, num_heads=r["heads"], head_dim=r["dim"], value_dim=r["vdim"], decay=tuple(r["decay"]), norm_eps=1e-5,
+        dtype=dtype, device=DEV)
+    p = "l0.mix.right."
+    assert set(part.expected_tensors(p)) == {n for n in w if n.startswith(p)} - {p + "out"}
+    part.bind(p, fetcher(w, dtype))
+    store = fresh_store(part, 16, 1, dtype, 0.0, slots=4)
+    store.state["S"][1].fill_(5.0)
+    g = torch.Generator().manual_seed(6)
+    hs = {x: torch.randn(n, width, generator=g).to(dtype) for x, n in {"a": 330, "b": 40, "c": 7}.items()}
+    slots = {"a": 3, "b": 0, "c": 2}
+    got = cut_spans(part, store, hs, slots, {"a": [200, 1, 63, 2, 1, 1], "b": [2, 30, 1, 1], "c": [1, 1, 2]})
+    for x, h in hs.items():
+        close(got[x], plain.lightning_attention(h.double(), double(w), p, r, 1e-5).float(), dtype, slack=2.0)
+        q, k = (plain.silu(h.double() @ double(w)[p + n].T).view(len(h), r["heads"], r["dim"]) for n in ("q", "k"))
+        v = plain.silu(h.double() @ double(w)[p + "v"].T).view(len(h), r["heads"], r["vdim"])
+        _, state = plain.fixed_decay_scan(q, k, v, torch.tensor(r["decay"], dtype=torch.float64))
+        held = store.state["S"][slots[x]].cpu().permute(0, 2, 1, 3).reshape(r["heads"], r["dim"], -1)
+        close(held[:, :, :r["vdim"]], state.float(), dtype, slack=2.0)
+    assert bool((store.state["S"][1] == 5.0).all())
+
+
+LEFTS = {
+    "g2": dict(heads=4, kv_heads=2, dim=16, vdim=32, rot=8, chunk=24),
+    "equal": dict(heads=6, kv_heads=3, dim=64, vdim=64, rot=64, chunk=48),
+    "g4": dict(heads=8, kv_heads=2, dim=32, vdim=48, rot=16, chunk=100),
+    "odd": dict(heads=3, kv_heads=1, dim=20, vdim=36, rot=6, chunk=17, base=5e5),
+    "g1-norot": dict(heads=2, kv_heads=2, dim=40, vdim=16, rot=0, chunk=33),
+    "chunk1": dict(heads=2, kv_heads=1, dim=16, vdim=16, rot=4, chunk=1),
+    "causal": dict(heads=4, kv_heads=1, dim=128, vdim=128, rot=128, chunk=None),
+    "g16": dict(heads=16, kv_heads=1, dim=24, vdim=16, rot=24, chunk=70),
+}
+
+
+@BOTH
+@pytest.mark.parametrize("name", list(LEFTS))
+def test_chunked_gated_attention_with_biases_and_weighted_norms_alone(dtype, name):
+    """Portions that end inside pages and chunks, two tokens, then single tokens, pages scattered.  Leaving out a
+    bias, a norm's weight, the order of norm and rotation, the gate or the chunks would move the output."""
+    from tokamak_amd.config import get_part
+
+    m = left(**LEFTS[name])
+    width, page = 64, 16 if m["dim"] * m["heads"] >= 64 else 8
+    cfg = model_json([{"type": "parallel", "mixer": {"left": m, "right": right()}, "mlp": None}], width=width)
+    w = random_weights(cfg, seed=m["dim"] + m["heads"], sharp=3.0)
+    p = "l0.mix.left."
+    T = 230
+    h = torch.randn(T, width, generator=torch.Generator().manual_seed(2)).to(dtype)
+    want = plain.chunked_attention(h.double(), double(w), p, m, 1e-5)
+    for n in ("q.b", "k.b", "v.b", "o.b", "q.norm", "k.norm", "g"):
+        other = {k: (torch.ones_like(t) if n.endswith("norm") else torch.zeros_like(t)) if k == p + n else t for k, t in double(w).items()}
+        moved = float((plain.chunked_attention(h.double(), other, p, m, 1e-5) - want).abs().max() / want.abs().max())
+        assert moved > 0.02 or (m.get("mask") or {}).get("size") == 1, n      # (alone in its chunk a key weighs one whatever its score)
+    mask = m.get("mask")
+    part = get_part("mixer", "rotated_unit_attention")(
+        hidden_size=width, num_heads=m["heads"], num_kv_heads=m["kv_heads"], head_dim=m["dim"], value_dim=m["vdim"],
+        softmax_scale=m["scale"], norm_eps=1e-5, chunk=None if mask is None else mask["size"], norm_first=True,
+        norm_names=("q.norm", "k.norm"), bias_suffix=".b", gate_name="g", dtype=dtype, device=DEV)
+    position = None
+    if m.get("rot"):
+        position = get_part("position", "rotary_half")(rotary_dim=m["rot"]["dims"], theta=m["rot"]["base"], dtype=dtype, device=DEV)
+    assert set(part.expected_tensors(p)) == {n for n in w if n.startswith(p)} - {p + "out"}
+    part.bind(p, fetcher(w, dtype))
+    padded = (part.key_size, part.value_size) != (m["dim"], m["vdim"])
+    store = fresh_store(part, page, 40, dtype, 0.0 if padded else float("nan"))
+    table = [(7 * i + 3) % 40 for i in range(-(-T // page))]
+    out, at = [], 0
+    for n in [100, 41, 2, 33] + [1] * (T - 176):
+        batch = make_batch([(n, at, table)])
+        data = None if position is None else position.prepare(batch)
+        rows = h[at:at + n].to(DEV)
+        if at % 2:
+            out.append(summed(part.forward(rows, batch, store, True, data)))
+        else:      # (the last bias left to whoever adds the output to the stream)
+            out.append(summed(part.forward(rows, batch, store, True, data, defer_bias=True)) + part.output_bias.cpu())
+        at += n
+    close(torch.cat(out), want.float(), dtype, slack=2.0)
+    # a call that only reads the cache: the gate is a product of its own then
+    batch = make_batch([(1, T - 1, table)])
+    again = summed(part.forward(h[T - 1:].to(DEV), batch, store, False, None if position is None else position.prepare(batch)))
+    close(again, want[T - 1:].float(), dtype, slack=4.0)
+
+
+@BOTH
+@pytest.mark.parametrize("rows,width,ff", [(1, 64, 48), (5, 64, 48), (50, 256, 136), (70, 72, 40), (300, 256, 136)])
+def test_clamped_feed_forward(dtype, rows, width, ff):
+    """Both clamps bite on either side, the gate only from above; few rows (one fused kernel) and many."""
+    from tokamak_amd.config import get_part
+
+    cfg = model_json([delta(mlp=dense(ff, 0.9))], width=width)
+    w = random_weights(cfg, seed=ff)
+    part = get_part("feed_forward", "swiglu")(hidden_size=width, intermediate_size=ff, names=("gate", "up", "down"),
+                                              activation="clamped", limit=0.9, dtype=dtype, device=DEV)
+    part.bind("l0.mlp.", fetcher(w, dtype))
+    h = (2.0 * torch.randn(rows, width, generator=torch.Generator().manual_seed(1))).to(dtype)
+    want = plain.feed_forward(h.double(), double(w), "l0.mlp.", cfg["layers"][0]["mlp"]).float()
+    assert float((plain.feed_forward(h.double(), double(w), "l0.mlp.", {"limit": 1.1}).float() - want).abs().max() / want.abs().max()) > 0.02
+    close(summed(part.forward(h.to(DEV), None)), want, dtype)
+
+
+def test_parts_refuse_what_they_cannot_run():
+    from tokamak_amd.config import get_part
+
+    make = get_part("mixer", "channel_delta_rule")
+    sizes = dict(hidden_size=32, num_heads=4, num_kv_heads=2, head_dim=8, value_dim=8, conv_taps=4, norm_eps=1e-5,
+                 dtype=torch.float32, device=DEV)
+    for bad in (dict(num_kv_heads=3), dict(head_dim=513), dict(conv_taps=9), dict(conv_taps=0), dict(value_dim=0)):
+        with pytest.raises(ValueError):
+            make(**{**sizes, **bad})
+    with pytest.raises(ValueError, match="one decay a head"):
+        get_part("mixer", "fixed_decay_linear_attention")(hidden_size=32, num_heads=2, head_dim=8, value_dim=8, decay=(0.5,),
+                                                          norm_eps=1e-5, dtype=torch.float32, device=DEV)
+    with pytest.raises(ValueError, match="limit"):
+        get_part("feed_forward", "swiglu")(hidden_size=32, intermediate_size=32, activation="clamped", dtype=torch.float32, device=DEV)
+
+
+# -- whole models -------------------------------------------------------------------
+SHAPES = {
+    "base": dict(cfg=model_json([delta(), parallel(), delta(mlp=dense(40, 2.5)), delta(), parallel(dict(heads=8, kv_heads=1, chunk=40), mlp=None)]),
+                 page=16),
+    "odd": dict(cfg=model_json([parallel(dict(heads=3, kv_heads=3, dim=20, vdim=40, rot=12, chunk=19), dict(heads=3, dim=12, vdim=20)),
+                                delta(heads=3, kv_heads=1, dim=21, vdim=18, conv=3, mlp=dense(50, 0.5)),
+                                parallel(dict(heads=6, kv_heads=2, dim=8, vdim=16, rot=0, chunk=None, scale=0.6), dict(heads=1, dim=40, vdim=8), mlp=None),
+                                delta(heads=5, kv_heads=5, dim=12, vdim=30, conv=2)],
+                               vocab=131, width=72, eps=1e-6, logit_scale=None), page=8, ranks=(5, 12)),
+    "ones": dict(cfg=model_json([delta(heads=1, kv_heads=1, dim=4, vdim=4, conv=1, mlp=dense(16, 1.0)),
+                                 parallel(dict(heads=5, kv_heads=1, dim=8, vdim=16, rot=2, chunk=1), dict(heads=1, dim=2, vdim=4, decay=(1.0,)), dense(8, 3.0)),
+                                 parallel(dict(heads=2, kv_heads=1, dim=64, vdim=64, rot=64, chunk=64), dict(heads=4, dim=64, vdim=64)),
+                                 delta(heads=2, kv_heads=1, dim=64, vdim=16, conv=5)],
+                                vocab=97, width=40, eps=1e-4, logit_scale=2.0), page=16, ranks=(1, 3)),
+}
+LENGTHS = [1, 2, 23, 61, 150]
+
+
+@pytest.fixture(scope="module")
+def models(tmp_path_factory):
+    root = tmp_path_factory.mktemp("korazen")
+    out = {}
+    for name, spec in SHAPES.items():
+        w = random_weights(spec["cfg"], seed=len(name), ranks=spec.get("ranks", (8, 8)))
+        out[name] = (write_folder(root / name, spec["cfg"], w), spec["cfg"], w, spec["page"])
+    return out
+
+
+def runner_for(models, name, dtype, pool_tokens=1024, max_requests=4, **kw):
+    from tokamak_amd.engine.runner import ModelRunner
+
+    folder, cfg, w, page = models[name]
+    return ModelRunner.from_folder(folder, dtype=dtype, page_size=page, kv_pool_tokens=pool_tokens,
+                                   max_requests=max_requests, **kw), cfg, w
+
+
+def requests_for(cfg, seed=0):
+    return {f"r{i}": tokens(cfg["vocab"], n, 100 * seed + i) for i, n in enumerate(LENGTHS)}
+
+
+@pytest.fixture(scope="module")
+def oracle(models):
+    out = {}
+    for name, (folder, cfg, w, page) in models.items():
+        for seed in (0, 1):
+            requests = requests_for(cfg, seed)
+            if seed == 1:
+                requests.update({f"s{i}": tokens(cfg["vocab"], n, 900 + i) for i, n in enumerate([40, 64, 17])})
+            out[name, seed] = (requests, {rid: Expected(cfg, w, toks) for rid, toks in requests.items()})
+    return out
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", list(SHAPES))
+def test_every_cutting(models, oracle, name, dtype):
+    """Whole prompts; most of a prompt and its tail token by token (prefill against decoding through
+    the cache and the states); portions of 16 down to 2 tokens."""
+    runner, cfg, w = runner_for(models, name, dtype)
+    requests, expected = oracle[name, 0]
+    checked = 0
+    for steps in [whole(requests)] + [f(rid, toks) for rid, toks in requests.items() for f in (tail_one_by_one, portions)]:
+        checked += check_rows(steps, run_steps(runner, steps), expected, dtype, name)
+    assert checked == 3 * sum(LENGTHS)
+    runner.manager.check()
+    assert all(runner.manager.num_free_pages(g) == runner.manager.num_pages(g) for g in range(runner.num_groups))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", list(SHAPES))
+def test_mixed_batches_with_pages_and_slots_used_again(models, oracle, name, dtype):
+    """Up to four live requests, portions beside single tokens, requests left out of steps; eight
+    requests over four state slots and a pool that only holds what is live."""
+    requests, expected = oracle[name, 1]
+    steps, peak = mixed(requests, seed=5)
+    assert max(len(s["entries"]) for s in steps) >= 3
+    runner, _, _ = runner_for(models, name, dtype, pool_tokens=peak, max_requests=4)
+    check_rows(steps, run_steps(runner, steps), expected, dtype, name)
+    runner.manager.check()
+    alone = whole({"r4": requests["r4"]})
+    check_rows(alone, run_steps(runner, alone), expected, dtype, name)
+
+
+def test_edges_of_chunks_and_a_far_key_show(tmp_path):
+    """Attention so sharp that one key more or less at a chunk's edge, or chunks counted from the start of a portion
+    instead of the sequence, moves the logits by far more than the tolerance, in a prompt, in portions that
+    start in the middle of pages and chunks, and in decoding over the edge; chunks of less than a page, of several pages,
+    and one that holds a key hundreds of positions back."""
+    from tokamak_amd.engine.runner import ModelRunner
+
+    cfg = model_json([parallel(dict(heads=2, kv_heads=1, rot=16, chunk=11), mlp=None), delta(),
+                      parallel(dict(heads=4, kv_heads=1, dim=32, vdim=32, rot=8, chunk=400)),
+                      parallel(dict(heads=8, kv_heads=1, rot=4, chunk=70), mlp=dense(32))])
+    w = random_weights(cfg, seed=3, sharp=5.0)
+    folder = write_folder(tmp_path / "sharp", cfg, w)
+    toks = tokens(cfg["vocab"], 450, 7)
+    expected = {"x": Expected(cfg, w, toks)}
+    for layer, sizes in ((0, (10, 12)), (2, (399, 401)), (3, (69, 71))):
+        for size in sizes:
+            other = json.loads(json.dumps(cfg))
+            other["layers"][layer]["mixer"]["left"]["mask"]["size"] = size
+            assert np.abs(oracle_logits(other, w, toks) - expected["x"].logits).max() > 0.05, (layer, size)
+    for dtype, page in (("float32", 16), ("float32", 8), ("bfloat16", 16)):
+        runner = ModelRunner.from_folder(folder, dtype=dtype, page_size=page, kv_pool_tokens=512, max_requests=2)
+        for steps in (whole({"x": toks}), tail_one_by_one("x", toks, tail=64), portions("x", toks)):
+            check_rows(steps, run_steps(runner, steps), expected, dtype, page)
+
+
+def test_the_first_tokens_are_remembered_by_the_recurrences(tmp_path):
+    """Decays near one: the first token of a sequence still moves the logits 300 tokens later through the states alone
+    (no attention layer reaches it), whatever the cutting, and a slot that is used again forgets it."""
+    from tokamak_amd.engine.runner import ModelRunner
+
+    cfg = model_json([delta(), parallel(dict(chunk=4), dict(decay=(0.999, 0.9995))), delta(mlp=dense())])
+    w = random_weights(cfg, seed=21)
+    for name in w:
+        if name.endswith("dt_bias"):
+            w[name] = torch.full_like(w[name], -9.0)
+    folder = write_folder(tmp_path / "slow", cfg, w)
+    toks = tokens(cfg["vocab"], 300, 1)
+    other = [(toks[0] + 1) % cfg["vocab"]] + toks[1:]
+    expected = {"x": Expected(cfg, w, toks), "y": Expected(cfg, w, other)}
+    last = expected["x"].logits[-1]
+    assert np.abs(last - expected["y"].logits[-1]).max() / np.abs(last).max() > 20 * LIMIT
+    runner = ModelRunner.from_folder(folder, dtype="float32", page_size=16, kv_pool_tokens=320, max_requests=1)
+    for steps in (whole({"x": toks, "y": other}), tail_one_by_one("y", other, tail=250), portions("x", toks)):
+        check_rows(steps, run_steps(runner, steps), expected, "float32")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_decoding_through_recorded_steps(models, dtype):
+    """One prompt token, then 260 tokens one by one (the recorded step of each shape replayed many
+    times, two requests side by side at different lengths); and the same without recorded steps and
+    without recorded layers gives the same bits."""
+    runner, cfg, w = runner_for(models, "base", dtype)
+    assert runner.use_graphs
+    a, b = tokens(cfg["vocab"], 261, 11), tokens(cfg["vocab"], 200, 12)
+    expected = {"a": Expected(cfg, w, a), "b": Expected(cfg, w, b)}
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:1], "want": [0]}], "end": []}]
+    for i in range(1, 261):
+        entries = [{"id": "a", "tokens": [a[i]], "want": [0]}]
+        if i >= 61:
+            entries.append({"id": "b", "tokens": [b[i - 61]], "want": [0]})
+        steps.append({"step": i, "entries": entries, "end": []})
+    got = run_steps(runner, steps)
+    check_rows(steps, got, expected, dtype)
+    plain_runner, _, _ = runner_for(models, "base", dtype, use_graphs=False)
+    plain_runner.model.replay_layers = False
+    again = run_steps(plain_runner, steps)
+    for step in got:
+        assert np.array_equal(got[step], again[step]), step
+
+
+def test_layers_launched_from_a_recorded_layer_use_their_own_norms_and_biases(tmp_path):
+    """Several layers of each kind: those after the first are launched from its recorded list, and the gains and
+    the bias that each leaves to the next layer's add must be its own."""
+    from tokamak_amd.engine.runner import ModelRunner
+
+    cfg = model_json([parallel(mlp=None)] * 3 + [delta()] * 3 + [parallel()] * 3 + [delta(mlp=dense(40))] * 3)
+    w = random_weights(cfg, seed=8)
+    folder = write_folder(tmp_path / "many", cfg, w)
+    toks = tokens(cfg["vocab"], 90, 3)
+    expected = {"x": Expected(cfg, w, toks)}
+    runner = ModelRunner.from_folder(folder, dtype="float32", page_size=16, kv_pool_tokens=256, max_requests=2)
+    for steps in (whole({"x": toks}), portions("x", toks)):
+        check_rows(steps, run_steps(runner, steps), expected, "float32")
+
+
+def test_greedy_generation_through_the_entry_point(models):
+    """``LLM.generate``: scheduler, portions of prompts, batched decoding, greedy sampling; a pool so
+    tight that requests are evicted and computed again (their states start anew)."""
+    from tokamak_amd import LLM, SamplingParams
+
+    folder, cfg, w, page = models["base"]
+    prompts = [tokens(cfg["vocab"], n, 40 + n) for n in (3, 30, 17, 9, 1)]
+    new = 14
+
+    def greedy(prompt):
+        ids = list(prompt)
+        for _ in range(new):
+            ids.append(int(np.argmax(oracle_logits(cfg, w, ids)[-1])))
+        return ids[len(prompt):]
+
+    want = [greedy(p) for p in prompts]
+    params = SamplingParams(temperature=0.0, max_new_tokens=new)
+    for kwargs in (dict(kv_pool_tokens=512), dict(kv_pool_tokens=64, prefill_chunk=8, max_batch_size=3)):
+        llm = LLM(folder, dtype="float32", max_seq_len=64, block_size=page, **kwargs)
+        out = llm.generate(prompt_token_ids=prompts, sampling_params=params)
+        assert [o.output_token_ids for o in out] == want, kwargs
+
+
+def test_trace_runner_and_command_line(models, tmp_path):
+    from test_gpu_rorosun import run_trace_any
+
+    folder, cfg, w, page = models["odd"]
+    requests = {f"r{i}": tokens(cfg["vocab"], n, 300 + i) for i, n in enumerate([5, 33, 70, 12, 41])}
+    steps, peak = mixed(requests, seed=2)
+    expected = {rid: Expected(cfg, w, toks) for rid, toks in requests.items()}
+    got = run_trace_any(folder, "float32", steps, peak, tmp_path / "out", page, cfg["vocab"])
+    check_rows(steps, got, expected, "float32")
+    done = subprocess.run([sys.executable, "-m", "tokamak_amd.cli", "--model", str(folder), "--prompt-ids", "5,6,7",
+                           "--max-new-tokens", "4", "--dtype", "float32", "--temperature", "0", "--max-seq-len", "64",
+                           "--page-size", str(page), "--quiet"], cwd=ROOT, capture_output=True, text=True, timeout=240)
+    assert done.returncode == 0, done.stderr[-2000:]
+    ids = [5, 6, 7]
+    for _ in range(4):
+        ids.append(int(np.argmax(oracle_logits(cfg, w, ids)[-1])))
+    assert ",".join(map(str, ids[3:])) in done.stdout.replace(" ", ""), done.stdout
+    done = subprocess.run([sys.executable, "-m", "tokamak_amd.cli", "--random-weights", "korazen-tiny", "--prompt-ids",
+                           "1,2,3", "--max-new-tokens", "3", "--quiet"], cwd=ROOT, capture_output=True, text=True, timeout=240)
+    assert done.returncode == 0, done.stderr[-2000:]
+
+
+def test_layers_of_a_real_width(tmp_path):
+    """Four layers of the 0.6B-class preset (delta-rule heads of 128 x 128, attention heads of 128) with a small
+    vocabulary: the library products of long portions, the tuned attention kernels, the fixed-decay scan in chunks."""
+    import dataclasses
+
+    from tokamak_amd.config.registry import find_preset
+    from tokamak_amd.engine.runner import ModelRunner
+
+    arch, full = find_preset("korazen-0.6b")
+    cfg = arch.to_json(dataclasses.replace(arch.shorten(full, 4), vocab_size=512))
+    for layer in cfg["layers"]:
+        if layer["type"] == "parallel":
+            layer["mixer"]["left"]["mask"]["size"] = 90
+    w = random_weights(cfg, 5, ranks=(64, 64))
+    folder = write_folder(tmp_path / "wide", cfg, w)
+    toks = tokens(512, 200, 3)
+    expected = {"x": Expected(cfg, w, toks)}
+    for dtype in ("float32", "bfloat16"):
+        runner = ModelRunner.from_folder(folder, dtype=dtype, page_size=16, kv_pool_tokens=512, max_requests=2)
+        for steps in (whole({"x": toks}), tail_one_by_one("x", toks, tail=50), portions("x", toks, sizes=(70, 2, 65, 13, 50))):
+            check_rows(steps, run_steps(runner, steps), expected, dtype)
+        del runner
