@@ -35,7 +35,68 @@ struct DeltaShape {
 // A wave a unit (a q or k head, or a run of 64 * CPL channels of v or of the decays) and a segment of a request's
 // tokens: a lane walks CPL channels with the taps' inputs in registers.  grid (units / 4, requests, segments).
 // update: a request's tokens are this one segment, whose wave also writes the convolution's new state.
-template <typename T, int CPL>
+// WIDE: a lane's channels are neighbours and read and written as one piece (every width a multiple of CPL); else lane,
+// lane + 64, ...
+template <typename T, int N> struct Piece { using type = void; };
+template <> struct Piece<bf16_t, 1> { using type = uint16_t; };
+template <> struct Piece<bf16_t, 2> { using type = uint32_t; };
+template <> struct Piece<bf16_t, 4> { using type = uint2; };
+template <> struct Piece<float, 1> { using type = float; };
+template <> struct Piece<float, 2> { using type = float2; };
+template <> struct Piece<float, 4> { using type = float4; };
+
+// N neighbouring elements from idx on of rows in T, float32 or partial sums
+template <typename T, int N>
+__device__ __forceinline__ void load_piece(const RowsIn& in, size_t idx, float (&v)[N]) {
+  if (!in.f32) {
+    union { typename Piece<bf16_t, N>::type u; bf16_t e[N]; } p;
+    p.u = *reinterpret_cast<const typename Piece<bf16_t, N>::type*>(reinterpret_cast<const bf16_t*>(in.p) + idx);
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = bf16_to_float(p.e[i]);
+    return;
+  }
+  const float* f = reinterpret_cast<const float*>(in.p) + idx;
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = 0.f;
+  for (int k = 0; k < in.parts; ++k) {
+    union { typename Piece<float, N>::type u; float e[N]; } p;
+    p.u = *reinterpret_cast<const typename Piece<float, N>::type*>(f + (size_t)k * in.stride);
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] += p.e[i];
+  }
+}
+template <int N>
+__device__ __forceinline__ void store_piece(float* dst, const float (&v)[N]) {
+  union { typename Piece<float, N>::type u; float e[N]; } p;
+#pragma unroll
+  for (int i = 0; i < N; ++i) p.e[i] = v[i];
+  *reinterpret_cast<typename Piece<float, N>::type*>(dst) = p.u;
+}
+
+// A lane's CPL channels of a unit's `count`, from `at` on (channels that do not exist: zeros, not stored).
+template <typename T, int CPL, bool WIDE>
+__device__ __forceinline__ void load_channels(const RowsIn& in, size_t at, int lane, int count, float (&v)[CPL]) {
+  if constexpr (WIDE) {
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) v[i] = 0.f;
+    if (lane * CPL < count) load_piece<T, CPL>(in, at + lane * CPL, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < CPL; ++i) v[i] = i * kWave + lane < count ? load_in<T>(in, at + i * kWave + lane) : 0.f;
+  }
+}
+template <int CPL, bool WIDE>
+__device__ __forceinline__ void store_channels(float* dst, int lane, int count, const float (&v)[CPL]) {
+  if constexpr (WIDE) {
+    if (lane * CPL < count) store_piece<CPL>(dst + lane * CPL, v);
+  } else {
+#pragma unroll
+    for (int i = 0; i < CPL; ++i)
+      if (i * kWave + lane < count) dst[i * kWave + lane] = v[i];
+  }
+}
+
+template <typename T, int CPL, bool WIDE>
 __global__ __launch_bounds__(256) void delta_inputs_kernel(
     RowsIn proj, long ld, RowsIn up, long uld, const float* __restrict__ conv, float* __restrict__ state,
     const float* __restrict__ a_log, const float* __restrict__ dt_bias, const int* __restrict__ q_start,
@@ -55,14 +116,20 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
     if (unit >= gunits) return;
     // decays, and (its first unit) the heads' step sizes
     float* dst = out + C;
+    const int from = unit * RUN, count = min(RUN, gall - from);
+    float rate[CPL], bias[CPL];
 #pragma unroll
     for (int i = 0; i < CPL; ++i) {
-      const int c = unit * RUN + i * kWave + lane;
-      if (c < gall) {
-        const float rate = expf(a_log[c / sh.dim]), bias = dt_bias[c];
-        for (int t = t_lo; t < t_hi; ++t)
-          dst[(size_t)t * row + c] = expf(-rate * softplus(load_in<T>(up, (size_t)t * uld + c) + bias));
-      }
+      const int c = WIDE ? lane * CPL + i : i * kWave + lane;
+      rate[i] = c < count ? expf(a_log[(from + c) / sh.dim]) : 0.f;
+      bias[i] = c < count ? dt_bias[from + c] : 0.f;
+    }
+    for (int t = t_lo; t < t_hi; ++t) {
+      float z[CPL];
+      load_channels<T, CPL, WIDE>(up, (size_t)t * uld + from, lane, count, z);
+#pragma unroll
+      for (int i = 0; i < CPL; ++i) z[i] = expf(-rate[i] * softplus(z[i] + bias[i]));
+      store_channels<CPL, WIDE>(dst + (size_t)t * row + from, lane, count, z);
     }
     if (unit == 0) {
       for (int i = lane; i < (t_hi - t_lo) * sh.heads; i += kWave) {
@@ -78,57 +145,60 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
   const float scale = unit < sh.kv ? q_scale : 1.f;
   float* st = taps > 1 ? state + (size_t)state_slots[req] * (taps - 1) * C + col0 : nullptr;
   // taps and window sit at the END of arrays of kMaxTaps: index kMaxTaps - 1 is the token itself
-  float wv[CPL][kMaxTaps], win[CPL][kMaxTaps];
+  float wv[CPL][kMaxTaps], win[kMaxTaps][CPL];
 #pragma unroll
-  for (int i = 0; i < CPL; ++i) {
-    const int c = i * kWave + lane;
+  for (int k = 0; k < kMaxTaps; ++k) {
+    const int j = k - (kMaxTaps - taps);
 #pragma unroll
-    for (int k = 0; k < kMaxTaps; ++k) {
-      const int j = k - (kMaxTaps - taps);
+    for (int i = 0; i < CPL; ++i) {
+      const int c = WIDE ? lane * CPL + i : i * kWave + lane;
       wv[i][k] = (j >= 0 && c < count) ? conv[(size_t)(col0 + c) * taps + j] : 0.f;
-      win[i][k] = 0.f;
+      win[k][i] = 0.f;
     }
+  }
 #pragma unroll
-    for (int d = 1; d < kMaxTaps; ++d) {
-      if (d < taps && c < count) {
-        const int local = t_lo - first - d;     // the input d positions before the segment's first token
-        win[i][kMaxTaps - d] = local >= 0 ? load_in<T>(proj, (size_t)(t_lo - d) * ld + col0 + c)
-                                          : st[(size_t)(taps - 1 + local) * C + c];
+  for (int d = 1; d < kMaxTaps; ++d) {
+    if (d < taps) {
+      const int local = t_lo - first - d;     // the input d positions before the segment's first token
+      if (local >= 0) {
+        load_channels<T, CPL, WIDE>(proj, (size_t)(t_lo - d) * ld + col0, lane, count, win[kMaxTaps - d]);
+      } else {
+#pragma unroll
+        for (int i = 0; i < CPL; ++i) {
+          const int c = WIDE ? lane * CPL + i : i * kWave + lane;
+          win[kMaxTaps - d][i] = c < count ? st[(size_t)(taps - 1 + local) * C + c] : 0.f;
+        }
       }
     }
   }
   for (int t = t_lo; t < t_hi; ++t) {
+#pragma unroll
+    for (int k = 0; k < kMaxTaps - 1; ++k)
+#pragma unroll
+      for (int i = 0; i < CPL; ++i) win[k][i] = win[k + 1][i];
+    load_channels<T, CPL, WIDE>(proj, (size_t)t * ld + col0, lane, count, win[kMaxTaps - 1]);
     float y[CPL];
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < CPL; ++i) {
-      const int c = i * kWave + lane;
-#pragma unroll
-      for (int k = 0; k < kMaxTaps - 1; ++k) win[i][k] = win[i][k + 1];
-      win[i][kMaxTaps - 1] = c < count ? load_in<T>(proj, (size_t)t * ld + col0 + c) : 0.f;
       float acc = 0.f;
 #pragma unroll
-      for (int k = 0; k < kMaxTaps; ++k) acc = fmaf(wv[i][k], win[i][k], acc);
+      for (int k = 0; k < kMaxTaps; ++k) acc = fmaf(wv[i][k], win[k][i], acc);
       y[i] = silu(acc);        // (channels behind the unit's: zero)
       ss = fmaf(y[i], y[i], ss);
     }
-    float r = 1.f;
-    if (qk) r = scale / sqrtf(wave_sum(ss) + kUnitEps);
+    if (qk) {
+      const float r = scale / sqrtf(wave_sum(ss) + kUnitEps);
 #pragma unroll
-    for (int i = 0; i < CPL; ++i) {
-      const int c = i * kWave + lane;
-      if (c < count) out[(size_t)t * row + col0 + c] = y[i] * r;
+      for (int i = 0; i < CPL; ++i) y[i] *= r;
     }
+    store_channels<CPL, WIDE>(out + (size_t)t * row + col0, lane, count, y);
   }
   if (update) {      // (the window now ends at the request's last token)
 #pragma unroll
-    for (int i = 0; i < CPL; ++i) {
-      const int c = i * kWave + lane;
-#pragma unroll
-      for (int k = 1; k < kMaxTaps; ++k) {
-        const int j = k - (kMaxTaps - (taps - 1));
-        if (j >= 0 && c < count) st[(size_t)j * C + c] = win[i][k];
-      }
+    for (int k = 1; k < kMaxTaps; ++k) {
+      const int j = k - (kMaxTaps - (taps - 1));
+      if (j >= 0) store_channels<CPL, WIDE>(st + (size_t)j * C, lane, count, win[k]);
     }
   }
 }
@@ -189,6 +259,54 @@ __device__ __forceinline__ void fetch_round(const float* __restrict__ in, int ro
   beta = (int)threadIdx.x < tb ? in[(size_t)(t0 + threadIdx.x) * row + b_at] : 0.f;
 }
 
+// What a lane reads of a token of the round.
+template <int PIECES>
+struct DeltaToken {
+  f32x4 k[PIECES], q[PIECES], g[PIECES];
+  float beta, v;
+};
+
+template <int PIECES, int TB>
+__device__ __forceinline__ void read_token(const float* lds, const float* vv, const float* bb, int t, int ks, int jl,
+                                           DeltaToken<PIECES>& x) {
+  constexpr int DP = kLanes * 4 * PIECES, SET = TB * DP;
+#pragma unroll
+  for (int i = 0; i < PIECES; ++i) {
+    const int piece = t * DP + i * (kLanes * 4) + ks * 4;
+    x.k[i] = *reinterpret_cast<const f32x4*>(lds + piece);
+    x.g[i] = *reinterpret_cast<const f32x4*>(lds + 2 * SET + piece);
+    x.q[i] = *reinterpret_cast<const f32x4*>(lds + SET + piece);
+  }
+  x.beta = bb[t];
+  x.v = vv[t * kColumns + jl];
+}
+
+// The lane's rows of the state move on by a token; its output (the same number in all lanes of the column).
+template <int PIECES>
+__device__ __forceinline__ float delta_token(const DeltaToken<PIECES>& x, f32x4 (&s)[PIECES]) {
+  // Measured on 2,048 tokens of 32 heads of 128 x 128: operands read where they are used 450 us, in a loop that asks for
+  // them a token ahead 525 (copies and addresses), unrolled with the reads ahead 370; the rest is the chain itself.
+  float d0 = 0.f, d1 = 0.f, o0 = 0.f, o1 = 0.f;
+#pragma unroll
+  for (int i = 0; i < PIECES; ++i) {
+    s[i] *= x.g[i];
+    d0 = fmaf(s[i].x, x.k[i].x, d0);
+    d1 = fmaf(s[i].y, x.k[i].y, d1);
+    d0 = fmaf(s[i].z, x.k[i].z, d0);
+    d1 = fmaf(s[i].w, x.k[i].w, d1);
+  }
+  const float u = x.beta * (x.v - sum16(d0 + d1));
+#pragma unroll
+  for (int i = 0; i < PIECES; ++i) {
+    s[i] = f32x4{fmaf(x.k[i].x, u, s[i].x), fmaf(x.k[i].y, u, s[i].y), fmaf(x.k[i].z, u, s[i].z), fmaf(x.k[i].w, u, s[i].w)};
+    o0 = fmaf(s[i].x, x.q[i].x, o0);
+    o1 = fmaf(s[i].y, x.q[i].y, o1);
+    o0 = fmaf(s[i].z, x.q[i].z, o0);
+    o1 = fmaf(s[i].w, x.q[i].w, o1);
+  }
+  return sum16(o0 + o1);
+}
+
 // A block a (request, head, 16 value columns).  The 16 neighbouring lanes that share a column hold its rows of the
 // state in registers, PIECES pieces of four rows a lane (lane l: rows 64 i + 4 l .. + 4), so that both dot
 // products of a token are sums of 4 PIECES multiply-adds and four lane moves, with no LDS and no barrier in
@@ -197,7 +315,7 @@ __device__ __forceinline__ void fetch_round(const float* __restrict__ in, int ro
 // The state lies as [head][column][dim rounded up to 4].
 // WIDE: dim and vdim are multiples of four, so that rows are read in 16-byte pieces.
 template <int PIECES, int TB, bool WIDE>
-__global__ __launch_bounds__(kScanThreads) void delta_scan_kernel(
+__global__ __launch_bounds__(kScanThreads, 1) void delta_scan_kernel(
     const float* __restrict__ in, float* __restrict__ state, const int* __restrict__ q_start,
     const int* __restrict__ state_slots, float* __restrict__ y, DeltaShape sh) {
   constexpr int DP = kLanes * 4 * PIECES;      // rows with the padding (zeros behind dim)
@@ -242,37 +360,24 @@ __global__ __launch_bounds__(kScanThreads) void delta_scan_kernel(
     if (t0 + TB < end) fetch_round<PER, TB, DP, WIDE>(in, row, k_at, q_at, g_at, v_at, b_at, dim, vdim - col0, t0 + TB,
                                                       min(TB, end - t0 - TB), held, held_beta);
     float kept = 0.f;
-    for (int t = 0; t < tb; ++t) {
-      f32x4 k[PIECES], g[PIECES], q[PIECES];
+    DeltaToken<PIECES> x[2];
+    read_token<PIECES, TB>(lds, vv, bb, 0, ks, jl, x[0]);
+    if (tb == TB) {
+      // a whole round, unrolled: a token's operands are read while the token before it is computed (the barrier lets
+      // arithmetic pass, LDS reads not: left alone the compiler puts the reads right ahead of their use)
 #pragma unroll
-      for (int i = 0; i < PIECES; ++i) {
-        const int piece = t * DP + i * (kLanes * 4) + ks * 4;
-        k[i] = *reinterpret_cast<const f32x4*>(lds + piece);
-        g[i] = *reinterpret_cast<const f32x4*>(lds + 2 * SET + piece);
-        q[i] = *reinterpret_cast<const f32x4*>(lds + SET + piece);
+      for (int t = 0; t < TB; ++t) {
+        if (t + 1 < TB) read_token<PIECES, TB>(lds, vv, bb, t + 1, ks, jl, x[(t + 1) & 1]);
+        __builtin_amdgcn_sched_barrier(0x7);
+        const float o = delta_token<PIECES>(x[t & 1], s);
+        if (ks == t) kept = o;      // (lane t of a column keeps token t's output: one store a round)
       }
-      const float beta = bb[t], v = vv[t * kColumns + jl];
-      float d0 = 0.f, d1 = 0.f;
-#pragma unroll
-      for (int i = 0; i < PIECES; ++i) {
-        s[i] *= g[i];
-        d0 = fmaf(s[i].x, k[i].x, d0);
-        d1 = fmaf(s[i].y, k[i].y, d1);
-        d0 = fmaf(s[i].z, k[i].z, d0);
-        d1 = fmaf(s[i].w, k[i].w, d1);
+    } else {
+      for (int t = 0; t < tb; ++t) {
+        if (t > 0) read_token<PIECES, TB>(lds, vv, bb, t, ks, jl, x[0]);
+        const float o = delta_token<PIECES>(x[0], s);
+        if (ks == t) kept = o;
       }
-      const float u = beta * (v - sum16(d0 + d1));
-      float o0 = 0.f, o1 = 0.f;
-#pragma unroll
-      for (int i = 0; i < PIECES; ++i) {
-        s[i] = f32x4{fmaf(k[i].x, u, s[i].x), fmaf(k[i].y, u, s[i].y), fmaf(k[i].z, u, s[i].z), fmaf(k[i].w, u, s[i].w)};
-        o0 = fmaf(s[i].x, q[i].x, o0);
-        o1 = fmaf(s[i].y, q[i].y, o1);
-        o0 = fmaf(s[i].z, q[i].z, o0);
-        o1 = fmaf(s[i].w, q[i].w, o1);
-      }
-      const float o = sum16(o0 + o1);
-      if (ks == t) kept = o;      // (lane t of a column keeps token t's output: one store a round)
     }
     static_assert(TB <= kLanes, "a lane of a column keeps one token's output");
     if (owns && ks < tb) y[(size_t)(t0 + ks) * sh.heads * vdim + (size_t)head * vdim + j] = kept;
@@ -297,13 +402,19 @@ int launch_inputs(RowsIn proj, long ld, RowsIn up, long uld, const float* conv, 
   const long units = 2L * sh.kv + ((long)sh.heads * sh.vdim + run - 1) / run + ((long)sh.heads * sh.dim + run - 1) / run;
   const dim3 grid((unsigned)((units + 3) / 4), R, segments);
   if (grid.y > 65535 || grid.z > 65535) return -1;
-#define TK_DI(CPL)                                                                                              \
-  delta_inputs_kernel<T, CPL><<<grid, 256, 0, stream>>>(proj, ld, up, uld, conv, state, a_log, dt_bias, q_start, \
-                                                        slots, out, sh, q_scale, update)
-  if (cpl == 1) TK_DI(1);
-  else if (cpl == 2) TK_DI(2);
-  else if (cpl == 4) TK_DI(4);
-  else TK_DI(8);
+  // (every unit then starts on a border of CPL elements in all of its arrays)
+  const bool wide = cpl <= 4 && sh.dim % cpl == 0 && sh.heads * sh.vdim % cpl == 0 && ld % cpl == 0 && uld % cpl == 0 &&
+                    proj.stride % cpl == 0 && up.stride % cpl == 0 && (uintptr_t)proj.p % 16 == 0 &&
+                    (uintptr_t)up.p % 16 == 0 && (uintptr_t)state % 16 == 0 && (uintptr_t)out % 16 == 0;
+#define TK_DI(CPL, WIDE)                                                                                              \
+  delta_inputs_kernel<T, CPL, WIDE><<<grid, 256, 0, stream>>>(proj, ld, up, uld, conv, state, a_log, dt_bias, q_start, \
+                                                              slots, out, sh, q_scale, update)
+  if (cpl == 1) TK_DI(1, false);
+  else if (cpl == 2 && wide) TK_DI(2, true);
+  else if (cpl == 2) TK_DI(2, false);
+  else if (cpl == 4 && wide) TK_DI(4, true);
+  else if (cpl == 4) TK_DI(4, false);
+  else TK_DI(8, false);
 #undef TK_DI
   if (!update && sh.taps > 1) {
     const int C = sh.conv_channels();

@@ -772,7 +772,17 @@ __device__ __forceinline__ float4 branch_four(const NormBranch& b, size_t idx) {
   if (!b.f32) return Load4<T>::at(reinterpret_cast<const T*>(b.p) + idx);
   const float* f = reinterpret_cast<const float*>(b.p) + idx;
   float4 s = *reinterpret_cast<const float4*>(f);
-  for (int i = 1; i < b.parts; ++i) {
+  int i = 1;
+  for (; i + 4 <= b.parts; i += 4) {      // four partial sums in flight, added in split order
+    float4 q[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) q[u] = *reinterpret_cast<const float4*>(f + (size_t)(i + u) * b.stride);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      s.x += q[u].x; s.y += q[u].y; s.z += q[u].z; s.w += q[u].w;
+    }
+  }
+  for (; i < b.parts; ++i) {
     const float4 q = *reinterpret_cast<const float4*>(f + (size_t)i * b.stride);
     s.x += q.x; s.y += q.y; s.z += q.z; s.w += q.w;
   }
@@ -1007,6 +1017,12 @@ __global__ __launch_bounds__(1024) void add_normed_vec_kernel(
       sb += square_sum(bv[g]);
     }
   }
+  float4 gv[GROUPS];      // (the last gain is asked for with the rows, not behind the sums)
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    gv[g] = n.gain && d < H ? *reinterpret_cast<const float4*>(n.gain + d) : make_float4(1.f, 1.f, 1.f, 1.f);
+  }
   if (n.gain_a || n.gain_b) {      // (every thread of the block alike)
     block_sum2(sa, sb, scratch);
     const float ra = 1.f / sqrtf(sa / (float)H + n.eps), rb = 1.f / sqrtf(sb / (float)H + n.eps);
@@ -1033,7 +1049,7 @@ __global__ __launch_bounds__(1024) void add_normed_vec_kernel(
   for (int g = 0; g < GROUPS; ++g) {
     const int d = (g * blockDim.x + threadIdx.x) * 4;
     if (d < H) {
-      if (n.gain) scale_by(av[g], rstd, n.gain + d);
+      if (n.gain) av[g] = make_float4(av[g].x * rstd * gv[g].x, av[g].y * rstd * gv[g].y, av[g].z * rstd * gv[g].z, av[g].w * rstd * gv[g].w);
       xv[g].x += av[g].x; xv[g].y += av[g].y; xv[g].z += av[g].z; xv[g].w += av[g].w;
       if (write_resid) *reinterpret_cast<float4*>(x + d) = xv[g];
       ss += square_sum(xv[g]);

@@ -320,6 +320,46 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
   }
 }
 
+// The same for parts of 4 to 256 columns where a lane takes four neighbours: LANES = size / 4 lanes a part (a power
+// of two), 64 / LANES parts a wave.
+template <typename T, int LANES>
+__global__ __launch_bounds__(256) void gated_group_norm_four_kernel(
+    const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
+    T* __restrict__ out, long pairs, int inner, int groups, float eps, int shared, int after) {
+  constexpr int size = LANES * 4;
+  const long pair = ((long)blockIdx.x * blockDim.x + threadIdx.x) / LANES;
+  const int sub = threadIdx.x % LANES;
+  if (pair >= pairs) return;       // (whole groups of LANES lanes leave together)
+  const long n = pair / groups;
+  const int g = (int)(pair - n * groups);
+  const size_t at = (size_t)n * inner + (size_t)g * size + sub * 4;
+  const size_t zat = (size_t)n * ld + z_col + (size_t)g * size + sub * 4;
+  float z[4], v[4];
+  if (!z_in.f32) {
+    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(z_in.p) + zat);
+    z[0] = __uint_as_float(u.x << 16); z[1] = __uint_as_float(u.x & 0xffff0000u);
+    z[2] = __uint_as_float(u.y << 16); z[3] = __uint_as_float(u.y & 0xffff0000u);
+  } else {
+    const float* f = reinterpret_cast<const float*>(z_in.p) + zat;
+    float4 s = *reinterpret_cast<const float4*>(f);
+    for (int i = 1; i < z_in.parts; ++i) {
+      const float4 a = *reinterpret_cast<const float4*>(f + (size_t)i * z_in.stride);
+      s.x += a.x; s.y += a.y; s.z += a.z; s.w += a.w;
+    }
+    z[0] = s.x; z[1] = s.y; z[2] = s.z; z[3] = s.w;
+  }
+  const float4 y4 = *reinterpret_cast<const float4*>(y + at);
+  const float4 w4 = *reinterpret_cast<const float4*>(weight + (shared ? 0 : g * size) + sub * 4);
+  v[0] = before_norm(y4.x, z[0], after); v[1] = before_norm(y4.y, z[1], after);
+  v[2] = before_norm(y4.z, z[2], after); v[3] = before_norm(y4.w, z[3], after);
+  float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+#pragma unroll
+  for (int m = LANES / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, kWave);
+  const float rstd = 1.f / sqrtf(ss / (float)size + eps);
+  store_four<T>(out + at, behind_norm(v[0] * rstd * w4.x, z[0], after), behind_norm(v[1] * rstd * w4.y, z[1], after),
+                behind_norm(v[2] * rstd * w4.z, z[2], after), behind_norm(v[3] * rstd * w4.w, z[3], after), 4, true);
+}
+
 // The same for long parts of the row: a block a (token, part), a thread up to kHold elements in registers
 // (beyond that the products are formed again for the second pass).
 constexpr int kHold = 8;
@@ -512,6 +552,18 @@ TK_API int tk_gated_group_norm(int dtype, const float* y, const void* z, int z_f
     if (pairs > 0x7fffffffL) return -1;
     if (dtype == 0) gated_group_norm_block_kernel<float><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, inner, groups, eps, shared, after);
     else gated_group_norm_block_kernel<bf16_t><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, inner, groups, eps, shared, after);
+    return launch_status();
+  }
+  if ((size & (size - 1)) == 0 && size >= 4 && ld % 4 == 0 && z_col % 4 == 0 && z_stride % 4 == 0 && (uintptr_t)y % 16 == 0 &&
+      (uintptr_t)z % 16 == 0 && (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0 && pairs * (size / 4) <= 0x7fffffffL) {
+    const unsigned quads = (unsigned)((pairs * (size / 4) + 255) / 256);
+#define TK_GN(LANES)                                                                                                      \
+  case LANES * 4:                                                                                                         \
+    if (dtype == 0) gated_group_norm_four_kernel<float, LANES><<<quads, 256, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, pairs, inner, groups, eps, shared, after); \
+    else gated_group_norm_four_kernel<bf16_t, LANES><<<quads, 256, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, pairs, inner, groups, eps, shared, after);         \
+    break;
+    switch (size) { TK_GN(1) TK_GN(2) TK_GN(4) TK_GN(8) TK_GN(16) TK_GN(32) TK_GN(64) }
+#undef TK_GN
     return launch_status();
   }
   const unsigned blocks = (unsigned)((pairs + 3) / 4);

@@ -11,6 +11,8 @@ from tokamak_amd.parts.base import Fetch, Mixer, PositionData, StateArray
 from tokamak_amd.weights.spec import TensorSpec
 
 LOW = 8        # the low ranks are padded with rows of zeros to a multiple of this (16-byte rows of the second product)
+WHOLE = 256    # ... and a large first matrix to a multiple of this (the library's tiles: 2,048 rows of 4,096 into 12,576
+               # columns take 180 us, into 12,800 165)
 
 
 class ChannelDeltaRule(Mixer):
@@ -30,8 +32,8 @@ class ChannelDeltaRule(Mixer):
     the recurrence behind the products is float32.  The low ranks of W_a1 and W_g1 are read off the checkpoint unless
     ``decay_rank`` and ``gate_rank`` give them.
 
-    q, k, v and b are one product of h, the two low ranks a second one, and their two second matrices a third with the
-    pair side by side on a matrix that is zero where they do not meet.
+    q, k, v, b and the two low ranks are one product of h (not split over K: the low ranks are read back as rows), and
+    the second matrices of the low ranks a second one, on a matrix that is zero where the two do not meet.
     Tensors: q, k, v with ``.conv`` each, b, A_log, norm, a1, a2, dt_bias, g1, g2, o behind the part's prefix.
     """
 
@@ -54,7 +56,7 @@ class ChannelDeltaRule(Mixer):
         self.decay_rank = None if decay_rank is None else int(decay_rank)
         self.gate_rank = None if gate_rank is None else int(gate_rank)
         self.conv_channels = 2 * self.num_kv_heads * self.head_dim + self.num_heads * self.value_dim
-        self.qkvb = self.low = self.up = self.o = None
+        self.first = self.up = self.o = None
         self.conv = self.a_log = self.dt_bias = self.gain = None
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
@@ -76,17 +78,21 @@ class ChannelDeltaRule(Mixer):
         return out
 
     def bind(self, prefix: str, fetch: Fetch) -> None:
-        self.qkvb = torch.cat([fetch(prefix + n) for n in ("q", "k", "v", "b")]).contiguous()
         self.conv = torch.cat([fetch(prefix + n + ".conv") for n in ("q", "k", "v")]).contiguous()
         self.a_log, self.dt_bias, self.gain, self.o = (fetch(prefix + n) for n in ("A_log", "dt_bias", "norm", "o"))
         a1, a2, g1, g2 = (fetch(prefix + n) for n in ("a1", "a2", "g1", "g2"))
         for name, first, second in (("decay", a1, a2), ("gate", g1, g2)):
             if second.shape[1] != first.shape[0]:
                 raise ValueError(f"the two matrices of the {name} disagree on its rank: {tuple(first.shape)} and {tuple(second.shape)}")
+        rows = [fetch(prefix + n) for n in ("q", "k", "v", "b")]
         ra, rg = a1.shape[0], g1.shape[0]
-        wide = -(-(ra + rg) // LOW) * LOW
-        self.low = torch.zeros((wide, self.hidden_size), dtype=a1.dtype, device=a1.device)
-        self.low[:ra], self.low[ra:ra + rg] = a1, g1
+        self.low_at = -(-sum(t.shape[0] for t in rows) // LOW) * LOW
+        self.low_width = wide = -(-(ra + rg) // LOW) * LOW
+        total = self.low_at + wide
+        total = -(-total // WHOLE) * WHOLE if total >= 8 * WHOLE else total
+        self.first = torch.zeros((total, self.hidden_size), dtype=a1.dtype, device=a1.device)
+        torch.cat(rows, out=self.first[:sum(t.shape[0] for t in rows)])
+        self.first[self.low_at:self.low_at + ra], self.first[self.low_at + ra:self.low_at + ra + rg] = a1, g1
         self.up = torch.zeros((a2.shape[0] + g2.shape[0], wide), dtype=a2.dtype, device=a2.device)
         self.up[:a2.shape[0], :ra], self.up[a2.shape[0]:, ra:ra + rg] = a2, g2
 
@@ -98,10 +104,10 @@ class ChannelDeltaRule(Mixer):
 
     def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None):
         n, sizes = h.shape[0], dict(heads=self.num_heads, kv_heads=self.num_kv_heads, dim=self.head_dim, vdim=self.value_dim)
-        # (split products leave float32 partial sums, which the kernels below add as they load)
-        proj = linear(h, self.qkvb, allow_partials=True)
+        proj = linear(h, self.first)
+        low = proj[:, self.low_at:self.low_at + self.low_width]
         few = n <= ops.STREAM_MAX_ROWS      # (few rows: float32 from the streaming product, at no cost)
-        up = linear(linear(h, self.low), self.up, out_dtype=torch.float32 if few else None, allow_partials=True)
+        up = linear(low, self.up, out_dtype=torch.float32 if few else None, allow_partials=True)
         operands = torch.empty((n, ops.delta_row(**sizes)), dtype=torch.float32, device=h.device)
         ops.delta_inputs(proj, up, self.conv, store.state.get("conv"), self.a_log, self.dt_bias, operands, batch,
                          q_scale=self.head_dim ** -0.5, **sizes)
