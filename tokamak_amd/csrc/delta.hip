@@ -24,6 +24,7 @@ namespace {
 typedef float f32x4 __attribute__((ext_vector_type(4)));   // (arrays of HIP's float4 struct may end up in scratch)
 
 constexpr int kSegment = 16;      // tokens of a request that a wave of delta_inputs walks
+constexpr int kTogether = 4;      // of which a wave asks for this many together
 constexpr float kUnitEps = 1e-6f;
 
 struct DeltaShape {
@@ -96,7 +97,8 @@ __device__ __forceinline__ void store_channels(float* dst, int lane, int count, 
   }
 }
 
-template <typename T, int CPL, bool WIDE>
+// TAPS: at least the convolution's taps.  Four tokens' inputs are asked for together.
+template <typename T, int CPL, int TAPS, bool WIDE>
 __global__ __launch_bounds__(256) void delta_inputs_kernel(
     RowsIn proj, long ld, RowsIn up, long uld, const float* __restrict__ conv, float* __restrict__ state,
     const float* __restrict__ a_log, const float* __restrict__ dt_bias, const int* __restrict__ q_start,
@@ -124,12 +126,18 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
       rate[i] = c < count ? expf(a_log[(from + c) / sh.dim]) : 0.f;
       bias[i] = c < count ? dt_bias[from + c] : 0.f;
     }
-    for (int t = t_lo; t < t_hi; ++t) {
-      float z[CPL];
-      load_channels<T, CPL, WIDE>(up, (size_t)t * uld + from, lane, count, z);
+    for (int t0 = t_lo; t0 < t_hi; t0 += kTogether) {
+      float z[kTogether][CPL];
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) z[i] = expf(-rate[i] * softplus(z[i] + bias[i]));
-      store_channels<CPL, WIDE>(dst + (size_t)t * row + from, lane, count, z);
+      for (int u = 0; u < kTogether; ++u)      // (a row behind the last token's: the last token's again)
+        load_channels<T, CPL, WIDE>(up, (size_t)min(t0 + u, t_hi - 1) * uld + from, lane, count, z[u]);
+#pragma unroll
+      for (int u = 0; u < kTogether; ++u) {
+        if (t0 + u >= t_hi) break;
+#pragma unroll
+        for (int i = 0; i < CPL; ++i) z[u][i] = expf(-rate[i] * softplus(z[u][i] + bias[i]));
+        store_channels<CPL, WIDE>(dst + (size_t)(t0 + u) * row + from, lane, count, z[u]);
+      }
     }
     if (unit == 0) {
       for (int i = lane; i < (t_hi - t_lo) * sh.heads; i += kWave) {
@@ -144,60 +152,75 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
   const int count = qk ? sh.dim : min(RUN, vall - (unit - 2 * sh.kv) * RUN);
   const float scale = unit < sh.kv ? q_scale : 1.f;
   float* st = taps > 1 ? state + (size_t)state_slots[req] * (taps - 1) * C + col0 : nullptr;
-  // taps and window sit at the END of arrays of kMaxTaps: index kMaxTaps - 1 is the token itself
-  float wv[CPL][kMaxTaps], win[kMaxTaps][CPL];
+  // taps sit at the END of arrays of TAPS: index TAPS - 1 is the token itself; win holds the inputs of the TAPS - 1
+  // positions before a group of kTogether tokens, and then theirs
+  float wv[TAPS][CPL], win[TAPS - 1 + kTogether][CPL];
 #pragma unroll
-  for (int k = 0; k < kMaxTaps; ++k) {
-    const int j = k - (kMaxTaps - taps);
+  for (int k = 0; k < TAPS; ++k) {
+    const int j = k - (TAPS - taps);
 #pragma unroll
     for (int i = 0; i < CPL; ++i) {
       const int c = WIDE ? lane * CPL + i : i * kWave + lane;
-      wv[i][k] = (j >= 0 && c < count) ? conv[(size_t)(col0 + c) * taps + j] : 0.f;
-      win[k][i] = 0.f;
+      wv[k][i] = (j >= 0 && c < count) ? conv[(size_t)(col0 + c) * taps + j] : 0.f;
     }
   }
 #pragma unroll
-  for (int d = 1; d < kMaxTaps; ++d) {
-    if (d < taps) {
-      const int local = t_lo - first - d;     // the input d positions before the segment's first token
-      if (local >= 0) {
-        load_channels<T, CPL, WIDE>(proj, (size_t)(t_lo - d) * ld + col0, lane, count, win[kMaxTaps - d]);
-      } else {
+  for (int d = 1; d < TAPS; ++d) {
+    const int local = t_lo - first - d;       // the input d positions before the segment's first token
+    if (d < taps && local >= 0) {
+      load_channels<T, CPL, WIDE>(proj, (size_t)(t_lo - d) * ld + col0, lane, count, win[TAPS - 1 - d]);
+    } else {
 #pragma unroll
-        for (int i = 0; i < CPL; ++i) {
-          const int c = WIDE ? lane * CPL + i : i * kWave + lane;
-          win[kMaxTaps - d][i] = c < count ? st[(size_t)(taps - 1 + local) * C + c] : 0.f;
-        }
+      for (int i = 0; i < CPL; ++i) {
+        const int c = WIDE ? lane * CPL + i : i * kWave + lane;
+        win[TAPS - 1 - d][i] = d < taps && c < count ? st[(size_t)(taps - 1 + local) * C + c] : 0.f;
       }
     }
   }
-  for (int t = t_lo; t < t_hi; ++t) {
+  for (int t0 = t_lo; t0 < t_hi; t0 += kTogether) {
+    const int many = min(kTogether, t_hi - t0);
 #pragma unroll
-    for (int k = 0; k < kMaxTaps - 1; ++k)
+    for (int u = 0; u < kTogether; ++u)      // (a row behind the last token's: the last token's again, not used)
+      load_channels<T, CPL, WIDE>(proj, (size_t)min(t0 + u, t_hi - 1) * ld + col0, lane, count, win[TAPS - 1 + u]);
+    float y[kTogether][CPL], ss[kTogether];
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) win[k][i] = win[k + 1][i];
-    load_channels<T, CPL, WIDE>(proj, (size_t)t * ld + col0, lane, count, win[kMaxTaps - 1]);
-    float y[CPL];
-    float ss = 0.f;
+    for (int u = 0; u < kTogether; ++u) {
+      ss[u] = 0.f;
 #pragma unroll
-    for (int i = 0; i < CPL; ++i) {
-      float acc = 0.f;
+      for (int i = 0; i < CPL; ++i) {
+        float acc = 0.f;
 #pragma unroll
-      for (int k = 0; k < kMaxTaps; ++k) acc = fmaf(wv[i][k], win[k][i], acc);
-      y[i] = silu(acc);        // (channels behind the unit's: zero)
-      ss = fmaf(y[i], y[i], ss);
+        for (int k = 0; k < TAPS; ++k) acc = fmaf(wv[k][i], win[u + k][i], acc);
+        y[u][i] = silu(acc);        // (channels behind the unit's: zero)
+        ss[u] = fmaf(y[u][i], y[u][i], ss[u]);
+      }
     }
     if (qk) {
-      const float r = scale / sqrtf(wave_sum(ss) + kUnitEps);
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) y[i] *= r;
+      for (int u = 0; u < kTogether; ++u) {
+        const float r = scale / sqrtf(wave_sum(ss[u]) + kUnitEps);
+#pragma unroll
+        for (int i = 0; i < CPL; ++i) y[u][i] *= r;
+      }
     }
-    store_channels<CPL, WIDE>(out + (size_t)t * row + col0, lane, count, y);
+#pragma unroll
+    for (int u = 0; u < kTogether; ++u)
+      if (u < many) store_channels<CPL, WIDE>(out + (size_t)(t0 + u) * row + col0, lane, count, y[u]);
+    // the window moves on by the tokens that were there
+#pragma unroll
+    for (int u = 1; u <= kTogether; ++u) {
+      if (u == many) {
+#pragma unroll
+        for (int k = 0; k < TAPS - 1; ++k)
+#pragma unroll
+          for (int i = 0; i < CPL; ++i) win[k][i] = win[k + u][i];
+      }
+    }
   }
   if (update) {      // (the window now ends at the request's last token)
 #pragma unroll
-    for (int k = 1; k < kMaxTaps; ++k) {
-      const int j = k - (kMaxTaps - (taps - 1));
+    for (int k = 0; k < TAPS - 1; ++k) {
+      const int j = k - (TAPS - taps);
       if (j >= 0) store_channels<CPL, WIDE>(st + (size_t)j * C, lane, count, win[k]);
     }
   }
@@ -406,15 +429,21 @@ int launch_inputs(RowsIn proj, long ld, RowsIn up, long uld, const float* conv, 
   const bool wide = cpl <= 4 && sh.dim % cpl == 0 && sh.heads * sh.vdim % cpl == 0 && ld % cpl == 0 && uld % cpl == 0 &&
                     proj.stride % cpl == 0 && up.stride % cpl == 0 && (uintptr_t)proj.p % 16 == 0 &&
                     (uintptr_t)up.p % 16 == 0 && (uintptr_t)state % 16 == 0 && (uintptr_t)out % 16 == 0;
-#define TK_DI(CPL, WIDE)                                                                                              \
-  delta_inputs_kernel<T, CPL, WIDE><<<grid, 256, 0, stream>>>(proj, ld, up, uld, conv, state, a_log, dt_bias, q_start, \
-                                                              slots, out, sh, q_scale, update)
-  if (cpl == 1) TK_DI(1, false);
-  else if (cpl == 2 && wide) TK_DI(2, true);
-  else if (cpl == 2) TK_DI(2, false);
-  else if (cpl == 4 && wide) TK_DI(4, true);
-  else if (cpl == 4) TK_DI(4, false);
-  else TK_DI(8, false);
+#define TK_DI_AS(CPL, TAPS, WIDE)                                                                                      \
+  delta_inputs_kernel<T, CPL, TAPS, WIDE><<<grid, 256, 0, stream>>>(proj, ld, up, uld, conv, state, a_log, dt_bias, q_start, \
+                                                                    slots, out, sh, q_scale, update)
+#define TK_DI(CPL, WIDE)                        \
+  {                                             \
+    if (sh.taps <= 4) TK_DI_AS(CPL, 4, WIDE);   \
+    else TK_DI_AS(CPL, kMaxTaps, WIDE);         \
+  }
+  if (cpl == 1) TK_DI(1, false)
+  else if (cpl == 2 && wide) TK_DI(2, true)
+  else if (cpl == 2) TK_DI(2, false)
+  else if (cpl == 4 && wide) TK_DI(4, true)
+  else if (cpl == 4) TK_DI(4, false)
+  else TK_DI(8, false)
+#undef TK_DI_AS
 #undef TK_DI
   if (!update && sh.taps > 1) {
     const int C = sh.conv_channels();

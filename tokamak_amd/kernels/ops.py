@@ -293,6 +293,10 @@ _SIGS = {
         "tk_gated_group_norm": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_void_p, c_void_p,
                                 c_int, c_int, c_int, c_float, c_int, c_int, c_void_p],
     },
+    "linear_chunks": {
+        "tk_fixed_decay_chunks": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_void_p, c_void_p, c_void_p, c_void_p,
+                                  c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p],
+    },
     "delta": {
         "tk_delta_inputs": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_void_p, c_int, c_int, c_long, c_long,
                             c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
@@ -1091,6 +1095,11 @@ def ssd_scan(u: torch.Tensor, proj: torch.Tensor, dt_col: int, dt_bias: torch.Te
                                      batch.num_requests, heads, groups, state_size, vdim, *plan, _stream()), "ssd_scan")
 
 
+FIXED_CHUNK_TOKENS = 64          # tokens of a chunk (csrc/linear_chunks.hip: kChunk)
+FIXED_CHUNKS_MAX_DIM = 128
+FIXED_CHUNKS_FROM_TOKENS = 48    # a request's tokens in a step from which the step runs in chunks
+
+
 def fixed_decay_scan(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, y: torch.Tensor, batch, *, heads: int,
                      dim: int, vdim: int) -> None:
     """Linear attention with one constant decay a head: per request and head over the step's tokens in order
@@ -1107,6 +1116,17 @@ def fixed_decay_scan(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tenso
     dtype = torch.bfloat16 if proj.dtype == torch.bfloat16 else torch.float32
     pointer, is_f32, parts, stride, ld = _ssm_in(proj, n, dtype, "projections")
     _need(ld >= heads * (vdim + 2 * dim), "the projections hold v, k and q of every head")
+    if batch.max_q_len >= FIXED_CHUNKS_FROM_TOKENS and max(dim, vdim) <= FIXED_CHUNKS_MAX_DIM:
+        # long portions: chunks side by side on the matrix cores
+        max_chunks = -(-batch.max_q_len // FIXED_CHUNK_TOKENS)
+        chunk_state = torch.empty((n // FIXED_CHUNK_TOKENS + batch.num_requests, heads, -(-vdim // 4), dim, 4),
+                                  dtype=torch.float32, device=y.device)
+        _note(f"{n}x{heads}x{dim}x{vdim} chunks", n * heads * ((2 * dim + vdim) * proj.element_size() * parts + vdim * 4),
+              4.0 * n * heads * dim * vdim)
+        _check(_fn("linear_chunks", "tk_fixed_decay_chunks")(
+            _code(dtype), pointer, is_f32, parts, stride, ld, _p(decay), _p(state), _p(batch.q_start), _p(batch.state_slots),
+            _p(y), batch.num_requests, heads, dim, vdim, max_chunks, _p(chunk_state), _stream()), "fixed_decay_chunks")
+        return
     plan = _scan_chunks(batch, n, heads, dim, vdim, y.device)
     _note(f"{n}x{heads}x{dim}x{vdim}", n * heads * ((2 * dim + vdim) * proj.element_size() * parts + vdim * 4),
           4.0 * n * heads * dim * vdim)
