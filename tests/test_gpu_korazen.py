@@ -212,6 +212,28 @@ def test_delta_rule_in_portions_over_state_slots(dtype, name):
         assert bool((array[3] == 7.0).all()) and bool((array[1] == 0.0).all())
 
 
+def test_decays_are_exact_from_nearly_zero_to_nearly_one():
+    """exp(-exp(A_log) softplus(z)) for z from -30 to 30: where the decay is close to one its distance from one is
+    right too, as far as float32 holds it."""
+    from tokamak_amd.kernels import ops
+
+    heads, dim, n = 4, 16, 512
+    z = torch.linspace(-30.0, 30.0, n * heads * dim, dtype=torch.float64).view(n, heads * dim).float()
+    a_log = torch.tensor([-2.0, -0.5, 0.3, 1.5])
+    row = ops.delta_row(heads, 1, dim, 1)
+    out = torch.empty(n, row, dtype=torch.float32, device=DEV)
+    ops.delta_inputs(torch.zeros(n, 2 * dim + 2 * heads, device=DEV), z.to(DEV), torch.zeros(2 * dim + heads, 1, device=DEV), None,
+                     a_log.to(DEV), torch.zeros(heads * dim, device=DEV), out, make_batch([(n, 0, [0])]), heads=heads, kv_heads=1,
+                     dim=dim, vdim=1, q_scale=1.0)
+    got = out.cpu().double()[:, 2 * dim + heads:2 * dim + heads + heads * dim]
+    rate = torch.exp(a_log.double()).repeat_interleave(dim)
+    step = torch.clamp(z.double(), min=0) + torch.log1p(torch.exp(-z.double().abs()))
+    want = torch.exp(-rate * step)
+    assert float((got - want).abs().max()) < 3e-7
+    kept = want > 1e-30
+    assert float(((got - want).abs() / want)[kept].max()) < 2e-5
+
+
 @pytest.mark.parametrize("tokens_a", [40, 700])
 def test_delta_scan_remembers_one_write_and_replaces_it(tokens_a):
     """Decays of one: a value written under one key is read back hundreds of tokens later among writes under keys

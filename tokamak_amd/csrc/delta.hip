@@ -135,7 +135,7 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(
       for (int u = 0; u < kTogether; ++u) {
         if (t0 + u >= t_hi) break;
 #pragma unroll
-        for (int i = 0; i < CPL; ++i) z[u][i] = expf(-rate[i] * softplus(z[u][i] + bias[i]));
+        for (int i = 0; i < CPL; ++i) z[u][i] = __expf(-rate[i] * softplus(z[u][i] + bias[i]));
         store_channels<CPL, WIDE>(dst + (size_t)(t0 + u) * row + from, lane, count, z[u]);
       }
     }

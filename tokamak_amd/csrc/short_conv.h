@@ -33,7 +33,13 @@ __device__ __forceinline__ float load_in(const RowsIn& in, size_t idx) {
 
 __device__ __forceinline__ float sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
 __device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
-__device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+// log(1 + e^x) = max(x, 0) + log1p(e), e = e^-|x|, with log1p(e) = log(u) e / (u - 1), u = 1 + e rounded (the rounding
+// of u cancels in the quotient; the library's log1pf is several times the rest of a kernel that forms a decay
+// per channel: 126 against 60 us for 2,048 tokens of 4,096 channels)
+__device__ __forceinline__ float softplus(float x) {
+  const float e = expf(-fabsf(x)), u = 1.f + e;
+  return fmaxf(x, 0.f) + (u == 1.f ? e : __logf(u) * (e / (u - 1.f)));
+}
 
 // The state after a step: the last taps - 1 inputs of every request, from the step's rows or, where the
 // step brought fewer, from the state before it.  A thread a (request, channel): it reads what it needs, then writes.

@@ -322,6 +322,22 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
 
 // The same for parts of 4 to 256 columns where a lane takes four neighbours: LANES = size / 4 lanes a part (a power
 // of two), 64 / LANES parts a wave.
+template <typename T>
+__device__ __forceinline__ float4 load_four(const SsmIn& in, size_t at) {
+  if (!in.f32) {
+    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(in.p) + at);
+    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+                       __uint_as_float(u.y & 0xffff0000u));
+  }
+  const float* f = reinterpret_cast<const float*>(in.p) + at;
+  float4 s = *reinterpret_cast<const float4*>(f);
+  for (int i = 1; i < in.parts; ++i) {
+    const float4 a = *reinterpret_cast<const float4*>(f + (size_t)i * in.stride);
+    s.x += a.x; s.y += a.y; s.z += a.z; s.w += a.w;
+  }
+  return s;
+}
+
 template <typename T, int LANES>
 __global__ __launch_bounds__(256) void gated_group_norm_four_kernel(
     const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
@@ -334,20 +350,9 @@ __global__ __launch_bounds__(256) void gated_group_norm_four_kernel(
   const int g = (int)(pair - n * groups);
   const size_t at = (size_t)n * inner + (size_t)g * size + sub * 4;
   const size_t zat = (size_t)n * ld + z_col + (size_t)g * size + sub * 4;
-  float z[4], v[4];
-  if (!z_in.f32) {
-    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(z_in.p) + zat);
-    z[0] = __uint_as_float(u.x << 16); z[1] = __uint_as_float(u.x & 0xffff0000u);
-    z[2] = __uint_as_float(u.y << 16); z[3] = __uint_as_float(u.y & 0xffff0000u);
-  } else {
-    const float* f = reinterpret_cast<const float*>(z_in.p) + zat;
-    float4 s = *reinterpret_cast<const float4*>(f);
-    for (int i = 1; i < z_in.parts; ++i) {
-      const float4 a = *reinterpret_cast<const float4*>(f + (size_t)i * z_in.stride);
-      s.x += a.x; s.y += a.y; s.z += a.z; s.w += a.w;
-    }
-    z[0] = s.x; z[1] = s.y; z[2] = s.z; z[3] = s.w;
-  }
+  float v[4];
+  const float4 z4 = load_four<T>(z_in, zat);
+  const float z[4] = {z4.x, z4.y, z4.z, z4.w};
   const float4 y4 = *reinterpret_cast<const float4*>(y + at);
   const float4 w4 = *reinterpret_cast<const float4*>(weight + (shared ? 0 : g * size) + sub * 4);
   v[0] = before_norm(y4.x, z[0], after); v[1] = before_norm(y4.y, z[1], after);
@@ -397,6 +402,46 @@ __global__ __launch_bounds__(1024) void gated_group_norm_block_kernel(
     const float z = load_in<T>(z_in, zat + x);
     const float v = before_norm(y[at + x], z, after);
     Elem<T>::store(out + at + x, behind_norm(v * rstd * weight[shared ? x : g * size + x], z, after));
+  }
+}
+
+// The same for long parts whose size is a multiple of four: a thread up to kHoldFours pieces of four neighbours.
+constexpr int kHoldFours = 4;
+template <typename T>
+__global__ __launch_bounds__(1024) void gated_group_norm_block_four_kernel(
+    const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
+    T* __restrict__ out, int inner, int groups, float eps, int shared, int after) {
+  __shared__ float scratch[16];
+  const long pair = blockIdx.x;
+  const long n = pair / groups;
+  const int g = (int)(pair - n * groups), size = inner / groups;
+  const size_t at = (size_t)n * inner + (size_t)g * size;
+  const size_t zat = (size_t)n * ld + z_col + (size_t)g * size;
+  const float* w = weight + (shared ? 0 : g * size);
+  float4 held[kHoldFours], gate[kHoldFours];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < kHoldFours; ++i) {
+    const int x = (threadIdx.x + i * blockDim.x) * 4;
+    held[i] = gate[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (x < size) {
+      gate[i] = load_four<T>(z_in, zat + x);
+      const float4 v = *reinterpret_cast<const float4*>(y + at + x);
+      held[i] = make_float4(before_norm(v.x, gate[i].x, after), before_norm(v.y, gate[i].y, after),
+                            before_norm(v.z, gate[i].z, after), before_norm(v.w, gate[i].w, after));
+      ss += held[i].x * held[i].x + held[i].y * held[i].y + held[i].z * held[i].z + held[i].w * held[i].w;
+    }
+  }
+  ss = block_sum(ss, scratch);
+  const float rstd = 1.f / sqrtf(ss / (float)size + eps);
+#pragma unroll
+  for (int i = 0; i < kHoldFours; ++i) {
+    const int x = (threadIdx.x + i * blockDim.x) * 4;
+    if (x < size) {
+      const float4 w4 = *reinterpret_cast<const float4*>(w + x);
+      store_four<T>(out + at + x, behind_norm(held[i].x * rstd * w4.x, gate[i].x, after), behind_norm(held[i].y * rstd * w4.y, gate[i].y, after),
+                    behind_norm(held[i].z * rstd * w4.z, gate[i].z, after), behind_norm(held[i].w * rstd * w4.w, gate[i].w, after), 4, true);
+    }
   }
 }
 
@@ -545,6 +590,17 @@ TK_API int tk_gated_group_norm(int dtype, const float* y, const void* z, int z_f
   const SsmIn in{z, z_f32 || dtype == 0, z_parts, z_stride};
   const long pairs = (long)N * groups;
   const int size = inner / groups;
+  const bool fours = size % 4 == 0 && ld % 4 == 0 && z_col % 4 == 0 && z_stride % 4 == 0 && (uintptr_t)y % 16 == 0 &&
+                     (uintptr_t)z % 16 == 0 && (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0;
+  if (size > 256 && fours && size <= 4 * kHoldFours * 1024) {
+    if (pairs > 0x7fffffffL) return -1;
+    // one piece a thread when rows are few (short chain), up to four when many
+    int threads = 64;
+    while (threads < 1024 && threads * 4 * (pairs >= 512 ? kHoldFours : 1) < size) threads *= 2;
+    if (dtype == 0) gated_group_norm_block_four_kernel<float><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (float*)out, inner, groups, eps, shared, after);
+    else gated_group_norm_block_four_kernel<bf16_t><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, inner, groups, eps, shared, after);
+    return launch_status();
+  }
   if (size > 256) {
     // a block a (token, part): enough threads that each holds a few elements
     int threads = 64;
@@ -554,8 +610,7 @@ TK_API int tk_gated_group_norm(int dtype, const float* y, const void* z, int z_f
     else gated_group_norm_block_kernel<bf16_t><<<(unsigned)pairs, threads, 0, stream>>>(y, in, ld, z_col, weight, (bf16_t*)out, inner, groups, eps, shared, after);
     return launch_status();
   }
-  if ((size & (size - 1)) == 0 && size >= 4 && ld % 4 == 0 && z_col % 4 == 0 && z_stride % 4 == 0 && (uintptr_t)y % 16 == 0 &&
-      (uintptr_t)z % 16 == 0 && (uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0 && pairs * (size / 4) <= 0x7fffffffL) {
+  if (fours && (size & (size - 1)) == 0 && pairs * (size / 4) <= 0x7fffffffL) {
     const unsigned quads = (unsigned)((pairs * (size / 4) + 255) / 256);
 #define TK_GN(LANES)                                                                                                      \
   case LANES * 4:                                                                                                         \
