@@ -414,6 +414,15 @@ __global__ __launch_bounds__(kScanThreads, 1) void delta_scan_kernel(
   }
 }
 
+// out[n][c] = the sum of a split product's partial sums at column col0 + c, rounded to T
+template <typename T>
+__global__ __launch_bounds__(256) void sum_columns_kernel(RowsIn in, long ld, int col0, T* __restrict__ out, int width, long total) {
+  const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const long n = idx / width;
+  Elem<T>::store(out + idx, load_in<T>(in, (size_t)n * ld + col0 + (idx - n * width)));
+}
+
 template <typename T>
 int launch_inputs(RowsIn proj, long ld, RowsIn up, long uld, const float* conv, float* state, const float* a_log,
                   const float* dt_bias, const int* q_start, const int* slots, float* out, int R, DeltaShape sh,
@@ -453,6 +462,19 @@ int launch_inputs(RowsIn proj, long ld, RowsIn up, long uld, const float* conv, 
 }
 
 }  // namespace
+
+// in: float32 [parts, N, ld], parts part_stride elements apart; out [N, width] in dtype: the sums of columns col0 .. + width.
+TK_API int tk_sum_columns(int dtype, const void* in, int parts, long part_stride, long ld, int col0, void* out, int N, int width,
+                          hipStream_t stream) {
+  if (N <= 0 || width <= 0) return 0;
+  if (parts < 1 || col0 < 0 || ld < (long)col0 + width) return -1;
+  const RowsIn r{in, 1, parts, part_stride};
+  const long total = (long)N * width;
+  const unsigned blocks = (unsigned)((total + 255) / 256);
+  if (dtype == 0) sum_columns_kernel<float><<<blocks, 256, 0, stream>>>(r, ld, col0, (float*)out, width, total);
+  else sum_columns_kernel<bf16_t><<<blocks, 256, 0, stream>>>(r, ld, col0, (bf16_t*)out, width, total);
+  return launch_status();
+}
 
 // proj: [N, ld] in dtype, float32 (in_f32) or float32 partial sums, its columns [q: kv dim | k: kv dim | v: heads vdim |
 // b: heads | ...]; up: [N, uld] likewise, its first heads * dim columns the decays' pre-activations.  conv float32
@@ -501,5 +523,6 @@ TK_API int tk_delta_scan(const float* in, float* state, const int* q_start, cons
   return launch_status();
 }
 
+TK_SLOTS(tk_sum_columns)
 TK_SLOTS(tk_delta_inputs)
 TK_SLOTS(tk_delta_scan)

@@ -298,6 +298,7 @@ _SIGS = {
                                   c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p],
     },
     "delta": {
+        "tk_sum_columns": [c_int, c_void_p, c_int, c_long, c_long, c_int, c_void_p, c_int, c_int, c_void_p],
         "tk_delta_inputs": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_void_p, c_int, c_int, c_long, c_long,
                             c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                             c_int, c_int, c_int, c_float, c_int, c_void_p],
@@ -1160,6 +1161,17 @@ DELTA_MAX_DIM = 512          # key channels of a head of the delta-rule scan (cs
 def delta_row(heads: int, kv_heads: int, dim: int, vdim: int) -> int:
     """Numbers a token has in the row that ``delta_inputs`` leaves for ``delta_scan``."""
     return -(-(2 * kv_heads * dim + heads * (vdim + dim + 1)) // 4) * 4
+
+
+def sum_columns(partials: torch.Tensor, col0: int, out: torch.Tensor) -> None:
+    """out[n, c] = the sum of a split product's float32 partial sums [P, N, ld] at column col0 + c, in out's dtype."""
+    _gpu(partials, out)
+    n, width = out.shape
+    _need(partials.dim() == 3 and partials.dtype == torch.float32 and partials.shape[1] == n and 0 <= col0
+          and col0 + width <= partials.shape[2], "the summed columns lie outside the partial sums")
+    _note(f"{n}x{width}", n * width * (4 * partials.shape[0] + out.element_size()))
+    _check(_fn("delta", "tk_sum_columns")(_code(out.dtype), _p(partials), partials.shape[0], partials.stride(0), partials.shape[2],
+                                          int(col0), _p(out), n, width, _stream()), "sum_columns")
 
 
 def delta_inputs(proj: torch.Tensor, up: torch.Tensor, conv: torch.Tensor, conv_state: torch.Tensor | None, a_log: torch.Tensor,

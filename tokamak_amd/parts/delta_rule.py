@@ -13,6 +13,7 @@ from tokamak_amd.weights.spec import TensorSpec
 LOW = 8        # the low ranks are padded with rows of zeros to a multiple of this (16-byte rows of the second product)
 WHOLE = 256    # ... and a large first matrix to a multiple of this (the library's tiles: 2,048 rows of 4,096 into 12,576
                # columns take 180 us, into 12,800 165)
+SPLIT_FROM_ROWS = 16   # beyond so many rows the first product may be split over K (64 rows of 4,096: 29 + 3 us against 43; 8 rows level)
 
 
 class ChannelDeltaRule(Mixer):
@@ -32,8 +33,7 @@ class ChannelDeltaRule(Mixer):
     the recurrence behind the products is float32.  The low ranks of W_a1 and W_g1 are read off the checkpoint unless
     ``decay_rank`` and ``gate_rank`` give them.
 
-    q, k, v, b and the two low ranks are one product of h (not split over K: the low ranks are read back as rows), and
-    the second matrices of the low ranks a second one, on a matrix that is zero where the two do not meet.
+    q, k, v, b and the two low ranks are one product of h, and the second matrices of the low ranks a second one, on a matrix that is zero where the two do not meet.
     Tensors: q, k, v with ``.conv`` each, b, A_log, norm, a1, a2, dt_bias, g1, g2, o behind the part's prefix.
     """
 
@@ -104,8 +104,14 @@ class ChannelDeltaRule(Mixer):
 
     def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None):
         n, sizes = h.shape[0], dict(heads=self.num_heads, kv_heads=self.num_kv_heads, dim=self.head_dim, vdim=self.value_dim)
-        proj = linear(h, self.first)
-        low = proj[:, self.low_at:self.low_at + self.low_width]
+        # (a split product leaves float32 partial sums, which the kernels below add as they load; the low ranks' sum is
+        # a kernel of its own then, which pays from some rows on)
+        proj = linear(h, self.first, allow_partials=n > SPLIT_FROM_ROWS)
+        if proj.dim() == 3:
+            low = torch.empty((n, self.low_width), dtype=self.dtype, device=h.device)
+            ops.sum_columns(proj, self.low_at, low)
+        else:
+            low = proj[:, self.low_at:self.low_at + self.low_width]
         few = n <= ops.STREAM_MAX_ROWS      # (few rows: float32 from the streaming product, at no cost)
         up = linear(low, self.up, out_dtype=torch.float32 if few else None, allow_partials=True)
         operands = torch.empty((n, ops.delta_row(**sizes)), dtype=torch.float32, device=h.device)
