@@ -7,6 +7,31 @@
 
 using namespace tk;
 
+// four neighbouring elements as floats, one access
+template <typename TD> struct Load4;
+template <> struct Load4<float> {
+  static __device__ __forceinline__ float4 at(const float* p) { return *reinterpret_cast<const float4*>(p); }
+};
+template <> struct Load4<bf16_t> {
+  static __device__ __forceinline__ float4 at(const bf16_t* p) {
+    const uint2 u = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u),
+                       __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
+  }
+};
+template <typename T> struct Store4;
+template <> struct Store4<float> {
+  static __device__ __forceinline__ void at(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+};
+template <> struct Store4<bf16_t> {
+  static __device__ __forceinline__ void at(bf16_t* p, float4 v) {
+    uint2 u;
+    u.x = pack_bf16x2(v.x, v.y);
+    u.y = pack_bf16x2(v.z, v.w);
+    *reinterpret_cast<uint2*>(p) = u;
+  }
+};
+
 // ---------------------------------------------------------------------------
 // embedding: resid[n, :] = float(table[ids[n], :]) * scale, or with `accumulate`
 // resid[n, :] += float(table[ids[n], :]) * scale (the same rows added to the stream once
@@ -68,9 +93,65 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const T* __restrict__ t
   }
 }
 
+// The same, the row in registers: H a multiple of 4 and at most 16 * blockDim.
+template <typename T>
+__global__ __launch_bounds__(1024) void embed_norm_vec_kernel(const T* __restrict__ table, const int* __restrict__ ids,
+                                                              const float* __restrict__ weight, float* __restrict__ resid,
+                                                              int H, int V, float scale, float eps, int accumulate) {
+  constexpr int GROUPS = 4;
+  __shared__ float scratch[16];
+  const int n = blockIdx.x;
+  const int id = ids[n];
+  float* out = resid + (size_t)n * H;
+  if (id < 0 || id >= V) {      // (the whole block, before any barrier)
+    for (int d = threadIdx.x; d < H; d += blockDim.x) out[d] = __uint_as_float(0x7fc00000u);
+    return;
+  }
+  const T* row = table + (size_t)id * H;
+  float4 v[GROUPS], w[GROUPS];
+  float ss = 0.f;
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    v[g] = w[g] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (d < H) {
+      v[g] = Load4<T>::at(row + d);
+      w[g] = *reinterpret_cast<const float4*>(weight + d);
+    }
+  }
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    v[g].x *= scale; v[g].y *= scale; v[g].z *= scale; v[g].w *= scale;
+    ss += v[g].x * v[g].x + v[g].y * v[g].y + v[g].z * v[g].z + v[g].w * v[g].w;
+  }
+  ss = block_sum(ss, scratch);
+  const float rstd = 1.f / sqrtf(ss / (float)H + eps);
+#pragma unroll
+  for (int g = 0; g < GROUPS; ++g) {
+    const int d = (g * blockDim.x + threadIdx.x) * 4;
+    if (d < H) {
+      float4 o = make_float4(v[g].x * rstd * w[g].x, v[g].y * rstd * w[g].y, v[g].z * rstd * w[g].z, v[g].w * rstd * w[g].w);
+      if (accumulate) {
+        const float4 x = *reinterpret_cast<const float4*>(out + d);
+        o.x += x.x; o.y += x.y; o.z += x.z; o.w += x.w;
+      }
+      *reinterpret_cast<float4*>(out + d) = o;
+    }
+  }
+}
+
 TK_API int tk_embed_norm(int dtype, const void* table, const int* ids, const float* weight, float* resid, int N, int H,
                          int V, float scale, float eps, int accumulate, hipStream_t stream) {
   if (N <= 0) return 0;
+  int threads = 64;
+  while (threads < 1024 && threads * 4 < H) threads *= 2;
+  if (H % 4 == 0 && H <= threads * 16 && (uintptr_t)table % 16 == 0 && (uintptr_t)weight % 16 == 0 && (uintptr_t)resid % 16 == 0) {
+    if (dtype == 0)
+      embed_norm_vec_kernel<float><<<N, threads, 0, stream>>>((const float*)table, ids, weight, resid, H, V, scale, eps, accumulate);
+    else
+      embed_norm_vec_kernel<bf16_t><<<N, threads, 0, stream>>>((const bf16_t*)table, ids, weight, resid, H, V, scale, eps, accumulate);
+    return launch_status();
+  }
   if (dtype == 0)
     embed_norm_kernel<float><<<N, 256, 0, stream>>>((const float*)table, ids, weight, resid, H, V, scale, eps, accumulate);
   else
@@ -105,30 +186,6 @@ TK_API int tk_feed_tokens(int* ids, const int* sampled, const int* slots, const 
 // ---------------------------------------------------------------------------
 // delta may come as `parts` float32 partial sums, part_stride elements apart
 // (a split-K product's output): they are added in order.
-template <typename TD> struct Load4;
-template <> struct Load4<float> {
-  static __device__ __forceinline__ float4 at(const float* p) { return *reinterpret_cast<const float4*>(p); }
-};
-template <> struct Load4<bf16_t> {
-  static __device__ __forceinline__ float4 at(const bf16_t* p) {
-    const uint2 u = *reinterpret_cast<const uint2*>(p);
-    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u),
-                       __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xffff0000u));
-  }
-};
-template <typename T> struct Store4;
-template <> struct Store4<float> {
-  static __device__ __forceinline__ void at(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
-};
-template <> struct Store4<bf16_t> {
-  static __device__ __forceinline__ void at(bf16_t* p, float4 v) {
-    uint2 u;
-    u.x = pack_bf16x2(v.x, v.y);
-    u.y = pack_bf16x2(v.z, v.w);
-    *reinterpret_cast<uint2*>(p) = u;
-  }
-};
-
 // Vector form: H a multiple of 4 and at most 4 * kNormGroups * blockDim.  A thread
 // keeps its elements of the row in registers, and all loads of the partial sums
 // are issued before the first add, so a row costs about one memory round trip.
@@ -1170,12 +1227,34 @@ __global__ void sigmoid_gate_kernel(T* __restrict__ x, const void* __restrict__ 
   Elem<T>::store(at, Elem<T>::load(at) / (1.f + expf(-g)));
 }
 
+// four neighbouring columns a thread: vd, vdp, ld, col0 and part_stride multiples of four
+template <typename T>
+__global__ void sigmoid_gate_four_kernel(T* __restrict__ x, NormBranch gate, long ld, int col0, int width, int vd, int vdp, size_t total4) {
+  const size_t i4 = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i4 >= total4) return;
+  const int quads = width / 4;
+  const size_t n = i4 / quads;
+  const int c = (int)(i4 - n * quads) * 4;
+  const int head = c / vd, d = c - head * vd;
+  const float4 g = branch_four<T>(gate, n * ld + col0 + c);
+  T* at = x + n * ((size_t)(width / vd) * vdp) + (size_t)head * vdp + d;
+  const float4 v = Load4<T>::at(at);
+  Store4<T>::at(at, make_float4(v.x / (1.f + expf(-g.x)), v.y / (1.f + expf(-g.y)), v.z / (1.f + expf(-g.z)), v.w / (1.f + expf(-g.w))));
+}
+
 TK_API int tk_sigmoid_gate(int dtype, void* x, const void* gate, int f32, int parts, long part_stride, long ld, int col0,
                            int N, int heads, int vd, int vdp, hipStream_t stream) {
   if (N <= 0) return 0;
   if (heads < 1 || vd < 1 || vdp < vd || parts < 1 || (parts > 1 && !f32 && dtype != 0) || col0 < 0 || ld < (long)col0 + (long)heads * vd)
     return -1;
   const size_t total = (size_t)N * heads * vd;
+  if (vd % 4 == 0 && vdp % 4 == 0 && ld % 4 == 0 && col0 % 4 == 0 && part_stride % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)gate % 16 == 0) {
+    const unsigned quads = (unsigned)((total / 4 + 255) / 256);
+    const NormBranch g{gate, f32 || dtype == 0, parts, part_stride};
+    if (dtype == 0) sigmoid_gate_four_kernel<float><<<quads, 256, 0, stream>>>((float*)x, g, ld, col0, heads * vd, vd, vdp, total / 4);
+    else sigmoid_gate_four_kernel<bf16_t><<<quads, 256, 0, stream>>>((bf16_t*)x, g, ld, col0, heads * vd, vd, vdp, total / 4);
+    return launch_status();
+  }
   const unsigned blocks = (unsigned)((total + 255) / 256);
   if (dtype == 0)
     sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, gate, 1, parts, part_stride, ld, col0, heads * vd, vd, vdp, total);

@@ -107,6 +107,33 @@ __device__ __forceinline__ void sum_and_deal(float (&v)[32], int ks) {
   }
 }
 
+// four neighbouring elements from `at` on (a multiple of four, rows and partial sums likewise)
+template <typename T>
+__device__ __forceinline__ float4 load_four(const SsmIn& in, size_t at) {
+  if (!in.f32) {
+    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(in.p) + at);
+    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+                       __uint_as_float(u.y & 0xffff0000u));
+  }
+  const float* f = reinterpret_cast<const float*>(in.p) + at;
+  float4 s = *reinterpret_cast<const float4*>(f);
+  int i = 1;
+  for (; i + 3 < in.parts; i += 4) {      // four loads in flight; the sums in the order of the parts
+    float4 q[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) q[u] = *reinterpret_cast<const float4*>(f + (size_t)(i + u) * in.stride);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      s.x += q[u].x; s.y += q[u].y; s.z += q[u].z; s.w += q[u].w;
+    }
+  }
+  for (; i < in.parts; ++i) {
+    const float4 a = *reinterpret_cast<const float4*>(f + (size_t)i * in.stride);
+    s.x += a.x; s.y += a.y; s.z += a.z; s.w += a.w;
+  }
+  return s;
+}
+
 struct ScanShape {
   int heads, groups, ns, vdim;      // ns: the state's size per value channel
   int columns;                      // groups of four value columns that a block holds
@@ -322,22 +349,6 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(
 
 // The same for parts of 4 to 256 columns where a lane takes four neighbours: LANES = size / 4 lanes a part (a power
 // of two), 64 / LANES parts a wave.
-template <typename T>
-__device__ __forceinline__ float4 load_four(const SsmIn& in, size_t at) {
-  if (!in.f32) {
-    const uint2 u = *reinterpret_cast<const uint2*>(reinterpret_cast<const bf16_t*>(in.p) + at);
-    return make_float4(__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
-                       __uint_as_float(u.y & 0xffff0000u));
-  }
-  const float* f = reinterpret_cast<const float*>(in.p) + at;
-  float4 s = *reinterpret_cast<const float4*>(f);
-  for (int i = 1; i < in.parts; ++i) {
-    const float4 a = *reinterpret_cast<const float4*>(f + (size_t)i * in.stride);
-    s.x += a.x; s.y += a.y; s.z += a.z; s.w += a.w;
-  }
-  return s;
-}
-
 template <typename T, int LANES>
 __global__ __launch_bounds__(256) void gated_group_norm_four_kernel(
     const float* __restrict__ y, SsmIn z_in, long ld, int z_col, const float* __restrict__ weight,
