@@ -19,6 +19,7 @@
 // a second kernel merges the splits of each (token, head).
 #include "common.h"
 #include "slots.h"
+#include "soft_cap.h"
 
 using namespace tk;
 
@@ -123,14 +124,15 @@ __device__ __forceinline__ void decode_head_vector(const DecodeInputs& in, size_
 // call stores, the token's own key and value, which the block of the last split writes to
 // the page and every wave that meets the token's position takes from LDS) from the
 // projection's output: one kernel less a layer than with the separate q/k norm kernel.
-template <int HD, int WAVES, int D, bool FUSED>
+template <int HD, int WAVES, int D, bool FUSED, bool CAP>
 __global__ __launch_bounds__(WAVES * 64) void attention_decode_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache_in,
     const bf16_t* __restrict__ v_cache_in, const int* __restrict__ block_tables, int max_pages,
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ item_token, const int* __restrict__ item_count,
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int nsplit,
-    int split_keys, int nh, int nkv, int ps, float scale_log2, DecodeInputs in, const float* __restrict__ sinks) {
+    int split_keys, int nh, int nkv, int ps, float scale_log2, DecodeInputs in, const float* __restrict__ sinks,
+    SoftCap cap) {
   const bf16_t* __restrict__ k_cache = k_cache_in;
   const bf16_t* __restrict__ v_cache = v_cache_in;
   constexpr int KCH = HD / 32;  // 32-wide chunks of the head dim (QK^T steps)
@@ -284,7 +286,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_kernel(
       float sv[4];
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        sv[e] = sc[e] * scale_log2;
+        sv[e] = CAP ? cap.log2_score(sc[e]) : sc[e] * scale_log2;
         if (edge && c0 + kb * 4 + e > pos0) sv[e] = -INFINITY;
       }
       float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
@@ -484,7 +486,7 @@ constexpr int kPrefillThreads = 256;
 // OCC: waves a SIMD the compiler must leave room for.  Three (what OCC = 2 gives) are best
 // when tiles differ in length (a prompt from position zero: the longest tile's walk
 // decides); four (a few registers spilled) when every tile walks a long context.
-template <int HD, int HPB, int OCC>
+template <int HD, int HPB, int OCC, bool CAP>
 __global__ __launch_bounds__(kPrefillThreads) __attribute__((amdgpu_waves_per_eu(OCC)))
 void attention_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
@@ -492,8 +494,9 @@ void attention_prefill_kernel(
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ item_token, const int* __restrict__ item_count,
     bf16_t* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int nsplit,
-    int split_keys, int num_items, int nh, int nkv, int ps, float scale_log2, int chunk,
-    const float* __restrict__ sinks) {
+    int split_keys, int num_items, int nh, int nkv, int ps, float scale_arg, int chunk,
+    const float* __restrict__ sinks, SoftCap cap) {
+  const float scale_log2 = CAP ? 1.f : scale_arg;   // (capped scores are in units of log2 already)
   constexpr int KCH = HD / 32, DBL = HD / 16;
   constexpr int THREADS = kPrefillThreads;
   constexpr int GROUP_PIECES = 2 * HD;         // 16-byte pieces of K (and of V) per 16-key group
@@ -644,7 +647,7 @@ void attention_prefill_kernel(
         sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, qreg[c], sc, 0, 0, 0);
       }
 #pragma unroll
-      for (int i = 0; i < 4; ++i) sv[j][i] = sc[i];
+      for (int i = 0; i < 4; ++i) sv[j][i] = CAP ? cap.log2_score(sc[i]) : sc[i];
     }
     if (s0 + 63 > pos0 || s0 < first_of_last) {  // some key of this stage is hidden from some column, or is past the end
 #pragma unroll
@@ -751,15 +754,16 @@ void attention_prefill_kernel(
 // ---------------------------------------------------------------------------
 typedef float float16v __attribute__((ext_vector_type(16)));
 
-template <int HD, int HPB>
+template <int HD, int HPB, bool CAP>
 __global__ __launch_bounds__(kPrefillThreads) __attribute__((amdgpu_waves_per_eu(2)))
 void attention_prefill_wide_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int max_pages,
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ item_token, const int* __restrict__ item_count,
-    bf16_t* __restrict__ out, int num_items, int nh, int nkv, int ps, float scale_log2,
-    const float* __restrict__ sinks) {
+    bf16_t* __restrict__ out, int num_items, int nh, int nkv, int ps, float scale_arg,
+    const float* __restrict__ sinks, SoftCap cap) {
+  const float scale_log2 = CAP ? 1.f : scale_arg;   // (capped scores are in units of log2 already)
   constexpr int KST = HD / 16;  // 16-wide steps over the head dim (QK^T)
   constexpr int DB = HD / 32;   // 32-wide blocks of the head dim (PV outputs)
   constexpr int DBL = HD / 16;  // 16-dim blocks of a V page
@@ -878,6 +882,12 @@ void attention_prefill_wide_kernel(
         sc[kb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf.v, qreg[c], sc[kb], 0, 0, 0);
       }
     }
+    if constexpr (CAP) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) sc[kb][e] = cap.log2_score(sc[kb][e]);
+    }
     if (s0 + 63 > pos0) {  // some key of this stage is hidden from some query, or is past the end
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -968,15 +978,16 @@ void attention_prefill_wide_kernel(
 // prompt, leaves no CU with one long tile at a quarter of its waves: tiles are started
 // longest first, twice as many as there are CUs, and the short ones fill in behind.
 // ---------------------------------------------------------------------------
-template <int HD, int GB, int S>
+template <int HD, int GB, int S, bool CAP>
 __global__ __launch_bounds__(GB * S * 64)
 void attention_prefill_group_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int max_pages,
     const int* __restrict__ positions, const int* __restrict__ req_of_token,
     const int* __restrict__ item_token, const int* __restrict__ item_count,
-    bf16_t* __restrict__ out, int num_items, int nh, int nkv, int ps, float scale_log2,
-    const float* __restrict__ sinks) {
+    bf16_t* __restrict__ out, int num_items, int nh, int nkv, int ps, float scale_arg,
+    const float* __restrict__ sinks, SoftCap cap) {
+  const float scale_log2 = CAP ? 1.f : scale_arg;   // (capped scores are in units of log2 already)
   constexpr int KST = HD / 16;  // 16-wide steps over the head dim (QK^T)
   constexpr int DB = HD / 32;   // 32-wide blocks of the head dim (PV outputs)
   constexpr int DBL = HD / 16;  // 16-dim blocks of a V page
@@ -1163,6 +1174,12 @@ void attention_prefill_group_kernel(
       }
       __builtin_amdgcn_sched_group_barrier(0x008, KST, 0);
     }
+    if constexpr (CAP) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) sc[kb][e] = cap.log2_score(sc[kb][e]);
+    }
     if (w0 + 63 > pos0) {  // some key of these is hidden from some query, or is past the end
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -1290,13 +1307,14 @@ static int launch_prefill(const void* q, const void* k_cache, const void* v_cach
                           const int* req_of_token, const int* item_token, const int* item_count,
                           int num_items, void* out, float* part_o, float* part_ml, int nsplit,
                           int split_keys, int nh, int nkv, int ps, float scale, hipStream_t stream, int chunk,
-                          const float* sinks) {
+                          const float* sinks, float softcap) {
   const int G = nh / nkv;
+  auto* const kernel = softcap > 0.f ? &attention_prefill_kernel<HD, HPB, OCC, true> : &attention_prefill_kernel<HD, HPB, OCC, false>;
   dim3 grid(nkv * (G / HPB), num_items, nsplit);
-  attention_prefill_kernel<HD, HPB, OCC><<<grid, kPrefillThreads, 0, stream>>>(
+  kernel<<<grid, kPrefillThreads, 0, stream>>>(
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages,
       positions, req_of_token, item_token, item_count, (bf16_t*)out, part_o, part_ml, nsplit,
-      split_keys, num_items, nh, nkv, ps, scale * 1.4426950408889634f, chunk, sinks);
+      split_keys, num_items, nh, nkv, ps, scale * 1.4426950408889634f, chunk, sinks, soft_cap(scale, softcap));
   if (nsplit > 1) {
     dim3 mgrid(num_items * 16, nh);
     attention_merge_kernel<HD><<<mgrid, 64, 0, stream>>>(part_o, part_ml, positions, item_token, item_count,
@@ -1310,13 +1328,14 @@ static int launch_prefill_wide(const void* q, const void* k_cache, const void* v
                                const int* block_tables, int max_pages, const int* positions,
                                const int* req_of_token, const int* item_token, const int* item_count,
                                int num_items, void* out, int nh, int nkv, int ps, float scale,
-                               hipStream_t stream, const float* sinks) {
+                               hipStream_t stream, const float* sinks, float softcap) {
   const int G = nh / nkv;
+  auto* const kernel = softcap > 0.f ? &attention_prefill_wide_kernel<HD, HPB, true> : &attention_prefill_wide_kernel<HD, HPB, false>;
   dim3 grid(nkv * (G / HPB), num_items);
-  attention_prefill_wide_kernel<HD, HPB><<<grid, kPrefillThreads, 0, stream>>>(
+  kernel<<<grid, kPrefillThreads, 0, stream>>>(
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages,
       positions, req_of_token, item_token, item_count, (bf16_t*)out, num_items, nh, nkv, ps,
-      scale * 1.4426950408889634f, sinks);
+      scale * 1.4426950408889634f, sinks, soft_cap(scale, softcap));
   return launch_status();
 }
 
@@ -1325,29 +1344,31 @@ static int launch_prefill_group(const void* q, const void* k_cache, const void* 
                                 const int* block_tables, int max_pages, const int* positions,
                                 const int* req_of_token, const int* item_token, const int* item_count,
                                 int num_items, void* out, int nh, int nkv, int ps, float scale,
-                                hipStream_t stream, const float* sinks) {
+                                hipStream_t stream, const float* sinks, float softcap) {
   const int G = nh / nkv;
+  const bool capped = softcap > 0.f;
+  auto* const kernel = capped ? &attention_prefill_group_kernel<HD, GB, S, true> : &attention_prefill_group_kernel<HD, GB, S, false>;
   constexpr size_t one_stage = (size_t)S * 8 * HD * 16 * 2;                       // K and V of a stage
   constexpr size_t stage_bytes = 2 * one_stage <= 160 * 1024 ? 2 * one_stage : one_stage;  // two where they fit
   constexpr size_t merge_bytes = (size_t)(S - 1) * GB * ((HD / 2 + 2) * 64) * 4;  // the shares' results
   constexpr size_t lds = stage_bytes > merge_bytes ? stage_bytes : merge_bytes;
   static_assert(lds <= 160 * 1024, "a stage must fit the CU's LDS");
   if (lds > 48 * 1024) {
-    static bool raised = false;  // per template instance
-    if (!raised) {
-      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_prefill_group_kernel<HD, GB, S>),
-                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) {
+    static bool raised[2] = {false, false};  // per template instance
+    if (!raised[capped]) {
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) !=
+          hipSuccess) {
         (void)hipGetLastError();
         return -2;
       }
-      raised = true;
+      raised[capped] = true;
     }
   }
   dim3 grid(nkv * ((G + GB - 1) / GB), num_items);
-  attention_prefill_group_kernel<HD, GB, S><<<grid, GB * S * 64, lds, stream>>>(
+  kernel<<<grid, GB * S * 64, lds, stream>>>(
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages,
       positions, req_of_token, item_token, item_count, (bf16_t*)out, num_items, nh, nkv, ps,
-      scale * 1.4426950408889634f, sinks);
+      scale * 1.4426950408889634f, sinks, soft_cap(scale, softcap));
   return launch_status();
 }
 
@@ -1359,10 +1380,10 @@ static int launch_prefill_group_any(const void* q, const void* k_cache, const vo
                                     const int* block_tables, int max_pages, const int* positions,
                                     const int* req_of_token, const int* item_token, const int* item_count,
                                     int num_items, void* out, int nh, int nkv, int ps, float scale,
-                                    hipStream_t stream, const float* sinks) {
+                                    hipStream_t stream, const float* sinks, float softcap) {
 #define TK_GARGS                                                                                  \
   q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, item_token, item_count, \
-      num_items, out, nh, nkv, ps, scale, stream, sinks
+      num_items, out, nh, nkv, ps, scale, stream, sinks, softcap
   const int G = nh / nkv;
   const int nblk = (G + 7) / 8;
   const int gb = (G + nblk - 1) / nblk;  // heads a block: G itself up to 8, else an even share
@@ -1385,8 +1406,12 @@ static int launch(const void* q, const void* k_cache, const void* v_cache, const
                   int max_pages, const int* positions, const int* req_of_token,
                   const int* item_token, const int* item_count, int num_items, void* out,
                   float* part_o, float* part_ml, int nsplit, int split_keys, int nh, int nkv, int ps,
-                  float scale, hipStream_t stream, const float* sinks, DecodeInputs in = DecodeInputs{}) {
+                  float scale, hipStream_t stream, const float* sinks, float softcap, DecodeInputs in = DecodeInputs{}) {
   if (num_items > 65535) return -1;
+  // (the fused form has no capped instance: its entry point takes no cap)
+  const bool capped = !FUSED && softcap > 0.f;
+  auto* const kernel = capped ? &attention_decode_kernel<HD, kDecodeWaves, 1, FUSED, !FUSED>
+                              : &attention_decode_kernel<HD, kDecodeWaves, 1, FUSED, false>;
   dim3 grid(nkv, num_items, nsplit);
   const int G = nh / nkv;
   // sixteen waves a block and one tile a wave in flight measured best at every batch size
@@ -1394,20 +1419,20 @@ static int launch(const void* q, const void* k_cache, const void* v_cache, const
   const size_t lds = (size_t)(kDecodeWaves * G * HD + 2 * kDecodeWaves * 16) * 4 + (FUSED ? (size_t)(G + 2) * HD * 2 : 0);
   if (lds > 160 * 1024) return -2;
   if (lds > 48 * 1024) {  // beyond the default limit of dynamic LDS (groups of 7 heads and more)
-    static bool raised = false;  // per template instance
-    if (!raised) {
-      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_decode_kernel<HD, kDecodeWaves, 1, FUSED>),
-                              hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) {
+    static bool raised[2] = {false, false};  // per template instance
+    if (!raised[capped]) {
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) !=
+          hipSuccess) {
         (void)hipGetLastError();
         return -2;
       }
-      raised = true;
+      raised[capped] = true;
     }
   }
-  attention_decode_kernel<HD, kDecodeWaves, 1, FUSED><<<grid, kDecodeWaves * 64, lds, stream>>>(
+  kernel<<<grid, kDecodeWaves * 64, lds, stream>>>(
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages, positions,
       req_of_token, item_token, item_count, (bf16_t*)out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps,
-      scale * 1.4426950408889634f, in, sinks);
+      scale * 1.4426950408889634f, in, sinks, soft_cap(scale, softcap));
   if (nsplit > 1) {
     dim3 mgrid(num_items, nh);
     attention_merge_kernel<HD><<<mgrid, 64, 0, stream>>>(part_o, part_ml, positions, item_token, nullptr,
@@ -1428,6 +1453,7 @@ static int launch(const void* q, const void* k_cache, const void* v_cache, const
 // sinks: null, or float32 [nh]: head a's softmax has exp(sinks[a]) as one more term of its denominator
 // (no key, no value, not scaled); it is added where a row's sums are complete (the kernel's end, or
 // the merge of its splits).
+// softcap > 0: every score becomes softcap tanh(score / softcap) first (not the sink's), see soft_cap.h.
 // Returns -2 if this shape is not instantiated (the caller uses the generic kernel).
 TK_API int tk_attention_decode_waves() { return kDecodeWaves; }
 
@@ -1436,9 +1462,9 @@ TK_API int tk_attention_mfma(int mode, const void* q, const void* k_cache, const
                              const int* req_of_token, const int* item_token, const int* item_count,
                              int num_items, void* out, float* part_o, float* part_ml, int nsplit,
                              int split_keys, int nh, int nkv, int hd, int ps, float scale, int chunk,
-                             const float* sinks, hipStream_t stream) {
+                             const float* sinks, float softcap, hipStream_t stream) {
   if (num_items <= 0) return 0;
-  if (mode < 0 || mode > 4) return -1;
+  if (mode < 0 || mode > 4 || !(softcap >= 0.f)) return -1;
   // chunked visibility: the narrow form for tiles only, their keys not split over blocks
   if (chunk < 0 || (chunk > 0 && ((mode != 1 && mode != 2) || nsplit != 1))) return -1;
   if (nkv <= 0 || nh % nkv != 0 || ps < 16 || (ps & (ps - 1)) != 0 || split_keys % 16 != 0 || nsplit < 1) return -1;
@@ -1446,7 +1472,7 @@ TK_API int tk_attention_mfma(int mode, const void* q, const void* k_cache, const
   const int G = nh / nkv;
 #define TK_ARGS                                                                                   \
   q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, item_token, item_count, \
-      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, sinks
+      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, sinks, softcap
   if (mode == 0) {
     if (G > 16) return -2;
     if (hd == 128) return launch<128, false>(TK_ARGS);
@@ -1457,10 +1483,10 @@ TK_API int tk_attention_mfma(int mode, const void* q, const void* k_cache, const
     if (nsplit != 1) return -1;
     if (hd == 128) return launch_prefill_group_any<128>(q, k_cache, v_cache, block_tables, max_pages, positions,
                                                         req_of_token, item_token, item_count, num_items, out, nh,
-                                                        nkv, ps, scale, stream, sinks);
+                                                        nkv, ps, scale, stream, sinks, softcap);
     if (hd == 64) return launch_prefill_group_any<64>(q, k_cache, v_cache, block_tables, max_pages, positions,
                                                       req_of_token, item_token, item_count, num_items, out, nh,
-                                                      nkv, ps, scale, stream, sinks);
+                                                      nkv, ps, scale, stream, sinks, softcap);
     return -2;
   }
   const int hpb = (G % 4 == 0) ? 4 : (G % 2 == 0) ? 2 : 1;
@@ -1468,7 +1494,7 @@ TK_API int tk_attention_mfma(int mode, const void* q, const void* k_cache, const
     if (nsplit != 1) return -1;
 #define TK_WARGS                                                                                  \
   q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, item_token, item_count, \
-      num_items, out, nh, nkv, ps, scale, stream, sinks
+      num_items, out, nh, nkv, ps, scale, stream, sinks, softcap
     // (groups of three heads and more take the group form; blocks of two heads or one here)
     if (hd == 128) {
       if (G % 2 == 0) return launch_prefill_wide<128, 2>(TK_WARGS);
@@ -1485,7 +1511,7 @@ TK_API int tk_attention_mfma(int mode, const void* q, const void* k_cache, const
   if (nsplit > 1 && (split_keys % 64 != 0 || (long)num_items * 16 > 65535)) return -1;
 #define TK_PARGS                                                                                  \
   q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, item_token, item_count, \
-      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, chunk, sinks
+      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, chunk, sinks, softcap
   const bool dense = mode == 2;
   if (hd == 128) {
     if (hpb == 4) return dense ? launch_prefill<128, 4, 4>(TK_PARGS) : launch_prefill<128, 4, 2>(TK_PARGS);
@@ -1528,7 +1554,7 @@ TK_API int tk_attention_decode_fused(const void* qkv, int in_f32, int parts, lon
   DecodeInputs in{qkv, in_f32, parts, part_stride, q_weight, k_weight, cos_t, sin_t, rot, nkv_in, eps};
 #define TK_FARGS                                                                                       \
   nullptr, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, item_token, nullptr,  \
-      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, nullptr, in
+      num_items, out, part_o, part_ml, nsplit, split_keys, nh, nkv, ps, scale, stream, nullptr, 0.f, in
   if (hd == 128) return launch<128, true>(TK_FARGS);
   if (hd == 64) return launch<64, true>(TK_FARGS);
 #undef TK_FARGS

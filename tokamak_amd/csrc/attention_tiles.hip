@@ -18,12 +18,13 @@
 // positions, -C < 0 the positions of its own chunk of C; with a window, `keep` > 0 leaves the first
 // `keep` positions of the sequence visible too (their stages of 16 keys are walked first, then the walk
 // jumps to the window's first stage).  sinks: null, or float32 [nh]: exp(sinks[a])
-// is one more term of head a's denominator.
+// is one more term of head a's denominator.  CAP instances bound every score softly first (soft_cap.h).
 //
 // Cache pages: K [nkv][hd/8][ps][8], V [nkv][vd/16][ps/4][16][4]; ps a multiple of 16, so that 16
 // consecutive keys from a multiple of 16 lie in one page.
 #include "common.h"
 #include "slots.h"
+#include "soft_cap.h"
 
 using namespace tk;
 
@@ -48,13 +49,13 @@ constexpr int kHeadsPerBlock = 4;
 
 // KCH: 32-wide chunks of the key size the instance holds (hd <= 32 KCH); DBL: 16-wide blocks of the
 // value size (vd <= 16 DBL).  Chunks and blocks behind the true sizes are skipped (the same for every lane).
-template <int KCH, int DBL>
+template <int KCH, int DBL, bool CAP>
 __global__ __launch_bounds__(kHeadsPerBlock * 64) void attention_tiles_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ positions,
     const int* __restrict__ req_of_token, const int* __restrict__ tile_first, const int* __restrict__ tile_count,
     bf16_t* __restrict__ out, int nh, int nkv, int hd, int vd, int ps, float scale_log2, int span, int keep,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, SoftCap cap) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, kb = lane >> 4;
   const int head = blockIdx.y * kHeadsPerBlock + wave;
   if (head >= nh) return;   // (the waves of a block never wait for one another)
@@ -110,7 +111,7 @@ __global__ __launch_bounds__(kHeadsPerBlock * 64) void attention_tiles_kernel(
     for (int e = 0; e < 4; ++e) {
       const int key = c0 + kb * 4 + e;
       seen[e] = (key >= first || key < keep) && key <= pos;
-      sv[e] = seen[e] ? sc[e] * scale_log2 : -INFINITY;     // (a key that no token wrote may hold anything: chosen, not computed)
+      sv[e] = seen[e] ? (CAP ? cap.log2_score(sc[e]) : sc[e] * scale_log2) : -INFINITY;     // (a key that no token wrote may hold anything: chosen, not computed)
     }
     float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
@@ -172,13 +173,13 @@ __global__ __launch_bounds__(kHeadsPerBlock * 64) void attention_tiles_kernel(
 // stages: the next one is fetched into registers before this one's products and written after them,
 // one barrier a stage.  Operands are read from LDS per instruction, which leaves a wave under 256
 // registers: two waves a SIMD.
-template <int KCH, int DBL, int HB>
+template <int KCH, int DBL, int HB, bool CAP>
 __global__ __launch_bounds__(HB * 64) void attention_tiles_shared_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ positions,
     const int* __restrict__ req_of_token, const int* __restrict__ tile_first, const int* __restrict__ tile_count,
     bf16_t* __restrict__ out, int nh, int nkv, int hd, int vd, int ps, float scale_log2, int span, int keep,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, SoftCap cap) {
   extern __shared__ __attribute__((aligned(16))) bf16_t stage_s[];   // two stages of (hd + vd) * 16 elements
   constexpr int THREADS = HB * 64;
   constexpr int KPT = (KCH * 64 + THREADS - 1) / THREADS;    // 16-byte pieces of K (hd / 8 * 16 = 2 hd) a thread copies
@@ -282,7 +283,7 @@ __global__ __launch_bounds__(HB * 64) void attention_tiles_shared_kernel(
       for (int e = 0; e < 4; ++e) {
         const int key = c0 + kb * 4 + e;
         seen[e] = (key >= first || key < keep) && key <= pos;
-        sv[e] = seen[e] ? sc[e] * scale_log2 : -INFINITY;
+        sv[e] = seen[e] ? (CAP ? cap.log2_score(sc[e]) : sc[e] * scale_log2) : -INFINITY;
       }
       float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
@@ -342,17 +343,17 @@ __global__ __launch_bounds__(HB * 64) void attention_tiles_shared_kernel(
   }
 }
 
-template <int KCH, int DBL, int HB>
+template <int KCH, int DBL, int HB, bool CAP>
 static int launch_shared(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_pages,
                          const int* positions, const int* req_of_token, const int* tile_first, const int* tile_count,
                          int num_tiles, void* out, int nh, int nkv, int hd, int vd, int ps, float scale, int span, int keep,
-                         const float* sinks, hipStream_t stream) {
+                         const float* sinks, float softcap, hipStream_t stream) {
   const int group = nh / nkv;
   const size_t lds = (size_t)2 * (hd + vd) * 16 * sizeof(bf16_t);
   if (lds > 48 * 1024) {
     static bool raised = false;   // per template instance
     if (!raised) {
-      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_tiles_shared_kernel<KCH, DBL, HB>),
+      if (hipFuncSetAttribute(reinterpret_cast<const void*>(&attention_tiles_shared_kernel<KCH, DBL, HB, CAP>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024) != hipSuccess) {
         (void)hipGetLastError();
         return -2;
@@ -362,9 +363,10 @@ static int launch_shared(const void* q, const void* k_cache, const void* v_cache
   }
   const dim3 grid(num_tiles, nkv * ((group + HB - 1) / HB));
   if (grid.y > 65535) return -1;
-  attention_tiles_shared_kernel<KCH, DBL, HB><<<grid, HB * 64, lds, stream>>>(
+  attention_tiles_shared_kernel<KCH, DBL, HB, CAP><<<grid, HB * 64, lds, stream>>>(
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages, positions, req_of_token,
-      tile_first, tile_count, (bf16_t*)out, nh, nkv, hd, vd, ps, scale * 1.4426950408889634f, span, keep, sinks);
+      tile_first, tile_count, (bf16_t*)out, nh, nkv, hd, vd, ps, scale * 1.4426950408889634f, span, keep, sinks,
+      soft_cap(scale, softcap));
   return launch_status();
 }
 
@@ -374,13 +376,13 @@ static int launch_shared(const void* q, const void* k_cache, const void* v_cache
 // of four waves, operands straight from the pages.  Every wave leaves an unnormalised partial result
 // (its maximum, its sum, its output) and a second kernel merges a head's partials in their order and
 // adds the sink: no wave waits for another.
-template <int KCH, int DBL>
+template <int KCH, int DBL, bool CAP>
 __global__ __launch_bounds__(256) void attention_heads_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ positions,
     const int* __restrict__ req_of_token, const int* __restrict__ single, float* __restrict__ part_o,
     float* __restrict__ part_ml, int nsplit, int nh, int nkv, int hd, int vd, int ps, float scale_log2, int span,
-    int keep) {
+    int keep, SoftCap cap) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, kb = lane >> 4;
   const int group = nh / nkv, pieces = (group + 15) >> 4;
   const int kvh = blockIdx.y / pieces, in_group = (blockIdx.y % pieces) * 16 + col;
@@ -440,7 +442,7 @@ __global__ __launch_bounds__(256) void attention_heads_kernel(
     for (int e = 0; e < 4; ++e) {
       const int key = c0 + kb * 4 + e;
       seen[e] = (key >= first || key < keep) && key <= pos;
-      sv[e] = seen[e] ? sc[e] * scale_log2 : -INFINITY;
+      sv[e] = seen[e] ? (CAP ? cap.log2_score(sc[e]) : sc[e] * scale_log2) : -INFINITY;
     }
     float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
@@ -539,9 +541,9 @@ __global__ __launch_bounds__(256) void attention_heads_merge_kernel(
 TK_API int tk_attention_tiles(const void* q, const void* k_cache, const void* v_cache, const int* block_tables,
                               int max_pages, const int* positions, const int* req_of_token, const int* tile_first,
                               const int* tile_count, int num_tiles, void* out, int nh, int nkv, int hd, int vd, int ps,
-                              float scale, int span, int keep, const float* sinks, hipStream_t stream) {
+                              float scale, int span, int keep, const float* sinks, float softcap, hipStream_t stream) {
   if (num_tiles <= 0) return 0;
-  if (keep < 0 || (keep > 0 && span <= 0)) return -1;
+  if (keep < 0 || (keep > 0 && span <= 0) || !(softcap >= 0.f)) return -1;
   if (nkv <= 0 || nh % nkv != 0 || hd < 8 || hd % 8 != 0 || vd < 16 || vd % 16 != 0 || ps < 16 || ps % 16 != 0) return -2;
   if (hd > 512 || vd > 512 || (uintptr_t)q % 16 != 0 || (uintptr_t)k_cache % 16 != 0 || (uintptr_t)v_cache % 16 != 0 ||
       (uintptr_t)out % 8 != 0)
@@ -549,25 +551,35 @@ TK_API int tk_attention_tiles(const void* q, const void* k_cache, const void* v_
   const int group = nh / nkv;
   if (group >= 4) {
     // the heads of a kv head share its keys and values through LDS
-#define TK_SHARED(KCH_, DBL_, HB_)                                                                              \
-  launch_shared<KCH_, DBL_, HB_>(q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token, tile_first, \
-                                 tile_count, num_tiles, out, nh, nkv, hd, vd, ps, scale, span, keep, sinks, stream)
+#define TK_SHARED_AS(KCH_, DBL_, HB_, CAP_)                                                                     \
+  launch_shared<KCH_, DBL_, HB_, CAP_>(q, k_cache, v_cache, block_tables, max_pages, positions, req_of_token,   \
+                                       tile_first, tile_count, num_tiles, out, nh, nkv, hd, vd, ps, scale, span, \
+                                       keep, sinks, softcap, stream)
+#define TK_SHARED(KCH_, DBL_, HB_) \
+  (softcap > 0.f ? TK_SHARED_AS(KCH_, DBL_, HB_, true) : TK_SHARED_AS(KCH_, DBL_, HB_, false))
     if (hd <= 128 && vd <= 128) return group > 4 ? TK_SHARED(4, 8, 8) : TK_SHARED(4, 8, 4);
     if (hd <= 256 && vd <= 256) return group > 4 ? TK_SHARED(8, 16, 8) : TK_SHARED(8, 16, 4);
     return group > 4 ? TK_SHARED(16, 32, 8) : TK_SHARED(16, 32, 4);
 #undef TK_SHARED
+#undef TK_SHARED_AS
   }
   const dim3 grid(num_tiles, (nh + kHeadsPerBlock - 1) / kHeadsPerBlock);
   if (grid.y > 65535) return -1;
-#define TK_TILES(KCH_, DBL_)                                                                                   \
-  attention_tiles_kernel<KCH_, DBL_><<<grid, kHeadsPerBlock * 64, 0, stream>>>(                                \
+#define TK_TILES_AS(KCH_, DBL_, CAP_)                                                                          \
+  attention_tiles_kernel<KCH_, DBL_, CAP_><<<grid, kHeadsPerBlock * 64, 0, stream>>>(                          \
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages, positions,    \
       req_of_token, tile_first, tile_count, (bf16_t*)out, nh, nkv, hd, vd, ps, scale * 1.4426950408889634f,    \
-      span, keep, sinks)
+      span, keep, sinks, soft_cap(scale, softcap))
+#define TK_TILES(KCH_, DBL_)                          \
+  do {                                                \
+    if (softcap > 0.f) TK_TILES_AS(KCH_, DBL_, true); \
+    else TK_TILES_AS(KCH_, DBL_, false);              \
+  } while (0)
   if (hd <= 128 && vd <= 128) TK_TILES(4, 8);
   else if (hd <= 256 && vd <= 256) TK_TILES(8, 16);
   else TK_TILES(16, 32);
 #undef TK_TILES
+#undef TK_TILES_AS
   return launch_status();
 }
 
@@ -577,9 +589,9 @@ TK_API int tk_attention_heads(const void* q, const void* k_cache, const void* v_
                               int max_pages, const int* positions, const int* req_of_token, const int* single,
                               int num_single, void* out, float* part_o, float* part_ml, int nsplit, int nh, int nkv,
                               int hd, int vd, int ps, float scale, int span, int keep, const float* sinks,
-                              hipStream_t stream) {
+                              float softcap, hipStream_t stream) {
   if (num_single <= 0) return 0;
-  if (keep < 0 || (keep > 0 && span <= 0)) return -1;
+  if (keep < 0 || (keep > 0 && span <= 0) || !(softcap >= 0.f)) return -1;
   if (nkv <= 0 || nh % nkv != 0 || hd < 8 || hd % 8 != 0 || vd < 16 || vd % 16 != 0 || ps < 16 || ps % 16 != 0) return -2;
   if (hd > 512 || vd > 512 || (uintptr_t)q % 16 != 0 || (uintptr_t)k_cache % 16 != 0 || (uintptr_t)v_cache % 16 != 0 ||
       (uintptr_t)part_o % 16 != 0 || nsplit < 1 || nsplit > 16 || nh > 65535)    // (the merge: up to 64 parts)
@@ -587,14 +599,21 @@ TK_API int tk_attention_heads(const void* q, const void* k_cache, const void* v_
   const int group = nh / nkv;
   const dim3 grid(num_single, nkv * ((group + 15) / 16), nsplit);
   if (grid.y > 65535) return -1;
-#define TK_HEADS(KCH_, DBL_)                                                                                  \
-  attention_heads_kernel<KCH_, DBL_><<<grid, 256, 0, stream>>>(                                               \
+#define TK_HEADS_AS(KCH_, DBL_, CAP_)                                                                         \
+  attention_heads_kernel<KCH_, DBL_, CAP_><<<grid, 256, 0, stream>>>(                                         \
       (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, max_pages, positions,   \
-      req_of_token, single, part_o, part_ml, nsplit, nh, nkv, hd, vd, ps, scale * 1.4426950408889634f, span, keep)
+      req_of_token, single, part_o, part_ml, nsplit, nh, nkv, hd, vd, ps, scale * 1.4426950408889634f, span, keep, \
+      soft_cap(scale, softcap))
+#define TK_HEADS(KCH_, DBL_)                          \
+  do {                                                \
+    if (softcap > 0.f) TK_HEADS_AS(KCH_, DBL_, true); \
+    else TK_HEADS_AS(KCH_, DBL_, false);              \
+  } while (0)
   if (hd <= 128 && vd <= 128) TK_HEADS(4, 8);
   else if (hd <= 256 && vd <= 256) TK_HEADS(8, 16);
   else TK_HEADS(16, 32);
 #undef TK_HEADS
+#undef TK_HEADS_AS
   attention_heads_merge_kernel<<<dim3(num_single, nh), vd <= 64 ? 64 : vd <= 128 ? 128 : 256, 0, stream>>>(  // (whole waves)
       part_o, part_ml, single, (bf16_t*)out, nsplit * 4, nh, vd, sinks);
   return launch_status();

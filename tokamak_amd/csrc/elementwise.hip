@@ -687,6 +687,117 @@ __global__ void silu_mul_bf16x8_kernel(const bf16_t* __restrict__ gu, bf16_t* __
   *reinterpret_cast<uint4*>(out + n * I + i) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
 }
 
+// out[n, i] = max(x[n, i], 0)^2: x is T, float32, or float32 partial sums of a split product
+template <typename T>
+__device__ __forceinline__ float branch_value(const void* p, int f32, int parts, long part_stride, size_t idx);
+
+template <typename T>
+__global__ void squared_relu_kernel(const void* __restrict__ x, int f32, int parts, long part_stride, T* __restrict__ out,
+                                    size_t total) {
+  const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total) return;
+  const float v = fmaxf(branch_value<T>(x, f32, parts, part_stride, idx), 0.f);
+  Elem<T>::store(out + idx, v * v);
+}
+
+// 8 elements a thread
+__global__ void squared_relu_bf16x8_kernel(const bf16_t* __restrict__ x, bf16_t* __restrict__ out, size_t total8) {
+  const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total8) return;
+  const uint4 v = reinterpret_cast<const uint4*>(x)[idx];
+  const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+  uint32_t o[4];
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float a = fmaxf(__uint_as_float(w[k] << 16), 0.f), b = fmaxf(__uint_as_float(w[k] & 0xffff0000u), 0.f);
+    o[k] = pack_bf16x2(a * a, b * b);
+  }
+  reinterpret_cast<uint4*>(out)[idx] = make_uint4(o[0], o[1], o[2], o[3]);
+}
+
+TK_API int tk_squared_relu(int dtype, const void* x, int f32, int parts, long part_stride, void* out, long total,
+                           hipStream_t stream) {
+  if (total <= 0) return 0;
+  if (parts < 1 || (parts > 1 && !f32 && dtype != 0)) return -1;
+  if (dtype == 1 && !f32 && parts == 1 && total % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0) {
+    squared_relu_bf16x8_kernel<<<(unsigned)((total / 8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, (size_t)total / 8);
+    return launch_status();
+  }
+  const unsigned blocks = (unsigned)((total + 255) / 256);
+  if (dtype == 0) squared_relu_kernel<float><<<blocks, 256, 0, stream>>>(x, 1, parts, part_stride, (float*)out, (size_t)total);
+  else squared_relu_kernel<bf16_t><<<blocks, 256, 0, stream>>>(x, f32, parts, part_stride, (bf16_t*)out, (size_t)total);
+  return launch_status();
+}
+
+// ---------------------------------------------------------------------------
+// The difference of two attention maps, per token and head: with o = a_1 - lambda a_2 over the head's vd values,
+// out = o / sqrt(mean(o^2) + eps) * scale.  a: rows of 2 `heads` heads of vdp >= vd columns (map 1 and map 2 of
+// head 0, then of head 1, ...); out rows: `heads` heads of vd columns, dense.  lambda is one float32 number on the
+// device.  LANES neighbouring lanes take a head, four values each at a time.
+// ---------------------------------------------------------------------------
+template <typename T, int LANES>
+__global__ __launch_bounds__(256) void map_difference_kernel(const T* __restrict__ a, const float* __restrict__ lambda,
+                                                             T* __restrict__ out, int vd, int vdp, float eps, float scale,
+                                                             long items) {
+  constexpr int STEPS = 2;           // (16 lanes: heads of up to 128 values, 64 lanes: 512)
+  const long item = (long)blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
+  const int sub = threadIdx.x % LANES;
+  if (item >= items) return;         // (whole groups of lanes leave together)
+  const float lam = *lambda;
+  const T* p = a + (size_t)item * 2 * vdp;
+  float o[STEPS][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const int d = (s * LANES + sub) * 4;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[s][e] = 0.f;
+    if (d < vd) {
+      const float4 x = Load4<T>::at(p + d), y = Load4<T>::at(p + vdp + d);
+      const float xv[4] = {x.x, x.y, x.z, x.w}, yv[4] = {y.x, y.y, y.z, y.w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (d + e < vd) o[s][e] = xv[e] - lam * yv[e];
+        ss = fmaf(o[s][e], o[s][e], ss);
+      }
+    }
+  }
+#pragma unroll
+  for (int m = LANES / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, kWave);
+  const float factor = scale / sqrtf(ss / (float)vd + eps);
+  T* q = out + (size_t)item * vd;
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const int d = (s * LANES + sub) * 4;
+    if (d >= vd) continue;
+    if (vd % 4 == 0) {
+      Store4<T>::at(q + d, make_float4(o[s][0] * factor, o[s][1] * factor, o[s][2] * factor, o[s][3] * factor));
+    } else {
+      for (int e = 0; e < 4 && d + e < vd; ++e) Elem<T>::store(q + d + e, o[s][e] * factor);
+    }
+  }
+}
+
+TK_API int tk_map_difference(int dtype, const void* a, const float* lambda, void* out, int N, int heads, int vd, int vdp,
+                             float eps, float scale, hipStream_t stream) {
+  if (N <= 0) return 0;
+  if (heads < 1 || vd < 1 || vdp < vd || vdp % 16 != 0 || vdp > 512 || lambda == nullptr) return -1;
+  if ((uintptr_t)a % 16 != 0 || (uintptr_t)out % 16 != 0) return -1;
+  const long items = (long)N * heads;
+#define TK_MD(T_, LANES_)                                                                                       \
+  map_difference_kernel<T_, LANES_><<<(unsigned)((items + 256 / LANES_ - 1) / (256 / LANES_)), 256, 0, stream>>>( \
+      (const T_*)a, lambda, (T_*)out, vd, vdp, eps, scale, items)
+  if (vd <= 128) {
+    if (dtype == 0) TK_MD(float, 16);
+    else TK_MD(bf16_t, 16);
+  } else {
+    if (dtype == 0) TK_MD(float, 64);
+    else TK_MD(bf16_t, 64);
+  }
+#undef TK_MD
+  return launch_status();
+}
+
 TK_API int tk_add_bias(int dtype, void* x, const float* bias, int N, int H, hipStream_t stream) {
   if (N <= 0 || H <= 0) return 0;
   const size_t total = (size_t)N * H;
@@ -805,8 +916,9 @@ TK_API int tk_scaled_sum(int dtype, const void* a, int a_f32, int a_parts, long 
 //   x = resid[row] + scale * (a[row] + b[row] + c[row] + bias);  if write_resid: resid[row] = x
 //   center: out[m] = (x - mean(x)) * rsqrt(mean((x - mean(x))^2) + eps) * weight   (a layer norm without a bias)
 //   else:   out[m] = x * rsqrt(mean(x^2) + eps) * weight
-// A branch is T, float32, or float32 partial sums (added in order); each may be absent, and so may
-// the bias (float32 [H], one row for all).  The branches' sum is formed first, in float32, and
+// A branch is T, float32, or float32 partial sums (added in order); each may be absent; b and c may have a
+// float32 weight per row (a token's gate on a whole branch).  Absent may be the
+// bias too (float32 [H], one row for all).  The branches' sum is formed first, in float32, and
 // added to the stream once.  weight2 / out2 (both or neither): the same normalised row times a
 // second weight, for a layer whose two sub-layers each have a norm of their own over the same stream.
 // ---------------------------------------------------------------------------
@@ -815,6 +927,7 @@ struct NormBranch {
   int f32;
   int parts;
   long stride;
+  const float* row_weight;   // null, or [rows]: the branch's row times this number (add_norm2 only)
 };
 
 struct NormAdds {
@@ -848,16 +961,18 @@ __device__ __forceinline__ float4 branch_four(const NormBranch& b, size_t idx) {
 
 // scale * (a + b + c + bias) at four consecutive columns from d of a row that starts at `at`
 template <typename T>
-__device__ __forceinline__ float4 adds_four(const NormAdds& n, size_t at, int d) {
+__device__ __forceinline__ float4 adds_four(const NormAdds& n, size_t row, size_t at, int d) {
   float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
   if (n.a.p) s = branch_four<T>(n.a, at + d);
   if (n.b.p) {
     const float4 t = branch_four<T>(n.b, at + d);
-    s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w;
+    const float w = n.b.row_weight ? n.b.row_weight[row] : 1.f;
+    s.x = fmaf(w, t.x, s.x); s.y = fmaf(w, t.y, s.y); s.z = fmaf(w, t.z, s.z); s.w = fmaf(w, t.w, s.w);
   }
   if (n.c.p) {
     const float4 t = branch_four<T>(n.c, at + d);
-    s.x += t.x; s.y += t.y; s.z += t.z; s.w += t.w;
+    const float w = n.c.row_weight ? n.c.row_weight[row] : 1.f;
+    s.x = fmaf(w, t.x, s.x); s.y = fmaf(w, t.y, s.y); s.z = fmaf(w, t.z, s.z); s.w = fmaf(w, t.w, s.w);
   }
   if (n.bias) {
     const float4 t = *reinterpret_cast<const float4*>(n.bias + d);
@@ -868,11 +983,11 @@ __device__ __forceinline__ float4 adds_four(const NormAdds& n, size_t at, int d)
 }
 
 template <typename T>
-__device__ __forceinline__ float adds_value(const NormAdds& n, size_t at, int d) {
+__device__ __forceinline__ float adds_value(const NormAdds& n, size_t row, size_t at, int d) {
   float s = 0.f;
   if (n.a.p) s = branch_value<T>(n.a.p, n.a.f32, n.a.parts, n.a.stride, at + d);
-  if (n.b.p) s += branch_value<T>(n.b.p, n.b.f32, n.b.parts, n.b.stride, at + d);
-  if (n.c.p) s += branch_value<T>(n.c.p, n.c.f32, n.c.parts, n.c.stride, at + d);
+  if (n.b.p) s = fmaf(n.b.row_weight ? n.b.row_weight[row] : 1.f, branch_value<T>(n.b.p, n.b.f32, n.b.parts, n.b.stride, at + d), s);
+  if (n.c.p) s = fmaf(n.c.row_weight ? n.c.row_weight[row] : 1.f, branch_value<T>(n.c.p, n.c.f32, n.c.parts, n.c.stride, at + d), s);
   if (n.bias) s += n.bias[d];
   return n.scale != 1.f ? s * n.scale : s;
 }
@@ -902,7 +1017,7 @@ __global__ __launch_bounds__(1024) void add_norm2_vec_kernel(
     if (d < H) {
       float4 v = *reinterpret_cast<const float4*>(x + d);
       if (adding) {
-        const float4 s = adds_four<T>(adds, row * H, d);
+        const float4 s = adds_four<T>(adds, row, row * H, d);
         v.x += s.x; v.y += s.y; v.z += s.z; v.w += s.w;
         if (write_resid) *reinterpret_cast<float4*>(x + d) = v;
       }
@@ -955,7 +1070,7 @@ __global__ void add_norm2_kernel(float* __restrict__ resid, NormAdds adds,
   for (int d = threadIdx.x; d < H; d += blockDim.x) {
     float v = x[d];
     if (adding) {
-      v += adds_value<T>(adds, row * H, d);
+      v += adds_value<T>(adds, row, row * H, d);
       if (write_resid) x[d] = v;      // (the passes below then read the sum back)
     }
     sum += v;
@@ -966,7 +1081,7 @@ __global__ void add_norm2_kernel(float* __restrict__ resid, NormAdds adds,
   float ss = 0.f;
   for (int d = threadIdx.x; d < H; d += blockDim.x) {
     float v = x[d];
-    if (again) v += adds_value<T>(adds, row * H, d);
+    if (again) v += adds_value<T>(adds, row, row * H, d);
     ss += (v - mean) * (v - mean);
   }
   ss = block_sum(ss, scratch);
@@ -974,7 +1089,7 @@ __global__ void add_norm2_kernel(float* __restrict__ resid, NormAdds adds,
   T* o = out + (size_t)m * H;
   for (int d = threadIdx.x; d < H; d += blockDim.x) {
     float v = x[d];
-    if (again) v += adds_value<T>(adds, row * H, d);
+    if (again) v += adds_value<T>(adds, row, row * H, d);
     Elem<T>::store(o + d, (v - mean) * rstd * weight[d]);
     if (out2) Elem<T>::store(out2 + (size_t)m * H + d, (v - mean) * rstd * weight2[d]);
   }
@@ -982,15 +1097,15 @@ __global__ void add_norm2_kernel(float* __restrict__ resid, NormAdds adds,
 
 TK_API int tk_add_norm2(int dtype, float* resid, const void* a, int a_f32, int a_parts, long a_stride,
                         const void* b, int b_f32, int b_parts, long b_stride, const void* c, int c_f32, int c_parts,
-                        long c_stride, const float* bias, float scale, const int* rows,
-                        const float* weight, void* out, const float* weight2, void* out2, int M, int H, float eps,
+                        long c_stride, const float* b_rows, const float* c_rows, const float* bias, float scale,
+                        const int* rows, const float* weight, void* out, const float* weight2, void* out2, int M, int H, float eps,
                         int write_resid, int center, hipStream_t stream) {
   if (M <= 0) return 0;
   if (rows && write_resid) return -1;
   if ((weight2 == nullptr) != (out2 == nullptr)) return -1;
   if (a_parts < 1 || b_parts < 1 || c_parts < 1 || (a_parts > 1 && !a_f32) || (b_parts > 1 && !b_f32) || (c_parts > 1 && !c_f32)) return -1;
-  const NormAdds adds{{a, a_f32 || dtype == 0, a_parts, a_stride}, {b, b_f32 || dtype == 0, b_parts, b_stride},
-                      {c, c_f32 || dtype == 0, c_parts, c_stride}, bias, scale};
+  const NormAdds adds{{a, a_f32 || dtype == 0, a_parts, a_stride, nullptr}, {b, b_f32 || dtype == 0, b_parts, b_stride, b_rows},
+                      {c, c_f32 || dtype == 0, c_parts, c_stride, c_rows}, bias, scale};
   int threads = 64;
   while (threads < 1024 && threads * 4 * (M >= 512 ? kNormGroups : 1) < H) threads *= 2;
   const bool vec = H % 4 == 0 && H <= threads * 4 * kNormGroups && a_stride % 4 == 0 && b_stride % 4 == 0 && c_stride % 4 == 0 &&
@@ -1210,56 +1325,67 @@ TK_API int tk_add_normed(int dtype, float* resid, const void* a, int a_f32, int 
 }
 
 // ---------------------------------------------------------------------------
-// x[n, head, d] *= sigmoid(gate[n, head * vd + d]) in place: the gate behind attention.  x rows hold `heads`
+// x[n, head, d] *= sigmoid(gate[n, head * vd + d]) in place: the gate behind attention (per_head: the gate holds
+// one number a head instead, gate[n, head]).  x rows hold `heads`
 // heads of vdp >= vd columns (those behind vd stay as they are); gate rows are ld long and start at column col0,
 // in T, float32, or float32 partial sums.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void sigmoid_gate_kernel(T* __restrict__ x, const void* __restrict__ gate, int f32, int parts, long part_stride,
-                                    long ld, int col0, int width, int vd, int vdp, size_t total) {
+                                    long ld, int col0, int width, int vd, int vdp, int per_head, size_t total) {
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const size_t n = idx / width;
   const int c = (int)(idx - n * width);
   const int head = c / vd, d = c - head * vd;
-  const float g = branch_value<T>(gate, f32, parts, part_stride, n * ld + col0 + c);
+  const float g = branch_value<T>(gate, f32, parts, part_stride, n * ld + col0 + (per_head ? head : c));
   T* at = x + n * ((size_t)(width / vd) * vdp) + (size_t)head * vdp + d;
   Elem<T>::store(at, Elem<T>::load(at) / (1.f + expf(-g)));
 }
 
-// four neighbouring columns a thread: vd, vdp, ld, col0 and part_stride multiples of four
+// four neighbouring columns a thread: vd and vdp multiples of four, and with a gate per column ld, col0 and
+// part_stride too
 template <typename T>
-__global__ void sigmoid_gate_four_kernel(T* __restrict__ x, NormBranch gate, long ld, int col0, int width, int vd, int vdp, size_t total4) {
+__global__ void sigmoid_gate_four_kernel(T* __restrict__ x, NormBranch gate, long ld, int col0, int width, int vd, int vdp,
+                                         int per_head, size_t total4) {
   const size_t i4 = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i4 >= total4) return;
   const int quads = width / 4;
   const size_t n = i4 / quads;
   const int c = (int)(i4 - n * quads) * 4;
   const int head = c / vd, d = c - head * vd;
-  const float4 g = branch_four<T>(gate, n * ld + col0 + c);
+  float4 g;
+  if (per_head) {
+    g.x = branch_value<T>(gate.p, gate.f32, gate.parts, gate.stride, n * ld + col0 + head);
+    g.y = g.z = g.w = g.x;
+  } else {
+    g = branch_four<T>(gate, n * ld + col0 + c);
+  }
   T* at = x + n * ((size_t)(width / vd) * vdp) + (size_t)head * vdp + d;
   const float4 v = Load4<T>::at(at);
   Store4<T>::at(at, make_float4(v.x / (1.f + expf(-g.x)), v.y / (1.f + expf(-g.y)), v.z / (1.f + expf(-g.z)), v.w / (1.f + expf(-g.w))));
 }
 
 TK_API int tk_sigmoid_gate(int dtype, void* x, const void* gate, int f32, int parts, long part_stride, long ld, int col0,
-                           int N, int heads, int vd, int vdp, hipStream_t stream) {
+                           int N, int heads, int vd, int vdp, int per_head, hipStream_t stream) {
   if (N <= 0) return 0;
-  if (heads < 1 || vd < 1 || vdp < vd || parts < 1 || (parts > 1 && !f32 && dtype != 0) || col0 < 0 || ld < (long)col0 + (long)heads * vd)
+  if (heads < 1 || vd < 1 || vdp < vd || parts < 1 || (parts > 1 && !f32 && dtype != 0) || col0 < 0 ||
+      ld < (long)col0 + (long)heads * (per_head ? 1 : vd))
     return -1;
   const size_t total = (size_t)N * heads * vd;
-  if (vd % 4 == 0 && vdp % 4 == 0 && ld % 4 == 0 && col0 % 4 == 0 && part_stride % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)gate % 16 == 0) {
+  const bool gate_wide = ld % 4 == 0 && col0 % 4 == 0 && part_stride % 4 == 0 && (uintptr_t)gate % 16 == 0;
+  if (vd % 4 == 0 && vdp % 4 == 0 && (per_head || gate_wide) && (uintptr_t)x % 16 == 0) {
     const unsigned quads = (unsigned)((total / 4 + 255) / 256);
-    const NormBranch g{gate, f32 || dtype == 0, parts, part_stride};
-    if (dtype == 0) sigmoid_gate_four_kernel<float><<<quads, 256, 0, stream>>>((float*)x, g, ld, col0, heads * vd, vd, vdp, total / 4);
-    else sigmoid_gate_four_kernel<bf16_t><<<quads, 256, 0, stream>>>((bf16_t*)x, g, ld, col0, heads * vd, vd, vdp, total / 4);
+    const NormBranch g{gate, f32 || dtype == 0, parts, part_stride, nullptr};
+    if (dtype == 0) sigmoid_gate_four_kernel<float><<<quads, 256, 0, stream>>>((float*)x, g, ld, col0, heads * vd, vd, vdp, per_head, total / 4);
+    else sigmoid_gate_four_kernel<bf16_t><<<quads, 256, 0, stream>>>((bf16_t*)x, g, ld, col0, heads * vd, vd, vdp, per_head, total / 4);
     return launch_status();
   }
   const unsigned blocks = (unsigned)((total + 255) / 256);
   if (dtype == 0)
-    sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, gate, 1, parts, part_stride, ld, col0, heads * vd, vd, vdp, total);
+    sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)x, gate, 1, parts, part_stride, ld, col0, heads * vd, vd, vdp, per_head, total);
   else
-    sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)x, gate, f32, parts, part_stride, ld, col0, heads * vd, vd, vdp, total);
+    sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)x, gate, f32, parts, part_stride, ld, col0, heads * vd, vd, vdp, per_head, total);
   return launch_status();
 }
 
@@ -1279,6 +1405,11 @@ TK_API int tk_sigmoid_gate(int dtype, void* x, const void* gate, int f32, int pa
 // Values may be mixed with those another layer made for the same tokens (v_keep, float32
 // [N, nkv * vd]): v_mode 1 leaves this layer's values there as they are projected; v_mode 2
 // caches (1 - lambda) v + lambda v_keep with lambda = *v_lambda.
+// maps > 1: every head of q and k comes as `maps` heads of hd beside one another, each rotated and normed by
+// itself (nh and the key heads of the input count them all, nkv key heads of the pages hold maps * hd channels,
+// map m at channel m hd).  q_out row `head` then has its hd numbers at channel (head % maps) hd and zeros
+// elsewhere: its score with a page's whole key is the score of its own map.
+// v_from_k: there are no values in the input; a kv head's values are its key as projected (with its bias).
 // One wave per (token, head), four waves a block, each with an LDS row of its own.
 // ---------------------------------------------------------------------------
 template <typename T, typename TIN>
@@ -1289,18 +1420,22 @@ __global__ void rope_norm_store_kernel(
     const int* __restrict__ block_tables, T* __restrict__ q_out, T* __restrict__ k_cache,
     T* __restrict__ v_cache, int nh, int nkv_in, int nkv, int hd, int vd, int hdp, int vdp, int rot, int ps,
     int max_pages, int unit, float eps, int num_pairs, int interleaved, float* __restrict__ v_keep, int v_mode,
-    const float* __restrict__ v_lambda, long in_ld, const float* __restrict__ bias, int norm_first) {
+    const float* __restrict__ v_lambda, long in_ld, const float* __restrict__ bias, int norm_first, int maps,
+    int v_from_k) {
   __shared__ float vecs[kPairsPerBlock][kMaxHeadDim];
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
-  const int heads = nh + 2 * nkv_in;
+  const int nk_in = nkv_in * maps;
+  const int heads = nh + nk_in + nkv_in;
   const int pair = blockIdx.x * kPairsPerBlock + wave;
   if (pair >= num_pairs) return;  // nothing below synchronises across waves
   const int n = pair / heads, head = pair - n * heads;
   float* vec = vecs[wave];
   const bool is_q = head < nh;
-  const bool is_k = !is_q && head < nh + nkv_in;
+  const bool is_k = !is_q && head < nh + nk_in;
   const int width = (is_q || is_k) ? hd : vd;
-  const size_t head_at = (is_q || is_k) ? (size_t)head * hd : (size_t)(nh + nkv_in) * hd + (size_t)(head - nh - nkv_in) * vd;
+  const size_t head_at = (is_q || is_k) ? (size_t)head * hd
+                         : v_from_k     ? (size_t)(head - nk_in) * hd
+                                        : (size_t)(nh + nk_in) * hd + (size_t)(head - nh - nk_in) * vd;
   const TIN* src = qkv + (size_t)n * in_ld + head_at;
   for (int d = lane; d < width; d += kWave) {
     float v = bias ? bias[head_at + d] : 0.f;
@@ -1339,19 +1474,20 @@ __global__ void rope_norm_store_kernel(
   }
   if (is_q) {
     T* dst = q_out + ((size_t)n * nh + head) * hdp;
-    for (int d = lane; d < hdp; d += kWave) Elem<T>::store(dst + d, d < hd ? vec[d] : 0.f);
+    const int at = (head % maps) * hd;
+    for (int d = lane; d < hdp; d += kWave) Elem<T>::store(dst + d, (d >= at && d < at + hd) ? vec[d - at] : 0.f);
     return;
   }
   const int pos = positions[n];
   const int page = block_tables[(size_t)req_of_token[n] * max_pages + pos / ps];
   const int off = pos % ps;
   if (is_k) {
-    const int kvh = head - nh;
+    const int kvh = (head - nh) / maps, at = ((head - nh) % maps) * hd;
     T* base = k_cache + (size_t)page * ((size_t)nkv * hdp * ps) + (size_t)kvh * hdp * ps;
     for (int d = lane; d < hd; d += kWave)
-      Elem<T>::store(base + ((size_t)(d >> 3) * ps + off) * 8 + (d & 7), vec[d]);
+      Elem<T>::store(base + ((size_t)((at + d) >> 3) * ps + off) * 8 + ((at + d) & 7), vec[d]);
   } else {
-    const int kvh = head - nh - nkv_in;
+    const int kvh = head - nh - nk_in;
     T* base = v_cache + (size_t)page * ((size_t)nkv * vdp * ps) + (size_t)kvh * vdp * ps;
     float* keep = v_keep + ((size_t)n * nkv + kvh) * vd;
     const float lambda = v_mode == 2 ? *v_lambda : 0.f;
@@ -1372,23 +1508,24 @@ TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts,
                               int N, int nh, int nkv_in, int nkv, int hd, int vd, int hdp, int vdp, int rot,
                               int ps, int max_pages, int unit, float eps, int interleaved, float* v_keep,
                               int v_mode, const float* v_lambda, long in_ld, const float* bias, int norm_first,
-                              hipStream_t stream) {
+                              int maps, int v_from_k, hipStream_t stream) {
   if (N <= 0) return 0;
-  if (hdp > kMaxHeadDim || vdp > kMaxHeadDim || hd < 1 || vd < 1 || hdp < hd || vdp < vd || hdp % 8 != 0 ||
+  if (maps < 1 || nh % maps != 0 || (v_from_k && (maps != 1 || vd != hd))) return -1;
+  if (hdp > kMaxHeadDim || vdp > kMaxHeadDim || hd < 1 || vd < 1 || (long)hdp < (long)maps * hd || vdp < vd || hdp % 8 != 0 ||
       vdp % 16 != 0 || ps % 4 != 0 || rot > hd || rot % 2 != 0)
     return -1;
   if (v_mode < 0 || v_mode > 2 || (v_mode != 0 && v_keep == nullptr) || (v_mode == 2 && v_lambda == nullptr)) return -1;
   if (nkv_in != 0 && nkv_in != nkv) return -1;
   if (parts < 1 || (parts > 1 && !in_f32 && dtype != 0)) return -1;
-  if (in_ld < (long)(nh + nkv_in) * hd + (long)nkv_in * vd) return -1;
-  const long pairs = (long)N * (nh + 2 * nkv_in);
+  if (in_ld < ((long)nh + (long)nkv_in * maps) * hd + (v_from_k ? 0L : (long)nkv_in * vd)) return -1;
+  const long pairs = (long)N * (nh + (long)nkv_in * (maps + 1));
   if (pairs > 0x7fffffffL) return -1;
   const unsigned grid = (unsigned)((pairs + kPairsPerBlock - 1) / kPairsPerBlock);
 #define TK_RN(T_, TIN_)                                                                          \
   rope_norm_store_kernel<T_, TIN_><<<grid, kWave * kPairsPerBlock, 0, stream>>>(                 \
       (const TIN_*)qkv, parts, part_stride, q_weight, k_weight, cos_t, sin_t, positions,         \
       req_of_token, block_tables, (T_*)q_out, (T_*)k_cache, (T_*)v_cache, nh, nkv_in, nkv, hd,   \
-      vd, hdp, vdp, rot, ps, max_pages, unit, eps, (int)pairs, interleaved, v_keep, v_mode, v_lambda, in_ld, bias, norm_first)
+      vd, hdp, vdp, rot, ps, max_pages, unit, eps, (int)pairs, interleaved, v_keep, v_mode, v_lambda, in_ld, bias, norm_first, maps, v_from_k)
   if (dtype == 0) TK_RN(float, float);
   else if (in_f32) TK_RN(bf16_t, float);
   else TK_RN(bf16_t, bf16_t);
@@ -1422,6 +1559,8 @@ TK_SLOTS(tk_rope_tables)
 TK_SLOTS(tk_qknorm_rope_store)
 TK_SLOTS(tk_silu_mul)
 TK_SLOTS(tk_add_bias)
+TK_SLOTS(tk_squared_relu)
+TK_SLOTS(tk_map_difference)
 TK_SLOTS(tk_scaled_sum)
 TK_SLOTS(tk_rope_norm_store)
 TK_SLOTS(tk_scale_softcap)

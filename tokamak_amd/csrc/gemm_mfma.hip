@@ -246,7 +246,8 @@ struct RowScale {
   const float* sumsq;  // [slabs][M]: sums of squares of the rows over slabs of columns; nullptr: no scaling
   int slabs;
   float eps;
-  int act;             // the gated form's activation: 0 silu, 1 the tanh form of gelu, 2 the clamped gate
+  int act;             // the gated form's activation: 0 silu, 1 the tanh form of gelu, 2 the clamped gate;
+                       // the plain form's: 0 none, 3 the square of relu
   float limit;         // of the clamped gate
 };
 
@@ -451,6 +452,16 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_stream_kernel(
     }
   }
 
+  if (!GATED && scale.act == 3) {
+#pragma unroll
+    for (int j = 0; j < MT; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float v = fmaxf(acc[j][e], 0.f);
+        acc[j][e] = v * v;
+      }
+  }
+
   // acc[j][e] = C[batch row j*16 + r][column n_wave + kb*4 + e]: four columns a store
   const bool wide = rows_take_wide_stores(C, ldc);
 #pragma unroll
@@ -510,14 +521,16 @@ static int launch_stream(int waves, const void* A, const void* W, void* C, int M
 // waves: 4 or 8 waves a block.  splits: shares of K.  With splits > 1 the output must be float32 and C holds
 // `splits` partial results, split_stride elements apart, that the reader adds.
 // sumsq (may be null), slabs, eps: the rows' scale, see RowScale; then M <= 16.
+// act: 0, or 3 for the square of relu on the result (one split).
 // Returns the number of splits actually used (<= splits; no split is empty), or < 0.
 TK_API int tk_gemm_stream(int out_dtype, const void* A, const void* W, void* C, int M, int N, int K,
                           long lda, long ldw, long ldc, int splits, long split_stride, int waves,
-                          const float* sumsq, int slabs, float eps, hipStream_t stream) {
+                          const float* sumsq, int slabs, float eps, int act, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
+  if ((act != 0 && act != 3) || (act != 0 && splits != 1)) return -1;
   if (M > (waves >= 8 ? 128 : 64) || K < 8 || K % 8 != 0 || lda % 8 != 0 || ldw % 8 != 0 || splits < 1 || splits > 65535) return -1;
   if (sumsq != nullptr && (M > 16 || slabs < 1 || slabs > kRowScaleSlabs || waves >= 6)) return -1;
-  const RowScale scale{sumsq, slabs, eps, 0};
+  const RowScale scale{sumsq, slabs, eps, act, 0.f};
   if (splits > 1 && out_dtype != 0) return -1;
   const int total_chunks = (K + SBK - 1) / SBK;
   const int cps = (total_chunks + splits - 1) / splits;

@@ -60,12 +60,17 @@ template <> struct Vec<bf16_t> {
 //     two largest choice scores (of its one, if it has one expert); only experts of the `keep` groups
 //     with the largest scores can be chosen (the others count as minus infinity).
 //   normalise: the chosen experts' weights are divided by their sum (+ 1e-20); then all times `scale`.
+//   bias (null or float32 [E]): added to the logits before anything else.
+//   scoring 2: the choice is made by the logits, the weights are the softmax over the chosen ones' logits.
+//   gate (null or float32 [N]): the router has one more row, E, whose product with h is the logit of a token's own
+//     gate: gate[n] = its sigmoid (a shared expert's weight, say), from the same walk over h.
 template <typename T>
 __global__ __launch_bounds__(kRouteWaves * kWave) void moe_route_kernel(
     const T* __restrict__ h, const float* __restrict__ router, int* __restrict__ chosen,
-    float* __restrict__ weight, int N, int W, int E, int top, int softmax, const float* __restrict__ correction,
-    int groups, int keep, int normalise, float scale) {
+    float* __restrict__ weight, int N, int W, int E, int top, int scoring, const float* __restrict__ correction,
+    int groups, int keep, int normalise, float scale, const float* __restrict__ bias, float* __restrict__ gate) {
   extern __shared__ float score[];     // [E] scores, [E] choice scores, [groups] group scores
+  const int rows = gate ? E + 1 : E;
   float* choice = score + E;
   float* group_score = choice + E;
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
@@ -73,10 +78,10 @@ __global__ __launch_bounds__(kRouteWaves * kWave) void moe_route_kernel(
   const T* row = h + (size_t)n * W;
   constexpr int V = Vec<T>::N;
   const bool wide = W % V == 0 && (reinterpret_cast<uintptr_t>(h) % 16 == 0) && (reinterpret_cast<uintptr_t>(router) % 16 == 0);
-  for (int e = 2 * wave; e < E; e += 2 * kRouteWaves) {
+  for (int e = 2 * wave; e < rows; e += 2 * kRouteWaves) {
     // the sums run over k in the same order whichever path loads them
     const float* r0 = router + (size_t)e * W;
-    const float* r1 = router + (size_t)min(e + 1, E - 1) * W;
+    const float* r1 = router + (size_t)min(e + 1, rows - 1) * W;
     float a0 = 0.f, a1 = 0.f;
     if (wide) {
       for (int d = lane * V; d < W; d += kWave * V) {
@@ -99,13 +104,21 @@ __global__ __launch_bounds__(kRouteWaves * kWave) void moe_route_kernel(
     a0 = wave_sum(a0);
     a1 = wave_sum(a1);
     if (lane == 0) {
-      score[e] = softmax ? a0 : 1.f / (1.f + expf(-a0));
-      if (e + 1 < E) score[e + 1] = softmax ? a1 : 1.f / (1.f + expf(-a1));
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const float a = u ? a1 : a0;
+        if (e + u < E) {
+          const float z = bias ? a + bias[e + u] : a;
+          score[e + u] = scoring ? z : 1.f / (1.f + expf(-z));
+        } else if (e + u < rows) {
+          gate[n] = 1.f / (1.f + expf(-a));
+        }
+      }
     }
   }
   __syncthreads();
   if (wave != 0) return;
-  if (softmax) {
+  if (scoring == 1) {
     // scores = softmax of the logits over all experts
     float top_z = -INFINITY;
     for (int e = lane; e < E; e += kWave) top_z = fmaxf(top_z, score[e]);
@@ -174,6 +187,21 @@ __global__ __launch_bounds__(kRouteWaves * kWave) void moe_route_kernel(
       choice[at] = -INFINITY;
     }
     wave_lds_sync();
+  }
+  if (scoring == 2) {
+    // (lane 0 has written the chosen logits and reads them back)
+    if (lane == 0) {
+      float* w = weight + (size_t)n * top;
+      float best = w[0];
+      for (int k = 1; k < top; ++k) best = fmaxf(best, w[k]);
+      float sum = 0.f;
+      for (int k = 0; k < top; ++k) {
+        w[k] = expf(w[k] - best);
+        sum += w[k];
+      }
+      for (int k = 0; k < top; ++k) w[k] = w[k] / sum * scale;
+    }
+    return;
   }
   if (lane == 0 && (normalise || scale != 1.f)) {
     const float factor = normalise ? scale / (total + 1e-20f) : scale;
@@ -593,21 +621,23 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void m
 }  // namespace
 
 // h [N, W] in dtype; router [E, W] float32; chosen [N, top] int32 and weight [N, top] float32 out
-// softmax: the scores are the softmax of the logits over all experts, else their sigmoids
+// scoring 0: the scores are the logits' sigmoids; 1: their softmax over all experts; 2: the logits themselves, and
+// the weights the softmax over the chosen ones.  gate: null, or float32 [N] (then router is [E + 1, W]).
 TK_API int tk_moe_route(int dtype, const void* h, const float* router, int* chosen, float* weight, int N,
-                        int W, int E, int top, int softmax, const float* correction, int groups, int keep,
-                        int normalise, float scale, hipStream_t stream) {
+                        int W, int E, int top, int scoring, const float* correction, int groups, int keep,
+                        int normalise, float scale, const float* bias, float* gate, hipStream_t stream) {
   if (N <= 0) return 0;
+  if (scoring < 0 || scoring > 2 || (scoring == 2 && normalise)) return -1;
   if (E < 1 || top < 1 || top > E || W < 1 || (size_t)E * 12 > 60 * 1024) return -1;
   if (groups < 0 || (groups > 0 && (E % groups != 0 || keep < 1 || keep > groups || (long)keep * (E / groups) < top))) return -1;
   const unsigned blocks = (unsigned)N;
   const size_t lds = ((size_t)2 * E + (size_t)groups) * sizeof(float);
   if (dtype == 0)
-    moe_route_kernel<float><<<blocks, kRouteWaves * kWave, lds, stream>>>((const float*)h, router, chosen, weight, N, W, E, top, softmax,
-                                                                         correction, groups, keep, normalise, scale);
+    moe_route_kernel<float><<<blocks, kRouteWaves * kWave, lds, stream>>>((const float*)h, router, chosen, weight, N, W, E, top, scoring,
+                                                                         correction, groups, keep, normalise, scale, bias, gate);
   else
-    moe_route_kernel<bf16_t><<<blocks, kRouteWaves * kWave, lds, stream>>>((const bf16_t*)h, router, chosen, weight, N, W, E, top, softmax,
-                                                                          correction, groups, keep, normalise, scale);
+    moe_route_kernel<bf16_t><<<blocks, kRouteWaves * kWave, lds, stream>>>((const bf16_t*)h, router, chosen, weight, N, W, E, top, scoring,
+                                                                          correction, groups, keep, normalise, scale, bias, gate);
   return launch_status();
 }
 

@@ -291,7 +291,7 @@ def decode_attention_fused(qkv, q_weight, k_weight, cos, sin, k_cache, v_cache, 
 
 def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads, num_kv_heads,
                     head_dim, page_size, scale, window=None, value_dim=None, chunk=None, sinks=None,
-                    keep_first=0) -> None:
+                    keep_first=0, softcap=None) -> None:
     """out[n] = softmax(q[n] . K[0..pos_n] * scale) V, per head, over the pages
     of each token's request.
 
@@ -308,7 +308,8 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
     single tokens (which read a chunk at most) and everything else in the generic kernel.
     ``sinks``: float32 [num_heads], one more term exp(sinks[a]) of head a's denominator, added where
     a row's sums are complete (every kernel has it).  ``keep_first``: with a window, the first so many
-    positions of a sequence stay visible (the window kernels take it).
+    positions of a sequence stay visible (the window kernels take it).  ``softcap`` c: every score becomes
+    c tanh(score / c) before the softmax (every kernel has it).
     bfloat16 at other shapes (key and value sizes that differ or are not 64 or 128, a window), with pages
     of a multiple of 16 tokens: the portions' tiles on the matrix cores with operands straight from the
     pages, or through LDS for the heads of one kv head (``ops.attention_tiles``); tokens that run alone
@@ -332,7 +333,7 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
     if not chunk and value_dim == head_dim and mfma_fits(q.dtype, head_dim, page_size, num_heads // num_kv_heads, window):
         if _paged_attention_mfma(q, k_cache, v_cache, block_tables, batch, work, out, num_heads=num_heads,
                                  num_kv_heads=num_kv_heads, head_dim=head_dim, page_size=page_size, scale=scale,
-                                 sinks=sinks, note=(decode_keys, tile_keys, tile_pairs, kv_token_bytes, flops_per_pair) if profiling else None):
+                                 sinks=sinks, softcap=softcap, note=(decode_keys, tile_keys, tile_pairs, kv_token_bytes, flops_per_pair) if profiling else None):
             return
     tiles = (work.tile_first, work.tile_count, work.num_tiles, work.single, work.num_single)
     if (chunk and work.num_tiles and value_dim == head_dim
@@ -342,13 +343,13 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
         if ops.attention_mfma("tokens", q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token,
                               work.tile_first, work.tile_count, work.num_tiles, out, num_heads=num_heads,
                               num_kv_heads=num_kv_heads, head_dim=head_dim, page_size=page_size, scale=scale, chunk=chunk,
-                              sinks=sinks):
+                              sinks=sinks, softcap=softcap):
             if profiling and work.num_single:
                 ops._note(f"{work.num_single} tokens", decode_keys * kv_token_bytes, decode_keys * flops_per_pair)
             ops.paged_attention_generic(
                 q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token, out,
                 num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim, page_size=page_size,
-                scale=scale, value_dim=value_dim, chunk=chunk, tiles=tiles, only_single=True, sinks=sinks)
+                scale=scale, value_dim=value_dim, chunk=chunk, tiles=tiles, only_single=True, sinks=sinks, softcap=softcap)
             return
     group = num_heads // num_kv_heads
     heads_form = group >= HEADS_FORM_FROM_GROUP and work.num_single > 0
@@ -367,7 +368,7 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
             if not ops.attention_tiles(q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token, work.tile_first,
                                        work.tile_count, work.num_tiles, out, num_heads=num_heads, num_kv_heads=num_kv_heads,
                                        head_dim=head_dim, value_dim=value_dim, page_size=page_size, scale=scale, window=window,
-                                       chunk=chunk, sinks=sinks, keep_first=keep_first):
+                                       chunk=chunk, sinks=sinks, keep_first=keep_first, softcap=softcap):
                 raise ops.KernelError("the tile kernel refused a shape it was asked about")
         if profiling and work.num_single:
             ops._note(f"{work.num_single} tokens {head_dim}/{value_dim}", decode_keys * kv_token_bytes, decode_keys * flops_per_pair)
@@ -375,7 +376,7 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
             ops.attention_heads(q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token, work.single,
                                 work.num_single, out, num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim,
                                 value_dim=value_dim, page_size=page_size, scale=scale, window=window, chunk=chunk, sinks=sinks,
-                                keep_first=keep_first,
+                                keep_first=keep_first, softcap=softcap,
                                 num_splits=heads_form_splits(work.num_single, num_kv_heads, group, work.max_single_len,
                                                              window + keep_first if window else window, chunk))
         elif work.num_single:
@@ -383,7 +384,7 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
                 q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token, out,
                 num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim, page_size=page_size,
                 scale=scale, window=window, value_dim=value_dim, chunk=chunk, tiles=tiles, only_single=True, sinks=sinks,
-                keep_first=keep_first)
+                keep_first=keep_first, softcap=softcap)
         return
     if profiling:
         ops._note(f"{batch.num_tokens} tokens", (decode_keys + tile_keys) * kv_token_bytes,
@@ -391,16 +392,17 @@ def paged_attention(q, k_cache, v_cache, block_tables, batch, out, *, num_heads,
     ops.paged_attention_generic(
         q, k_cache, v_cache, block_tables, batch.positions, batch.req_of_token, out,
         num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim, page_size=page_size,
-        scale=scale, window=window, value_dim=value_dim, chunk=chunk, tiles=tiles, sinks=sinks, keep_first=keep_first)
+        scale=scale, window=window, value_dim=value_dim, chunk=chunk, tiles=tiles, sinks=sinks, keep_first=keep_first,
+        softcap=softcap)
 
 
 def _paged_attention_mfma(q, k_cache, v_cache, block_tables, batch, work, out, *, num_heads, num_kv_heads,
-                          head_dim, page_size, scale, note, sinks=None) -> bool:
+                          head_dim, page_size, scale, note, sinks=None, softcap=None) -> bool:
     """The matrix-core kernels over the step's single tokens and tiles.  False if the
     library has no instance for the shape: nothing of ``out`` counts then, and the caller
     runs the generic kernel over the whole step."""
     common = dict(num_heads=num_heads, num_kv_heads=num_kv_heads, head_dim=head_dim,
-                  page_size=page_size, scale=scale, sinks=sinks)
+                  page_size=page_size, scale=scale, sinks=sinks, softcap=softcap)
     if note is not None:
         decode_keys, tile_keys, tile_pairs, kv_token_bytes, flops_per_pair = note
     if work.num_single:

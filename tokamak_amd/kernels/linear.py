@@ -132,6 +132,31 @@ def _sink_fits(sink: StreamSink, m: int, n: int) -> bool:
             and (g is None or (g.dtype == torch.float32 and g.numel() == n and g.is_contiguous() and g.data_ptr() % 16 == 0)))
 
 
+ACTIVATED_SPLIT_FROM = 3    # shares of K that the product would be cut in from which it is, and the activation runs behind it
+
+
+def activated_linear(x: torch.Tensor, weight: torch.Tensor, activation: str = "squared_relu") -> torch.Tensor:
+    """act(x @ weight^T) -> [M, N]; ``activation`` "squared_relu": max(z, 0)^2.
+
+    bfloat16 with up to 64 rows and enough weight rows to fill the GPU unsplit: in the streaming product's
+    epilogue.  Otherwise the product (in partial sums where that pays), then the activation's kernel, which adds
+    partial sums before it."""
+    from tokamak_amd.kernels import gemm_bf16
+
+    if activation != "squared_relu":
+        raise ValueError(f"unknown activation {activation!r}")
+    m, (n, k) = x.shape[0], weight.shape
+    out = torch.empty((m, n), dtype=x.dtype, device=x.device)
+    if m == 0:
+        return out
+    if (x.dtype == torch.bfloat16 and m <= gemm_bf16.SKINNY_MAX_ROWS and n >= gemm_bf16.STREAM_MIN_ROWS_OUT
+            and gemm_bf16.skinny_fits(x, weight) and gemm_bf16.stream_splits(n, k, m) < ACTIVATED_SPLIT_FROM):
+        ops.gemm_stream(x, weight, out, activation=activation)
+    else:
+        ops.squared_relu(linear(x, weight, allow_partials=True), out)
+    return out
+
+
 def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activation: str = "silu",
                  limit: float | None = None) -> torch.Tensor:
     """act(x @ gate^T) * (x @ up^T) for ``gate_up`` = [gate; up] ([2I, K]) -> [M, I].

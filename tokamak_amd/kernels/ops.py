@@ -172,12 +172,12 @@ _SIGS = {
         "tk_add_rmsnorm": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p,
                            c_void_p, c_int, c_int, c_float, c_int, c_void_p],
         "tk_add_norm2": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_int, c_int, c_long,
-                         c_void_p, c_int, c_int, c_long, c_void_p, c_float, c_void_p,
+                         c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_float, c_void_p,
                          c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_int, c_void_p],
         "tk_add_normed": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_float,
                           c_void_p, c_int, c_int, c_long, c_void_p, c_float, c_void_p, c_float, c_void_p,
                           c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
-        "tk_sigmoid_gate": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p],
+        "tk_sigmoid_gate": [c_int, c_void_p, c_void_p, c_int, c_int, c_long, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
         "tk_rope_tables": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p],
         "tk_qknorm_rope_store": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                  c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
@@ -185,10 +185,12 @@ _SIGS = {
         "tk_rope_norm_store": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                               c_int, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_void_p],
+                               c_int, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
         "tk_scale_softcap": [c_void_p, c_long, c_float, c_float, c_void_p],
         "tk_silu_mul": [c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p],
         "tk_add_bias": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
+        "tk_squared_relu": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_long, c_void_p],
+        "tk_map_difference": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p],
         "tk_scaled_sum": [c_int, c_void_p, c_int, c_int, c_long, c_float, c_void_p, c_int, c_int, c_long, c_float,
                           c_void_p, c_void_p, c_int, c_int, c_void_p],
     },
@@ -224,7 +226,7 @@ _SIGS = {
     },
     "moe": {
         "tk_moe_route": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p,
-                         c_int, c_int, c_int, c_float, c_void_p],
+                         c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p],
         "tk_moe_gate_up": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
                            c_void_p],
         "tk_moe_down": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
@@ -240,7 +242,7 @@ _SIGS = {
     },
     "gemm_mfma": {
         "tk_gemm_stream": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long,
-                           c_long, c_int, c_long, c_int, c_void_p, c_int, c_float, c_void_p],
+                           c_long, c_int, c_long, c_int, c_void_p, c_int, c_float, c_int, c_void_p],
         "tk_gemm_stream_swiglu": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long, c_long,
                                   c_int, c_void_p, c_int, c_float, c_int, c_float, c_void_p],
         "tk_gemm_skinny": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long,
@@ -261,7 +263,7 @@ _SIGS = {
         "tk_paged_attention_generic": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                        c_float, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p,
-                                       c_void_p],
+                                       c_float, c_void_p],
     },
     "latent": {
         "tk_latent_prepare": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -273,14 +275,14 @@ _SIGS = {
     "attention_mfma": {
         "tk_attention_mfma": [c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                               c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
-                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p],
+                              c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_float, c_void_p],
     },
     "attention_tiles": {
         "tk_attention_tiles": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
-                               c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p],
+                               c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p],
         "tk_attention_heads": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
-                               c_void_p, c_void_p],
+                               c_void_p, c_float, c_void_p],
     },
     "ssm": {
         "tk_conv_silu": [c_int, c_void_p, c_int, c_int, c_long, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -488,13 +490,18 @@ def add_rmsnorm(resid: torch.Tensor, delta: torch.Tensor | None, weight: torch.T
 def add_norm2(resid: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | None, weight: torch.Tensor, eps: float,
               out: torch.Tensor, *, center: bool, rows: torch.Tensor | None = None, write_resid: bool = True,
               c: torch.Tensor | None = None, bias: torch.Tensor | None = None, scale: float = 1.0,
-              weight2: torch.Tensor | None = None, out2: torch.Tensor | None = None) -> None:
+              weight2: torch.Tensor | None = None, out2: torch.Tensor | None = None,
+              b_rows: torch.Tensor | None = None, c_rows: torch.Tensor | None = None) -> None:
     """x = resid[row] + scale * (a[row] + b[row] + c[row] + bias), optionally stored back; ``center``: out =
     (x - mean) / sqrt(mean((x - mean)^2) + eps) * weight (a layer norm without a bias), else the RMS norm.
     ``a``, ``b`` and ``c`` are each None, [M, H] in the compute dtype or float32, or float32 partial sums
-    [P, M, H]; ``bias`` is None or float32 [H].  ``weight2`` and ``out2`` (both or neither): the same normalised
+    [P, M, H]; ``bias`` is None or float32 [H].  ``b_rows``, ``c_rows``: None, or float32 [M]: the branch's rows are
+    multiplied by these numbers first.  ``weight2`` and ``out2`` (both or neither): the same normalised
     row times a second weight, for two sub-layers that each norm the same stream."""
-    _gpu(resid, a, b, c, bias, weight, out, rows, weight2, out2)
+    _gpu(resid, a, b, c, bias, weight, out, rows, weight2, out2, b_rows, c_rows)
+    for branch, numbers in ((b, b_rows), (c, c_rows)):
+        _need(numbers is None or (branch is not None and numbers.dtype == torch.float32 and numbers.numel() >= resid.shape[0]),
+              "a branch's row weights are float32, one for every row of the stream")
     h = resid.shape[-1]
     m = out.shape[0] if rows is None else rows.numel()
     _need(resid.dtype == torch.float32 and weight.dtype == torch.float32, "residual and norm weight are float32")
@@ -516,7 +523,7 @@ def add_norm2(resid: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | Non
     _note(f"{m}x{h}", m * h * (4 + (8 if write_resid and adds else 0) + out.element_size() * (2 if out2 is not None else 1))
           + sum(t.element_size() * parts * m * h for t, parts in ((a, na), (b, nb), (c, nc)) if t is not None))
     _check(_fn("elementwise", "tk_add_norm2")(_code(out.dtype), _p(resid), pa, fa, na, sa, pb, fb, nb, sb, pc, fc, nc, sc,
-                                              _p(bias), float(scale), _p(rows), _p(weight), _p(out), _p(weight2), _p(out2),
+                                              _p(b_rows), _p(c_rows), _p(bias), float(scale), _p(rows), _p(weight), _p(out), _p(weight2), _p(out2),
                                               m, h, float(eps), int(bool(write_resid)), int(bool(center)), _stream()),
            "add_norm2")
 
@@ -551,17 +558,20 @@ def add_normed(resid: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | No
         int(bool(write_resid)), _stream()), "add_normed")
 
 
-def sigmoid_gate(x: torch.Tensor, gate: torch.Tensor, col0: int, *, heads: int, vdim: int, vdim_padded: int) -> None:
-    """x[n, head, d] *= sigmoid(gate[n, col0 + head * vdim + d]) in place.  x [N, heads * vdim_padded]; ``gate`` [N, ld]
+def sigmoid_gate(x: torch.Tensor, gate: torch.Tensor, col0: int, *, heads: int, vdim: int, vdim_padded: int,
+                 per_head: bool = False) -> None:
+    """x[n, head, d] *= sigmoid(gate[n, col0 + head * vdim + d]) in place (``per_head``: one number a head instead,
+    gate[n, col0 + head]).  x [N, heads * vdim_padded]; ``gate`` [N, ld]
     in x's dtype or float32, or float32 partial sums [P, N, ld]."""
     _gpu(x, gate)
     n = x.shape[0]
     _need(x.shape == (n, heads * vdim_padded) and 1 <= vdim <= vdim_padded, "the gated heads' shape disagrees")
     pointer, is_f32, parts, stride, ld = _ssm_in(gate, n, x.dtype, "gate")
-    _need(0 <= col0 and col0 + heads * vdim <= ld, "the gate lies outside the projections")
-    _note(f"{n}x{heads * vdim}", n * heads * vdim * (2 * x.element_size() + gate.element_size() * parts))
+    columns = heads * (1 if per_head else vdim)
+    _need(0 <= col0 and col0 + columns <= ld, "the gate lies outside the projections")
+    _note(f"{n}x{heads * vdim}", n * (heads * vdim * 2 * x.element_size() + columns * gate.element_size() * parts))
     _check(_fn("elementwise", "tk_sigmoid_gate")(_code(x.dtype), _p(x), pointer, is_f32, parts, stride, ld, int(col0), n,
-                                                 heads, vdim, vdim_padded, _stream()), "sigmoid_gate")
+                                                 heads, vdim, vdim_padded, int(bool(per_head)), _stream()), "sigmoid_gate")
 
 
 def rope_tables(positions: torch.Tensor, inv_freq: torch.Tensor, cos: torch.Tensor,
@@ -622,7 +632,7 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
                     head_dim: int, value_dim: int, rotary_dim: int, page_size: int, unit_norm: bool, eps: float,
                     store: bool = True, interleaved: bool = False, value_keep: torch.Tensor | None = None,
                     value_mode: int = 0, value_lambda: torch.Tensor | None = None, bias: torch.Tensor | None = None,
-                    norm_first: bool = False) -> None:
+                    norm_first: bool = False, maps: int = 1, values_are_keys: bool = False) -> None:
     """Rotation of the first ``rotary_dim`` dims of every q and k head, then (``unit_norm``) each
     head divided by its root mean square over ``head_dim`` (times a weight, if given); q written to
     q_out, k and v into pages.  Values are ``value_dim`` wide.  ``rotary_dim`` 0: no rotation.
@@ -631,7 +641,11 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
     j + rotary_dim / 2.  ``value_mode`` 1: the values, as projected, are also left in ``value_keep`` (float32
     [N, kv heads * value_dim]); 2: what is cached is (1 - lambda) v + lambda value_keep with lambda =
     ``value_lambda`` (one float32 number on the device).  ``norm_first``: the norm comes before the rotation.
-    ``bias``: float32, one number per q, k and v column, added first.  Rows of ``qkv`` may be longer than
+    ``bias``: float32, one number per q, k and v column, added first.  ``maps``: every head of q and k is that many
+    heads of ``head_dim`` side by side (``num_heads`` counts the maps of all query heads, ``num_kv_heads`` the key
+    heads of the pages, whose keys hold the maps' keys one after the other); each is rotated and normed by itself, and a
+    row of q_out, as wide as a page's key, holds its map's numbers in its map's place and zeros elsewhere.
+    ``values_are_keys``: the input holds no values; a kv head's values are its keys as projected.  Rows of ``qkv`` may be longer than
     q, k and v together (what lies behind them is not read)."""
     _gpu(qkv, q_weight, k_weight, cos, sin, positions, req_of_token, block_tables, q_out, k_cache, v_cache,
          value_keep, value_lambda, bias)
@@ -646,12 +660,14 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
     if value_mode == 2:
         _need(value_lambda is not None and value_lambda.dtype == torch.float32 and value_lambda.numel() == 1,
               "the mixing weight is one float32 number")
-    width = (num_heads + nkv_in) * head_dim + nkv_in * value_dim
+    _need(maps >= 1 and num_heads % maps == 0 and (not values_are_keys or (maps == 1 and value_dim == head_dim and value_mode == 0)),
+          "values that are the keys go with one map and equal sizes; heads come in whole sets of maps")
+    width = (num_heads + nkv_in * maps) * head_dim + (0 if values_are_keys else nkv_in * value_dim)
     ld = qkv.shape[-1]
     _need(ld >= width, f"qkv rows hold {ld} columns, q, k and v are {width}")
     in_f32, parts, stride = _partials(qkv, n, ld, q_out.dtype, "qkv")
     _need(bias is None or (bias.dtype == torch.float32 and bias.numel() >= width), "the bias is float32, one number a column")
-    hdp, vdp = padded_sizes(head_dim, value_dim)
+    hdp, vdp = padded_sizes(maps * head_dim, value_dim)
     _need(q_out.numel() >= n * num_heads * hdp, "q_out too small")
     _need(min(head_dim, value_dim) >= 1 and max(hdp, vdp) <= 512 and page_size % 8 == 0,
           "head sizes are 1 to 512, page_size a multiple of 8")
@@ -670,13 +686,15 @@ def rope_norm_store(qkv: torch.Tensor, q_weight: torch.Tensor | None, k_weight: 
         _need(k_cache.numel() % (num_kv_heads * hdp * page_size) == 0
               and v_cache.numel() % (num_kv_heads * vdp * page_size) == 0
               and k_cache.numel() // hdp == v_cache.numel() // vdp, "cache size is not whole pages")
-    _note(f"{n}x{width}", n * width * (qkv.element_size() * parts + q_out.element_size()))
+    _note(f"{n}x{width}", n * (width * qkv.element_size() * parts
+                               + (num_heads * hdp + nkv_in * (maps * head_dim + value_dim)) * q_out.element_size()))
     _check(_fn("elementwise", "tk_rope_norm_store")(
         _code(q_out.dtype), _p(qkv), in_f32, parts, stride, _p(q_weight), _p(k_weight), _p(cos), _p(sin), _p(positions),
         _p(req_of_token), _p(block_tables), _p(q_out), _p(k_cache), _p(v_cache), n, num_heads,
         nkv_in, num_kv_heads, head_dim, value_dim, hdp, vdp, rotary_dim, page_size, block_tables.shape[1],
         int(bool(unit_norm)), float(eps), int(bool(interleaved)), _p(value_keep if value_mode else None), int(value_mode),
-        _p(value_lambda if value_mode == 2 else None), ld, _p(bias), int(bool(norm_first)), _stream()), "rope_norm_store")
+        _p(value_lambda if value_mode == 2 else None), ld, _p(bias), int(bool(norm_first)), int(maps),
+        int(bool(values_are_keys)), _stream()), "rope_norm_store")
 
 
 def padded_sizes(head_dim: int, value_dim: int) -> tuple[int, int]:
@@ -719,6 +737,33 @@ def add_bias(x: torch.Tensor, bias: torch.Tensor) -> None:
     _need(bias.dtype == torch.float32 and bias.numel() == h, "the bias is float32 [H]")
     _note(f"{n}x{h}", 2 * n * h * x.element_size())
     _check(_fn("elementwise", "tk_add_bias")(_code(x.dtype), _p(x), _p(bias), n, h, _stream()), "add_bias")
+
+
+def squared_relu(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = max(x, 0)^2; ``x`` [N, F] in out's dtype or float32, or float32 partial sums [P, N, F]."""
+    _gpu(x, out)
+    n, f = out.shape
+    _need(out.is_contiguous(), "the output is contiguous")
+    pointer, is_f32, parts, stride = _branch(x, n, f, out.dtype, "x")
+    _note(f"{n}x{f}", n * f * (x.element_size() * parts + out.element_size()))
+    _check(_fn("elementwise", "tk_squared_relu")(_code(out.dtype), pointer, is_f32, parts, stride, _p(out), n * f, _stream()),
+           "squared_relu")
+
+
+def map_difference(attended: torch.Tensor, weight: torch.Tensor, out: torch.Tensor, *, heads: int, vdim: int,
+                   vdim_padded: int, eps: float, scale: float) -> None:
+    """Per token and head, from the outputs a1, a2 of two attention maps: o = a1 - weight a2, out = o / sqrt(mean(o^2)
+    + eps) * scale.  ``attended`` [N, heads * 2 * vdim_padded] (a head's first map, then its second), ``weight`` one
+    float32 number on the device, out [N, heads * vdim]."""
+    _gpu(attended, weight, out)
+    n = out.shape[0]
+    _need(attended.shape == (n, heads * 2 * vdim_padded) and out.shape == (n, heads * vdim) and out.dtype == attended.dtype
+          and attended.is_contiguous() and out.is_contiguous(), "the maps' outputs and their difference disagree in shape")
+    _need(weight.dtype == torch.float32 and weight.numel() == 1, "the second map's weight is one float32 number")
+    _need(1 <= vdim <= vdim_padded <= 512 and vdim_padded % 16 == 0, "value heads of 1 to 512, padded to blocks of 16")
+    _note(f"{n}x{heads}x{vdim}", n * heads * vdim * 3 * out.element_size())
+    _check(_fn("elementwise", "tk_map_difference")(_code(out.dtype), _p(attended), _p(weight), _p(out), n, heads, vdim,
+                                                   vdim_padded, float(eps), float(scale), _stream()), "map_difference")
 
 
 def _branch(t: torch.Tensor | None, rows: int, width: int, dtype: torch.dtype, what: str):
@@ -1247,21 +1292,31 @@ def gated_group_norm(y: torch.Tensor, proj: torch.Tensor, z_col: int, weight: to
 MOE_LDS_BYTES = 96 * 1024      # of a row of activations in float32 that a block of the expert kernels stages
 
 
+ROUTER_SCORES = {"sigmoid": 0, "softmax": 1, "chosen_softmax": 2}
+
+
 def moe_route(h: torch.Tensor, router: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, top: int,
               scoring: str = "sigmoid", *, correction: torch.Tensor | None = None, groups: tuple[int, int] | None = None,
-              normalise: bool = False, scale: float = 1.0) -> None:
+              normalise: bool = False, scale: float = 1.0, bias: torch.Tensor | None = None,
+              gate: torch.Tensor | None = None) -> None:
     """Per token the ``top`` experts with the largest scores, float32 throughout: the scores are
     sigmoid(router . h), or with ``scoring="softmax"`` the softmax of router . h over all experts;
     chosen [N, top] int32 (largest first, the lower index on ties), weight [N, top] float32 their scores.
     ``correction`` (float32 [experts]): the choice goes by score + correction, the weights stay the scores.
     ``groups`` = (count, keep): the experts form ``count`` equal groups of neighbours, a group's score is the
     sum of its two largest choice scores, and only experts of the ``keep`` best groups can be chosen.
-    ``normalise``: the chosen weights are divided by their sum (+ 1e-20); then all are multiplied by ``scale``."""
-    _need(scoring in ("sigmoid", "softmax"), "the router's scores are sigmoids or a softmax")
-    _gpu(h, router, chosen, weight, correction)
+    ``normalise``: the chosen weights are divided by their sum (+ 1e-20); then all are multiplied by ``scale``.
+    ``scoring="chosen_softmax"``: the choice goes by the logits, the weights are the softmax over the chosen ones.
+    ``bias`` (float32 [experts]) is added to the logits first.  ``gate`` (float32 [N]): the router has one row more,
+    behind the experts', and gate[n] = sigmoid of that row's product with h[n]."""
+    _need(scoring in ROUTER_SCORES, f"the router's scores are one of {sorted(ROUTER_SCORES)}")
+    _gpu(h, router, chosen, weight, correction, bias, gate)
     n, w = h.shape
-    e = router.shape[0]
-    _need(router.dtype == torch.float32 and router.shape == (e, w), "the router is float32 [experts, width]")
+    e = router.shape[0] - (1 if gate is not None else 0)
+    _need(router.dtype == torch.float32 and router.shape[1] == w and router.is_contiguous(), "the router is float32 [experts, width]")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == e), "the router's bias is float32 [experts]")
+    _need(gate is None or (gate.dtype == torch.float32 and gate.numel() >= n), "the gates are float32, one a token")
+    _need(not (normalise and scoring == "chosen_softmax"), "a softmax over the chosen experts is normalised already")
     _need(1 <= top <= e and chosen.dtype == torch.int32 and weight.dtype == torch.float32
           and chosen.numel() >= n * top and weight.numel() >= n * top, "lists of chosen experts too small")
     _need(correction is None or (correction.dtype == torch.float32 and correction.numel() == e),
@@ -1271,8 +1326,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, chosen: torch.Tensor, weigh
         _need(count >= 1 and e % count == 0 and 1 <= keep <= count and keep * (e // count) >= top,
               "groups divide the experts evenly and the kept ones hold at least `top` experts")
     _check(_fn("moe", "tk_moe_route")(_code(h.dtype), _p(h), _p(router), _p(chosen), _p(weight), n, w, e, top,
-                                      int(scoring == "softmax"), _p(correction), int(count), int(keep),
-                                      int(bool(normalise)), float(scale), _stream()), "moe_route")
+                                      ROUTER_SCORES[scoring], _p(correction), int(count), int(keep),
+                                      int(bool(normalise)), float(scale), _p(bias), _p(gate), _stream()), "moe_route")
 
 
 def moe_gate_up(h: torch.Tensor, gate_up: torch.Tensor, chosen: torch.Tensor, weight: torch.Tensor, act: torch.Tensor,
@@ -1494,7 +1549,7 @@ def _row_scale(sumsq: torch.Tensor | None, m: int, what: str) -> int:
 
 
 def gemm_stream(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, splits: int = 1, waves: int = 0,
-                sumsq: torch.Tensor | None = None, eps: float = 0.0) -> int:
+                sumsq: torch.Tensor | None = None, eps: float = 0.0, activation: str | None = None) -> int:
     """out = a[M, K] @ w[N, K]^T for M <= 64 with the LDS-staged weight-streaming
     MFMA kernel (``waves``: 4, 6 or 8 waves a block; 0 chooses by the shape).  ``splits == 1``: out is
     [M, N], bfloat16 or float32.  More:
@@ -1502,7 +1557,8 @@ def gemm_stream(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, splits: 
     them were written (the reader adds out[:returned]).  ``sumsq`` [slabs, M] (M <= 16): row m
     of the result is multiplied by rsqrt(sum_s sumsq[s, m] / K + eps): ``a`` is then
     bf16(x * gamma) of an RMSNorm and ``sumsq`` the sums of squares of x's rows over slabs of
-    columns (``gemm_wholek_add`` leaves both)."""
+    columns (``gemm_wholek_add`` leaves both).  ``activation`` "squared_relu" (one split): out = max(., 0)^2."""
+    _need(activation in (None, "squared_relu") and (activation is None or splits == 1), "the product's activation is squared_relu, in one split")
     for t in (a, w):
         _need(t.is_cuda and t.dim() == 2 and t.stride(1) == 1, "gemm operands are 2-D GPU tensors with unit inner stride")
     m, k = a.shape
@@ -1525,7 +1581,7 @@ def gemm_stream(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, *, splits: 
     _note(f"{m}x{n}x{k}", (n * k + m * k) * 2 + splits * m * n * out.element_size(), 2.0 * m * n * k)
     used = _fn("gemm_mfma", "tk_gemm_stream")(_code(out.dtype), _p(a), _p(w), _p(out), m, n, k, a.stride(0),
                                               w.stride(0), ldc, splits, stride, waves,
-                                              _p(sumsq), slabs, float(eps), _stream())
+                                              _p(sumsq), slabs, float(eps), 3 if activation else 0, _stream())
     if used < 1:
         raise KernelError(f"gemm_stream failed with status {used}")
     return used
@@ -1762,7 +1818,8 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
                             window: int | None = None, tiles: tuple | None = None,
                             share_heads: bool | None = None, value_dim: int | None = None,
                             chunk: int | None = None, only_single: bool = False,
-                            sinks: torch.Tensor | None = None, keep_first: int = 0) -> None:
+                            sinks: torch.Tensor | None = None, keep_first: int = 0,
+                            softcap: float | None = None) -> None:
     """Causal attention of each query token over its request's pages.  ``tiles``:
     (tile_first, tile_count, num_tiles, single_tokens, num_single), the step's work lists (tiles
     of up to 16 consecutive tokens of one request, and token rows that run alone), which together
@@ -1774,7 +1831,9 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     (counted from position 0); not together with ``window``.  ``only_single``: the tokens of the tiles
     are left to another kernel.  ``sinks``: float32 [num_heads]; head a's softmax has exp(sinks[a]) as one
     more term of its denominator, with no key and no value.  ``keep_first``: with a window, the first so many
-    positions of a sequence stay visible whatever the distance."""
+    positions of a sequence stay visible whatever the distance.  ``softcap`` c: every score becomes
+    c tanh(score / c) first (the sinks do not)."""
+    _need(softcap is None or softcap > 0, "a soft cap is positive")
     _gpu(q, k_cache, v_cache, block_tables, positions, req_of_token, out, sinks)
     _need(keep_first >= 0 and (keep_first == 0 or window), "kept first positions go with a window")
     _need(sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == num_heads), "sinks are float32 [num_heads]")
@@ -1812,7 +1871,7 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
         _code(q.dtype), _p(q), _p(k_cache), _p(v_cache), _p(block_tables), _p(positions),
         _p(req_of_token), _p(out), n, num_heads, num_kv_heads, head_dim, vd, page_size,
         block_tables.shape[1], float(scale), span, int(keep_first), _p(tile_first), _p(tile_count), num_tiles,
-        _p(single), num_single, -1 if share_heads is None else int(share_heads), _p(sinks), _stream()),
+        _p(single), num_single, -1 if share_heads is None else int(share_heads), _p(sinks), float(softcap or 0.0), _stream()),
         "paged_attention_generic")
 
 
@@ -1823,10 +1882,11 @@ def attention_tiles(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     positions: torch.Tensor, req_of_token: torch.Tensor, tile_first: torch.Tensor,
                     tile_count: torch.Tensor, num_tiles: int, out: torch.Tensor, *, num_heads: int, num_kv_heads: int,
                     head_dim: int, value_dim: int, page_size: int, scale: float, window: int | None = None,
-                    chunk: int | None = None, sinks: torch.Tensor | None = None, keep_first: int = 0) -> bool:
+                    chunk: int | None = None, sinks: torch.Tensor | None = None, keep_first: int = 0,
+                    softcap: float | None = None) -> bool:
     """bf16 attention of the tiles of prompt portions (up to 16 consecutive tokens of one request each) on
     the matrix cores, for keys and values of unlike sizes (up to 512; keys in pieces of 8, values in blocks
-    of 16), any group, a window or chunks, sinks; pages of a multiple of 16 tokens.  Returns False
+    of 16), any group, a window or chunks, sinks, scores under a soft cap; pages of a multiple of 16 tokens.  Returns False
     (nothing launched) for a shape it does not take."""
     _gpu(q, k_cache, v_cache, block_tables, positions, req_of_token, tile_first, tile_count, out, sinks)
     n = positions.numel()
@@ -1846,7 +1906,7 @@ def attention_tiles(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     status = _fn("attention_tiles", "tk_attention_tiles")(
         _p(q), _p(k_cache), _p(v_cache), _p(block_tables), block_tables.shape[1], _p(positions), _p(req_of_token),
         _p(tile_first), _p(tile_count), num_tiles, _p(out), num_heads, num_kv_heads, head_dim, value_dim, page_size,
-        float(scale), span, int(keep_first if window else 0), _p(sinks), _stream())
+        float(scale), span, int(keep_first if window else 0), _p(sinks), float(softcap or 0.0), _stream())
     if status == NOT_INSTANTIATED:
         return False
     _check(status, "attention_tiles")
@@ -1858,7 +1918,7 @@ def attention_mfma(mode: str, q: torch.Tensor, k_cache: torch.Tensor, v_cache: t
                    item_token: torch.Tensor, item_count: torch.Tensor | None, num_items: int,
                    out: torch.Tensor, *, num_heads: int, num_kv_heads: int, head_dim: int,
                    page_size: int, scale: float, split_keys: int = 256, num_splits: int = 1,
-                   chunk: int | None = None, sinks: torch.Tensor | None = None) -> bool:
+                   chunk: int | None = None, sinks: torch.Tensor | None = None, softcap: float | None = None) -> bool:
     """bf16 attention on the matrix cores.  ``mode`` "heads": every item is one
     decode token; "tokens": every item is up to 16 consecutive tokens of one
     request ("tokens_dense": the same, with the kernel variant for tiles that all
@@ -1869,7 +1929,8 @@ def attention_mfma(mode: str, q: torch.Tensor, k_cache: torch.Tensor, v_cache: t
     second kernel merges the pieces (in "heads" mode the sixteen waves of a block share a piece, so
     ``split_keys`` is a multiple of 256).  ``chunk`` ("tokens" and "tokens_dense" without splits): a
     query sees the keys of its own chunk of that many positions only.  ``sinks``: float32
-    [num_heads], one more term exp(sinks[a]) of head a's denominator.  Returns False (nothing
+    [num_heads], one more term exp(sinks[a]) of head a's denominator.  ``softcap`` c: every score becomes
+    c tanh(score / c) first.  Returns False (nothing
     launched) if the shape is not instantiated."""
     _gpu(q, k_cache, v_cache, block_tables, positions, req_of_token, item_token, item_count, out, sinks)
     _need(sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == num_heads), "sinks are float32 [num_heads]")
@@ -1904,7 +1965,7 @@ def attention_mfma(mode: str, q: torch.Tensor, k_cache: torch.Tensor, v_cache: t
         {"heads": 0, "tokens": 1, "tokens_dense": 2, "tokens_wide": 3, "tokens_group": 4}[mode], _p(q), _p(k_cache), _p(v_cache), _p(block_tables),
         block_tables.shape[1], _p(positions), _p(req_of_token), _p(item_token), _p(item_count),
         num_items, _p(out), _p(part_o), _p(part_ml), num_splits, split_keys, num_heads, num_kv_heads,
-        head_dim, page_size, float(scale), int(chunk or 0), _p(sinks), _stream())
+        head_dim, page_size, float(scale), int(chunk or 0), _p(sinks), float(softcap or 0.0), _stream())
     if status == NOT_INSTANTIATED:
         return False
     _check(status, "attention_mfma")
@@ -1921,7 +1982,8 @@ def attention_heads(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     positions: torch.Tensor, req_of_token: torch.Tensor, single: torch.Tensor, num_single: int,
                     out: torch.Tensor, *, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
                     page_size: int, scale: float, num_splits: int, window: int | None = None,
-                    chunk: int | None = None, sinks: torch.Tensor | None = None, keep_first: int = 0) -> None:
+                    chunk: int | None = None, sinks: torch.Tensor | None = None, keep_first: int = 0,
+                    softcap: float | None = None) -> None:
     """bf16 attention of tokens that run alone (``single``: their rows) on the matrix cores, the 16 columns of
     a product being 16 query heads of one kv head, for the shapes of ``attention_tiles``.  Each token's visible
     keys are dealt, 16 at a time, to the four waves of ``num_splits`` blocks; a second kernel merges the waves'
@@ -1946,7 +2008,8 @@ def attention_heads(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _check(_fn("attention_tiles", "tk_attention_heads")(
         _p(q), _p(k_cache), _p(v_cache), _p(block_tables), block_tables.shape[1], _p(positions), _p(req_of_token),
         _p(single), num_single, _p(out), _p(part_o), _p(part_ml), num_splits, num_heads, num_kv_heads, head_dim,
-        value_dim, page_size, float(scale), span, int(keep_first if window else 0), _p(sinks), _stream()), "attention_heads")
+        value_dim, page_size, float(scale), span, int(keep_first if window else 0), _p(sinks), float(softcap or 0.0),
+        _stream()), "attention_heads")
 
 
 FUSED_DECODE_MAX_GROUP = 14   # query heads per kv head the fused decode kernel takes (two waves make the key and value)

@@ -147,7 +147,19 @@ class RotatedUnitAttention(Mixer):
     projection's tensor name plus this suffix), float32; the last one may be left to whoever adds the output to
     the residual stream (``output_bias``, ``forward(defer_bias=True)``).  ``gate_name``: the concatenated heads are
     multiplied by sigmoid(W_g h) ahead of the o projection (W_g: the tensor of this name, [heads * value_dim, H]; one
-    product with q, k and v).
+    product with q, k and v); with ``gate_per_head`` by one number a head (W_g [heads, H]).
+
+    ``softcap`` = c: every score becomes c tanh(score / c) before the softmax.  ``unit_sink``: one is added to the softmax's
+    denominator (a sink of score 0 that is no tensor).  ``values_are_keys``: there is no W_v; a kv head's values are
+    its keys as projected (with their bias), before norm and rotation; ``names``' third name is not used.
+    ``own_keys`` False: the layer has no W_k and W_v (no biases and norm of theirs): it attends, with its own queries,
+    over the keys and values that the layer whose cache slot it is called with has stored.
+    ``maps``: queries and keys come as that many maps a head, side by side: q has heads * maps * head_dim rows, k
+    kv heads * maps * head_dim, laid out head by head; norm and rotation act on each map of a head by itself.  Every
+    map is an attention of its own over the head's values; what becomes of their outputs is the subclass's
+    (``_joined``).  A page holds the maps of a key side by side, and a map's query has zeros in the other maps'
+    places: its score with the whole key is its own map's, and all maps of a kv head's query heads share the keys
+    and values they load.
     """
 
     capturable = True
@@ -159,19 +171,21 @@ class RotatedUnitAttention(Mixer):
                  sink: bool = False, value_mix: str | None = None,
                  extra_names: tuple[str, str] = ("sink", "vmix"), keep_first: int = 0, norm_first: bool = False,
                  norm_names: tuple[str, str] | None = None, bias_suffix: str | None = None,
-                 gate_name: str | None = None) -> None:
+                 gate_name: str | None = None, gate_per_head: bool = False, softcap: float | None = None,
+                 unit_sink: bool = False, values_are_keys: bool = False, own_keys: bool = True, maps: int = 1) -> None:
         super().__init__(dtype=dtype, device=device)
         if num_heads < 1 or num_kv_heads < 1 or num_heads % num_kv_heads:
             raise ValueError(f"num_heads ({num_heads}) must be a multiple of num_kv_heads ({num_kv_heads})")
-        if min(head_dim, value_dim) < 1 or max(ops.padded_sizes(head_dim, value_dim)) > 512:
-            raise ValueError(f"head_dim and value_dim must be 1 to 512; got {head_dim}, {value_dim}")
+        if min(head_dim, value_dim, maps) < 1 or max(ops.padded_sizes(maps * head_dim, value_dim)) > 512:
+            raise ValueError(f"head_dim (times the maps of a head) and value_dim must be 1 to 512; got {head_dim} x {maps}, {value_dim}")
         if chunk is not None and chunk < 1:
             raise ValueError(f"chunk must be >= 1, got {chunk}")
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.head_dim, self.value_dim = int(head_dim), int(value_dim)
         # cache pages, queries and attention outputs are laid out for keys in pieces of 8 channels and
         # values in blocks of 16: sizes that do not fill them are padded with zeros, which add nothing
-        self.key_size, self.value_size = ops.padded_sizes(self.head_dim, self.value_dim)
+        self.maps = int(maps)
+        self.key_size, self.value_size = ops.padded_sizes(self.maps * self.head_dim, self.value_dim)
         self.softmax_scale = float(softmax_scale)
         self.norm_eps = None if norm_eps is None else float(norm_eps)
         self.chunk = None if chunk is None else int(chunk)
@@ -190,10 +204,21 @@ class RotatedUnitAttention(Mixer):
         self.names = tuple(names)
         if (norm_first or norm_names is not None) and norm_eps is None:
             raise ValueError("norm_first and norm_names go with norm_eps")
+        if softcap is not None and not softcap > 0:
+            raise ValueError(f"softcap must be positive, got {softcap}")
+        if sink and unit_sink:
+            raise ValueError("a learned sink or a unit one, not both")
+        if values_are_keys and (value_dim != head_dim or value_mix is not None or maps != 1):
+            raise ValueError("values that are the keys have the keys' size, one map, and are not mixed")
+        if gate_per_head and gate_name is None:
+            raise ValueError("gate_per_head goes with gate_name")
+        self.softcap = None if softcap is None else float(softcap)
+        self.unit_sink, self.values_are_keys, self.own_keys = bool(unit_sink), bool(values_are_keys), bool(own_keys)
+        self.gate_per_head = bool(gate_per_head)
         self.norm_first, self.gate_name = bool(norm_first), gate_name
         self.norm_names = None if norm_names is None else tuple(norm_names)
         self.bias_suffix = None if bias_suffix is None else str(bias_suffix)
-        self.qkv: torch.Tensor | None = None        # with a gate: [q; k; v; gate]
+        self.qkv: torch.Tensor | None = None        # [q; k; v; gate], of these what the layer has
         self.o: torch.Tensor | None = None
         self.qkv_bias: torch.Tensor | None = None
         self.output_bias: torch.Tensor | None = None
@@ -201,45 +226,61 @@ class RotatedUnitAttention(Mixer):
         self.k_norm: torch.Tensor | None = None
 
     def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
-        h, nh, nkv, hd, vd = self.hidden_size, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
-        q, k, v, o = self.names
-        out = {prefix + q: TensorSpec((nh * hd, h)), prefix + k: TensorSpec((nkv * hd, h)),
-               prefix + v: TensorSpec((nkv * vd, h)), prefix + o: TensorSpec((h, nh * vd))}
+        h, nh, vd = self.hidden_size, self.num_heads, self.value_dim
+        o = self.names[3]
+        out = {prefix + name: TensorSpec((rows, h)) for name, rows in self._projections()}
+        out[prefix + o] = TensorSpec((h, nh * vd))
         if self.has_sink:
-            out[prefix + self.extra_names[0]] = TensorSpec((nh,), role="vector")
+            out[prefix + self.extra_names[0]] = TensorSpec((nh * self.maps,), role="vector")
         if self.value_mix is not None:
             out[prefix + self.extra_names[1]] = TensorSpec((), role="vector")
         if self.bias_suffix is not None:
-            for name, width in ((q, nh * hd), (k, nkv * hd), (v, nkv * vd), (o, h)):
+            for name, width in (*self._projections(), (o, h)):
                 out[prefix + name + self.bias_suffix] = TensorSpec((width,), held="float32")
         if self.norm_names is not None:
-            for name in self.norm_names:
-                out[prefix + name] = TensorSpec((hd,), role="vector")
+            for name in self.norm_names[:2 if self.own_keys else 1]:
+                out[prefix + name] = TensorSpec((self.head_dim,), role="vector")
         if self.gate_name is not None:
-            out[prefix + self.gate_name] = TensorSpec((nh * vd, h))
+            out[prefix + self.gate_name] = TensorSpec((nh if self.gate_per_head else nh * vd, h))
+        return out
+
+    def _projections(self) -> list[tuple[str, int]]:
+        """(name, rows) of the query, key and value projections that the layer has."""
+        q, k, v, _ = self.names
+        out = [(q, self.num_heads * self.maps * self.head_dim)]
+        if self.own_keys:
+            out.append((k, self.num_kv_heads * self.maps * self.head_dim))
+            if not self.values_are_keys:
+                out.append((v, self.num_kv_heads * self.value_dim))
         return out
 
     def bind(self, prefix: str, fetch: Fetch) -> None:
-        q, k, v, o = self.names
-        gate = () if self.gate_name is None else (self.gate_name,)
-        self.qkv = torch.cat([fetch(prefix + n) for n in (q, k, v, *gate)], dim=0).contiguous()
+        o = self.names[3]
+        projections = [name for name, _ in self._projections()]
+        gate = [] if self.gate_name is None else [self.gate_name]
+        self.qkv = torch.cat([fetch(prefix + n) for n in projections + gate], dim=0).contiguous()
         self.o = fetch(prefix + o)
         if self.bias_suffix is not None:
-            self.qkv_bias = torch.cat([fetch(prefix + n + self.bias_suffix) for n in (q, k, v)]).contiguous()
+            self.qkv_bias = torch.cat([fetch(prefix + n + self.bias_suffix) for n in projections]).contiguous()
             self.output_bias = fetch(prefix + o + self.bias_suffix)
         if self.norm_names is not None:
-            self.q_norm, self.k_norm = (fetch(prefix + n) for n in self.norm_names)
+            self.q_norm = fetch(prefix + self.norm_names[0])
+            self.k_norm = fetch(prefix + self.norm_names[1]) if self.own_keys else None
         if self.has_sink:
             self.sink = fetch(prefix + self.extra_names[0])
+        elif self.unit_sink:
+            self.sink = torch.zeros((self.num_heads * self.maps,), dtype=torch.float32, device=self.qkv.device)   # exp(0)
         if self.value_mix is not None:
             self.vmix = fetch(prefix + self.extra_names[1]).reshape(1).contiguous()
-        if self.value_size != self.value_dim:
+        if self.value_size != self.value_dim and self.maps == 1:
             # (the attention's output has the padded value size: columns of zeros in between)
             wide = torch.zeros((self.hidden_size, self.num_heads, self.value_size), dtype=self.o.dtype, device=self.o.device)
             wide[:, :, :self.value_dim] = self.o.view(self.hidden_size, self.num_heads, self.value_dim)
             self.o = wide.view(self.hidden_size, self.num_heads * self.value_size).contiguous()
 
-    def cache_request(self) -> CacheRequest:
+    def cache_request(self) -> CacheRequest | None:
+        if not self.own_keys:
+            return None
         return CacheRequest.of(window=self.window, keep_first=self.keep_first, k=self.num_kv_heads * self.key_size,
                                v=self.num_kv_heads * self.value_size)
 
@@ -250,7 +291,7 @@ class RotatedUnitAttention(Mixer):
         check_page_size(page_size)
 
     def pair_flops(self) -> float:
-        return 2.0 * self.num_heads * (self.head_dim + self.value_dim)
+        return 2.0 * self.num_heads * self.maps * (self.head_dim + self.value_dim)
 
     def visible_keys(self, position: int) -> int:
         if self.window is not None:
@@ -275,13 +316,15 @@ class RotatedUnitAttention(Mixer):
 
     def forward(self, h, batch, store, writes_cache: bool = True, position: PositionData | None = None,
                 defer_bias: bool = False):
-        nh, nkv, hd, vd = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
+        nh, nkv, hd, vd = self.num_heads * self.maps, self.num_kv_heads, self.head_dim, self.value_dim
         n = h.shape[0]
-        behind = (nh + nkv) * hd + nkv * vd     # rows of the matrix ahead of the gate's
-        weight = self.qkv if writes_cache else self.qkv[: nh * hd]
+        behind = sum(rows for _, rows in self._projections())     # rows of the matrix ahead of the gate's
+        if writes_cache and not self.own_keys:
+            raise ops.KernelError("a layer without keys of its own attends over another's and stores none")
+        weight = self.qkv if writes_cache or not self.own_keys else self.qkv[: nh * hd]
         qkv = linear(h, weight, allow_partials=True)
         gate, gate_at = qkv, behind
-        if self.gate_name is not None and not writes_cache:
+        if self.gate_name is not None and not writes_cache and self.own_keys:
             gate, gate_at = linear(h, self.qkv[behind:], allow_partials=True), 0
         cos = sin = None
         rotary_dim, interleaved = 0, False
@@ -297,14 +340,16 @@ class RotatedUnitAttention(Mixer):
             store.arrays["v"], num_heads=nh, num_kv_heads=nkv, head_dim=hd, value_dim=vd, rotary_dim=rotary_dim,
             page_size=store.page_size, unit_norm=self.norm_eps is not None, eps=self.norm_eps or 0.0, store=writes_cache,
             interleaved=interleaved, value_keep=kept, value_mode=value_mode, value_lambda=self.vmix, bias=self.qkv_bias,
-            norm_first=self.norm_first)
+            norm_first=self.norm_first, maps=self.maps, values_are_keys=self.values_are_keys)
         attended = torch.empty((n, nh * self.value_size), dtype=h.dtype, device=h.device)
         paged_attention(q, store.arrays["k"], store.arrays["v"], tables, batch, attended, num_heads=nh,
                         num_kv_heads=nkv, head_dim=self.key_size, value_dim=self.value_size, page_size=store.page_size,
                         scale=self.softmax_scale, chunk=self.chunk, window=self.window, sinks=self.sink,
-                        keep_first=self.keep_first)
+                        keep_first=self.keep_first, softcap=self.softcap)
+        attended = self._joined(attended)
         if self.gate_name is not None:
-            ops.sigmoid_gate(attended, gate, gate_at, heads=nh, vdim=vd, vdim_padded=self.value_size)
+            ops.sigmoid_gate(attended, gate, gate_at, heads=self.num_heads, vdim=vd,
+                             vdim_padded=self.value_size if self.maps == 1 else vd, per_head=self.gate_per_head)
         if self.output_bias is None or defer_bias:
             # (a deferred bias: the caller adds ``output_bias`` where it adds the output to the stream)
             return linear(attended, self.o, allow_partials=True)
@@ -313,5 +358,46 @@ class RotatedUnitAttention(Mixer):
         return out
 
 
+    def _joined(self, attended: torch.Tensor) -> torch.Tensor:
+        """The heads' outputs, from those of their maps ([N, heads * maps * value size in blocks of 16]); with several
+        maps [N, heads * value_dim]."""
+        if self.maps != 1:
+            raise NotImplementedError("what becomes of several maps' outputs is a subclass's")
+        return attended
+
+
+class DifferentialAttention(RotatedUnitAttention):
+    """Two attention maps a head over the same values, of which the second is subtracted: with a1 and a2 the maps'
+    outputs and lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + ``difference`` (one number for the layer, from four vectors
+    of ``head_dim``: tensors ``lambda_names``), o = a1 - lambda a2, divided by its root mean square over the head's
+    values (``output_eps`` under the root) and multiplied by 1 - ``difference``; the o projection follows.  Queries,
+    keys, values, their norms and rotation as in ``RotatedUnitAttention`` with two maps."""
+
+    def __init__(self, *, difference: float, output_eps: float,
+                 lambda_names: tuple[str, str, str, str] = ("lq1", "lk1", "lq2", "lk2"), **params) -> None:
+        super().__init__(maps=2, **params)
+        self.difference, self.output_eps = float(difference), float(output_eps)
+        self.lambda_names = tuple(lambda_names)
+        self.second_weight: torch.Tensor | None = None      # lambda, one float32 number on the device
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        out = super().expected_tensors(prefix)
+        out.update({prefix + name: TensorSpec((self.head_dim,), held="float32") for name in self.lambda_names})
+        return out
+
+    def bind(self, prefix: str, fetch: Fetch) -> None:
+        super().bind(prefix, fetch)
+        q1, k1, q2, k2 = (fetch(prefix + name).double() for name in self.lambda_names)
+        weight = torch.exp((q1 * k1).sum()) - torch.exp((q2 * k2).sum()) + self.difference
+        self.second_weight = weight.float().reshape(1).contiguous()
+
+    def _joined(self, attended):
+        out = torch.empty((attended.shape[0], self.num_heads * self.value_dim), dtype=attended.dtype, device=attended.device)
+        ops.map_difference(attended, self.second_weight, out, heads=self.num_heads, vdim=self.value_dim,
+                           vdim_padded=self.value_size, eps=self.output_eps, scale=1.0 - self.difference)
+        return out
+
+
 register_part("mixer", "gqa_attention", GQAAttention)
 register_part("mixer", "rotated_unit_attention", RotatedUnitAttention)
+register_part("mixer", "differential_attention", DifferentialAttention)

@@ -157,7 +157,8 @@ class PositionData:
 class BranchPair:
     """The outputs of up to three sub-layers (or terms of one) that belong to one residual add, not
     yet added to the stream: each [N, H] in the compute dtype or float32, or float32 partial sums
-    [P, N, H]; ``second`` and ``third`` may be None.  ``bias``: None or float32 [H], one more term,
+    [P, N, H]; ``second`` and ``third`` may be None, and may have a float32 number a row ([N], ``second_rows``,
+    ``third_rows``) that multiplies the row.  ``bias``: None or float32 [H], one more term,
     the same for every row.  The norm that reads the stream next forms
     scale * (first + second + third + bias) in float32 and adds it to the stream once."""
 
@@ -166,6 +167,26 @@ class BranchPair:
     third: torch.Tensor | None = None
     bias: torch.Tensor | None = None
     scale: float = 1.0
+    second_rows: torch.Tensor | None = None
+    third_rows: torch.Tensor | None = None
+
+    @classmethod
+    def of(cls, first, *terms, bias=None, scale: float = 1.0) -> "BranchPair":
+        """Of up to three terms, of which the later ones may be ``RowWeighted``."""
+        if len(terms) > 2 or isinstance(first, RowWeighted):
+            raise ValueError("a residual add takes up to three terms, the first one without row weights")
+        values = [t.value if isinstance(t, RowWeighted) else t for t in terms] + [None] * (2 - len(terms))
+        rows = [t.rows if isinstance(t, RowWeighted) else None for t in terms] + [None] * (2 - len(terms))
+        return cls(first, *values, bias=bias, scale=scale, second_rows=rows[0], third_rows=rows[1])
+
+
+@dataclass
+class RowWeighted:
+    """A term of a sub-layer's output whose rows are still to be multiplied by one float32 number each (a token's
+    gate on a whole expert): whoever adds the term to the stream does it."""
+
+    value: torch.Tensor
+    rows: torch.Tensor
 
 
 @dataclass
@@ -243,7 +264,8 @@ class Mixer(Part):
 
 class FeedForward(Part):
     """``forward`` returns the sub-layer's output, or a tuple of up to two terms whose sum it is (a
-    mixture's routed experts and its shared expert): whoever adds the output to the stream adds the terms."""
+    mixture's routed experts and its shared expert, the second possibly ``RowWeighted``): whoever adds the output
+    to the stream adds the terms."""
 
     def forward(self, h: torch.Tensor, batch) -> "torch.Tensor | tuple[torch.Tensor, ...]":
         raise NotImplementedError

@@ -52,7 +52,7 @@ class PreNormBlock(Block):
 
 def _whole(out):
     """A feed-forward's output as one pending sub-layer output (its terms, if it has several, as a pair)."""
-    return BranchPair(*out) if isinstance(out, tuple) else out
+    return BranchPair.of(*out) if isinstance(out, tuple) else out
 
 
 def _normed(norm, resid, pending, consumer):
@@ -125,7 +125,8 @@ class ParallelSublayersBlock(Block):
     its own over the same x: x = x + branch_scale * (mixer(norm(x)) + feed_forward(feed_forward_norm(x)));
     where the two norms agree on everything but their weights one kernel makes both outputs.  The
     feed-forward may be absent: x = x + branch_scale * mixer(h).  A feed-forward may return two terms
-    (routed and shared experts) and leave a bias of its last product to the add (``output_bias``).
+    (routed and shared experts), and it or the mixer may leave a bias of its last product to the add (``output_bias``;
+    the add takes one: with two the mixer adds its own).
     An optional ``position`` part prepares the step's position data for the mixer.
     """
 
@@ -159,15 +160,19 @@ class ParallelSublayersBlock(Block):
     def forward(self, resid, pending, batch, store, writes_cache):
         position = None if self.position is None else self.position.prepare(batch)
         h, h_ff = self._normed(resid, pending)
-        mixed = self.mixer.forward(h, batch, store, writes_cache, position)
+        if getattr(self.feed_forward, "output_bias", None) is None:
+            mixed, bias = _biasless(self.mixer, h, batch, store, writes_cache, position)
+        else:
+            mixed, bias = self.mixer.forward(h, batch, store, writes_cache, position), None
         if self.feed_forward is None:
-            return mixed if self.branch_scale == 1.0 else BranchPair(mixed, scale=self.branch_scale)
-        bias = getattr(self.feed_forward, "output_bias", None)
-        out = self.feed_forward.forward(h_ff, batch, defer_bias=True) if bias is not None else self.feed_forward.forward(h_ff, batch)
+            if bias is None and self.branch_scale == 1.0:
+                return mixed
+            return BranchPair(mixed, bias=bias, scale=self.branch_scale)
+        out, ff_bias = _biasless(self.feed_forward, h_ff, batch)
         terms = out if isinstance(out, tuple) else (out,)
         if len(terms) > 2:
             raise ValueError("a feed-forward hands on two terms at most")
-        return BranchPair(mixed, *terms, bias=bias, scale=self.branch_scale)
+        return BranchPair.of(mixed, *terms, bias=bias if ff_bias is None else ff_bias, scale=self.branch_scale)
 
 
 class PostNormBlock(Block):

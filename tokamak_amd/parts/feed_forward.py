@@ -6,7 +6,7 @@ import torch
 
 from tokamak_amd.config.registry import register_part
 from tokamak_amd.kernels import ops
-from tokamak_amd.kernels.linear import gated_linear, linear
+from tokamak_amd.kernels.linear import activated_linear, gated_linear, linear
 from tokamak_amd.kernels.ops import GATE_ACTIVATIONS
 from tokamak_amd.parts.base import FeedForward, Fetch
 from tokamak_amd.weights.spec import TensorSpec
@@ -83,4 +83,35 @@ class SwiGLU(FeedForward):
         return out
 
 
+class ActivatedFeedForward(FeedForward):
+    """down(act(up(x))), no gate and no biases.  ``activation``: ``"squared_relu"``, max(z, 0)^2."""
+
+    capturable = True
+    replayable = True
+
+    def __init__(self, *, hidden_size: int, intermediate_size: int, dtype, device,
+                 names: tuple[str, str] = ("up_proj.weight", "down_proj.weight"), activation: str = "squared_relu") -> None:
+        super().__init__(dtype=dtype, device=device)
+        if activation != "squared_relu":
+            raise ValueError(f"activation is 'squared_relu', got {activation!r}")
+        self.activation = activation
+        self.hidden_size = int(hidden_size)
+        self.intermediate_size = int(intermediate_size)
+        self.names = tuple(names)       # up, down behind the part's prefix
+        self.up: torch.Tensor | None = None
+        self.down: torch.Tensor | None = None
+
+    def expected_tensors(self, prefix: str) -> dict[str, TensorSpec]:
+        h, i = self.hidden_size, self.intermediate_size
+        up, down = self.names
+        return {prefix + up: TensorSpec((i, h)), prefix + down: TensorSpec((h, i))}
+
+    def bind(self, prefix: str, fetch: Fetch) -> None:
+        self.up, self.down = (fetch(prefix + name) for name in self.names)
+
+    def forward(self, h, batch):
+        return linear(activated_linear(h, self.up, self.activation), self.down, allow_partials=True)
+
+
 register_part("feed_forward", "swiglu", SwiGLU)
+register_part("feed_forward", "activated", ActivatedFeedForward)

@@ -17,6 +17,8 @@ def _normed_sum(pending) -> NormedSum | None:
         return pending
     if not isinstance(pending, BranchPair):
         return NormedSum(pending)
+    if pending.second_rows is not None:
+        raise ops.KernelError("a term with a weight a row is added by a norm, not by a bare reading of the stream")
     if pending.third is not None:
         raise ops.KernelError("a sum of three terms is added by a norm, not by a bare reading of the stream")
     return NormedSum(pending.first, pending.second, bias=pending.bias, first_weight=pending.scale, second_weight=pending.scale)
@@ -102,7 +104,8 @@ class RMSNorm(Norm):
         if isinstance(delta, BranchPair):
             # branches that belong to one residual add: their sum is formed first, then added
             ops.add_norm2(resid, delta.first, delta.second, self.weight, self.eps, out, center=False, rows=rows,
-                          write_resid=write_resid, c=delta.third, bias=delta.bias, scale=delta.scale)
+                          write_resid=write_resid, c=delta.third, bias=delta.bias, scale=delta.scale,
+                          b_rows=delta.second_rows, c_rows=delta.third_rows)
             return out
         ops.add_rmsnorm(resid, delta, self.weight, self.eps, out, rows=rows, write_resid=write_resid)
         return out
@@ -121,7 +124,8 @@ class RMSNorm(Norm):
         out2 = torch.empty_like(out)
         ops.add_norm2(resid, pair.first if pair else None, pair.second if pair else None, self.weight, self.eps, out,
                       center=False, c=pair.third if pair else None, bias=pair.bias if pair else None,
-                      scale=pair.scale if pair else 1.0, weight2=other.weight, out2=out2)
+                      scale=pair.scale if pair else 1.0, weight2=other.weight, out2=out2,
+                      b_rows=pair.second_rows if pair else None, c_rows=pair.third_rows if pair else None)
         return out, out2
 
 
@@ -166,7 +170,8 @@ class LayerNorm(Norm):
         m = resid.shape[0] if rows is None else rows.numel()
         out = torch.empty((m, self.dim), dtype=self.dtype, device=resid.device)
         ops.add_norm2(resid, pair.first, pair.second, self.weight, self.eps, out, center=True, rows=rows,
-                      write_resid=write_resid, c=pair.third, bias=pair.bias, scale=pair.scale)
+                      write_resid=write_resid, c=pair.third, bias=pair.bias, scale=pair.scale,
+                      b_rows=pair.second_rows, c_rows=pair.third_rows)
         return out
 
 

@@ -7,7 +7,7 @@ import torch
 from tokamak_amd.config.registry import register_part
 from tokamak_amd.kernels import ops
 from tokamak_amd.kernels.linear import gated_linear, linear
-from tokamak_amd.parts.base import FeedForward, Fetch
+from tokamak_amd.parts.base import FeedForward, Fetch, RowWeighted
 from tokamak_amd.weights.spec import TensorSpec
 
 
@@ -15,10 +15,12 @@ class RoutedExperts(FeedForward):
     """``num_experts`` feed-forwards down(silu(gate x) * up x) without biases, of which every token
     uses ``top``.
 
-    The router's logits z = W_r h and the scores are float32: s = sigmoid(z), or with
+    The router's logits z = W_r h (+ b, with ``logit_bias``: the tensor of that name) and the scores are float32:
+    s = sigmoid(z), or with
     ``scoring="softmax"`` the softmax of z over all experts; the ``top`` experts
     with the largest scores are chosen (the lower index on a tie) and weighted by their scores
-    as they are, not renormalised.  ``weight_on`` says where a weight w acts: ``"input"``, the
+    as they are, not renormalised.  ``scoring="chosen_softmax"``: the largest logits are chosen and the weights are
+    the softmax over the chosen ones.  ``weight_on`` says where a weight w acts: ``"input"``, the
     expert sees w * h (out = sum expert(w h)), or ``"output"``, out = sum w * expert(h).  On the
     input the kernels use gate(w h) = w gate(h): the weight scales the two first products in
     float32; on the output they use w down(a) = down(w a): the weight scales the activations.  Tensors: router, e<i>.gate, e<i>.up, e<i>.down; an expert's gate and up are held as
@@ -31,7 +33,10 @@ class RoutedExperts(FeedForward):
     are divided by their sum (+ 1e-20).  ``weight_scale``: all weights times this number.
     ``shared_size``: one more expert of that inner size (tensors ``shared.gate``, ``shared.up``,
     ``shared.down``) that every token uses with weight one; ``forward`` then returns two terms, the routed
-    experts' partial sums and the shared expert's output.
+    experts' partial sums and the shared expert's output.  ``shared_gate``: a tensor of that name behind
+    ``shared_prefix`` [1, H]; the shared expert's output is multiplied by the sigmoid of its product with h, one
+    float32 number a token, which the router's kernel forms (its matrix is held as the router's last row) and the
+    residual add applies (``RowWeighted``).
     """
 
     capturable = True
@@ -41,7 +46,8 @@ class RoutedExperts(FeedForward):
                  weight_on: str = "input", scoring: str = "sigmoid", dtype, device,
                  names: tuple[str, str, str, str, str] = ("router", "e{}.", "gate", "up", "down"),
                  correction: str | None = None, groups: tuple[int, int] | None = None, normalise: bool = False,
-                 weight_scale: float = 1.0, shared_size: int | None = None, shared_prefix: str = "shared.") -> None:
+                 weight_scale: float = 1.0, shared_size: int | None = None, shared_prefix: str = "shared.",
+                 logit_bias: str | None = None, shared_gate: str | None = None) -> None:
         super().__init__(dtype=dtype, device=device)
         self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
         self.num_experts, self.top = int(num_experts), int(top)
@@ -49,8 +55,8 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"top ({top}) must be between 1 and the number of experts ({num_experts})")
         if weight_on not in ("input", "output"):
             raise ValueError(f"weight_on is 'input' or 'output', got {weight_on!r}")
-        if scoring not in ("sigmoid", "softmax"):
-            raise ValueError(f"scoring is 'sigmoid' or 'softmax', got {scoring!r}")
+        if scoring not in ops.ROUTER_SCORES:
+            raise ValueError(f"scoring is one of {sorted(ops.ROUTER_SCORES)}, got {scoring!r}")
         self.weight_on, self.scoring = weight_on, scoring
         self.names = tuple(names)
         self.correction_name = None if correction is None else str(correction)
@@ -65,6 +71,10 @@ class RoutedExperts(FeedForward):
         if self.shared_size is not None and self.shared_size < 1:
             raise ValueError(f"shared_size must be >= 1, got {shared_size}")
         self.shared_prefix = str(shared_prefix)
+        if shared_gate is not None and shared_size is None:
+            raise ValueError("a gate on the shared expert goes with a shared expert")
+        self.logit_bias_name, self.shared_gate_name = logit_bias, shared_gate
+        self.logit_bias: torch.Tensor | None = None
         self.router = self.gate_up = self.down = None
         self.correction = self.shared_gate_up = self.shared_down = None
 
@@ -80,6 +90,10 @@ class RoutedExperts(FeedForward):
         if self.shared_size is not None:
             base, s = prefix + self.shared_prefix, self.shared_size
             out.update({base + gate: TensorSpec((s, h)), base + up: TensorSpec((s, h)), base + down: TensorSpec((h, s))})
+            if self.shared_gate_name is not None:
+                out[base + self.shared_gate_name] = TensorSpec((1, h), held="float32")
+        if self.logit_bias_name is not None:
+            out[prefix + self.logit_bias_name] = TensorSpec((self.num_experts,), held="float32")
         return out
 
     def bind(self, prefix: str, fetch: Fetch) -> None:
@@ -94,6 +108,10 @@ class RoutedExperts(FeedForward):
             base = prefix + self.shared_prefix
             self.shared_gate_up = torch.cat([fetch(base + gate), fetch(base + up)], dim=0).contiguous()
             self.shared_down = fetch(base + down)
+            if self.shared_gate_name is not None:
+                self.router = torch.cat([self.router, fetch(base + self.shared_gate_name)], dim=0).contiguous()
+        if self.logit_bias_name is not None:
+            self.logit_bias = fetch(prefix + self.logit_bias_name)
 
     def matrix_share(self, tokens: int) -> tuple[float, float]:
         e, top = self.num_experts, self.top
@@ -107,17 +125,21 @@ class RoutedExperts(FeedForward):
         """Float32 partial sums [top, N, width]: layer k holds every token's k-th chosen expert's output;
         whoever adds the sub-layer's output to the stream sums them in that order.  With a shared expert a
         tuple: those, and the shared expert's output."""
-        routed = self._routed(h)
+        token_gate = None
+        if self.shared_gate_name is not None:
+            token_gate = torch.empty((h.shape[0],), dtype=torch.float32, device=h.device)
+        routed = self._routed(h, token_gate)
         if self.shared_size is None:
             return routed
-        return routed, linear(gated_linear(h, self.shared_gate_up), self.shared_down, allow_partials=True)
+        shared = linear(gated_linear(h, self.shared_gate_up), self.shared_down, allow_partials=True)
+        return routed, shared if token_gate is None else RowWeighted(shared, token_gate)
 
-    def _routed(self, h):
+    def _routed(self, h, token_gate):
         n, top = h.shape[0], self.top
         chosen = torch.empty((n, top), dtype=torch.int32, device=h.device)
         weight = torch.empty((n, top), dtype=torch.float32, device=h.device)
         ops.moe_route(h, self.router, chosen, weight, top, self.scoring, correction=self.correction, groups=self.groups,
-                      normalise=self.normalise, scale=self.weight_scale)
+                      normalise=self.normalise, scale=self.weight_scale, bias=self.logit_bias, gate=token_gate)
         on_output = self.weight_on == "output"
         act = torch.empty((n * top, self.intermediate_size), dtype=h.dtype, device=h.device)
         out = torch.empty((top, n, self.hidden_size), dtype=torch.float32, device=h.device)
