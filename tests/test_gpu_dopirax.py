@@ -354,7 +354,7 @@ def test_router_over_logits_with_a_bias_and_a_gated_shared_expert(dtype, name):
     cfg = model_json([capped(mlp=mlp)], width=width)
     w = random_weights(cfg, seed=r["n"] + r["top"])
     part = built(cfg, 0, w, dtype)["feed_forward"]
-    for rows in (3, 200):
+    for rows in (3, 200) + ((1030,) if name in ("base", "odd") else ()):      # (from 1,024 on several tokens a block)
         h = (2.0 * torch.randn(rows, width, generator=torch.Generator().manual_seed(rows))).to(dtype)
         margins: list = []
         chosen, weight = plain.route(h.double(), double(w), "l0.mlp.", mlp["router"], margins)
@@ -377,6 +377,26 @@ def test_router_over_logits_with_a_bias_and_a_gated_shared_expert(dtype, name):
     if r["shared"] is not None:
         ungated = dict(double(w), **{"l0.mlp.shared.sg": torch.zeros(1, width, dtype=torch.float64)})
         assert float((plain.experts_ff(h.double(), ungated, "l0.mlp.", mlp) - plain.experts_ff(h.double(), double(w), "l0.mlp.", mlp)).abs().max()) > 0.05
+
+
+@BOTH
+@pytest.mark.parametrize("rows", [1, 8, 33])
+def test_gated_product_of_few_weight_rows_is_split(dtype, rows):
+    """A gated product too small to fill the GPU under the gate: split over K, the gate adds the partial sums."""
+    from tokamak_amd.kernels import ops
+    from tokamak_amd.kernels.linear import gated_linear
+
+    g = torch.Generator().manual_seed(rows)
+    k, inter = 4096, 2304
+    w = (torch.randn(2 * inter, k, generator=g) * k ** -0.5).to(dtype)
+    h = torch.randn(rows, k, generator=g).to(dtype)
+    z = h.double() @ w.double().T
+    want = plain.silu(z[:, :inter]) * z[:, inter:]
+    close(gated_linear(h.to(DEV), w.to(DEV)).float().cpu(), want.float(), dtype)
+    parts = torch.stack([0.25 * z, 0.5 * z, 0.125 * z, 0.0625 * z, 0.0625 * z]).float().contiguous().to(DEV)
+    out = torch.empty((rows, inter), dtype=dtype, device=DEV)
+    ops.silu_mul(parts, out)
+    close(out.float().cpu(), want.float(), dtype)
 
 
 # -- whole models -------------------------------------------------------------------

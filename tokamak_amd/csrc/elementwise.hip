@@ -642,6 +642,50 @@ __device__ __forceinline__ float gated_value(float z, float u, int act, float li
   return g / (1.f + expf(-1.702f * g)) * (fminf(fmaxf(u, -limit), limit) + 1.f);
 }
 
+// The gate over float32 partial sums of a split product, four columns a thread: I and part_stride multiples of four.
+template <typename T>
+__global__ __launch_bounds__(256) void silu_mul_parts_kernel(const float* __restrict__ gu, int parts, long part_stride,
+                                                             T* __restrict__ out, int I, size_t total4, int act, float limit) {
+  const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= total4) return;
+  const int per_row = I / 4;
+  const size_t n = idx / per_row;
+  const int i = (int)(idx - n * per_row) * 4;
+  const float* g = gu + n * 2 * I + i;
+  float gv[4] = {0.f, 0.f, 0.f, 0.f}, uv[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int p = 0; p < parts; p += 4) {       // four partial sums of each half in flight, added in split order
+    float4 a[4], b[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (p + k < parts) {
+        a[k] = *reinterpret_cast<const float4*>(g + (size_t)(p + k) * part_stride);
+        b[k] = *reinterpret_cast<const float4*>(g + (size_t)(p + k) * part_stride + I);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (p + k < parts) {
+        gv[0] += a[k].x; gv[1] += a[k].y; gv[2] += a[k].z; gv[3] += a[k].w;
+        uv[0] += b[k].x; uv[1] += b[k].y; uv[2] += b[k].z; uv[3] += b[k].w;
+      }
+    }
+  }
+  Store4<T>::at(out + n * I + i, make_float4(gated_value(gv[0], uv[0], act, limit), gated_value(gv[1], uv[1], act, limit),
+                                             gated_value(gv[2], uv[2], act, limit), gated_value(gv[3], uv[3], act, limit)));
+}
+
+TK_API int tk_silu_mul_parts(int dtype, const float* gu, int parts, long part_stride, void* out, int N, int I, int act,
+                             float limit, hipStream_t stream) {
+  if (N <= 0 || I <= 0) return 0;
+  if (act < 0 || act > 2 || parts < 1 || I % 4 != 0 || part_stride % 4 != 0 || (uintptr_t)gu % 16 != 0 || (uintptr_t)out % 16 != 0)
+    return -1;
+  const size_t total4 = (size_t)N * I / 4;
+  const unsigned blocks = (unsigned)((total4 + 255) / 256);
+  if (dtype == 0) silu_mul_parts_kernel<float><<<blocks, 256, 0, stream>>>(gu, parts, part_stride, (float*)out, I, total4, act, limit);
+  else silu_mul_parts_kernel<bf16_t><<<blocks, 256, 0, stream>>>(gu, parts, part_stride, (bf16_t*)out, I, total4, act, limit);
+  return launch_status();
+}
+
 template <typename T>
 __global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total, int act,
                                 float limit, const float* __restrict__ bias) {
@@ -942,19 +986,17 @@ __device__ __forceinline__ float4 branch_four(const NormBranch& b, size_t idx) {
   if (!b.f32) return Load4<T>::at(reinterpret_cast<const T*>(b.p) + idx);
   const float* f = reinterpret_cast<const float*>(b.p) + idx;
   float4 s = *reinterpret_cast<const float4*>(f);
-  int i = 1;
-  for (; i + 4 <= b.parts; i += 4) {      // four partial sums in flight, added in split order
-    float4 q[4];
+  for (int i = 1; i < b.parts; i += 8) {      // eight partial sums in flight, added in split order
+    float4 q[8];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) q[u] = *reinterpret_cast<const float4*>(f + (size_t)(i + u) * b.stride);
+    for (int u = 0; u < 8; ++u)
+      if (i + u < b.parts) q[u] = *reinterpret_cast<const float4*>(f + (size_t)(i + u) * b.stride);
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      s.x += q[u].x; s.y += q[u].y; s.z += q[u].z; s.w += q[u].w;
+    for (int u = 0; u < 8; ++u) {
+      if (i + u < b.parts) {
+        s.x += q[u].x; s.y += q[u].y; s.z += q[u].z; s.w += q[u].w;
+      }
     }
-  }
-  for (; i < b.parts; ++i) {
-    const float4 q = *reinterpret_cast<const float4*>(f + (size_t)i * b.stride);
-    s.x += q.x; s.y += q.y; s.z += q.z; s.w += q.w;
   }
   return s;
 }
@@ -1410,7 +1452,8 @@ TK_API int tk_sigmoid_gate(int dtype, void* x, const void* gate, int f32, int pa
 // map m at channel m hd).  q_out row `head` then has its hd numbers at channel (head % maps) hd and zeros
 // elsewhere: its score with a page's whole key is the score of its own map.
 // v_from_k: there are no values in the input; a kv head's values are its key as projected (with its bias).
-// One wave per (token, head), four waves a block, each with an LDS row of its own.
+// This form takes any size: one wave per (token, head), four waves a block, each with an LDS row of its own; the
+// next one takes what comes in pieces of eight channels.
 // ---------------------------------------------------------------------------
 template <typename T, typename TIN>
 __global__ void rope_norm_store_kernel(
@@ -1500,6 +1543,250 @@ __global__ void rope_norm_store_kernel(
   }
 }
 
+// The same in pieces of eight channels: a lane owns eight neighbouring channels of a head (head sizes that are
+// multiples of 8, up to 8 LK channels for queries and keys and 8 LV for values; half-split rotations of multiples of
+// 16 dims).  The rotation's partner is in the lane (interleaved pairs) or rot / 16 lanes away.  Blocks of 256 threads:
+// the first `key_blocks` take queries, token by token, and behind them the keys, each head with its tokens in order;
+// the rest take the values likewise, so that neighbouring lanes hold neighbouring tokens of one head and the cache writes
+// fall next to each other; the values of four tokens that fill one quad of a page are exchanged through LDS inside the
+// wave and written as the page's own 16-byte pieces of two dims by four keys (bfloat16).
+struct RopeNormArgs {
+  const float* q_weight;
+  const float* k_weight;
+  const float* cos_t;
+  const float* sin_t;
+  const int* positions;
+  const int* req_of_token;
+  const int* block_tables;
+  const float* bias;
+  float* v_keep;
+  const float* v_lambda;
+  long part_stride, in_ld;
+  int parts, N, nh, nkv_in, nkv, hd, vd, hdp, vdp, rot, ps, max_pages, unit, interleaved, v_mode, norm_first, maps, v_from_k;
+  float eps;
+};
+
+template <typename TIN>
+__device__ __forceinline__ void load_piece(const TIN* src, int parts, long part_stride, const float* bias, float (&x)[8]) {
+  if (bias) {
+    const float4 a = *reinterpret_cast<const float4*>(bias), b = *reinterpret_cast<const float4*>(bias + 4);
+    x[0] = a.x; x[1] = a.y; x[2] = a.z; x[3] = a.w;
+    x[4] = b.x; x[5] = b.y; x[6] = b.z; x[7] = b.w;
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = 0.f;
+  }
+  for (int p = 0; p < parts; p += 4) {      // four partial sums in flight, added in split order
+    float4 a[4], b[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (p + u < parts) {
+        a[u] = Load4<TIN>::at(src + (size_t)(p + u) * part_stride);
+        b[u] = Load4<TIN>::at(src + (size_t)(p + u) * part_stride + 4);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (p + u < parts) {
+        x[0] += a[u].x; x[1] += a[u].y; x[2] += a[u].z; x[3] += a[u].w;
+        x[4] += b[u].x; x[5] += b[u].y; x[6] += b[u].z; x[7] += b[u].w;
+      }
+    }
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ void store_piece(T* p, const float (&x)[8]) {
+  if constexpr (sizeof(T) == 2) {
+    *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]), pack_bf16x2(x[4], x[5]),
+                                              pack_bf16x2(x[6], x[7]));
+  } else {
+    *reinterpret_cast<float4*>(p) = make_float4(x[0], x[1], x[2], x[3]);
+    *reinterpret_cast<float4*>(p + 4) = make_float4(x[4], x[5], x[6], x[7]);
+  }
+}
+
+template <typename T, typename TIN, int LK, int LV>
+__global__ __launch_bounds__(256) void rope_norm_store_vec_kernel(const TIN* __restrict__ in, T* __restrict__ q_out,
+                                                                  T* __restrict__ k_cache, T* __restrict__ v_cache,
+                                                                  RopeNormArgs A, int key_blocks) {
+  __shared__ uint4 s_quad[sizeof(T) == 2 ? 256 : 1];
+  const int nk_in = A.nkv_in * A.maps;
+  if ((int)blockIdx.x < key_blocks) {
+    const unsigned slot = (blockIdx.x * 256u + threadIdx.x) / LK;
+    const unsigned q_pairs = (unsigned)A.N * (unsigned)A.nh;
+    if (slot >= q_pairs + (unsigned)A.N * (unsigned)nk_in) return;     // (whole groups of LK lanes leave together)
+    const int sub = threadIdx.x % LK, d0 = sub * 8;
+    int n, head;
+    if (slot < q_pairs) {
+      n = (int)(slot / (unsigned)A.nh);
+      head = (int)(slot - (unsigned)n * (unsigned)A.nh);
+    } else {
+      const unsigned behind = slot - q_pairs, k = behind / (unsigned)A.N;
+      n = (int)(behind - k * (unsigned)A.N);
+      head = A.nh + (int)k;
+    }
+    const bool is_q = head < A.nh, mine = d0 < A.hd;      // (lanes behind the head's end bring zeros)
+    const size_t at = (size_t)head * A.hd + d0;
+    float x[8];
+    if (mine) {
+      load_piece<TIN>(in + (size_t)n * A.in_ld + at, A.parts, A.part_stride, A.bias ? A.bias + at : nullptr, x);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = 0.f;
+    }
+    auto norm_head = [&]() {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+#pragma unroll
+      for (int m = LK / 2; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, kWave);
+      const float rstd = 1.f / sqrtf(ss / (float)A.hd + A.eps);
+      const float* w = is_q ? A.q_weight : A.k_weight;
+      if (w && mine) {
+        const float4 w0 = *reinterpret_cast<const float4*>(w + d0), w1 = *reinterpret_cast<const float4*>(w + d0 + 4);
+        const float wv[8] = {w0.x, w0.y, w0.z, w0.w, w1.x, w1.y, w1.z, w1.w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = x[e] * rstd * wv[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] *= rstd;
+      }
+    };
+    if (A.unit && A.norm_first) norm_head();
+    const int half = A.rot / 2;
+    if (A.interleaved) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int j = d0 / 2 + e;
+        if (j < half) {
+          const float c = A.cos_t[(size_t)n * half + j], s = A.sin_t[(size_t)n * half + j];
+          const float a = x[2 * e], b = x[2 * e + 1];
+          x[2 * e] = a * c - b * s;
+          x[2 * e + 1] = b * c + a * s;
+        }
+      }
+    } else if (half > 0) {
+      // (half is a multiple of 8: a lane's piece lies wholly in the first half, the second, or behind)
+      const bool first = d0 < half, turns = d0 < A.rot;
+      const int partner = (threadIdx.x & 63) + (first ? half / 8 : turns ? -(half / 8) : 0);
+      float c[8], s[8];
+      if (turns) {
+        const size_t j = (size_t)n * half + (first ? d0 : d0 - half);
+        const float4 c0 = *reinterpret_cast<const float4*>(A.cos_t + j), c1 = *reinterpret_cast<const float4*>(A.cos_t + j + 4);
+        const float4 s0 = *reinterpret_cast<const float4*>(A.sin_t + j), s1 = *reinterpret_cast<const float4*>(A.sin_t + j + 4);
+        c[0] = c0.x; c[1] = c0.y; c[2] = c0.z; c[3] = c0.w; c[4] = c1.x; c[5] = c1.y; c[6] = c1.z; c[7] = c1.w;
+        s[0] = s0.x; s[1] = s0.y; s[2] = s0.z; s[3] = s0.w; s[4] = s1.x; s[5] = s1.y; s[6] = s1.z; s[7] = s1.w;
+      }
+      const float sign = first ? -1.f : 1.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float other = __shfl(x[e], partner, kWave);
+        if (turns) x[e] = x[e] * c[e] + sign * other * s[e];
+      }
+    }
+    if (A.unit && !A.norm_first) norm_head();
+    if (!mine) return;
+    if (is_q) {
+      T* dst = q_out + ((size_t)n * A.nh + head) * A.hdp + d0;
+      const int map = head % A.maps;
+      const float zero[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      for (int m = 0; m < A.maps; ++m) {
+        if (m == map) store_piece<T>(dst + m * A.hd, x);
+        else store_piece<T>(dst + m * A.hd, zero);
+      }
+      return;
+    }
+    const int pos = A.positions[n];
+    const int page = A.block_tables[(size_t)A.req_of_token[n] * A.max_pages + pos / A.ps], off = pos % A.ps;
+    const int kvh = (head - A.nh) / A.maps, piece = ((head - A.nh) % A.maps) * (A.hd / 8) + sub;
+    store_piece<T>(k_cache + (size_t)page * ((size_t)A.nkv * A.hdp * A.ps) + (size_t)kvh * A.hdp * A.ps +
+                       ((size_t)piece * A.ps + off) * 8, x);
+    return;
+  }
+  const unsigned slot = ((blockIdx.x - (unsigned)key_blocks) * 256u + threadIdx.x) / LV;
+  if (slot >= (unsigned)A.N * (unsigned)A.nkv_in) return;
+  const int sub = threadIdx.x % LV, d0 = sub * 8;
+  const int kvh = (int)(slot / (unsigned)A.N), n = (int)(slot - (unsigned)kvh * (unsigned)A.N);
+  const bool mine = d0 < A.vd;
+  const size_t at = A.v_from_k ? (size_t)(A.nh + kvh) * A.hd + d0 : (size_t)(A.nh + nk_in) * A.hd + (size_t)kvh * A.vd + d0;
+  float x[8];
+  if (mine) {
+    load_piece<TIN>(in + (size_t)n * A.in_ld + at, A.parts, A.part_stride, A.bias ? A.bias + at : nullptr, x);
+    if (A.v_mode) {
+      float* keep = A.v_keep + ((size_t)n * A.nkv + kvh) * A.vd + d0;
+      const float lambda = A.v_mode == 2 ? *A.v_lambda : 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        if (A.v_mode == 1) keep[e] = x[e];
+        else x[e] = (1.f - lambda) * x[e] + lambda * keep[e];
+      }
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = 0.f;
+  }
+  const int pos = A.positions[n], req = A.req_of_token[n];
+  const int page = A.block_tables[(size_t)req * A.max_pages + pos / A.ps], off = pos % A.ps;
+  T* base = v_cache + (size_t)page * ((size_t)A.nkv * A.vdp * A.ps) + (size_t)kvh * A.vdp * A.ps;
+  if constexpr (sizeof(T) == 2 && LV <= 16) {
+    // four tokens in a row (a "quad" of this wave) of one request and head that fill one quad of keys in a page?
+    constexpr int QL = 4 * LV;
+    const int lane = threadIdx.x & 63, t = (lane / LV) & 3;
+    const int lead = lane / QL * QL + sub;             // the lane with these dims in the quad's first token
+    const bool fits = n == __shfl(n, lead, kWave) + t && pos == __shfl(pos, lead, kWave) + t &&
+                      req == __shfl(req, lead, kWave) && kvh == __shfl(kvh, lead, kWave) && ((pos - t) & 3) == 0;
+    const unsigned long long all = QL == 64 ? ~0ull : ((1ull << (QL & 63)) - 1) << (lane / QL * QL);
+    if ((__builtin_amdgcn_ballot_w64(fits) & all) == all) {
+      s_quad[threadIdx.x] = make_uint4(pack_bf16x2(x[0], x[1]), pack_bf16x2(x[2], x[3]), pack_bf16x2(x[4], x[5]),
+                                       pack_bf16x2(x[6], x[7]));
+      wave_lds_sync();
+      const unsigned* words = reinterpret_cast<const unsigned*>(s_quad);
+      const int quad0 = (int)threadIdx.x / QL * QL + sub;
+      unsigned r[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) r[k] = words[(quad0 + k * LV) * 4 + t];      // token k: dims d, d + 1
+      const int d = d0 + 2 * t;
+      uint4 piece;      // [dim d: keys 0..3][dim d + 1: keys 0..3]
+      piece.x = (r[0] & 0xffffu) | (r[1] << 16);
+      piece.y = (r[2] & 0xffffu) | (r[3] << 16);
+      piece.z = (r[0] >> 16) | (r[1] & 0xffff0000u);
+      piece.w = (r[2] >> 16) | (r[3] & 0xffff0000u);
+      if (mine) *reinterpret_cast<uint4*>(base + ((size_t)(d >> 4) * (A.ps >> 2) + (off >> 2)) * 64 + (d & 15) * 4) = piece;
+      return;
+    }
+  }
+  if (!mine) return;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int d = d0 + e;
+    Elem<T>::store(base + ((size_t)(d >> 4) * (A.ps >> 2) + (off >> 2)) * 64 + (d & 15) * 4 + (off & 3), x[e]);
+  }
+}
+
+static bool rope_norm_vec_fits(const RopeNormArgs& A, const void* in, const void* q_out, const void* k_cache, const void* v_cache,
+                               int in_bytes) {
+  auto aligned = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  return A.hd % 8 == 0 && A.hd <= 256 && A.hdp == A.maps * A.hd && (A.nkv_in == 0 || (A.vd % 8 == 0 && A.vd <= 256)) &&
+         (A.interleaved || (A.rot / 2) % 8 == 0) && A.in_ld * in_bytes % 16 == 0 && A.part_stride * in_bytes % 16 == 0 &&
+         A.ps % 8 == 0 && aligned(in) && aligned(q_out) && aligned(k_cache) && aligned(v_cache) && aligned(A.cos_t) &&
+         aligned(A.sin_t) && aligned(A.bias) && aligned(A.q_weight) && aligned(A.k_weight);
+}
+
+template <typename T, typename TIN, int LK>
+static void launch_rope_norm_vec(const void* in, void* q_out, void* k_cache, void* v_cache, const RopeNormArgs& A, hipStream_t stream) {
+  const long key_pairs = (long)A.N * (A.nh + (long)A.nkv_in * A.maps), value_pairs = (long)A.N * A.nkv_in;
+  const int lv = A.vd <= 64 ? 8 : A.vd <= 128 ? 16 : 32;
+  const long key_blocks = (key_pairs * LK + 255) / 256, value_blocks = (value_pairs * lv + 255) / 256;
+#define TK_RV(LV_)                                                                                                   \
+  rope_norm_store_vec_kernel<T, TIN, LK, LV_><<<(unsigned)(key_blocks + value_blocks), 256, 0, stream>>>(            \
+      (const TIN*)in, (T*)q_out, (T*)k_cache, (T*)v_cache, A, (int)key_blocks)
+  if (lv == 8) TK_RV(8);
+  else if (lv == 16) TK_RV(16);
+  else TK_RV(32);
+#undef TK_RV
+}
+
 // in_f32: qkv is float32 (possibly `parts` partial sums, part_stride elements apart)
 TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts, long part_stride,
                               const float* q_weight, const float* k_weight, const float* cos_t,
@@ -1520,6 +1807,22 @@ TK_API int tk_rope_norm_store(int dtype, const void* qkv, int in_f32, int parts,
   if (in_ld < ((long)nh + (long)nkv_in * maps) * hd + (v_from_k ? 0L : (long)nkv_in * vd)) return -1;
   const long pairs = (long)N * (nh + (long)nkv_in * (maps + 1));
   if (pairs > 0x7fffffffL) return -1;
+  const RopeNormArgs args{q_weight, k_weight, cos_t, sin_t, positions, req_of_token, block_tables, bias, v_keep, v_lambda,
+                          part_stride, in_ld, parts, N, nh, nkv_in, nkv, hd, vd, hdp, vdp, rot, ps, max_pages, unit,
+                          interleaved, v_mode, norm_first, maps, v_from_k, eps};
+  if (rope_norm_vec_fits(args, qkv, q_out, k_cache, v_cache, dtype == 0 || in_f32 ? 4 : 2) && pairs <= (1L << 26)) {
+#define TK_RK(T_, TIN_)                                                                                        \
+  {                                                                                                            \
+    if (hd <= 64) launch_rope_norm_vec<T_, TIN_, 8>(qkv, q_out, k_cache, v_cache, args, stream);               \
+    else if (hd <= 128) launch_rope_norm_vec<T_, TIN_, 16>(qkv, q_out, k_cache, v_cache, args, stream);        \
+    else launch_rope_norm_vec<T_, TIN_, 32>(qkv, q_out, k_cache, v_cache, args, stream);                       \
+  }
+    if (dtype == 0) TK_RK(float, float)
+    else if (in_f32) TK_RK(bf16_t, float)
+    else TK_RK(bf16_t, bf16_t)
+#undef TK_RK
+    return launch_status();
+  }
   const unsigned grid = (unsigned)((pairs + kPairsPerBlock - 1) / kPairsPerBlock);
 #define TK_RN(T_, TIN_)                                                                          \
   rope_norm_store_kernel<T_, TIN_><<<grid, kWave * kPairsPerBlock, 0, stream>>>(                 \
@@ -1558,6 +1861,7 @@ TK_SLOTS(tk_sigmoid_gate)
 TK_SLOTS(tk_rope_tables)
 TK_SLOTS(tk_qknorm_rope_store)
 TK_SLOTS(tk_silu_mul)
+TK_SLOTS(tk_silu_mul_parts)
 TK_SLOTS(tk_add_bias)
 TK_SLOTS(tk_squared_relu)
 TK_SLOTS(tk_map_difference)

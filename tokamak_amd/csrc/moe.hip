@@ -28,7 +28,8 @@ using namespace tk;
 
 namespace {
 
-constexpr int kRouteWaves = 8;     // waves of a block of the router, which share a token's experts
+constexpr int kRouteWaves = 16;    // waves of a block of the router, which share its tokens' experts
+constexpr int kRouteTokens = 4;    // tokens of a block where there are many
 constexpr int kRows = 8;           // weight rows a wave walks at once
 
 template <typename T> struct Vec;
@@ -52,8 +53,8 @@ template <> struct Vec<bf16_t> {
   }
 };
 
-// A block a token: its waves take the experts two at a time (lanes stride the width), then the
-// first wave picks the largest scores.
+// A block takes TOK tokens: its waves take the router's rows two at a time for all of them (lanes stride the width; the
+// rows are read once a block), then a wave a token picks the largest scores.
 //   correction (null or float32 [E]): the choice is made by score + correction, the weights are the
 //     scores without it.
 //   groups > 0: the experts form `groups` equal groups of neighbours; a group's score is the sum of its
@@ -64,60 +65,94 @@ template <> struct Vec<bf16_t> {
 //   scoring 2: the choice is made by the logits, the weights are the softmax over the chosen ones' logits.
 //   gate (null or float32 [N]): the router has one more row, E, whose product with h is the logit of a token's own
 //     gate: gate[n] = its sigmoid (a shared expert's weight, say), from the same walk over h.
-template <typename T>
+template <typename T, int TOK>
 __global__ __launch_bounds__(kRouteWaves * kWave) void moe_route_kernel(
     const T* __restrict__ h, const float* __restrict__ router, int* __restrict__ chosen,
     float* __restrict__ weight, int N, int W, int E, int top, int scoring, const float* __restrict__ correction,
     int groups, int keep, int normalise, float scale, const float* __restrict__ bias, float* __restrict__ gate) {
-  extern __shared__ float score[];     // [E] scores, [E] choice scores, [groups] group scores
+  // per token: [E] scores, [E] choice scores, [groups] group scores
+  extern __shared__ float route_lds[];
+  const int per_token = 2 * E + groups;
   const int rows = gate ? E + 1 : E;
-  float* choice = score + E;
-  float* group_score = choice + E;
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
-  const int n = blockIdx.x;
-  const T* row = h + (size_t)n * W;
+  const int n0 = blockIdx.x * TOK;
   constexpr int V = Vec<T>::N;
+  constexpr int AHEAD = TOK == 1 ? 4 : 1;      // steps of the walk asked for together (a token alone is bound by round trips)
   const bool wide = W % V == 0 && (reinterpret_cast<uintptr_t>(h) % 16 == 0) && (reinterpret_cast<uintptr_t>(router) % 16 == 0);
-  for (int e = 2 * wave; e < rows; e += 2 * kRouteWaves) {
-    // the sums run over k in the same order whichever path loads them
-    const float* r0 = router + (size_t)e * W;
-    const float* r1 = router + (size_t)min(e + 1, rows - 1) * W;
-    float a0 = 0.f, a1 = 0.f;
-    if (wide) {
-      for (int d = lane * V; d < W; d += kWave * V) {
-        float x[V];
-        Vec<T>::load(row + d, x);
+  const T* row[TOK];
 #pragma unroll
-        for (int i = 0; i < V; i += 4) {
-          const float4 p = *reinterpret_cast<const float4*>(r0 + d + i), q = *reinterpret_cast<const float4*>(r1 + d + i);
-          a0 = fmaf(x[i], p.x, a0); a0 = fmaf(x[i + 1], p.y, a0); a0 = fmaf(x[i + 2], p.z, a0); a0 = fmaf(x[i + 3], p.w, a0);
-          a1 = fmaf(x[i], q.x, a1); a1 = fmaf(x[i + 1], q.y, a1); a1 = fmaf(x[i + 2], q.z, a1); a1 = fmaf(x[i + 3], q.w, a1);
+  for (int t = 0; t < TOK; ++t) row[t] = h + (size_t)min(n0 + t, N - 1) * W;
+  for (int e = 2 * wave; e < rows; e += 2 * kRouteWaves) {
+    // the sums run over k in the same order whichever path loads them, and whatever else the block holds
+    const float* r[2] = {router + (size_t)e * W, router + (size_t)min(e + 1, rows - 1) * W};
+    float a[TOK][2];
+#pragma unroll
+    for (int t = 0; t < TOK; ++t) a[t][0] = a[t][1] = 0.f;
+    if (wide) {
+      for (int d0 = lane * V; d0 < W; d0 += AHEAD * kWave * V) {
+        float4 p[AHEAD][2][V / 4];
+        float x[AHEAD][TOK][V];
+#pragma unroll
+        for (int s = 0; s < AHEAD; ++s) {
+          const int d = d0 + s * kWave * V;
+          if (d < W) {
+#pragma unroll
+            for (int t = 0; t < TOK; ++t) Vec<T>::load(row[t] + d, x[s][t]);
+#pragma unroll
+            for (int u = 0; u < 2; ++u)
+#pragma unroll
+              for (int i = 0; i < V / 4; ++i) p[s][u][i] = *reinterpret_cast<const float4*>(r[u] + d + 4 * i);
+          }
+        }
+#pragma unroll
+        for (int s = 0; s < AHEAD; ++s) {
+          if (d0 + s * kWave * V < W) {
+#pragma unroll
+            for (int t = 0; t < TOK; ++t)
+#pragma unroll
+              for (int u = 0; u < 2; ++u)
+#pragma unroll
+                for (int i = 0; i < V / 4; ++i) {
+                  a[t][u] = fmaf(x[s][t][4 * i], p[s][u][i].x, a[t][u]);
+                  a[t][u] = fmaf(x[s][t][4 * i + 1], p[s][u][i].y, a[t][u]);
+                  a[t][u] = fmaf(x[s][t][4 * i + 2], p[s][u][i].z, a[t][u]);
+                  a[t][u] = fmaf(x[s][t][4 * i + 3], p[s][u][i].w, a[t][u]);
+                }
+          }
         }
       }
     } else {
       for (int d = lane; d < W; d += kWave) {
-        const float x = Elem<T>::load(row + d);
-        a0 = fmaf(x, r0[d], a0);
-        a1 = fmaf(x, r1[d], a1);
+#pragma unroll
+        for (int t = 0; t < TOK; ++t) {
+          const float x = Elem<T>::load(row[t] + d);
+          a[t][0] = fmaf(x, r[0][d], a[t][0]);
+          a[t][1] = fmaf(x, r[1][d], a[t][1]);
+        }
       }
     }
-    a0 = wave_sum(a0);
-    a1 = wave_sum(a1);
-    if (lane == 0) {
+#pragma unroll
+    for (int t = 0; t < TOK; ++t) {
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        const float a = u ? a1 : a0;
-        if (e + u < E) {
-          const float z = bias ? a + bias[e + u] : a;
-          score[e + u] = scoring ? z : 1.f / (1.f + expf(-z));
-        } else if (e + u < rows) {
-          gate[n] = 1.f / (1.f + expf(-a));
+        const float sum = wave_sum(a[t][u]);
+        if (lane != 0) {
+          // (lane 0 writes)
+        } else if (e + u < E) {
+          const float z = bias ? sum + bias[e + u] : sum;
+          route_lds[t * per_token + e + u] = scoring ? z : 1.f / (1.f + expf(-z));
+        } else if (e + u < rows && n0 + t < N) {
+          gate[n0 + t] = 1.f / (1.f + expf(-sum));
         }
       }
     }
   }
   __syncthreads();
-  if (wave != 0) return;
+  if (wave >= TOK || n0 + wave >= N) return;
+  const int n = n0 + wave;
+  float* score = route_lds + wave * per_token;
+  float* choice = score + E;
+  float* group_score = choice + E;
   if (scoring == 1) {
     // scores = softmax of the logits over all experts
     float top_z = -INFINITY;
@@ -630,14 +665,19 @@ TK_API int tk_moe_route(int dtype, const void* h, const float* router, int* chos
   if (scoring < 0 || scoring > 2 || (scoring == 2 && normalise)) return -1;
   if (E < 1 || top < 1 || top > E || W < 1 || (size_t)E * 12 > 60 * 1024) return -1;
   if (groups < 0 || (groups > 0 && (E % groups != 0 || keep < 1 || keep > groups || (long)keep * (E / groups) < top))) return -1;
-  const unsigned blocks = (unsigned)N;
-  const size_t lds = ((size_t)2 * E + (size_t)groups) * sizeof(float);
-  if (dtype == 0)
-    moe_route_kernel<float><<<blocks, kRouteWaves * kWave, lds, stream>>>((const float*)h, router, chosen, weight, N, W, E, top, scoring,
-                                                                         correction, groups, keep, normalise, scale, bias, gate);
-  else
-    moe_route_kernel<bf16_t><<<blocks, kRouteWaves * kWave, lds, stream>>>((const bf16_t*)h, router, chosen, weight, N, W, E, top, scoring,
-                                                                          correction, groups, keep, normalise, scale, bias, gate);
+  // many tokens: several a block, which read the router's rows once (the same sums: a token's result is its own)
+  const int tok = N >= 1024 && ((size_t)2 * E + groups) * kRouteTokens * sizeof(float) <= 60 * 1024 ? kRouteTokens : 1;
+  const unsigned blocks = (unsigned)((N + tok - 1) / tok);
+  const size_t lds = ((size_t)2 * E + (size_t)groups) * tok * sizeof(float);
+#define TK_ROUTE(T_, TOK_)                                                                                      \
+  moe_route_kernel<T_, TOK_><<<blocks, kRouteWaves * kWave, lds, stream>>>((const T_*)h, router, chosen, weight, N, W, E, top, \
+                                                                          scoring, correction, groups, keep, normalise,  \
+                                                                          scale, bias, gate)
+  if (dtype == 0 && tok == 1) TK_ROUTE(float, 1);
+  else if (dtype == 0) TK_ROUTE(float, kRouteTokens);
+  else if (tok == 1) TK_ROUTE(bf16_t, 1);
+  else TK_ROUTE(bf16_t, kRouteTokens);
+#undef TK_ROUTE
   return launch_status();
 }
 

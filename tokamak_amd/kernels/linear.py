@@ -26,6 +26,7 @@ from tokamak_amd.kernels import ops
 # longer K the split product and the norm kernel after it are as fast (measured: the o
 # projection of an 8B-shaped layer gains 2 us, its down projection nothing).
 ADD_INTO_MAX_K = 16 * 256
+GATED_SPLIT_UP_TO_BLOCKS = 160      # blocks of the gated streaming product up to which K is split instead, the gate behind it
 GATED_WHOLEK_MAX_BYTES = 32 << 20   # gate and up together, up to which the whole-K form takes the gated product
 
 
@@ -157,6 +158,22 @@ def activated_linear(x: torch.Tensor, weight: torch.Tensor, activation: str = "s
     return out
 
 
+def _gated_split(x: torch.Tensor, gate_up: torch.Tensor, out: torch.Tensor, activation: str, limit: float | None) -> bool:
+    """The gated product of few rows as a product split over K and a gate that adds the partial sums.  The gated
+    streaming kernel cannot split K under the gate: a matrix of few rows (a shared expert: 8,192 of 4,096, 128 blocks) leaves
+    half of the CUs idle and takes 24 us, split 19."""
+    from tokamak_amd.kernels import gemm_bf16
+
+    m, (n, k) = x.shape[0], gate_up.shape
+    blocks = -(-n // (16 * ops.stream_waves(m, k, True, n // 2)))
+    splits = gemm_bf16.stream_splits(n, k, m)
+    if blocks > GATED_SPLIT_UP_TO_BLOCKS or splits < 3 or n % 8:
+        return False
+    parts = torch.empty((splits, m, n), dtype=torch.float32, device=x.device)
+    ops.silu_mul(parts[:ops.gemm_stream(x, gate_up, parts, splits=splits)], out, activation, limit=limit)
+    return True
+
+
 def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activation: str = "silu",
                  limit: float | None = None) -> torch.Tensor:
     """act(x @ gate^T) * (x @ up^T) for ``gate_up`` = [gate; up] ([2I, K]) -> [M, I].
@@ -175,7 +192,8 @@ def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activati
         from tokamak_amd.kernels import gemm_bf16
 
         if x.dtype == torch.bfloat16 and m <= 64 and gemm_bf16.skinny_fits(x, gate_up):
-            ops.gemm_stream_swiglu(x, gate_up, out, activation=activation, limit=limit)
+            if not _gated_split(x, gate_up, out, activation, limit):
+                ops.gemm_stream_swiglu(x, gate_up, out, activation=activation, limit=limit)
         else:
             ops.silu_mul(linear(x, gate_up), out, activation, limit=limit)
         return out
@@ -203,7 +221,7 @@ def gated_linear(x: torch.Tensor | DeferredNorm, gate_up: torch.Tensor, activati
         if gemm_bf16.skinny_fits(x, gate_up):
             if small and _few_rows_fit(m, x, gate_up, ops.WHOLEK_MAX_ROWS):
                 ops.gemm_wholek(x, gate_up, out, gated=True)
-            else:
+            elif small or not _gated_split(x, gate_up, out, activation, limit):
                 ops.gemm_stream_swiglu(x, gate_up, out)
             return out
     ops.silu_mul(linear(x, gate_up), out)

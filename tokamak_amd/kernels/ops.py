@@ -188,6 +188,7 @@ _SIGS = {
                                c_int, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
         "tk_scale_softcap": [c_void_p, c_long, c_float, c_float, c_void_p],
         "tk_silu_mul": [c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p],
+        "tk_silu_mul_parts": [c_int, c_void_p, c_int, c_long, c_void_p, c_int, c_int, c_int, c_float, c_void_p],
         "tk_add_bias": [c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
         "tk_squared_relu": [c_int, c_void_p, c_int, c_int, c_long, c_void_p, c_long, c_void_p],
         "tk_map_difference": [c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p],
@@ -718,9 +719,18 @@ def silu_mul(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu",
              limit: float | None = None) -> None:
     """out[n, i] = act(gate_up[n, i]) * gate_up[n, I + i]; act is silu, or the tanh form of gelu.  ``bias``:
     float32 [2 I], added to both halves before the activation.  "clamped": with g = min(gate_up[n, i], limit) and
-    u = clamp(gate_up[n, I + i], -limit, limit), out = g sigmoid(1.702 g) (u + 1)."""
+    u = clamp(gate_up[n, I + i], -limit, limit), out = g sigmoid(1.702 g) (u + 1).  ``gate_up`` [N, 2 I] in out's
+    dtype, or (without a bias, I a multiple of 4) float32 partial sums [P, N, 2 I]."""
     _need((activation == "clamped") == (limit is not None), "a limit goes with the clamped gate")
     _gpu(gate_up, out, bias)
+    if gate_up.dim() == 3:
+        parts, n, two_i = gate_up.shape
+        _need(bias is None and gate_up.dtype == torch.float32 and two_i % 8 == 0 and out.shape == (n, two_i // 2)
+              and out.is_contiguous() and gate_up[0].is_contiguous() and activation in GATE_ACTIVATIONS, "silu_mul shapes disagree")
+        _note(f"{n}x{two_i // 2}", n * two_i * (4 * parts + 0.5 * out.element_size()))
+        _check(_fn("elementwise", "tk_silu_mul_parts")(_code(out.dtype), _p(gate_up), parts, gate_up.stride(0), _p(out), n, two_i // 2,
+                                                       GATE_ACTIVATIONS[activation], float(limit or 0.0), _stream()), "silu_mul_parts")
+        return
     _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == gate_up.shape[1]), "the bias is float32 [2 I]")
     n, two_i = gate_up.shape
     _need(two_i % 2 == 0 and out.shape == (n, two_i // 2) and out.dtype == gate_up.dtype, "silu_mul shapes disagree")
